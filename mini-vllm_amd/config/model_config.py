@@ -1257,3 +1257,259 @@ class FuranexConfig(ModelConfig):
         if self.max_position_embeddings != (1 << 24):
             d["max_position_embeddings"] = self.max_position_embeddings
         return d
+
+
+# ---------------------------------------------------------------------------------------
+# Sorulix
+# ---------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class SorulixAttention:
+    """The softmax side of a "parallel" layer. ``q_temp`` = (coef, every) or None; ``softcap`` None: scores are not capped."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: Optional[float] = None
+    q_temp: Optional[Tuple[float, int]] = None
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+                             "softcap": self.softcap,
+                             "q_temp": None if self.q_temp is None else {"coef": self.q_temp[0], "every": self.q_temp[1]}}
+        return {k: v for k, v in d.items() if v is not None and v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SorulixLinear:
+    """The linear-attention side of a "parallel" layer, with one decay for each head."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: Tuple[float, ...] = ()
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "decay": list(self.decay)}
+        return {k: v for k, v in d.items() if v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SorulixDelta:
+    """A "channel_delta" mixer; ``decay_rank`` and ``gate_rank`` are the widths between the two matrices of its low-rank
+    projections (the stored tensors state them; the keys may be left out of config.json)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    decay_rank: int = UNSTATED
+    gate_rank: int = UNSTATED
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "conv": self.conv,
+             "decay_rank": self.decay_rank, "gate_rank": self.gate_rank}
+        return {k: v for k, v in d.items() if v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SorulixLayer:
+    """``left`` and ``right`` for a "parallel" layer, ``delta`` for a "channel_delta" layer. ``ff`` is the width of the
+    feed-forward, None for a layer without one; ``limit`` its clamp."""
+    type: str
+    left: Optional[SorulixAttention] = None
+    right: Optional[SorulixLinear] = None
+    delta: Optional[SorulixDelta] = None
+    ff: Optional[int] = None
+    limit: float = 0.0
+
+    def to_dict(self) -> Dict[str, Any]:
+        mixer = self.delta.to_dict() if self.type == "channel_delta" else {"left": self.left.to_dict(), "right": self.right.to_dict()}
+        mlp = None
+        if self.ff is not None:
+            mlp = {"kind": "dense", "limit": self.limit}
+            if self.ff != UNSTATED:
+                mlp["ff"] = self.ff
+        return {"type": self.type, "mixer": mixer, "mlp": mlp}
+
+
+@dataclass(frozen=True)
+class SorulixConfig(ModelConfig):
+    """Sorulix: a pre-norm decoder whose ``layers`` are listed one by one; each has a mixer (``type``: "parallel", softmax
+    attention beside linear attention with constant decays, or "channel_delta", the gated delta rule with a decay per
+    key channel) and a clamped gated feed-forward or none. ``loop`` = (start, stop, times): layers start .. stop - 1 run
+    ``times`` times in a row. The output head is the embedding's table. Keys: ``vocab``, ``width``, ``layers``, ``loop``,
+    ``norm.eps``. Sizes that config.json leaves out are UNSTATED until ``completed`` fills them in from the stored
+    tensors' shapes."""
+
+    architecture: ClassVar[str] = "Sorulix"
+
+    vocab_size: int = UNSTATED
+    hidden_size: int = UNSTATED
+    layers: Tuple[SorulixLayer, ...] = ()
+    loop: Optional[Tuple[int, int, int]] = None
+    norm_eps: float = 1e-6
+    max_position_embeddings: int = 1 << 24
+    dtype: str = "bfloat16"
+    eos_token_ids: Tuple[int, ...] = ()
+
+    @staticmethod
+    def _left(m: Dict[str, Any], mw: str) -> SorulixAttention:
+        cap = m.get("softcap")
+        temp = _section(m, "q_temp", mw, optional=True)
+        q_temp = None
+        if temp is not None:
+            every = _require(temp, "every", float, mw + ".q_temp")
+            if every < 1 or every != int(every):
+                raise ConfigError(f"{mw}.q_temp: every must be a whole number >= 1, got {every}")
+            q_temp = (_require(temp, "coef", float, mw + ".q_temp"), int(every))
+        return SorulixAttention(heads=_require(m, "heads", int, mw), kv_heads=_size(m, "kv_heads", mw), dim=_size(m, "dim", mw),
+                                vdim=_size(m, "vdim", mw), scale=_require(m, "scale", float, mw),
+                                softcap=None if cap is None else _typed(cap, "softcap", float, mw), q_temp=q_temp)
+
+    @staticmethod
+    def _right(m: Dict[str, Any], mw: str) -> SorulixLinear:
+        decay = m.get("decay")
+        if not isinstance(decay, (list, tuple)) or not decay:
+            raise ConfigError(f"{mw}: 'decay' must list one number for each head")
+        decays = tuple(_typed(v, "decay", float, mw) for v in decay)
+        heads = _size(m, "heads", mw)
+        return SorulixLinear(heads=len(decays) if heads == UNSTATED else heads, dim=_size(m, "dim", mw), vdim=_size(m, "vdim", mw),
+                             decay=decays)
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any], where: str = "config.json") -> "SorulixConfig":
+        raw_layers = d.get("layers")
+        if not isinstance(raw_layers, (list, tuple)) or not raw_layers:
+            raise ConfigError(f"{where}: 'layers' must be a non-empty list")
+        layers = []
+        for i, entry in enumerate(raw_layers):
+            lw = f"{where}: layers[{i}]"
+            if not isinstance(entry, dict):
+                raise ConfigError(f"{lw} must be an object")
+            kind = entry.get("type")
+            m, mw = _section(entry, "mixer", lw), lw + ".mixer"
+            left = right = delta = None
+            if kind == "parallel":
+                left = cls._left(_section(m, "left", mw), mw + ".left")
+                right = cls._right(_section(m, "right", mw), mw + ".right")
+            elif kind == "channel_delta":
+                delta = SorulixDelta(heads=_size(m, "heads", mw), kv_heads=_size(m, "kv_heads", mw), dim=_size(m, "dim", mw),
+                                     vdim=_size(m, "vdim", mw), conv=_size(m, "conv", mw), decay_rank=_size(m, "decay_rank", mw),
+                                     gate_rank=_size(m, "gate_rank", mw))
+            else:
+                raise ConfigError(f"{lw}: layer type {kind!r} is not supported (parallel, channel_delta)")
+            mlp = _section(entry, "mlp", lw, optional=True)
+            ff, limit = None, 0.0
+            if mlp is not None:
+                pw = lw + ".mlp"
+                if mlp.get("kind", "dense") != "dense":
+                    raise ConfigError(f"{pw}: kind {mlp.get('kind')!r} is not supported (dense)")
+                ff, limit = _size(mlp, "ff", pw), _require(mlp, "limit", float, pw)
+            layers.append(SorulixLayer(type=kind, left=left, right=right, delta=delta, ff=ff, limit=limit))
+        loop = _section(d, "loop", where, optional=True)
+        runs = None
+        if loop is not None:
+            runs = tuple(_require(loop, key, int, where + ".loop") for key in ("start", "stop", "times"))
+        dtype = d.get("dtype", d.get("torch_dtype", "bfloat16")) or "bfloat16"
+        if str(dtype) not in _DTYPE_NAMES:
+            raise ConfigError(f"{where}: unknown dtype {dtype!r}")
+        eos = d.get("eos_token_id")
+        eos_ids: Tuple[int, ...] = ()
+        if isinstance(eos, int) and not isinstance(eos, bool):
+            eos_ids = (eos,)
+        elif isinstance(eos, (list, tuple)) and all(isinstance(e, int) for e in eos):
+            eos_ids = tuple(eos)
+        elif eos is not None:
+            raise ConfigError(f"{where}: eos_token_id must be an integer or a list of integers, got {eos!r}")
+        max_pos = d.get("max_position_embeddings")
+        cfg = cls(
+            vocab_size=_size(d, "vocab", where), hidden_size=_size(d, "width", where), layers=tuple(layers), loop=runs,
+            norm_eps=_require(_section(d, "norm", where), "eps", float, where + ".norm"),
+            max_position_embeddings=(1 << 24) if max_pos is None else _typed(max_pos, "max_position_embeddings", int, where),
+            dtype=_DTYPE_NAMES[str(dtype)],
+            eos_token_ids=eos_ids,
+        )
+        cfg.validate(where)
+        return cfg
+
+    def completed(self, sizes=None, where: str = "config") -> "SorulixConfig":
+        """The configuration with nothing UNSTATED. ``sizes(name) -> shape or None`` looks a stored tensor's shape up."""
+        import dataclasses
+        sizes = sizes or (lambda name: None)
+
+        def need(value: int, name: str, axis: int, what: str, per: int = 1, default: Optional[int] = None) -> int:
+            if value != UNSTATED:
+                return value
+            shape = sizes(name)
+            if shape is not None and len(shape) > axis and shape[axis] % per == 0:
+                return int(shape[axis]) // per
+            if default is not None:
+                return default
+            raise ConfigError(f"{where}: {what} is stated neither in config.json nor by a stored tensor's shape")
+
+        layers = []
+        for i, l in enumerate(self.layers):
+            p, lw = f"l{i}.mix.", f"layers[{i}]"
+            if l.type == "parallel":
+                a, b = l.left, l.right
+                dim = need(a.dim, p + "left.q", 0, lw + ".left.dim", a.heads)
+                kv = need(a.kv_heads, p + "left.k", 0, lw + ".left.kv_heads", dim, a.heads)
+                a = dataclasses.replace(a, dim=dim, kv_heads=kv, vdim=need(a.vdim, p + "left.v", 0, lw + ".left.vdim", kv, dim))
+                b_dim = need(b.dim, p + "right.q", 0, lw + ".right.dim", b.heads)
+                b = dataclasses.replace(b, dim=b_dim, vdim=need(b.vdim, p + "right.v", 0, lw + ".right.vdim", b.heads, b_dim))
+                l = dataclasses.replace(l, left=a, right=b)
+            else:
+                m = l.delta
+                heads = need(m.heads, p + "A_log", 0, lw + ".heads")
+                dim = need(m.dim, p + "dt_bias", 0, lw + ".dim", heads)
+                l = dataclasses.replace(l, delta=SorulixDelta(
+                    heads=heads, dim=dim, kv_heads=need(m.kv_heads, p + "q", 0, lw + ".kv_heads", dim, heads),
+                    vdim=need(m.vdim, p + "norm", 0, lw + ".vdim", 1, dim), conv=need(m.conv, p + "q.conv", 1, lw + ".conv"),
+                    decay_rank=need(m.decay_rank, p + "a1", 0, lw + ".decay_rank"),
+                    gate_rank=need(m.gate_rank, p + "g1", 0, lw + ".gate_rank")))
+            if l.ff is not None:
+                l = dataclasses.replace(l, ff=need(l.ff, f"l{i}.mlp.gate", 0, lw + ".mlp.ff"))
+            layers.append(l)
+        done = dataclasses.replace(self, vocab_size=need(self.vocab_size, "embed", 0, "vocab"),
+                                   hidden_size=need(self.hidden_size, "embed", 1, "width"), layers=tuple(layers))
+        done.validate(where)
+        return done
+
+    def validate(self, where: str = "config") -> None:
+        positive = lambda *values: all(v == UNSTATED or v > 0 for v in values)
+        if not positive(self.vocab_size, self.hidden_size):
+            raise ConfigError(f"{where}: vocab and width must be positive")
+        if self.norm_eps <= 0:
+            raise ConfigError(f"{where}: norm.eps must be positive, got {self.norm_eps}")
+        if self.loop is not None:
+            start, stop, times = self.loop
+            if not (0 <= start < stop <= len(self.layers)) or times < 1:
+                raise ConfigError(f"{where}: loop {self.loop} does not name a run of the {len(self.layers)} layers and a count >= 1")
+        for i, l in enumerate(self.layers):
+            lw = f"{where}: layers[{i}]"
+            for part in (l.left, l.delta):
+                if part is not None and (not positive(part.heads, part.kv_heads, part.dim, part.vdim) or (
+                        UNSTATED not in (part.heads, part.kv_heads) and part.heads % part.kv_heads)):
+                    raise ConfigError(f"{lw}: sizes must be positive, and {part.heads} heads a multiple of {part.kv_heads} kv_heads")
+            if l.left is not None and (not l.left.scale > 0 or (l.left.softcap is not None and not l.left.softcap > 0)):
+                raise ConfigError(f"{lw}: scale and softcap must be positive")
+            if l.right is not None and (not positive(l.right.heads, l.right.dim, l.right.vdim) or len(l.right.decay) != l.right.heads):
+                raise ConfigError(f"{lw}: the linear side needs positive sizes and one decay for each of its {l.right.heads} heads")
+            if l.delta is not None and not positive(l.delta.conv, l.delta.decay_rank, l.delta.gate_rank):
+                raise ConfigError(f"{lw}: taps and ranks must be positive")
+            if l.ff is not None and (not positive(l.ff) or not l.limit > 0):
+                raise ConfigError(f"{lw}: the feed-forward's width and limit must be positive")
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {"architecture": self.architecture, "layers": [l.to_dict() for l in self.layers],
+                             "norm": {"eps": self.norm_eps}, "torch_dtype": self.dtype}
+        for key, value in (("vocab", self.vocab_size), ("width", self.hidden_size)):
+            if value != UNSTATED:
+                d[key] = value
+        if self.loop is not None:
+            d["loop"] = dict(zip(("start", "stop", "times"), self.loop))
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids) if len(self.eos_token_ids) > 1 else self.eos_token_ids[0]
+        if self.max_position_embeddings != (1 << 24):
+            d["max_position_embeddings"] = self.max_position_embeddings
+        return d

@@ -30,12 +30,14 @@ def named_shapes() -> Dict[str, Dict[str, Any]]:
     shapes["dutilix-tiny"] = dutilix_tiny_shape()
     shapes["zedudra-tiny"] = zedudra_tiny_shape()
     shapes["furanex-tiny"] = furanex_tiny_shape()
+    shapes["sorulix-tiny"] = sorulix_tiny_shape()
     for name in QWEN3_SHAPES:
         if name != "tiny":
             shapes[f"bolapel-{name}"] = bolapel_shape(name)
             shapes[f"dutilix-{name}"] = dutilix_shape(name)
             shapes[f"zedudra-{name}"] = zedudra_shape(name)
             shapes[f"furanex-{name}"] = furanex_shape(name)
+            shapes[f"sorulix-{name}"] = sorulix_shape(name)
     return shapes
 
 
@@ -216,3 +218,43 @@ def furanex_tiny_shape() -> Dict[str, Any]:
             "layers": [{"type": "attention", "mixer": dict(attention), "mlp": dict(moe)},
                        {"type": "latent_attention", "mixer": dict(latent), "mlp": None},
                        {"type": "attention", "mixer": dict(attention), "mlp": dict(moe)}]}
+
+
+def sorulix_shape(name: str, layers: int = None, state_head_dim: int = 64, rank: int = 64, conv: int = 4, loops: int = 1,
+                  softcap: float = 50.0, limit: float = 7.0) -> Dict[str, Any]:
+    """A Sorulix configuration with the width, feed-forward, vocabulary, head counts, head size and number of layers of the
+    named Qwen3 shape: every second layer (from the first) has softmax attention with the shape's heads beside linear
+    attention with heads of ``state_head_dim``, the others are the channel-wise delta rule with heads of that size and
+    low-rank projections of ``rank``; every feed-forward has the shape's dense width. With ``loops`` > 1 the middle half
+    of the layers runs that many times. For random-weights models at sizes that resemble a real model's layers."""
+    q = QWEN3_SHAPES[name]
+    n = layers or q["num_hidden_layers"]
+    hid, hd = q["hidden_size"], q["head_dim"]
+    state_heads = hid // state_head_dim
+    parallel = {"left": {"heads": q["num_attention_heads"], "kv_heads": q["num_key_value_heads"], "dim": hd, "vdim": hd,
+                         "scale": hd ** -0.5, "softcap": softcap, "q_temp": {"coef": 0.1, "every": 4096}},
+                "right": {"heads": state_heads, "dim": state_head_dim, "vdim": state_head_dim,
+                          "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * (h + 1) / state_heads) for h in range(state_heads)]}}
+    delta = {"heads": state_heads, "kv_heads": state_heads, "dim": state_head_dim, "vdim": state_head_dim, "conv": conv,
+             "decay_rank": rank, "gate_rank": rank}
+    mlp = {"kind": "dense", "ff": q["intermediate_size"], "limit": limit}
+    out = [{"type": "channel_delta" if i % 2 else "parallel", "mixer": dict(delta if i % 2 else parallel), "mlp": dict(mlp)}
+           for i in range(n)]
+    d = {"architecture": "Sorulix", "vocab": q["vocab_size"], "width": hid, "layers": out, "norm": {"eps": q["rms_norm_eps"]}}
+    if loops > 1:
+        d["loop"] = {"start": n // 4, "stop": n // 4 + max(1, n // 2), "times": loops}
+    return d
+
+
+def sorulix_tiny_shape() -> Dict[str, Any]:
+    """A Sorulix model of a few thousand weights: both kinds of layers, a run of two layers that runs three times, a
+    layer without a feed-forward."""
+    mlp = {"kind": "dense", "ff": 88, "limit": 2.0}
+    parallel = {"left": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "scale": 0.25, "softcap": 12.0,
+                         "q_temp": {"coef": 0.2, "every": 16}},
+                "right": {"heads": 3, "dim": 12, "vdim": 8, "decay": [0.8, 0.95, 0.995]}}
+    delta = {"heads": 4, "kv_heads": 2, "dim": 12, "vdim": 16, "conv": 3, "decay_rank": 10, "gate_rank": 6}
+    return {"architecture": "Sorulix", "vocab": 256, "width": 64, "norm": {"eps": 1e-5}, "loop": {"start": 1, "stop": 3, "times": 3},
+            "layers": [{"type": "channel_delta", "mixer": dict(delta), "mlp": None},
+                       {"type": "parallel", "mixer": parallel, "mlp": dict(mlp)},
+                       {"type": "channel_delta", "mixer": dict(delta, kv_heads=4), "mlp": dict(mlp)}]}

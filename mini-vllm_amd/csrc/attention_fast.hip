@@ -25,8 +25,10 @@
 // probability zero; value slots that were never written are read as zero. With `kept.first` > 0
 // (a window, finished queries) the sequence's first positions stay visible however far back they lie:
 // the blocks that hold them are dealt out in front of the window's blocks, the blocks between are
-// never touched. With `kept.gate`, head h's output is multiplied by sigmoid(gate[token][h]).
+// never touched. With `kept.gate`, head h's output is multiplied by sigmoid(gate[token][h]). SCORED variants
+// cap the scores, take a distance bias off and add a sink to the denominator (see attention_score.h).
 #include "dispatch.h"
+#include "attention_score.h"
 
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float floatx4_t __attribute__((ext_vector_type(4)));
@@ -129,14 +131,14 @@ struct KeptArgs {
 // can be asked for together with the position. A split whose blocks all lie outside the sequence's
 // keys ends at once; the others leave their partial results and count themselves in, and the one
 // that counts last adds the partial results up (see the end of the kernel).
-template <int D, int W, bool FUSED, int OCC>
+template <int D, int W, bool FUSED, int OCC, bool SCORED>
 __global__ void __launch_bounds__(64 * W) __attribute__((amdgpu_waves_per_eu(OCC * W / 4, OCC * W / 4)))
 attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restrict__ out, long out_stride,
                       const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
                       const int* __restrict__ block_table, int bt_width, int page_size,
                       const int* __restrict__ positions, const int* __restrict__ cu_seqlens, int n_seqs,
                       int H, int Hkv, float scale, int window, float* __restrict__ partials,
-                      int* __restrict__ counters, int nsplit, int max_pages, FusedInput fz, KeptArgs kept) {
+                      int* __restrict__ counters, int nsplit, int max_pages, FusedInput fz, KeptArgs kept, ScoreForm form) {
     constexpr int DS = D / 32;
     constexpr int DT = D / 16;
     constexpr int NT = 1;      // column tiles of a wave (the group's heads fit one tile)
@@ -311,6 +313,8 @@ attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restr
     const int n_active = hi_w < 0 ? 0 : (g1 - g0 + 1 < nsplit ? g1 - g0 + 1 : nsplit);
     if (nsplit > 1 && (split - z_first + nsplit) % nsplit >= n_active) return;
     const float sc_mul = scale * LOG2E;
+    const ScoreBase2 scored(form, scale);
+    const float slope2 = (SCORED && form.slopes != nullptr) ? form.slopes[col_head[0]] * LOG2E : 0.f;
 
     // (FUSED) the wave that meets the newest position among its keys takes the new key and value
     // from the step's rows, not from the page
@@ -435,7 +439,8 @@ attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restr
             for (int r = 0; r < 4; ++r) {
                 const int key = base + 8 * g + 4 * t + r;
                 const bool ok = v_live && col_ok[0] && key <= col_pos[0] && (key >= col_lo[0] || key < kept_first);
-                p[t][r] = ok ? sacc[r] * sc_mul : -INFINITY;
+                if constexpr (SCORED) p[t][r] = ok ? fmaf(-slope2, (float)(col_pos[0] - key), scored.of(sacc[r])) : -INFINITY;
+                else p[t][r] = ok ? sacc[r] * sc_mul : -INFINITY;
             }
         }
         // online softmax per column
@@ -545,10 +550,12 @@ attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restr
         sm_l[wave][i] = l_run[0];
     }
     __syncthreads();
-    float m_fin = -INFINITY;
+    // (a sink counts once: here, or where the splits' partial results are added up)
+    const bool sink_here = SCORED && form.sink && (OCC != 1 || nsplit == 1);
+    float m_fin = sink_here ? 0.f : -INFINITY;
 #pragma unroll
     for (int w = 0; w < W; ++w) m_fin = fmaxf(m_fin, sm_m[w][i]);
-    float f[W], l_fin = 0.f;
+    float f[W], l_fin = sink_here ? exp2f(-m_fin) : 0.f;
 #pragma unroll
     for (int w = 0; w < W; ++w) {
         const float mw = sm_m[w][i];
@@ -630,7 +637,7 @@ attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restr
         const int col = idx / D, d = idx - col * D;
         const int tok = t0 + col / G, head = kvh * G + col % G;
         const float* base = partials + ((size_t)tok * H + head) * nsplit * (D + 2);
-        float m = -INFINITY, l = 0.f, a = 0.f;
+        float m = SCORED && form.sink ? 0.f : -INFINITY, l = SCORED && form.sink ? 1.f : 0.f, a = 0.f;
         for (int j0 = 0; j0 < n_active; j0 += MB) {
             float v[MB], mz[MB], lz[MB];
 #pragma unroll
@@ -664,16 +671,16 @@ attention_decode_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restr
 #undef AF_PEEK
 }
 
-template <int D, int W, bool FUSED, int OCC>
+template <int D, int W, bool FUSED, int OCC, bool SCORED = false>
 static void launch_decode(dim3 grid, hipStream_t stream, const void* q, long q_stride, void* out, long out_stride,
                           const void* k_pages, const void* v_pages, const int* block_table, int bt_width,
                           int page_size, const int* positions, const int* cu_seqlens, int n_seqs, int H, int Hkv,
                           float scale, int window, float* partials, int* counters, int nsplit, int max_pages,
-                          const FusedInput& fz, const KeptArgs& kept) {
-    hipLaunchKernelGGL((attention_decode_kernel<D, W, FUSED, OCC>), grid, dim3(64 * W), 0, stream, (const bf16*)q, q_stride,
+                          const FusedInput& fz, const KeptArgs& kept, const ScoreForm& form = ScoreForm{0.f, nullptr, 0}) {
+    hipLaunchKernelGGL((attention_decode_kernel<D, W, FUSED, OCC, SCORED>), grid, dim3(64 * W), 0, stream, (const bf16*)q, q_stride,
                        (bf16*)out, out_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, bt_width,
                        page_size, positions, cu_seqlens, n_seqs, H, Hkv, scale, window, partials, counters, nsplit, max_pages,
-                       fz, kept);
+                       fz, kept, form);
 }
 
 static int check_common(const char* what, long q_stride, long out_stride, int page_size, int bt_width, int H, int Hkv,
@@ -692,7 +699,8 @@ static int decode_common(bool fused, const FusedInput& fz, const void* q, long q
                          const void* k_pages, const void* v_pages, const int* block_table, int bt_width,
                          int page_size, const int* positions, const int* cu_seqlens, int n_seqs, int H, int Hkv, int D,
                          float scale, int window, float* partials, int* counters, int nsplit, int max_pages, int waves,
-                         const int* token_seq, hipStream_t stream, KeptArgs kept = KeptArgs{0, nullptr, 0}) {
+                         const int* token_seq, hipStream_t stream, KeptArgs kept = KeptArgs{0, nullptr, 0},
+                         ScoreForm form = ScoreForm{0.f, nullptr, 0}) {
     MV_REQUIRE(kept.first >= 0 && (kept.gate == nullptr || kept.gate_stride >= H) && (!fused || kept.first == 0),
                "attention_decode: bad count of kept first positions (none with raw rows) or gate rows too short");
     if (window < 0) kept.first = 0;          // without a window every key is seen anyway
@@ -723,6 +731,19 @@ static int decode_common(bool fused, const FusedInput& fz, const void* q, long q
                                      bt_width, page_size, positions, cu_seqlens, n_seqs, H, Hkv, scale, window,   \
                                      part, counters, nsplit, max_pages, fz, kept);                                \
     } while (0)
+    if (form.cap > 0.f || form.slopes != nullptr || form.sink) {
+        MV_REQUIRE(!fused && waves == 4, "attention_decode: capped or biased scores and sinks take finished rows and 4 waves");
+#define AF_SCORED(DD, OO)                                                                                             \
+    launch_decode<DD, 4, false, OO, true>(grid, stream, q, q_stride, out, out_stride, k_pages, v_pages, block_table,  \
+                                          bt_width, page_size, positions, cu_seqlens, n_seqs, H, Hkv, scale, window,  \
+                                          part, counters, nsplit, max_pages, fz, kept, form)
+        if (D == 128 && occ == 2) AF_SCORED(128, 2);
+        else if (D == 128) AF_SCORED(128, 1);
+        else if (occ == 2) AF_SCORED(64, 2);
+        else AF_SCORED(64, 1);
+#undef AF_SCORED
+        return mv_check_launch("attention_decode");
+    }
     if (fused) {
         MV_REQUIRE(waves == 4, "attention_decode_fused: %d waves per workgroup (4 only)", waves);
         if (D == 128) AF_LAUNCH(128, 4, true);
@@ -749,11 +770,12 @@ extern "C" int mv_attention_decode(const void* q, long q_stride, void* out, long
                                    const int* positions, const int* cu_seqlens, int n_seqs, int H, int Hkv, int D,
                                    float scale, int window, float* partials, int* counters, int nsplit,
                                    int max_pages, int waves, const int* token_seq, int first, const void* gate,
-                                   long gate_stride, hipStream_t stream) {
+                                   long gate_stride, float cap, const float* slopes, int sink, hipStream_t stream) {
     if (int rc = check_common("attention_decode", q_stride, out_stride, page_size, bt_width, H, Hkv, D)) return rc;
     return decode_common(false, FusedInput{}, q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_width,
                          page_size, positions, cu_seqlens, n_seqs, H, Hkv, D, scale, window, partials, counters, nsplit,
-                         max_pages, waves, token_seq, stream, KeptArgs{first, (const bf16*)gate, gate_stride});
+                         max_pages, waves, token_seq, stream, KeptArgs{first, (const bf16*)gate, gate_stride},
+                         ScoreForm{cap, slopes, sink});
 }
 
 // The same for a decode step whose queries, keys and values are still the raw rows of the

@@ -32,7 +32,7 @@
 // walk of a unit with many keys takes half as many rounds.
 //
 // Layouts: K[page][kv_head][slot][d], V[page][kv_head][d][slot]; page size a multiple of 16.
-#include "common.h"
+#include "attention_score.h"
 
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float floatx4_t __attribute__((ext_vector_type(4)));
@@ -78,13 +78,14 @@ struct SigmoidArgs {
     int first;                 // kept first positions (softmax weights with a window; 0: none)
 };
 
-template <int D, int NT, int KW, bool SIG = false>
+// SCORED (softmax weights): capped scores, a distance bias, a sink in the denominator (see attention_score.h).
+template <int D, int NT, int KW, bool SIG = false, bool SCORED = false>
 __global__ void __launch_bounds__(AP_THREADS * KW) __attribute__((amdgpu_waves_per_eu(2, 2)))
 attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __restrict__ out, long out_stride,
                          const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
                          const int* __restrict__ block_table, int bt_width, int page_size, int page_shift,
                          const int* __restrict__ positions, const int* __restrict__ cu_seqlens, int n_seqs, int H,
-                         int Hkv, float scale, int window, int fold, SigmoidArgs sig) {
+                         int Hkv, float scale, int window, int fold, SigmoidArgs sig, ScoreForm form) {
     constexpr int DS = D / 32;                 // k-steps of the score product
     constexpr int DT = D / 16;                 // d tiles of the output product
     constexpr int COLS = 16 * AP_WAVES * NT;   // columns of a workgroup
@@ -157,7 +158,7 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
     // ---- this lane's columns
     int col_tok[NT], col_head[NT], col_pos[NT], col_lo[NT];
     bool col_ok[NT];
-    float col_bias[NT];         // SIG: the head's score bias, in the base-2 domain
+    float col_bias[NT];         // SIG: the head's score bias, SCORED: its distance slope, in the base-2 domain
     Frag qop[NT][DS];
     int hi_w = -1, lo_w = 0x7fffffff;
 #pragma unroll
@@ -176,6 +177,9 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
                 col_lo[ct] = c0 > col_lo[ct] ? c0 : col_lo[ct];
             }
             if (sig.bias != nullptr) col_bias[ct] = sig.bias[col_head[ct]] * LOG2E;
+        }
+        if constexpr (SCORED) {
+            if (form.slopes != nullptr) col_bias[ct] = form.slopes[col_head[ct]] * LOG2E;
         }
         if (col_ok[ct]) {
             hi_w = col_pos[ct] > hi_w ? col_pos[ct] : hi_w;
@@ -222,7 +226,9 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) acc_o[ct][dt] = floatx4_t{0.f, 0.f, 0.f, 0.f};
     }
-    const float sc_mul = scale * LOG2E;
+    // (SCORED: the scores come in the base-2 domain already)
+    const float sc_mul = SCORED ? 1.f : scale * LOG2E;
+    const ScoreBase2 scored(form, scale);
 
     // ---- a block's way from the pages into LDS.
     // A load instruction of a wave fills 64 consecutive 16-byte chunks of LDS, one per lane, from
@@ -393,8 +399,8 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
     };
     // The two products with the softmax between them. ask_k / ask_v: behind the score product, ask
     // for the keys of the next block (from k_next into op_next) and for this block's values (from
-    // v_now into vo_w, which is `vo`).
-    auto compute = [&](int j, const KOps& op, const VOps& vo, const uint4* k_next, KOps& op_next, const uint4* v_now, VOps& vo_w, const bool ask_k, const bool ask_v) {
+    // v_now into vo_w, which is `vo`). Inlined always: as a call it would keep the accumulators in memory.
+    auto compute = [&](int j, const KOps& op, const VOps& vo, const uint4* k_next, KOps& op_next, const uint4* v_now, VOps& vo_w, const bool ask_k, const bool ask_v) __attribute__((always_inline)) {
         const int base = 32 * block_of(j);
         const bool masked = block_of(j) > bm_hi || block_of(j) < bm_lo;
         // scores^T for the two 16-key tiles
@@ -417,6 +423,16 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
         if (ask_v) read_v(v_now, vo_w);
         if (ask_k) read_k(k_next, op_next);
         __builtin_amdgcn_sched_barrier(0);
+        if constexpr (SCORED) {
+#pragma unroll
+            for (int ct = 0; ct < NT; ++ct) {
+                const float ahead = (float)(col_pos[ct] - base - 8 * g);      // how far the lane's first key lies behind
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) p[ct][t][r] = fmaf(-col_bias[ct], ahead - (float)(4 * t + r), scored.of(p[ct][t][r]));
+            }
+        }
         if (masked) {
 #pragma unroll
             for (int ct = 0; ct < NT; ++ct)
@@ -668,7 +684,13 @@ attention_prefill_kernel(const bf16* __restrict__ q, long q_stride, bf16* __rest
                 inv = 1.f / (1.f + __expf(-z));
             }
         } else {
-            inv = 1.f / l_run[ct];
+            if (SCORED && form.sink) {          // one more score, 0, without a value
+                const float m_fin = fmaxf(m_run[ct], 0.f);
+                const float f = exp2f(m_run[ct] - m_fin);
+                inv = f / fmaf(f, l_run[ct], exp2f(-m_fin));
+            } else {
+                inv = 1.f / l_run[ct];
+            }
             if (sig.gate != nullptr) {
                 const float z = to_f(sig.gate[(size_t)col_tok[ct] * sig.gate_stride + col_head[ct]]);
                 inv *= 1.f / (1.f + __expf(-z));
@@ -691,15 +713,16 @@ extern "C" int mv_attention_prefill_unit_tokens(int group, int nt) {
     return group > 0 && group <= cols ? cols / group : 0;
 }
 
-template <int D, int NT, int KW, bool SIG = false>
+template <int D, int NT, int KW, bool SIG = false, bool SCORED = false>
 static int launch_prefill(dim3 grid, hipStream_t stream, const void* q, long q_stride, void* out, long out_stride,
                           const void* k_pages, const void* v_pages, const int* block_table, int bt_width,
                           int page_size, int page_shift, const int* positions, const int* cu_seqlens, int n_seqs,
-                          int H, int Hkv, float scale, int window, int fold, SigmoidArgs sig = SigmoidArgs{0, nullptr, nullptr, 0, 0}) {
+                          int H, int Hkv, float scale, int window, int fold, SigmoidArgs sig = SigmoidArgs{0, nullptr, nullptr, 0, 0},
+                          ScoreForm form = ScoreForm{0.f, nullptr, 0}) {
     // the stages of K and V tiles are static LDS (four of 16 KiB per key group with D = 128)
-    hipLaunchKernelGGL((attention_prefill_kernel<D, NT, KW, SIG>), grid, dim3(AP_THREADS * KW), 0, stream, (const bf16*)q,
+    hipLaunchKernelGGL((attention_prefill_kernel<D, NT, KW, SIG, SCORED>), grid, dim3(AP_THREADS * KW), 0, stream, (const bf16*)q,
                        q_stride, (bf16*)out, out_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table,
-                       bt_width, page_size, page_shift, positions, cu_seqlens, n_seqs, H, Hkv, scale, window, fold, sig);
+                       bt_width, page_size, page_shift, positions, cu_seqlens, n_seqs, H, Hkv, scale, window, fold, sig, form);
     return 0;
 }
 
@@ -713,7 +736,8 @@ extern "C" int mv_attention_prefill(const void* q, long q_stride, void* out, lon
                                     const void* v_pages, const int* block_table, int bt_width, int page_size,
                                     const int* positions, const int* cu_seqlens, int n_seqs, int n_units, int n_busy,
                                     int nt, int kw, int H, int Hkv, int D, float scale, int window, int first,
-                                    const void* gate, long gate_stride, hipStream_t stream) {
+                                    const void* gate, long gate_stride, float cap, const float* slopes, int sink,
+                                    hipStream_t stream) {
     MV_REQUIRE(kw == 1 || kw == 2, "attention_prefill: %d key groups per workgroup (1 or 2)", kw);
     MV_REQUIRE(first >= 0 && (gate == nullptr || gate_stride >= H), "attention_prefill: bad count of kept first positions or "
                "gate rows too short");
@@ -741,10 +765,15 @@ extern "C" int mv_attention_prefill(const void* q, long q_stride, void* out, lon
     if (n_busy <= 0 || n_busy > n_units) n_busy = n_units;
     const int fold = (kw == 1 && (long)Hkv * n_busy <= 2L * cus) ? 1 : 0;
     int rc = 0;
+    const ScoreForm form{cap, slopes, sink};
+    const bool scored = cap > 0.f || slopes != nullptr || sink;
 #define AP_LAUNCH(DD, NN, KK)                                                                                      \
-    rc = launch_prefill<DD, NN, KK>(grid, stream, q, q_stride, out, out_stride, k_pages, v_pages, block_table,       \
-                                    bt_width, page_size, page_shift, positions, cu_seqlens, n_seqs, H, Hkv, scale,  \
-                                    window, fold, extra)
+    rc = scored ? launch_prefill<DD, NN, KK, false, true>(grid, stream, q, q_stride, out, out_stride, k_pages, v_pages,   \
+                                                          block_table, bt_width, page_size, page_shift, positions,      \
+                                                          cu_seqlens, n_seqs, H, Hkv, scale, window, fold, extra, form) \
+                : launch_prefill<DD, NN, KK>(grid, stream, q, q_stride, out, out_stride, k_pages, v_pages, block_table, \
+                                             bt_width, page_size, page_shift, positions, cu_seqlens, n_seqs, H, Hkv,    \
+                                             scale, window, fold, extra)
     if (kw == 2) {
         if (D == 128 && nt == 2) AP_LAUNCH(128, 2, 2);
         else if (D == 128) AP_LAUNCH(128, 1, 2);

@@ -8,12 +8,14 @@
 // in tiles of 128 starting at the first visible key (the kept first positions in front of the
 // window's), so the order of additions depends only on the query's position, the window and
 // `first`, never on how the step was batched. With `gate`, head h's output row is multiplied by
-// sigmoid(gate[token][h]).
+// sigmoid(gate[token][h]). Scores may be capped, lose a distance bias, and meet a sink (see
+// attention_score.h).
 //
 // Layouts:  K[page][kv_head][slot][d]   V[page][kv_head][dv][slot]   (a value row may have another size, Dv, than a key's)
 // This kernel takes every head size up to 512 and every page size; it is the float32
 // path's attention and the fall-back of the bfloat16 path.
 #include "dispatch.h"
+#include "attention_score.h"
 
 #define AR_THREADS 128
 #define AR_MAX_D 512
@@ -24,7 +26,7 @@ attention_ref_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ out
                      const T* __restrict__ k_pages, const T* __restrict__ v_pages,
                      const int* __restrict__ block_table, int bt_width, int page_size,
                      const int* __restrict__ positions, const int* __restrict__ token_seq, int H, int Hkv, int D, int Dv,
-                     float scale, int window, int first, const T* __restrict__ gate, long gate_stride) {
+                     float scale, int window, int first, const T* __restrict__ gate, long gate_stride, ScoreForm form) {
     __shared__ float qs[AR_MAX_D];
     __shared__ float ps[AR_THREADS];
     __shared__ long voff[AR_THREADS];
@@ -53,7 +55,9 @@ attention_ref_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ out
     for (int d = tid; d < D; d += AR_THREADS) qs[d] = to_f(qrow[d]);
     __syncthreads();
 
-    float m = -INFINITY, l = 0.f;
+    // a sink is a first score of 0 whose exponential belongs to no key
+    float m = form.sink ? 0.f : -INFINITY, l = form.sink ? 1.f : 0.f;
+    const float slope = form.slopes != nullptr ? form.slopes[head] : 0.f;
     float acc[AR_MAX_D / AR_THREADS];
 #pragma unroll
     for (int i = 0; i < AR_MAX_D / AR_THREADS; ++i) acc[i] = 0.f;
@@ -71,6 +75,8 @@ attention_ref_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ out
             float dot = 0.f;
             for (int d = 0; d < D; ++d) dot = fmaf(qs[d], to_f(krow[d]), dot);
             s = dot * scale;
+            if (form.cap > 0.f) s = form.cap * tanhf(s / form.cap);
+            if (form.slopes != nullptr) s -= slope * (float)(pos - j);
             vo = (long)(((size_t)page * Hkv + kvh) * Dv) * page_size + slot;
         }
         const float tmax = block_max(s, scratch);
@@ -107,8 +113,8 @@ attention_ref_kernel(const T* __restrict__ q, long q_stride, T* __restrict__ out
 extern "C" int mv_attention_ref(const void* q, long q_stride, void* out, long out_stride, const void* k_pages,
                                 const void* v_pages, const int* block_table, int bt_width, int page_size,
                                 const int* positions, const int* token_seq, int n, int H, int Hkv, int D, int Dv,
-                                float scale, int window, int first, const void* gate, long gate_stride, int dtype,
-                                hipStream_t stream) {
+                                float scale, int window, int first, const void* gate, long gate_stride, float cap,
+                                const float* slopes, int sink, int dtype, hipStream_t stream) {
     MV_REQUIRE(n >= 0 && H > 0 && Hkv > 0 && D > 0, "attention: bad sizes n=%d H=%d Hkv=%d D=%d", n, H, Hkv, D);
     MV_REQUIRE(H % Hkv == 0, "attention: %d query heads are not a multiple of %d key/value heads", H, Hkv);
     MV_REQUIRE(D <= AR_MAX_D && Dv > 0 && Dv <= AR_MAX_D, "attention: head sizes %d / %d exceed the supported maximum %d", D, Dv, AR_MAX_D);
@@ -122,6 +128,6 @@ extern "C" int mv_attention_ref(const void* q, long q_stride, void* out, long ou
                   hipLaunchKernelGGL(attention_ref_kernel<T>, dim3(n, H), dim3(AR_THREADS), 0, stream, (const T*)q,
                                      q_stride, (T*)out, out_stride, (const T*)k_pages, (const T*)v_pages,
                                      block_table, bt_width, page_size, positions, token_seq, H, Hkv, D, Dv, scale,
-                                     window, first, (const T*)gate, gate_stride));
+                                     window, first, (const T*)gate, gate_stride, ScoreForm{cap, slopes, sink}));
     return mv_check_launch("attention");
 }

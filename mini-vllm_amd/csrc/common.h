@@ -184,6 +184,21 @@ __device__ __forceinline__ float block_max(float v, float* scratch) {
 }
 
 // ---------------------------------------------------------------------------------------
+// The gated pair of a feed-forward: silu(g) * u, or with a `limit` > 0 the clamped pair
+// g' = min(g, limit), u' = clamp(u, -limit, limit), g' * sigmoid(slope * g') * (u' + 1).
+// ---------------------------------------------------------------------------------------
+struct GatedPair {
+    float limit, slope;
+    __device__ __forceinline__ float of(float g, float u) const {
+        if (limit > 0.f) {
+            const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit);
+            return gc / (1.f + expf(-slope * gc)) * (uc + 1.f);
+        }
+        return g / (1.f + expf(-g)) * u;
+    }
+};
+
+// ---------------------------------------------------------------------------------------
 // Host side: error reporting of the extern "C" entry points. Each returns 0 on success;
 // otherwise mv_last_error() holds the reason.
 // ---------------------------------------------------------------------------------------

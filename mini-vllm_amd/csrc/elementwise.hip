@@ -835,21 +835,21 @@ extern "C" int mv_store_v_pages(const void* qkv, long row_stride, int v_off, con
 }
 
 // ---------------------------------------------------------------------------------------
-// SwiGLU: out[n, i] = silu(gu[n, i]) * gu[n, I + i],  silu(z) = z / (1 + exp(-z))
+// The gated pair: out[n, i] = pair(gu[n, i], gu[n, I + i]), silu(g) * u or the clamped pair (GatedPair)
 // ---------------------------------------------------------------------------------------
 template <typename T>
-__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, long total, int I) {
+__global__ void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, long total, int I, GatedPair pair) {
     const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const long row = idx / I;
     const int col = (int)(idx - row * I);
     const float g = to_f(gu[row * 2 * I + col]);
     const float u = to_f(gu[row * 2 * I + I + col]);
-    out[idx] = from_f<T>(g / (1.f + expf(-g)) * u);
+    out[idx] = from_f<T>(pair.of(g, u));
 }
 
 template <typename T>
-__global__ void swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, long total8, int I8) {
+__global__ void swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, long total8, int I8, GatedPair pair) {
     const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;   // eight columns each
     if (idx >= total8) return;
     const long row = idx / I8;
@@ -859,25 +859,25 @@ __global__ void swiglu_vec_kernel(const T* __restrict__ gu, T* __restrict__ out,
     Vec8<T>::load(gu + row * 2 * I + col, g);
     Vec8<T>::load(gu + row * 2 * I + I + col, u);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) y[e] = g[e] / (1.f + expf(-g[e])) * u[e];
+    for (int e = 0; e < 8; ++e) y[e] = pair.of(g[e], u[e]);
     Vec8<T>::store(out + row * I + col, y);
 }
 
-extern "C" int mv_swiglu(const void* gate_up, void* out, int n, int I, int dtype, hipStream_t stream) {
+extern "C" int mv_swiglu(const void* gate_up, void* out, int n, int I, float limit, float slope, int dtype, hipStream_t stream) {
     MV_REQUIRE(n >= 0 && I > 0, "swiglu: bad sizes n=%d I=%d", n, I);
     if (n == 0) return 0;
     if (I % 8 == 0 && ((uintptr_t)gate_up % 16) == 0 && ((uintptr_t)out % 16) == 0) {
         const long total8 = (long)n * (I / 8);
         MV_DISPATCH_T(dtype, "swiglu",
                       hipLaunchKernelGGL(swiglu_vec_kernel<T>, dim3((unsigned)((total8 + 255) / 256)), dim3(256), 0,
-                                         stream, (const T*)gate_up, (T*)out, total8, I / 8));
+                                         stream, (const T*)gate_up, (T*)out, total8, I / 8, GatedPair{limit, slope}));
         return mv_check_launch("swiglu");
     }
     const long total = (long)n * I;
     const unsigned blocks = (unsigned)((total + 255) / 256);
     MV_DISPATCH_T(dtype, "swiglu",
                   hipLaunchKernelGGL(swiglu_kernel<T>, dim3(blocks), dim3(256), 0, stream, (const T*)gate_up,
-                                     (T*)out, total, I));
+                                     (T*)out, total, I, GatedPair{limit, slope}));
     return mv_check_launch("swiglu");
 }
 

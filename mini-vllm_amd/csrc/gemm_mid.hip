@@ -179,11 +179,12 @@ gemm_mid_kernel(const bf16* __restrict__ A, long lda, const bf16* __restrict__ W
         }
 }
 
-// out[m][n] = sum_f part[f][m][n] (+ bias[n]), or with `swiglu` out[m][i] = silu(gate) * up with
-// gate = sum_f part[f][m][i], up = sum_f part[f][m][I + i], N = 2 I.
+// out[m][n] = sum_f part[f][m][n] (+ bias[n]), or with `swiglu` out[m][i] = pair(gate, up) (GatedPair) with
+// gate = sum_f part[f][m][i] (+ bias[i]), up = sum_f part[f][m][I + i] (+ bias[I + i]), N = 2 I.
 template <typename TC>
 __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, const bf16* __restrict__ bias,
-                                       TC* __restrict__ C, long ldc, int M, int N, int F, int swiglu) {
+                                       TC* __restrict__ C, long ldc, int M, int N, int F, int swiglu,
+                                       GatedPair pair) {
     const int n_out = swiglu ? N / 2 : N;
     const long idx = (long)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= (long)M * n_out) return;
@@ -196,7 +197,11 @@ __global__ void gemm_mid_reduce_kernel(const float* __restrict__ part, const bf1
     }
     float v;
     if (swiglu) {
-        v = a / (1.f + expf(-a)) * b;
+        if (bias) {
+            a += to_f(bias[n]);
+            b += to_f(bias[n_out + n]);
+        }
+        v = pair.of(a, b);
     } else {
         v = a;
         if (bias) v += to_f(bias[n]);
@@ -285,25 +290,26 @@ extern "C" int mv_gemm_mid_sums(const void* A, long lda, const void* W, int M, i
 // The second half alone: C = sum over f < F of work[f] (+ bias), or the gated activation of the two
 // halves of the sum. c_dtype: MV_BF16 or MV_F32.
 extern "C" int mv_gemm_mid_reduce(const float* work, const void* bias, void* C, long ldc, int c_dtype, int M, int N,
-                                  int F, int swiglu, hipStream_t stream) {
+                                  int F, int swiglu, float limit, float slope, hipStream_t stream) {
     MV_REQUIRE(M > 0 && N > 0 && F > 0 && work != nullptr && C != nullptr, "gemm_mid: bad sizes M=%d N=%d F=%d", M, N, F);
-    MV_REQUIRE(!swiglu || (N % 2 == 0 && bias == nullptr), "gemm_mid: the gated form takes an even N and no bias");
+    MV_REQUIRE(!swiglu || N % 2 == 0, "gemm_mid: the gated form takes an even N");
     MV_REQUIRE(ldc >= (swiglu ? N / 2 : N), "gemm_mid: ldc=%ld too small for N=%d", ldc, N);
     MV_REQUIRE(c_dtype == MV_F32 || c_dtype == MV_BF16, "gemm_mid: bad output dtype %d", c_dtype);
     const long total = (long)M * (swiglu ? N / 2 : N);
     const unsigned blocks = (unsigned)((total + 255) / 256);
     if (c_dtype == MV_F32)
         hipLaunchKernelGGL(gemm_mid_reduce_kernel<float>, dim3(blocks), dim3(256), 0, stream, work, (const bf16*)bias,
-                           (float*)C, ldc, M, N, F, swiglu);
+                           (float*)C, ldc, M, N, F, swiglu, GatedPair{limit, slope});
     else
         hipLaunchKernelGGL(gemm_mid_reduce_kernel<bf16>, dim3(blocks), dim3(256), 0, stream, work, (const bf16*)bias,
-                           (bf16*)C, ldc, M, N, F, swiglu);
+                           (bf16*)C, ldc, M, N, F, swiglu, GatedPair{limit, slope});
     return mv_check_launch("gemm_mid (reduce)");
 }
 
 // Both halves. With `swiglu`, W is the packed gate/up weight [N = 2 I, K] and C is [M, I].
 extern "C" int mv_gemm_mid(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int c_dtype,
-                           int M, int N, int K, int swiglu, float* work, long work_floats, hipStream_t stream) {
+                           int M, int N, int K, int swiglu, float* work, long work_floats, float limit, float slope,
+                           hipStream_t stream) {
     if (int rc = mv_gemm_mid_sums(A, lda, W, M, N, K, work, work_floats, stream)) return rc;
-    return mv_gemm_mid_reduce(work, bias, C, ldc, c_dtype, M, N, mid_plan(N, K).F, swiglu, stream);
+    return mv_gemm_mid_reduce(work, bias, C, ldc, c_dtype, M, N, mid_plan(N, K).F, swiglu, limit, slope, stream);
 }

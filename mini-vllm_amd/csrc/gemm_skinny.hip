@@ -27,7 +27,8 @@
 // the same (weight row, token) pairs, the other two quarters are not used.
 //
 // A fused variant computes the gated activation of a feed-forward in the same pass:
-//     out[M, I] = silu(A Wg^T) * (A Wu^T)  with Wg = W[0:I], Wu = W[I:2I].
+//     out[M, I] = pair(A Wg^T, A Wu^T)  with Wg = W[0:I], Wu = W[I:2I] (biases likewise), pair(g, u) =
+//     silu(g) * u or the clamped pair (GatedPair).
 //
 // Two more variants take a residual add and an RMSNorm between two products apart, for steps
 // with too many rows to normalise them in every workgroup of the second product. The product in
@@ -63,7 +64,7 @@ template <int R, int TM, bool SWIGLU, bool NORM, typename TC, int EPI = EPI_NONE
 __global__ void __launch_bounds__(64 * SK_MAX_WAVES)
 gemm_skinny_kernel(const bf16* __restrict__ A, long lda, const bf16* __restrict__ W, const bf16* __restrict__ bias,
                    TC* __restrict__ C, long ldc, int M, int N, int K, int groups, int blocks, int rows,
-                   NormInput norm, RowsInput fold) {
+                   NormInput norm, RowsInput fold, GatedPair pair) {
     extern __shared__ float red[];  // [S - 1][R * TM][64][4], then (NORM) bf16 [M][K + 8], or (SCALED) float [16 * TM]
     // The tokens may be dealt out to `groups` workgroups per weight tile (16 * TM tokens each): with
     // few weight tiles that fills more compute units, and each unit pulls fewer activation rows.
@@ -550,8 +551,12 @@ gemm_skinny_kernel(const bf16* __restrict__ A, long lda, const bf16* __restrict_
             for (int e = 0; e < 4; ++e) {
                 const int col = n_base + 4 * g + e;
                 if (col >= n_end) continue;
-                const float gate = acc[0][t][e], up = acc[R - 1][t][e];
-                store_c<TC>(C + (size_t)tok * ldc + col, gate / (1.f + expf(-gate)) * up);
+                float gate = acc[0][t][e], up = acc[R - 1][t][e];
+                if (bias) {
+                    gate += to_f(bias[col]);
+                    up += to_f(bias[N + col]);
+                }
+                store_c<TC>(C + (size_t)tok * ldc + col, pair.of(gate, up));
             }
         }
     } else {
@@ -589,7 +594,8 @@ static bool skinny_paired(int M, long weight_rows, int K) {
 
 template <int R, int TM, bool SWIGLU, typename TC, int EPI = EPI_NONE>
 static void launch_skinny(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int M, int N,
-                          int K, int S, int rows, hipStream_t stream, const RowsInput& fold = RowsInput{}) {
+                          int K, int S, int rows, hipStream_t stream, const RowsInput& fold = RowsInput{},
+                          GatedPair pair = GatedPair{0.f, 1.f}) {
     const int blocks = skinny_blocks(N, rows);
     const int groups = (M + 16 * TM - 1) / (16 * TM);
     const int grid = groups > 1 ? (blocks + 7) / 8 * 8 * groups : blocks;
@@ -599,22 +605,22 @@ static void launch_skinny(const void* A, long lda, const void* W, const void* bi
             if (M <= 8)
                 hipLaunchKernelGGL((gemm_skinny_kernel<R, TM, SWIGLU, false, TC, EPI, 2>), dim3(grid), dim3(64 * S), lds,
                                    stream, (const bf16*)A, lda, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N, K,
-                                   groups, blocks, rows, NormInput{}, fold);
+                                   groups, blocks, rows, NormInput{}, fold, pair);
             else
                 hipLaunchKernelGGL((gemm_skinny_kernel<R, TM, SWIGLU, false, TC, EPI, 1>), dim3(grid), dim3(64 * S), lds,
                                    stream, (const bf16*)A, lda, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N, K,
-                                   groups, blocks, rows, NormInput{}, fold);
+                                   groups, blocks, rows, NormInput{}, fold, pair);
             return;
         }
     }
     hipLaunchKernelGGL((gemm_skinny_kernel<R, TM, SWIGLU, false, TC, EPI>), dim3(grid), dim3(64 * S), lds, stream,
                        (const bf16*)A, lda, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N, K, groups, blocks,
-                       rows, NormInput{}, fold);
+                       rows, NormInput{}, fold, pair);
 }
 
 template <int R, bool SWIGLU, typename TC>
 static void launch_skinny_norm(const NormInput& norm, const void* W, const void* bias, void* C, long ldc, int M, int N,
-                               int K, int S, hipStream_t stream) {
+                               int K, int S, hipStream_t stream, GatedPair pair = GatedPair{0.f, 1.f}) {
     const int rows = SWIGLU ? 16 : 16 * R;
     const int blocks = skinny_blocks(N, rows);
     const size_t lds = skinny_lds_bytes(S, R, 1, true, M, K);
@@ -622,21 +628,21 @@ static void launch_skinny_norm(const NormInput& norm, const void* W, const void*
         if (M <= 8)
             hipLaunchKernelGGL((gemm_skinny_kernel<R, 1, SWIGLU, true, TC, EPI_NONE, 2>), dim3(blocks), dim3(64 * S), lds,
                                stream, (const bf16*)nullptr, (long)K, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N,
-                               K, 1, blocks, rows, norm, RowsInput{});
+                               K, 1, blocks, rows, norm, RowsInput{}, pair);
         else
             hipLaunchKernelGGL((gemm_skinny_kernel<R, 1, SWIGLU, true, TC, EPI_NONE, 1>), dim3(blocks), dim3(64 * S), lds,
                                stream, (const bf16*)nullptr, (long)K, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N,
-                               K, 1, blocks, rows, norm, RowsInput{});
+                               K, 1, blocks, rows, norm, RowsInput{}, pair);
         return;
     }
     hipLaunchKernelGGL((gemm_skinny_kernel<R, 1, SWIGLU, true, TC>), dim3(blocks), dim3(64 * S), lds, stream,
                        (const bf16*)nullptr, (long)K, (const bf16*)W, (const bf16*)bias, (TC*)C, ldc, M, N, K, 1, blocks,
-                       rows, norm, RowsInput{});
+                       rows, norm, RowsInput{}, pair);
 }
 
 template <int R, bool SWIGLU, typename TC, int EPI = EPI_NONE>
 static int dispatch_tm(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int M, int N, int K,
-                       int S, int rows, hipStream_t stream, const RowsInput& fold = RowsInput{}) {
+                       int S, int rows, hipStream_t stream, const RowsInput& fold = RowsInput{}, GatedPair pair = GatedPair{0.f, 1.f}) {
     // Token tiles per workgroup: all of them (the weights pass each compute unit once), or fewer
     // with the tokens dealt out to several workgroups per weight tile. A compute unit pulls
     // R + TM operand rows of 16 per workgroup it runs; the choice with the least per unit wins.
@@ -653,10 +659,10 @@ static int dispatch_tm(const void* A, long lda, const void* W, const void* bias,
             best_tm = tm;
         }
     }
-    if (best_tm == 1) launch_skinny<R, 1, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold);
-    else if (best_tm == 2) launch_skinny<R, 2, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold);
-    else if (best_tm == 3) launch_skinny<R, 3, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold);
-    else launch_skinny<R, 4, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold);
+    if (best_tm == 1) launch_skinny<R, 1, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold, pair);
+    else if (best_tm == 2) launch_skinny<R, 2, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold, pair);
+    else if (best_tm == 3) launch_skinny<R, 3, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold, pair);
+    else launch_skinny<R, 4, SWIGLU, TC, EPI>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, fold, pair);
     return 0;
 }
 
@@ -725,7 +731,7 @@ extern "C" int mv_gemm_skinny_fold(const void* A, long lda, const void* W, const
 // sqrt(sum_p partial[m][p] / K + eps). bf16 out.
 extern "C" int mv_gemm_skinny_scaled(const void* A, long lda, const void* W, const void* bias, void* C, long ldc,
                                      const float* partial, int P, float eps, int M, int N, int K, int swiglu,
-                                     hipStream_t stream) {
+                                     float limit, float slope, hipStream_t stream) {
     if (int rc = check_skinny("gemm_skinny_scaled", A, lda, W, ldc, M, N, K)) return rc;
     MV_REQUIRE(partial != nullptr && P > 0 && eps > 0.f, "gemm_skinny_scaled: bad partial sums (P=%d) or eps", P);
     if (M == 0) return 0;
@@ -733,8 +739,8 @@ extern "C" int mv_gemm_skinny_scaled(const void* A, long lda, const void* W, con
     int rc = 0;
     if (swiglu) {
         const int S = pick_waves(K);
-        rc = dispatch_tm<2, true, bf16, EPI_SCALED>(A, lda, W, nullptr, C, ldc, M, N, K, S,
-                                                    M <= 16 ? pick_rows(N, 16) : 16, stream, fold);
+        rc = dispatch_tm<2, true, bf16, EPI_SCALED>(A, lda, W, bias, C, ldc, M, N, K, S,
+                                                    M <= 16 ? pick_rows(N, 16) : 16, stream, fold, GatedPair{limit, slope});
     } else {
         int S, R, rows;
         skinny_shape(M, N, K, S, R, rows);
@@ -746,13 +752,14 @@ extern "C" int mv_gemm_skinny_scaled(const void* A, long lda, const void* W, con
     return mv_check_launch("gemm_skinny_scaled");
 }
 
-// out[M, I] = silu(A Wgu[0:I]^T) * (A Wgu[I:2I]^T), bf16 in and out.
-extern "C" int mv_gemm_skinny_swiglu(const void* A, long lda, const void* Wgu, void* out, long ldo, int M, int I,
-                                     int K, hipStream_t stream) {
+// out[M, I] = pair(A Wgu[0:I]^T + bias[0:I], A Wgu[I:2I]^T + bias[I:2I]), bf16 in and out (GatedPair).
+extern "C" int mv_gemm_skinny_swiglu(const void* A, long lda, const void* Wgu, const void* bias, void* out, long ldo, int M, int I,
+                                     int K, float limit, float slope, hipStream_t stream) {
     if (int rc = check_skinny("gemm_skinny_swiglu", A, lda, Wgu, ldo, M, I, K)) return rc;
     if (M == 0) return 0;
     const int S = pick_waves(K);
-    int rc = dispatch_tm<2, true, bf16>(A, lda, Wgu, nullptr, out, ldo, M, I, K, S, M <= 16 ? pick_rows(I, 16) : 16, stream);
+    int rc = dispatch_tm<2, true, bf16>(A, lda, Wgu, bias, out, ldo, M, I, K, S, M <= 16 ? pick_rows(I, 16) : 16, stream,
+                                        RowsInput{}, GatedPair{limit, slope});
     if (rc) return rc;
     return mv_check_launch("gemm_skinny_swiglu");
 }
@@ -766,7 +773,7 @@ extern "C" int mv_gemm_skinny_swiglu(const void* A, long lda, const void* Wgu, v
 extern "C" int mv_gemm_skinny_norm(const float* resid_in, const void* delta, float* resid_out, const void* norm_weight,
                                    int norm_weight_dtype, float eps, int unit_offset, const void* W, const void* bias,
                                    void* C, long ldc, int c_dtype, int M, int N, int K, int swiglu,
-                                   hipStream_t stream) {
+                                   float limit, float slope, hipStream_t stream) {
     MV_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm_skinny_norm: bad sizes M=%d N=%d K=%d", M, N, K);
     MV_REQUIRE(mv_valid_dtype(norm_weight_dtype) && norm_weight != nullptr && ((uintptr_t)norm_weight % 16) == 0,
                "gemm_skinny_norm: the norm weight is missing, of an unknown type or not 16-byte aligned");
@@ -786,7 +793,7 @@ extern "C" int mv_gemm_skinny_norm(const float* resid_in, const void* delta, flo
         return 2;
     }
     NormInput norm{resid_in, (const bf16*)delta, resid_out, WeightPtr{norm_weight, norm_weight_dtype}, eps, unit_offset};
-    if (swiglu) launch_skinny_norm<2, true, bf16>(norm, W, nullptr, C, ldc, M, N, K, S, stream);
+    if (swiglu) launch_skinny_norm<2, true, bf16>(norm, W, bias, C, ldc, M, N, K, S, stream, GatedPair{limit, slope});
     else if (c_dtype == MV_F32) launch_skinny_norm<1, false, float>(norm, W, bias, C, ldc, M, N, K, S, stream);
     else launch_skinny_norm<1, false, bf16>(norm, W, bias, C, ldc, M, N, K, S, stream);
     return mv_check_launch("gemm_skinny_norm");

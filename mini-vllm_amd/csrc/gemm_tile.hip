@@ -69,6 +69,7 @@ struct TileArgs {
     const float* partial;
     int P;
     float eps;
+    GatedPair pair;       // GATED: what becomes of the two products (with biases [2 I] added where given)
 };
 
 template <int WM, int WN, bool GATED, int STAGES, int OCC>
@@ -259,11 +260,14 @@ gemm_tile_kernel(TileArgs a) {
 #pragma unroll
     for (int t = 0; t < TOUT; ++t) {
         const int col = n0 + 16 * ((GATED ? WN / 2 : WN) * wn + t) + 4 * g;
-        float bv[4] = {0.f, 0.f, 0.f, 0.f};
-        if (!GATED && a.bias != nullptr) {
+        float bv[4] = {0.f, 0.f, 0.f, 0.f}, bu[4] = {0.f, 0.f, 0.f, 0.f};
+        if (a.bias != nullptr) {
 #pragma unroll
             for (int e = 0; e < 4; ++e)
-                if (col + e < n_out) bv[e] = to_f(a.bias[col + e]);
+                if (col + e < n_out) {
+                    bv[e] = to_f(a.bias[col + e]);
+                    if (GATED) bu[e] = to_f(a.bias[n_out + col + e]);
+                }
         }
 #pragma unroll
         for (int u = 0; u < WM; ++u) {
@@ -274,8 +278,7 @@ gemm_tile_kernel(TileArgs a) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
                 if (GATED) {
-                    const float gt = acc[t][u][e] * rinv, up = acc[t + WN / 2][u][e] * rinv;
-                    v[e] = gt / (1.f + expf(-gt)) * up;
+                    v[e] = a.pair.of(fmaf(acc[t][u][e], rinv, bv[e]), fmaf(acc[t + WN / 2][u][e], rinv, bu[e]));
                 } else {
                     v[e] = acc[t][u][e] * rinv + bv[e];
                 }
@@ -403,21 +406,21 @@ extern "C" int mv_gemm_tile_splits(int M, int N, int K, int gated, int force) {
 
 // (gemm_mid.hip) C = sum over f < F of work[f] (+ bias), or the gated activation of the two halves of the sum
 extern "C" int mv_gemm_mid_reduce(const float* work, const void* bias, void* C, long ldc, int c_dtype, int M, int N,
-                                  int F, int swiglu, hipStream_t stream);
+                                  int F, int swiglu, float limit, float slope, hipStream_t stream);
 
-// C[M, N] = A W^T (+ bias), or with `gated` C[M, N / 2] = silu(A Wg^T) * (A Wu^T) for the packed weight
+// C[M, N] = A W^T (+ bias), or with `gated` C[M, N / 2] = pair(A Wg^T (+ bias), A Wu^T (+ bias)) for the packed weight
 // [N = 2 I, K]. bf16 A (row stride lda) and W (contiguous rows of K), C bf16 or float (c_dtype).
 // K a multiple of 64. `work`: the float area mv_gemm_tile_workspace asks for (may be null when it
 // asks for none).
 static int tile_launch(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int c_dtype, int M,
                        int N, int K, int gated, float* work, long work_floats, int force, bool reduce,
-                       const float* partial, int P, float eps, hipStream_t stream) {
+                       const float* partial, int P, float eps, hipStream_t stream, GatedPair pair = GatedPair{0.f, 1.f}) {
     MV_REQUIRE(M > 0 && N > 0 && K > 0 && K % GT_KC == 0, "gemm_tile: K=%d must be a positive multiple of %d (M=%d, N=%d)",
                K, GT_KC, M, N);
     MV_REQUIRE(lda >= K && lda % 8 == 0, "gemm_tile: lda=%ld must be a multiple of 8 and at least K=%d", lda, K);
     MV_REQUIRE(((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0, "gemm_tile: operands must be 16-byte aligned");
     MV_REQUIRE(c_dtype == MV_F32 || c_dtype == MV_BF16, "gemm_tile: bad output dtype %d", c_dtype);
-    MV_REQUIRE(!gated || (N % 2 == 0 && bias == nullptr), "gemm_tile: the gated form takes an even N and no bias");
+    MV_REQUIRE(!gated || N % 2 == 0, "gemm_tile: the gated form takes an even N");
     MV_REQUIRE(ldc >= (gated ? N / 2 : N), "gemm_tile: ldc=%ld too small for N=%d", ldc, N);
     MV_REQUIRE((long)M * N < (1L << 31), "gemm_tile: %d x %d outputs exceed the index range", M, N);
     const TilePlan p = tile_plan(M, gated ? N / 2 : N, K, gated != 0, force);
@@ -428,7 +431,7 @@ static int tile_launch(const void* A, long lda, const void* W, const void* bias,
     MV_REQUIRE(partial == nullptr || (p.F == 1 && P > 0 && eps > 0.f),
                "gemm_tile: rows without their norm's division need an unsplit K (F=%d), their sums (P=%d) and eps", p.F, P);
     TileArgs a{(const bf16*)A, lda, (const bf16*)W, (const bf16*)bias, C, ldc, c_dtype == MV_F32, p.F > 1 ? work : nullptr,
-               M, N, K, p.F, p.chunks_per_split, p.tiles_m, p.tiles_n, gated ? N / 2 : 0, partial, P, eps};
+               M, N, K, p.F, p.chunks_per_split, p.tiles_m, p.tiles_n, gated ? N / 2 : 0, partial, P, eps, pair};
     const dim3 grid((unsigned)((long)p.tiles_m * p.tiles_n * p.F));
     // rings: 128 x 128 tiles 2 stages of 32 KB with two workgroups a compute unit, or 4 with one;
     // 64 x 128 and 128 x 64 3 stages of 24 KB, 64 x 64 4 stages of 16 KB, two workgroups a unit
@@ -448,15 +451,15 @@ static int tile_launch(const void* A, long lda, const void* W, const void* bias,
     }
 #undef GT_LAUNCH
     if (int rc = mv_check_launch("gemm_tile")) return rc;
-    if (p.F > 1 && reduce) return mv_gemm_mid_reduce(work, bias, C, ldc, c_dtype, M, N, p.F, gated, stream);
+    if (p.F > 1 && reduce) return mv_gemm_mid_reduce(work, bias, C, ldc, c_dtype, M, N, p.F, gated, pair.limit, pair.slope, stream);
     return 0;
 }
 
 extern "C" int mv_gemm_tile(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int c_dtype,
-                            int M, int N, int K, int gated, float* work, long work_floats, int force,
-                            hipStream_t stream) {
+                            int M, int N, int K, int gated, float* work, long work_floats, int force, float limit,
+                            float slope, hipStream_t stream) {
     return tile_launch(A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, true, nullptr, 0, 0.f,
-                       stream);
+                       stream, GatedPair{limit, slope});
 }
 
 // The same for rows that a product in front left weighted but not yet divided by their root mean
@@ -464,9 +467,10 @@ extern "C" int mv_gemm_tile(const void* A, long lda, const void* W, const void* 
 // Only for shapes whose K is not split (mv_gemm_tile_splits == 1).
 extern "C" int mv_gemm_tile_scaled(const void* A, long lda, const void* W, const void* bias, void* C, long ldc,
                                    int c_dtype, int M, int N, int K, int gated, const float* partial, int P, float eps,
-                                   hipStream_t stream) {
+                                   float limit, float slope, hipStream_t stream) {
     MV_REQUIRE(partial != nullptr, "gemm_tile_scaled: the partial sums are missing");
-    return tile_launch(A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, nullptr, 0, 0, true, partial, P, eps, stream);
+    return tile_launch(A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, nullptr, 0, 0, true, partial, P, eps, stream,
+                       GatedPair{limit, slope});
 }
 
 // The partial sums alone, for a shape whose K is split (mv_gemm_tile_splits > 1): work[f][m][n] =

@@ -167,11 +167,7 @@ struct MoeWeights {
 };
 
 __device__ __forceinline__ float moe_pair(float w, float g, float u, float limit, float slope) {
-    if (limit > 0.f) {
-        const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit);
-        return w * (gc / (1.f + expf(-slope * gc))) * (uc + 1.f);
-    }
-    return w * (g / (1.f + expf(-g))) * u;
+    return w * GatedPair{limit, slope}.of(g, u);
 }
 
 template <typename T>

@@ -10,7 +10,7 @@
 // cu_seqlens[s] .. cu_seqlens[s+1] are the rows of request s, state_slots[s] its row of the state
 // tensors. States are float (the shift's row has the activation type, it is a copy); decays,
 // rates, unit keys and the recurrence are float whatever the activation type T is.
-#include "dispatch.h"
+#include "recurrent.h"
 
 // ---------------------------------------------------------------------------------------
 // Token shift. One workgroup per row. The thread that serves column c of a request's first row
@@ -79,30 +79,6 @@ extern "C" int mv_token_shift(const void* h, long ldh, void* out, long ldo, cons
 #define DP_TOKENS 8
 #define DP_MAX_RANK 512
 #define DP_MAX_HEADS 260      // heads that 256 channels can touch, for head sizes >= 1
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-
-// NT sums over j in [j0, j1) of w2t[j][c] * th[t][j] (th rows `pitch` floats apart), the weight's element
-// type known at compile time and eight loads in flight at a time; the additions run in the order of j
-template <typename W, int NT>
-__device__ __forceinline__ void decay_dots(const W* __restrict__ w2t_c, size_t inner, const float* th, int pitch, int j0,
-                                           int j1, float (&acc)[NT]) {
-    int j = j0;
-    for (; j + 8 <= j1; j += 8) {
-        float w[8];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) w[e] = to_f(w2t_c[(size_t)(j + e) * inner]);
-#pragma unroll
-        for (int e = 0; e < 8; ++e)
-#pragma unroll
-            for (int t = 0; t < NT; ++t) acc[t] = fmaf(w[e], th[t * pitch + j + e], acc[t]);
-    }
-    for (; j < j1; ++j) {
-        const float w = to_f(w2t_c[(size_t)j * inner]);
-#pragma unroll
-        for (int t = 0; t < NT; ++t) acc[t] = fmaf(w, th[t * pitch + j], acc[t]);
-    }
-}
 
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -204,19 +180,6 @@ extern "C" int mv_delta_prepare(const void* packed, long ld, int n, int H, int D
 // computed. The request's state is read at the start and written at the end.
 // ---------------------------------------------------------------------------------------
 
-// the sum of a value over the L lanes that share a column (L = 4, 8 or 16 neighbouring lanes of a row
-// of 16): exchanges inside the row by data-parallel moves; every lane ends with the sum
-template <int L>
-__device__ __forceinline__ float lanes_sum(float v) {
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));   // quad [1,0,3,2]
-    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));   // quad [2,3,0,1]
-    if constexpr (L >= 8)
-        v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));  // mirror of 8
-    if constexpr (L >= 16)
-        v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));  // mirror of 16
-    return v;
-}
-
 template <int R>
 struct DeltaTokenRegs {
     float w[R], au[R], u[R], k[R], r[R], v;
@@ -251,37 +214,6 @@ __device__ __forceinline__ float delta_update(float (&s)[R], const DeltaTokenReg
         o = fmaf(t.r[e], x, o);
     }
     return lanes_sum<L>(o);
-}
-
-// a lane's R rows of its column, between registers and the column's D floats in memory (rows
-// sub*R .. sub*R+R-1; rows beyond D are zero and are not stored)
-template <int R, bool STORE>
-__device__ __forceinline__ void delta_state_io(float (&s)[R], float* column, int sub, int D, bool live) {
-    const int i0 = sub * R;
-    if ((D & 3) == 0) {
-#pragma unroll
-        for (int e = 0; e < R; e += 4) {
-            const bool ok = live && i0 + e < D;
-            float4* p = reinterpret_cast<float4*>(column + (i0 + e < D ? i0 + e : 0));
-            if constexpr (STORE) {
-                if (ok) *p = float4{s[e], s[e + 1], s[e + 2], s[e + 3]};
-            } else {
-                const float4 v = *p;                  // always issued (a valid address either way), dropped where it does not count
-                s[e] = ok ? v.x : 0.f; s[e + 1] = ok ? v.y : 0.f; s[e + 2] = ok ? v.z : 0.f; s[e + 3] = ok ? v.w : 0.f;
-            }
-        }
-    } else {
-#pragma unroll
-        for (int e = 0; e < R; ++e) {
-            const bool ok = live && i0 + e < D;
-            if constexpr (STORE) {
-                if (ok) column[i0 + e] = s[e];
-            } else {
-                const float v = column[i0 + e < D ? i0 + e : 0];
-                s[e] = ok ? v : 0.f;
-            }
-        }
-    }
 }
 
 // V4: the head size is a multiple of four, so the staged vectors come in 16 bytes a lane: a run of tokens
@@ -398,17 +330,6 @@ delta_scan_kernel(const T* __restrict__ packed, long ld, const float* __restrict
         __syncthreads();
     }
     delta_state_io<R, true>(s, S, sub, D, live);
-}
-
-// how a head of size D is dealt out: (rows a lane keeps, lanes a column); 0 when D is not served
-static void delta_scan_shape(int D, int& R, int& L) {
-    // few rows a lane and many lanes a column: a token costs the fewest instructions of the one wave a
-    // SIMD runs, and a head is spread over the most workgroups
-    if (D <= 16) { R = 4; L = 4; }
-    else if (D <= 32) { R = 4; L = 8; }
-    else if (D <= 64) { R = 4; L = 16; }
-    else if (D <= 128) { R = 8; L = 16; }
-    else { R = 16; L = 16; }
 }
 
 extern "C" int mv_delta_scan(const void* packed, long ld, const float* coef, float* state, const int* cu_seqlens,
@@ -651,22 +572,6 @@ extern "C" int mv_delta_finish(const float* raw, const void* packed, long ld, co
 // from the packed projection rows, the scan runs the recurrence request by request, the finish
 // kernel divides each head's output by its root mean square, applies weight and gate.
 // =======================================================================================
-#define MS_MAX_TAPS 16
-
-__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-// log(sigmoid(z)) without overflow
-__device__ __forceinline__ float logsigmoid_f(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
-
-// One input of the causal convolution: row r of the step when the request's rows reach back that far,
-// else the request's kept inputs (hist[slot][taps-1][C], the last one the newest).
-template <typename T>
-__device__ __forceinline__ float conv_input(const T* __restrict__ rows, long ld, const T* __restrict__ hist, int C, int taps,
-                                            int first, int r, int c) {
-    if (r >= first) return to_f(rows[(size_t)r * ld + c]);
-    return to_f(hist[(size_t)(taps - 1 + (r - first)) * C + c]);
-}
-
 // ---------------------------------------------------------------------------------------
 // Gated delta rule, prepare. Packed rows: [q (G*DK) | k (G*DK) | v (H*DV) | g (H*DV) | b (H) | a (H)].
 // q, k and v pass a causal convolution over time per channel (taps[c][j], the last tap the current
@@ -722,26 +627,6 @@ gdelta_prepare_kernel(const T* __restrict__ packed, long ld, int H, int G, int D
         g[2] = 0.f;
         g[3] = 0.f;
     }
-}
-
-// The convolution's kept inputs after the step: the last taps-1 inputs of each request, from the step's
-// rows and, where the step brought fewer, from what was kept before. Thread (request, channel) reads all
-// it needs before it writes, and no other thread touches its channel.
-template <typename T>
-__global__ void __launch_bounds__(256)
-conv_state_kernel(const T* __restrict__ packed, long ld, int C, int taps, T* __restrict__ conv_state,
-                  const int* __restrict__ cu_seqlens, const int* __restrict__ state_slots) {
-    const int seq = blockIdx.x;
-    const int c = blockIdx.y * 256 + threadIdx.x;
-    const int first = cu_seqlens[seq], end = cu_seqlens[seq + 1];
-    if (end <= first || c >= C) return;
-    T* hist = conv_state + (size_t)state_slots[seq] * (taps - 1) * C;
-    T keep[MS_MAX_TAPS];
-    for (int i = 0; i < taps - 1; ++i) {
-        const int r = end - (taps - 1) + i;
-        keep[i] = r >= first ? packed[(size_t)r * ld + c] : hist[(size_t)(taps - 1 + (r - first)) * C + c];
-    }
-    for (int i = 0; i < taps - 1; ++i) hist[(size_t)i * C + c] = keep[i];
 }
 
 // A causal convolution over time added to its own input, channel by channel:
@@ -1111,11 +996,13 @@ extern "C" int mv_state_scan(const float* qk, const float* vals, const float* ga
 // Finish. One wave per (row, head): the head's DV outputs (of DVS columns the scan wrote), with
 // `normaliser` divided by max(|column DV|, gates[2]) + denom_eps first; then
 //     y[d] = o[d] / sqrt(mean(o^2) + eps) * weight[shared ? d : head * DV + d] * act(g[head * DV + d])
-// act = SiLU (silu_gate) or the logistic function; g at column g_off of the packed rows.
+// act = SiLU (silu_gate) or the logistic function; g at column g_off of the packed rows (whose element type is
+// gate_dtype: the activation type, or float where another product made the gates). `gates` may be null without a
+// normaliser.
 // ---------------------------------------------------------------------------------------
 template <typename T>
 __global__ void __launch_bounds__(256)
-state_finish_kernel(const float* __restrict__ raw, const float* __restrict__ gates, const T* __restrict__ packed, long ld,
+state_finish_kernel(const float* __restrict__ raw, const float* __restrict__ gates, WeightPtr packed, long ld,
                     long g_off, WeightPtr weight, int shared_weight, int silu_gate, int normaliser, float denom_eps, int H,
                     int DV, int DVS, float eps, const int* __restrict__ token_seq, T* __restrict__ out, long ldo, int n) {
     const int lane = threadIdx.x % MV_WAVE;
@@ -1137,9 +1024,9 @@ state_finish_kernel(const float* __restrict__ raw, const float* __restrict__ gat
     }
     ss = wave_sum(ss);
     const float rinv = scale / sqrtf(ss / (float)DV + eps);
-    const T* g = packed + (size_t)t * ld + g_off + (size_t)head * DV;
+    const size_t g = (size_t)t * ld + g_off + (size_t)head * DV;
     for (int d = lane; d < DV; d += MV_WAVE) {
-        const float z = to_f(g[d]);
+        const float z = packed.at(g + d);
         const float act = silu_gate ? silu_f(z) : sigmoid_f(z);
         y[d] = from_f<T>(o[d] * rinv * weight.at(shared_weight ? d : (size_t)head * DV + d) * act);
     }
@@ -1148,16 +1035,17 @@ state_finish_kernel(const float* __restrict__ raw, const float* __restrict__ gat
 extern "C" int mv_state_finish(const float* raw, const float* gates, const void* packed, long ld, long g_off,
                                const void* weight, int weight_dtype, int shared_weight, int silu_gate, int normaliser,
                                float denom_eps, int n, int H, int DV, float eps, const int* token_seq, void* out, long ldo,
-                               int dtype, hipStream_t stream) {
+                               int gate_dtype, int dtype, hipStream_t stream) {
     MV_REQUIRE(n >= 0 && H > 0 && DV > 0 && eps > 0.f, "state_finish: bad sizes n=%d H=%d DV=%d", n, H, DV);
     MV_REQUIRE(g_off >= 0 && ld >= g_off + (long)H * DV && ldo >= (long)H * DV, "state_finish: row pitches too small");
-    MV_REQUIRE(mv_valid_dtype(weight_dtype) && raw && gates && packed && weight && token_seq && out, "state_finish: missing operand");
+    MV_REQUIRE(mv_valid_dtype(weight_dtype) && mv_valid_dtype(gate_dtype) && raw && (gates || !normaliser) && packed && weight && token_seq && out,
+               "state_finish: missing operand");
     if (n == 0) return 0;
     const long units = (long)n * H;
     WeightPtr w{weight, weight_dtype};
     MV_DISPATCH_T(dtype, "state_finish",
                   hipLaunchKernelGGL(state_finish_kernel<T>, dim3((unsigned)((units + 3) / 4)), dim3(256), 0, stream, raw, gates,
-                                     (const T*)packed, ld, g_off, w, shared_weight, silu_gate, normaliser, denom_eps, H, DV,
+                                     WeightPtr{packed, gate_dtype}, ld, g_off, w, shared_weight, silu_gate, normaliser, denom_eps, H, DV,
                                      DV + (normaliser ? 1 : 0), eps, token_seq, (T*)out, ldo, n));
     return mv_check_launch("state_finish");
 }

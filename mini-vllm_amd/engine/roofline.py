@@ -80,6 +80,15 @@ KERNELS_OF: Dict[str, Tuple[str, Optional[str], int]] = {
     "mv_qkv_rotate_norm_store": (r"\bqkv_rotate_norm_store(_vec)?_kernel", r"\bstore_v_pages_kernel", 2),
     "mv_moe_table_route": (r"\bmoe_table_route_kernel", None, 1),
     "mv_add_rows": (r"\badd_rows_kernel", None, 1),
+    "mv_qkv_row_norm_store": (r"\bqkv_row_norm_store_kernel", r"\bstore_v_pages_kernel", 2),
+    "mv_constant_prepare": (r"\bconstant_prepare_kernel", None, 1),
+    "mv_row_gate_finish": (r"\brow_gate_finish_kernel", None, 1),
+    "mv_constant_step": (r"\bconstant_step_kernel", None, 1),
+    "mv_pair_norm_add_norm": (r"\bpair_norm_add_norm_kernel", None, 1),
+    "mv_stream_entry": (r"\bstream_entry_kernel", None, 1),
+    "mv_channel_prepare": (r"\bchannel_prepare_kernel", r"\bconv_state_kernel", 2),
+    "mv_channel_scan": (r"\bchannel_scan_kernel", None, 1),
+    "mv_channel_step": (r"\bchannel_step_kernel", r"\bconv_state_kernel", 2),
 }
 _OURS = re.compile("|".join(f"(?:{p})" for spec in KERNELS_OF.values() for p in spec[:2] if p))
 

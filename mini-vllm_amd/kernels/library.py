@@ -40,20 +40,59 @@ _SIGNATURES = {
                                       c_void_p, c_int, c_int, c_int, c_int, c_void_p]),  # table, rot, inter, store, dtype
     "mv_store_v_pages": (c_int, [c_void_p, c_long, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
                                  c_int, c_int, c_int, c_int, c_void_p]),
-    "mv_swiglu": (c_int, [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
+    "mv_swiglu": (c_int, [c_void_p, c_void_p, c_int, c_int, c_float, c_float, c_int, c_void_p]),
     "mv_gemm_ref": (c_int, [c_void_p, c_long, c_int, c_void_p, c_long, c_int, c_void_p, c_void_p, c_long, c_int,
                             c_int, c_int, c_int, c_void_p]),
     # q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_width, page_size, positions, token_seq, n, H, Hkv, D,
-    # Dv, scale, window, first, gate, gate_stride, dtype, stream
+    # Dv, scale, window, first, gate, gate_stride, cap, slopes, sink, dtype, stream
     "mv_attention_ref": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                  c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_long,
-                                 c_int, c_void_p]),
+                                 c_float, c_void_p, c_int, c_int, c_void_p]),
     # qkv, stride, q_off, k_off, v_off, positions, token_seq, block_table, bt_width, page_size, k_pages, v_pages, n, H, Hkv, D,
     # Dv, q_weight, k_weight, weight_dtype, unit_norm, eps, table, rot_dim, interleaved, mix_rows, mix_stride, mix_weight,
     # mix_weight_dtype, dtype, stream
     "mv_qkv_rotate_norm_store": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                          c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int,
                                          c_float, c_void_p, c_int, c_int, c_void_p, c_long, c_void_p, c_int, c_int, c_void_p]),
+    # rows, stride, q_off, k_off, v_off, positions, token_seq, block_table, bt_width, page_size, k_pages, v_pages, n, H, Hkv,
+    # D, Dv, q_weight, k_weight, weight_dtype, eps, temp_coef, temp_every, dtype, stream
+    "mv_qkv_row_norm_store": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
+                                      c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_float,
+                                      c_int, c_int, c_void_p]),
+    # packed, ld, off, n, H, DK, DV, decay, token_seq, qk, vals, gates, dtype, stream
+    "mv_constant_prepare": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                                    c_void_p, c_int, c_void_p]),
+    # raw, packed, ld, g_off, weight, weight_dtype, n, W, eps, token_seq, out, ldo, dtype, stream
+    "mv_row_gate_finish": (c_int, [c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p,
+                                   c_long, c_int, c_void_p]),
+    # packed, ld, off, n, H, DK, DV, decay, weight, weight_dtype, state, token_seq, state_slots, out, ldo, sums, then the row
+    # norm beside it: rows, stride, q_off, k_off, v_off, positions, block_table, bt_width, page_size, k_pages, v_pages, H, Hkv,
+    # D, Dv, q_weight, k_weight, norm_dtype, eps, temp_coef, temp_every, dtype, stream
+    "mv_constant_step": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
+                                 c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p,
+                                 c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_float,
+                                 c_float, c_int, c_int, c_void_p]),
+    # ya, lda, wa, sums_a, parts_a, inner_a, yb, ldb, wb, sums_b, parts_b, inner_b, pair_dtype, eps, inner_eps, resid, wn,
+    # wn_dtype, eps_n, unit_n, out, ldo, n, h, dtype, stream
+    "mv_pair_norm_add_norm": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p,
+                                      c_int, c_int, c_int, c_float, c_float, c_void_p, c_void_p, c_int, c_float, c_int, c_void_p,
+                                      c_long, c_int, c_int, c_int, c_void_p]),
+    # resid, delta, ldd, ids, table, table_dtype, vocab, scale, step, step_dtype, wn, wn_dtype, eps, unit, out, n, h, dtype, stream
+    "mv_stream_entry": (c_int, [c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_void_p,
+                                c_int, c_float, c_int, c_void_p, c_int, c_int, c_int, c_void_p]),
+    # packed, ld, n, n_seqs, H, G, DK, DV, taps, b_off, conv_w, a_log, dt_bias, weight_dtype, conv_state, unit_eps, token_seq,
+    # cu_seqlens, state_slots, qk, vals, beta, z, ldz, dtype, stream
+    "mv_channel_prepare": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
+                                   c_void_p, c_int, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                   c_void_p, c_long, c_int, c_void_p]),
+    # qk, vals, beta, decay, ldz, state, cu_seqlens, state_slots, n_seqs, n, H, G, DK, DV, out, stream
+    "mv_channel_scan": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                                c_int, c_int, c_int, c_void_p, c_void_p]),
+    # packed, ld, n, n_seqs, H, G, DK, DV, taps, b_off, low_off, ra, rg, conv_w, a_log, dt_bias, a2t, g2t, norm_w, weight_dtype,
+    # conv_state, state, unit_eps, eps, token_seq, cu_seqlens, state_slots, out, ldo, dtype, stream
+    "mv_channel_step": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float,
+                                c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p]),
     # lanes, plane, first, S, n, W, y, ldy, w_mix, w_out, w_in, w_norm, norm_dtype, eps, h, ldh, total, dtype, stream
     "mv_hyper_step": (c_int, [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p,
                               c_void_p, c_int, c_float, c_void_p, c_long, c_void_p, c_int, c_void_p]),
@@ -123,18 +162,20 @@ _OPTIONAL_SIGNATURES = {
                                c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_float, c_float, c_void_p]),
     "mv_gemm_skinny": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int,
                                c_int, c_int, c_int, c_void_p]),
-    "mv_gemm_skinny_swiglu": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_void_p]),
+    # A, lda, W, bias, out, ldo, M, I, K, limit, slope, stream
+    "mv_gemm_skinny_swiglu": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_float, c_float,
+                                      c_void_p]),
     "mv_gemm_skinny_fold_parts": (c_int, [c_int, c_int, c_int]),
     # A, lda, W, bias, resid, ldr, norm_weight, norm_weight_dtype, unit_offset, weighted, ldw, partial, P, M, N, K, stream
     "mv_gemm_skinny_fold": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_int, c_int,
                                     c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
     # A, lda, W, bias, C, ldc, partial, P, eps, M, N, K, swiglu, stream
     "mv_gemm_skinny_scaled": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_int, c_float,
-                                      c_int, c_int, c_int, c_int, c_void_p]),
+                                      c_int, c_int, c_int, c_int, c_float, c_float, c_void_p]),
     # weighted, ldw, partial, P, eps, out, ldo, dtype, M, width, stream
     "mv_scale_rows": (c_int, [c_void_p, c_long, c_void_p, c_int, c_float, c_void_p, c_long, c_int, c_int, c_int, c_void_p]),
     "mv_gemm_skinny_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_float, c_int, c_void_p, c_void_p,
-                                    c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+                                    c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p]),
     "mv_gemm_lt_workspace": (c_long, []),
     # A, lda, W, bias, C, ldc, c_dtype, M, N, K, workspace, workspace_bytes, stream
     "mv_gemm_lt": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p,
@@ -143,30 +184,33 @@ _OPTIONAL_SIGNATURES = {
     "mv_gemm_mid_splits": (c_int, [c_int, c_int]),
     # A, lda, W, M, N, K, work, work_floats, stream
     "mv_gemm_mid_sums": (c_int, [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_void_p]),
-    # work, bias, C, ldc, c_dtype, M, N, F, swiglu, stream
-    "mv_gemm_mid_reduce": (c_int, [c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+    # work, bias, C, ldc, c_dtype, M, N, F, swiglu, limit, slope, stream
+    "mv_gemm_mid_reduce": (c_int, [c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_float, c_float,
+                                   c_void_p]),
     # resid, part, F, plane, bias, weight, weight_dtype, eps, unit_offset, out, rows, n_out, h, dtype, stream
     "mv_add_rmsnorm_split": (c_int, [c_void_p, c_void_p, c_int, c_long, c_void_p, c_void_p, c_int, c_float, c_int,
                                      c_void_p, c_void_p, c_int, c_int, c_int, c_void_p]),
     # A, lda, W, bias, C, ldc, c_dtype, M, N, K, swiglu, work, work_floats, stream
     "mv_gemm_mid": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int,
-                            c_void_p, c_long, c_void_p]),
+                            c_void_p, c_long, c_float, c_float, c_void_p]),
     "mv_device_compute_units": (c_int, []),
     "mv_gemm_tile_workspace": (c_long, [c_int, c_int, c_int, c_int, c_int]),
     "mv_gemm_tile_splits": (c_int, [c_int, c_int, c_int, c_int, c_int]),
-    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, stream
+    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, limit, slope, stream
     "mv_gemm_tile": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int,
-                             c_void_p, c_long, c_int, c_void_p]),
+                             c_void_p, c_long, c_int, c_float, c_float, c_void_p]),
     # A, lda, W, M, N, K, work, work_floats, force, stream
     "mv_gemm_tile_sums": (c_int, [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_void_p]),
-    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, partial, P, eps, stream
+    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, partial, P, eps, limit, slope, stream
     "mv_gemm_tile_scaled": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int,
-                                    c_int, c_void_p, c_int, c_float, c_void_p]),
+                                    c_int, c_void_p, c_int, c_float, c_float, c_float, c_void_p]),
     # q, q_stride, out, out_stride, k_pages, v_pages, block_table, bt_width, page_size, positions, cu_seqlens, n_seqs, H, Hkv,
-    # D, scale, window, partials, counters, nsplit, max_pages, waves, token_seq, first, gate, gate_stride, stream
+    # D, scale, window, partials, counters, nsplit, max_pages, waves, token_seq, first, gate, gate_stride, cap, slopes, sink,
+    # stream
     "mv_attention_decode": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                     c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_float, c_int,
-                                    c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_long, c_void_p]),
+                                    c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_long, c_float, c_void_p,
+                                    c_int, c_void_p]),
     # qkv, stride, q_off, k_off, v_off, out, out_stride, k_pages, v_pages, block_table, bt_width, page_size,
     # positions, cu_seqlens, n_seqs, H, Hkv, D, scale, window, q_weight, k_weight, weight_dtype, eps, unit_offset,
     # table, rows, store_kv, partials, counters, nsplit, max_pages, waves, token_seq, stream
@@ -177,10 +221,11 @@ _OPTIONAL_SIGNATURES = {
     # ids, table, table_dtype, resid, n, h, vocab, scale, ids2, table2, out2, h2, rows2, stream
     "mv_embedding_gather": (c_int, [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p,
                                     c_void_p, c_int, c_int, c_void_p]),
-    # ..., positions, cu_seqlens, n_seqs, n_units, n_busy, nt, kw, H, Hkv, D, scale, window, first, gate, gate_stride, stream
+    # ..., positions, cu_seqlens, n_seqs, n_units, n_busy, nt, kw, H, Hkv, D, scale, window, first, gate, gate_stride, cap, slopes,
+    # sink, stream
     "mv_attention_prefill": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int,
                                      c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                     c_float, c_int, c_int, c_void_p, c_long, c_void_p]),
+                                     c_float, c_int, c_int, c_void_p, c_long, c_float, c_void_p, c_int, c_void_p]),
     "mv_attention_prefill_unit_tokens": (c_int, [c_int, c_int]),
     # as mv_attention_prefill up to window, then chunk, bias, gate, gate_stride, stream
     "mv_attention_prefill_sigmoid": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int,
@@ -204,9 +249,9 @@ _OPTIONAL_SIGNATURES = {
                               c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_float,
                               c_float, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p]),
     # raw, gates, packed, ld, g_off, weight, weight_dtype, shared_weight, silu_gate, normaliser, denom_eps, n, H, DV, eps,
-    # token_seq, out, ldo, dtype, stream
+    # token_seq, out, ldo, gate_dtype, dtype, stream
     "mv_state_finish": (c_int, [c_void_p, c_void_p, c_void_p, c_long, c_long, c_void_p, c_int, c_int, c_int, c_int, c_float,
-                                c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_long, c_int, c_void_p]),
+                                c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_long, c_int, c_int, c_void_p]),
     # packed, ld, n, QR, R, DR, wq, wkv, weight_dtype, eps, table, table_rows, positions, token_seq, block_table, bt_width,
     # page_size, cq, ldq, pages, pages_t, dtype, stream
     "mv_latent_prepare": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_float, c_void_p,

@@ -149,7 +149,7 @@ class SplitSum:
             M, N = self.out.shape
             self.ops.lib.call("mv_gemm_mid_reduce", self.work.data_ptr(), _ptr(self.bias), self.out.data_ptr(),
                               self.out.stride(0) if M > 1 else N, _CODES[self.out.dtype], M, N, self.splits, 0,
-                              self.ops._stream())
+                              0.0, 1.0, self.ops._stream())
             self.discard()
         return self.out
 
@@ -188,6 +188,37 @@ class WeightedRows:
             self.ops.scale_rows(self.weighted, self.partial, self.P, self.eps, self.normed)
             self._done = True
         return self.normed
+
+
+class RowSums:
+    """Rows whose division by their root mean square is still to be done behind the linear map they go through:
+    ``sums`` float32 [rows, parts] are parts of each row's sum of squares over ``inner`` columns, ``eps`` is the norm's."""
+
+    def __init__(self, sums: torch.Tensor, inner: int, eps: float):
+        self.sums, self.inner, self.eps = sums, int(inner), float(eps)
+
+
+class NormedPair:
+    """A residual delta that exists only as the output rows of two parts that ran side by side: half the sum of
+    the two, each divided by its root mean square over the row and multiplied by a weight of its own. The next
+    residual add + norm takes it as it is (``Ops.add_rmsnorm``); anything else calls ``materialize``. ``sums``: per
+    side a ``RowSums`` when the rows that went into the side's linear map were not divided by theirs, or None."""
+
+    is_normed_pair = True
+
+    def __init__(self, ops: "Ops", sides, weights, eps: float, sums, out: torch.Tensor):
+        self.ops, self.sides, self.weights, self.eps, self.sums, self.out = ops, sides, weights, float(eps), sums, out
+        self.shape = out.shape
+        self.done = False
+
+    def materialize(self) -> torch.Tensor:
+        if not self.done:
+            self.ops.pair_norm(self, None, None, self.out)
+            self.done = True
+        return self.out
+
+    def discard(self) -> None:
+        self.done = True
 
 
 class Ops:
@@ -302,6 +333,12 @@ class Ops:
         n, h = resid.shape
         if isinstance(delta, SplitSum):
             if self._add_rmsnorm_split(resid, delta, weight, eps, out, rows, unit_offset):
+                return
+            delta = delta.materialize()
+        if isinstance(delta, NormedPair):
+            if rows is None and not delta.done:
+                self.pair_norm(delta, resid, None if out is None else (weight, eps, unit_offset), out)
+                delta.discard()
                 return
             delta = delta.materialize()
         if delta is not None:
@@ -793,28 +830,32 @@ class Ops:
         self.lib.call("mv_state_scan", qk.data_ptr(), vals.data_ptr(), gates.data_ptr(), state.data_ptr(), cu_seqlens.data_ptr(),
                       state_slots.data_ptr(), n_seqs, n, heads, groups, dk, dvs, int(bool(read)), out.data_ptr(), self._stream())
 
-    def state_finish(self, raw: torch.Tensor, gates: torch.Tensor, packed: torch.Tensor, gate_offset: int, weight: torch.Tensor,
+    def state_finish(self, raw: torch.Tensor, gates: Optional[torch.Tensor], packed: torch.Tensor, gate_offset: int, weight: torch.Tensor,
                      heads: int, dv: int, eps: float, token_seq: torch.Tensor, out: torch.Tensor, shared_weight: bool,
                      silu_gate: bool, normaliser: bool = False, denom_eps: float = 0.0) -> None:
         """out[t, h] = o / rms(o) * weight * act(g) per head, o = raw[t, h, :dv]; with ``normaliser`` o is first divided
         by max(|raw[t, h, dv]|, gates[t, h, 2]) + denom_eps. ``weight`` holds dv numbers shared by the heads or
-        heads*dv; act is SiLU or the logistic function; g are ``heads*dv`` columns of ``packed`` from ``gate_offset``."""
-        self._act(packed, "mixer rows"); self._act(out, "mixer output"); _dev(weight, "output norm weight")
+        heads*dv; act is SiLU or the logistic function; g are ``heads*dv`` columns of ``packed``
+        (activation type or float32) from ``gate_offset``."""
+        _dev(packed, "mixer rows"); self._act(out, "mixer output"); _dev(weight, "output norm weight")
+        if packed.dtype not in (self.dtype, torch.float32) or packed.stride(1) != 1:
+            raise KernelLibraryError(f"state_finish: gates of dtype {packed.dtype}, {self.dtype} or float32 are served")
         n, dvs = packed.shape[0], dv + (1 if normaliser else 0)
         if raw.dtype != torch.float32 or tuple(raw.shape) != (n, heads, dvs) or not raw.is_contiguous():
             raise KernelLibraryError(f"state_finish: the scan's output must be float32 [{n}, {heads}, {dvs}]")
-        if gates.dtype != torch.float32 or tuple(gates.shape) != (n, heads, 4) or not gates.is_contiguous():
+        if (gates is None and normaliser) or (gates is not None and (
+                gates.dtype != torch.float32 or tuple(gates.shape) != (n, heads, 4) or not gates.is_contiguous())):
             raise KernelLibraryError("state_finish: gates must be float32 [n, heads, 4]")
         if tuple(out.shape) != (n, heads * dv) or out.stride(1) != 1 or packed.shape[1] < gate_offset + heads * dv \
                 or weight.numel() != (dv if shared_weight else heads * dv) or not weight.is_contiguous():
             raise KernelLibraryError("state_finish: operands do not fit")
         self._ints(n, token_seq=(token_seq, n))
         self._note("mv_state_finish", self._size(raw, out) + n * heads * dv * packed.element_size(), 8 * n * heads * dv)
-        self.lib.call("mv_state_finish", raw.data_ptr(), gates.data_ptr(), packed.data_ptr(),
+        self.lib.call("mv_state_finish", raw.data_ptr(), _ptr(gates), packed.data_ptr(),
                       packed.stride(0) if n > 1 else packed.shape[1], int(gate_offset), weight.data_ptr(),
                       _weight_code(weight, "output norm weight"), int(shared_weight), int(silu_gate), int(normaliser),
                       float(denom_eps), n, heads, dv, float(eps), token_seq.data_ptr(), out.data_ptr(),
-                      out.stride(0) if n > 1 else heads * dv, self.code, self._stream())
+                      out.stride(0) if n > 1 else heads * dv, _CODES[packed.dtype], self.code, self._stream())
 
     def state_step(self, delta: bool, packed: torch.Tensor, heads: int, groups: int, dk: int, dv: int, norm_weight: torch.Tensor,
                    eps: float, state: torch.Tensor, token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor,
@@ -869,6 +910,315 @@ class Ops:
 
     # ------------------------------------------------------------------------------------
     # attention over a cached latent
+    # ------------------------------------------------------------------------------------
+    # gated delta rule with a decay per head and key channel
+    # ------------------------------------------------------------------------------------
+    def _channel_operands(self, what: str, packed: torch.Tensor, heads: int, groups: int, dk: int, dv: int, taps: int, b_off: int,
+                          conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, conv_state: Optional[torch.Tensor],
+                          token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int) -> int:
+        self._act(packed, "delta rows")
+        n, C = packed.shape[0], 2 * groups * dk + heads * dv
+        if packed.dim() != 2 or packed.stride(1) != 1 or b_off < C or packed.shape[1] < b_off + heads:
+            raise KernelLibraryError(f"{what}: rows {tuple(packed.shape)} are too short")
+        for t, shape, name in ((conv_w, (C, taps), "convolution taps"), (a_log, (heads,), "A_log"), (dt_bias, (heads * dk,), "dt_bias")):
+            _dev(t, name)
+            if tuple(t.shape) != shape or not t.is_contiguous() or t.dtype != conv_w.dtype:
+                raise KernelLibraryError(f"{what}: {name} must be a contiguous {shape} tensor of the taps' dtype")
+        if taps > 1:
+            self._act(conv_state, "convolution state")
+            if conv_state.dim() != 3 or tuple(conv_state.shape[1:]) != (taps - 1, C) or not conv_state.is_contiguous():
+                raise KernelLibraryError(f"{what}: the convolution's state must be [slots, {taps - 1}, {C}]")
+        self._ints(n, token_seq=(token_seq, n), cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        return n
+
+    def _matrix_state(self, what: str, state: torch.Tensor, heads: int, dv: int, dk: int) -> None:
+        _dev(state, "matrix state")
+        if state.dtype != torch.float32 or state.dim() != 4 or tuple(state.shape[1:]) != (heads, dv, dk) or not state.is_contiguous():
+            raise KernelLibraryError(f"{what}: the state must be float32 [slots, {heads}, {dv}, {dk}]")
+
+    def channel_prepare(self, packed: torch.Tensor, heads: int, groups: int, dk: int, dv: int, taps: int, b_off: int,
+                        conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, conv_state: Optional[torch.Tensor],
+                        unit_eps: float, token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int,
+                        qk: torch.Tensor, vals: torch.Tensor, beta: torch.Tensor, z: torch.Tensor) -> None:
+        """From rows [q (groups*dk) | k (groups*dk) | v (heads*dv) | ...] with b (heads) at column ``b_off``: q, k, v through
+        a causal convolution (conv_w [channels, taps], last tap the current token) and SiLU; q and k unit vectors per group
+        (q times dk^-1/2) into qk float32 [n, groups, 2, dk], v into vals [n, heads, dv], beta [n, heads] = sigmoid(b). The
+        first heads*dk columns of z (float32 rows) turn in place into exp(-exp(a_log[head]) softplus(z + dt_bias)).
+        conv_state [slots, taps-1, channels]: read for the rows in front of the step, then advanced."""
+        n = self._channel_operands("channel_prepare", packed, heads, groups, dk, dv, taps, b_off, conv_w, a_log, dt_bias, conv_state,
+                                   token_seq, cu_seqlens, state_slots, n_seqs)
+        for t, shape, name in ((qk, (n, groups, 2, dk), "queries and keys"), (vals, (n, heads, dv), "values"), (beta, (n, heads), "beta")):
+            _dev(t, name)
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"channel_prepare: {name} must be contiguous float32 {shape}")
+        _dev(z, "decay rows")
+        if z.dtype != torch.float32 or z.dim() != 2 or z.shape[0] != n or z.shape[1] < heads * dk or z.stride(1) != 1:
+            raise KernelLibraryError(f"channel_prepare: decay rows must be float32 [{n}, >= {heads * dk}]")
+        C = 2 * groups * dk + heads * dv
+        self._note("mv_channel_prepare", n * (C + heads) * packed.element_size() + self._size(qk, vals, beta) + 8 * n * heads * dk,
+                   2 * n * C * taps + 8 * n * C + 16 * n * heads * dk)
+        self.lib.call("mv_channel_prepare", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], n, n_seqs, heads, groups,
+                      dk, dv, taps, int(b_off), conv_w.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),
+                      _weight_code(conv_w, "convolution taps"), _ptr(conv_state), float(unit_eps), token_seq.data_ptr(),
+                      cu_seqlens.data_ptr(), state_slots.data_ptr(), qk.data_ptr(), vals.data_ptr(), beta.data_ptr(), z.data_ptr(),
+                      z.stride(0) if n > 1 else z.shape[1], self.code, self._stream())
+
+    def channel_scan(self, qk: torch.Tensor, vals: torch.Tensor, beta: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+                     cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int, heads: int, groups: int, dk: int, dv: int,
+                     out: torch.Tensor) -> None:
+        """Per request and head, token by token: S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; out = S^T q, g the
+        head's dk columns of ``decay`` (float32 rows). state float32 [slots, heads, dv, dk] is read and left advanced."""
+        n = vals.shape[0]
+        for t, shape, name in ((qk, (n, groups, 2, dk), "queries and keys"), (vals, (n, heads, dv), "values"), (beta, (n, heads), "beta"),
+                               (out, (n, heads, dv), "scan output")):
+            _dev(t, name)
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"channel_scan: {name} must be contiguous float32 {shape}")
+        _dev(decay, "decays")
+        if decay.dtype != torch.float32 or decay.dim() != 2 or decay.shape[0] != n or decay.shape[1] < heads * dk or decay.stride(1) != 1:
+            raise KernelLibraryError(f"channel_scan: decays must be float32 [{n}, >= {heads * dk}]")
+        self._matrix_state("channel_scan", state, heads, dv, dk)
+        self._ints(n, cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        self._note("mv_channel_scan", self._size(qk, vals, beta, out) + 4 * n * heads * dk
+                   + 2 * min(n_seqs, max(n, 1)) * heads * dv * dk * 4, 7 * n * heads * dv * dk)
+        self.lib.call("mv_channel_scan", qk.data_ptr(), vals.data_ptr(), beta.data_ptr(), decay.data_ptr(),
+                      decay.stride(0) if n > 1 else decay.shape[1], state.data_ptr(), cu_seqlens.data_ptr(), state_slots.data_ptr(),
+                      n_seqs, n, heads, groups, dk, dv, out.data_ptr(), self._stream())
+
+    def channel_step(self, packed: torch.Tensor, heads: int, groups: int, dk: int, dv: int, taps: int, b_off: int, low_off: int,
+                     conv_w: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor, a2t: torch.Tensor, g2t: torch.Tensor,
+                     norm_weight: torch.Tensor, conv_state: Optional[torch.Tensor], state: torch.Tensor, unit_eps: float, eps: float,
+                     token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int,
+                     out: torch.Tensor) -> bool:
+        """For a step in which every request brings one token: ``channel_prepare``, ``channel_scan``, the head's norm and the
+        output gate as one kernel per (row, head). The rows hold W_a1 h and W_g1 h side by side from column ``low_off``;
+        a2t [rank, heads*dk] and g2t [rank, heads*dv] are the transposed second matrices. False when the sizes are not
+        served (nothing was done)."""
+        n = self._channel_operands("channel_step", packed, heads, groups, dk, dv, taps, b_off, conv_w, a_log, dt_bias, conv_state,
+                                   token_seq, cu_seqlens, state_slots, n_seqs)
+        ra, rg = a2t.shape[0], g2t.shape[0]
+        for t, shape, name in ((a2t, (ra, heads * dk), "second decay matrix"), (g2t, (rg, heads * dv), "second gate matrix"),
+                               (norm_weight, (dv,), "output norm weight")):
+            _dev(t, name)
+            if tuple(t.shape) != shape or not t.is_contiguous() or t.dtype != conv_w.dtype:
+                raise KernelLibraryError(f"channel_step: the {name} must be a contiguous {shape} tensor of the taps' dtype")
+        self._act(out, "mixer output")
+        if packed.shape[1] < low_off + ra + rg or tuple(out.shape) != (n, heads * dv) or out.stride(1) != 1:
+            raise KernelLibraryError("channel_step: operands do not fit")
+        self._matrix_state("channel_step", state, heads, dv, dk)
+        if not self.lib.offer("mv_channel_step", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], n, n_seqs, heads,
+                              groups, dk, dv, taps, int(b_off), int(low_off), ra, rg, conv_w.data_ptr(), a_log.data_ptr(),
+                              dt_bias.data_ptr(), a2t.data_ptr(), g2t.data_ptr(), norm_weight.data_ptr(),
+                              _weight_code(conv_w, "convolution taps"), _ptr(conv_state), state.data_ptr(), float(unit_eps), float(eps),
+                              token_seq.data_ptr(), cu_seqlens.data_ptr(), state_slots.data_ptr(), out.data_ptr(),
+                              out.stride(0) if n > 1 else heads * dv, self.code, self._stream()):
+            return False
+        self._note("mv_channel_step", n * packed.shape[1] * packed.element_size() + self._size(out, a2t, g2t)
+                   + 2 * n * heads * dv * dk * 4, n * heads * (7 * dv * dk + 2 * (ra * dk + rg * dv)))
+        return True
+
+    # ------------------------------------------------------------------------------------
+    # linear attention with one constant decay per head; parts side by side; entries into the residual stream
+    # ------------------------------------------------------------------------------------
+    def _constant_rows(self, what: str, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, decay: torch.Tensor,
+                       token_seq: torch.Tensor) -> int:
+        self._act(packed, "mixer rows"); _dev(decay, "decays")
+        n = packed.shape[0]
+        if packed.dim() != 2 or packed.stride(1) != 1 or packed.shape[1] < offset + 2 * heads * (dk + dv):
+            raise KernelLibraryError(f"{what}: rows {tuple(packed.shape)} are too short")
+        if decay.dtype != torch.float32 or decay.numel() != heads or not decay.is_contiguous():
+            raise KernelLibraryError(f"{what}: the decays must be float32 [{heads}]")
+        self._ints(n, token_seq=(token_seq, n))
+        return n
+
+    def constant_prepare(self, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, decay: torch.Tensor,
+                         token_seq: torch.Tensor, qk: torch.Tensor, vals: torch.Tensor, gates: torch.Tensor) -> None:
+        """From rows [q | k (heads*dk each) | v (heads*dv) | ...] at column ``offset``: SiLU of q, k and v as floats, and
+        gates (decay[head], 1, 0, 0), in the layouts ``state_scan`` takes."""
+        n = self._constant_rows("constant_prepare", packed, offset, heads, dk, dv, decay, token_seq)
+        self._state_vectors(n, heads, heads, dk, dv, qk, vals, gates, "constant_prepare")
+        self._note("mv_constant_prepare", n * heads * (2 * dk + dv) * packed.element_size() + self._size(qk, vals, gates),
+                   6 * n * heads * (2 * dk + dv))
+        self.lib.call("mv_constant_prepare", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(offset), n, heads,
+                      dk, dv, decay.data_ptr(), token_seq.data_ptr(), qk.data_ptr(), vals.data_ptr(), gates.data_ptr(), self.code,
+                      self._stream())
+
+    def row_gate_finish(self, raw: torch.Tensor, packed: torch.Tensor, gate_offset: int, weight: torch.Tensor, eps: float,
+                        token_seq: torch.Tensor, out: torch.Tensor) -> None:
+        """out[t] = o / rms(o) * weight * sigmoid(g), the root mean square over the whole row of o = raw[t] (all heads
+        together); g are as many columns of ``packed`` from ``gate_offset``."""
+        self._act(packed, "mixer rows"); self._act(out, "mixer output"); _dev(weight, "output norm weight")
+        n, W = out.shape
+        if raw.dtype != torch.float32 or raw.numel() != n * W or not raw.is_contiguous() or packed.shape[0] != n \
+                or packed.shape[1] < gate_offset + W or packed.stride(1) != 1 or out.stride(1) != 1 or weight.numel() != W \
+                or not weight.is_contiguous():
+            raise KernelLibraryError("row_gate_finish: operands do not fit")
+        self._ints(n, token_seq=(token_seq, n))
+        self._note("mv_row_gate_finish", self._size(raw, out) + n * W * packed.element_size(), 8 * n * W)
+        self.lib.call("mv_row_gate_finish", raw.data_ptr(), packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1],
+                      int(gate_offset), weight.data_ptr(), _weight_code(weight, "output norm weight"), n, W, float(eps),
+                      token_seq.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else W, self.code, self._stream())
+
+    def constant_step(self, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, decay: torch.Tensor,
+                      weight: torch.Tensor, state: torch.Tensor, token_seq: torch.Tensor, state_slots: torch.Tensor,
+                      out: torch.Tensor, sums: torch.Tensor, beside: Optional[dict] = None) -> bool:
+        """For a step in which every request brings one token: the activations, the recurrence and the output gate of one
+        (row, head) in one workgroup. ``out`` is left without the division by the row's root mean square, which needs
+        every head: sums float32 [n, heads] are the heads' sums of o^2 (see ``RowSums``, ``scale_rows``). ``beside``: the
+        arguments of a ``qkv_row_norm_store`` on the same rows that runs in the same launch. False when the sizes are
+        not served (nothing was done)."""
+        n = self._constant_rows("constant_step", packed, offset, heads, dk, dv, decay, token_seq)
+        self._act(out, "mixer output"); _dev(weight, "output norm weight"); _dev(sums, "row sums")
+        if tuple(out.shape) != (n, heads * dv) or out.stride(1) != 1 or weight.numel() != heads * dv or not weight.is_contiguous() \
+                or sums.dtype != torch.float32 or tuple(sums.shape) != (n, heads) or not sums.is_contiguous():
+            raise KernelLibraryError("constant_step: operands do not fit")
+        self._matrix_state("constant_step", state, heads, dv, dk)
+        self._ints(n, state_slots=(state_slots, 1))
+        norm = [0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0.0, 0.0, 0]
+        if beside is not None:
+            a = self._row_norm_operands(token_seq=token_seq, **beside)
+            norm = [a["rows"], a["stride"], *a["offsets"], a["positions"], a["block_table"], a["bt_width"], a["page_size"], a["k_pages"],
+                    a["v_pages"], *a["sizes"], a["q_weight"], a["k_weight"], a["wcode"], a["eps"], a["coef"], a["every"]]
+        if not self.lib.offer("mv_constant_step", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(offset), n,
+                              heads, dk, dv, decay.data_ptr(), weight.data_ptr(), _weight_code(weight, "output norm weight"),
+                              state.data_ptr(), token_seq.data_ptr(), state_slots.data_ptr(), out.data_ptr(),
+                              out.stride(0) if n > 1 else heads * dv, sums.data_ptr(), *norm, self.code, self._stream()):
+            return False
+        extra = 0 if beside is None else self._row_norm_bytes(n, beside)
+        self._note("mv_constant_step", n * heads * (2 * dk + 3 * dv) * packed.element_size() + 2 * n * heads * dv * dk * 4 + extra,
+                   4 * n * heads * dv * dk)
+        return True
+
+    def _row_norm_operands(self, rows: torch.Tensor, offsets, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
+                           positions: torch.Tensor, token_seq: torch.Tensor, q_weight: torch.Tensor, k_weight: torch.Tensor,
+                           eps: float, temperature, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
+                           page_size: int) -> dict:
+        self._act(rows, "qkv rows"); self._act(k_pages, "key pages"); self._act(v_pages, "value pages"); _dev(block_table, "block table")
+        n = rows.shape[0]
+        q_dim, k_dim, v_dim = num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim
+        if rows.dim() != 2 or rows.stride(1) != 1 or rows.shape[1] < max(offsets[0] + q_dim, offsets[1] + k_dim, offsets[2] + v_dim):
+            raise KernelLibraryError(f"qkv_row_norm_store: rows {tuple(rows.shape)} are too short")
+        if tuple(k_pages.shape[1:]) != (num_kv_heads, page_size, head_dim) or tuple(v_pages.shape[1:]) != (num_kv_heads, value_dim, page_size) \
+                or not k_pages.is_contiguous() or not v_pages.is_contiguous():
+            raise KernelLibraryError(f"qkv_row_norm_store: pages {tuple(k_pages.shape)} / {tuple(v_pages.shape)} do not match "
+                                     f"[pages, {num_kv_heads}, {page_size}, {head_dim}] / [pages, {num_kv_heads}, {value_dim}, {page_size}]")
+        if block_table.dtype != torch.int32 or block_table.dim() != 2 or not block_table.is_contiguous():
+            raise KernelLibraryError("qkv_row_norm_store: the block table must be a contiguous int32 matrix")
+        for w, size, name in ((q_weight, q_dim, "query"), (k_weight, k_dim, "key")):
+            _dev(w, f"{name} norm weight")
+            if w.numel() != size or w.dtype != q_weight.dtype or not w.is_contiguous():
+                raise KernelLibraryError(f"qkv_row_norm_store: the {name} norm weight must hold {size} elements")
+        self._ints(n, positions=(positions, n), token_seq=(token_seq, n))
+        coef, every = (0.0, 0) if temperature is None else temperature
+        return {"rows": rows.data_ptr(), "stride": rows.stride(0) if n > 1 else rows.shape[1], "offsets": tuple(int(o) for o in offsets),
+                "positions": positions.data_ptr(), "block_table": block_table.data_ptr(), "bt_width": block_table.shape[1],
+                "page_size": page_size, "k_pages": k_pages.data_ptr(), "v_pages": v_pages.data_ptr(),
+                "sizes": (num_heads, num_kv_heads, head_dim, value_dim), "q_weight": q_weight.data_ptr(),
+                "k_weight": k_weight.data_ptr(), "wcode": _weight_code(q_weight, "query norm weight"), "eps": float(eps),
+                "coef": float(coef), "every": int(every)}
+
+    @staticmethod
+    def _row_norm_bytes(n: int, args: dict) -> int:
+        kv = args["num_kv_heads"] * (args["head_dim"] + args["value_dim"])
+        return 2 * n * (args["num_heads"] * args["head_dim"] + kv) * args["rows"].element_size()
+
+    def qkv_row_norm_store(self, token_seq: torch.Tensor, **args) -> None:
+        """On ``rows`` with q, k and v at the columns ``offsets``: q (all heads' channels together) is divided by its root
+        mean square over the row and multiplied by ``q_weight`` [heads*head_dim] and, with ``temperature`` = (coef, every),
+        by 1 + coef ln(floor((position + 1) / every) + 1); k likewise with ``k_weight``, without the temperature. q stays in
+        the rows; k and v (``value_dim`` a head) go to the cache pages."""
+        a = self._row_norm_operands(token_seq=token_seq, **args)
+        n = args["rows"].shape[0]
+        if n == 0:
+            return
+        self._note("mv_qkv_row_norm_store", self._row_norm_bytes(n, args), 6 * n * (args["num_heads"] + args["num_kv_heads"]) * args["head_dim"])
+        self.lib.call("mv_qkv_row_norm_store", a["rows"], a["stride"], *a["offsets"], a["positions"], token_seq.data_ptr(),
+                      a["block_table"], a["bt_width"], a["page_size"], a["k_pages"], a["v_pages"], n, *a["sizes"], a["q_weight"],
+                      a["k_weight"], a["wcode"], a["eps"], a["coef"], a["every"], self.code, self._stream())
+
+    def pair_norm(self, pair: "NormedPair", resid: Optional[torch.Tensor], norm_next, out: Optional[torch.Tensor]) -> None:
+        """resid += half the sum of the pair's two sides, each divided by its root mean square and times its weight; with
+        ``norm_next`` = (weight, eps, unit_offset), out = that norm of the new residual. Without ``resid``, out = the half
+        sum itself."""
+        (ya, yb), (wa, wb), (sa, sb) = pair.sides, pair.weights, pair.sums
+        n, h = pair.shape
+        for t, name in ((ya, "left"), (yb, "right")):
+            self._act(t, f"{name} output")
+            if tuple(t.shape) != (n, h) or t.stride(1) != 1:
+                raise KernelLibraryError(f"pair_norm: the {name} rows {tuple(t.shape)} are not [{n}, {h}]")
+        for w in (wa, wb):
+            _dev(w, "pair weight")
+            if w.numel() != h or w.dtype != wa.dtype or not w.is_contiguous():
+                raise KernelLibraryError(f"pair_norm: the weights must hold {h} elements of one dtype")
+        if sa is not None and sb is not None and sa.eps != sb.eps:
+            raise KernelLibraryError("pair_norm: both sides' rows are undivided with different eps")
+        for r in (sa, sb):
+            if r is not None and (r.sums.dtype != torch.float32 or r.sums.dim() != 2 or r.sums.shape[0] != n or not r.sums.is_contiguous()):
+                raise KernelLibraryError("pair_norm: the row sums must be contiguous float32 [rows, parts]")
+        if resid is not None:
+            _dev(resid, "residual")
+            if resid.dtype != torch.float32 or tuple(resid.shape) != (n, h) or not resid.is_contiguous():
+                raise KernelLibraryError("pair_norm: the residual must be a contiguous float32 [n, h]")
+        wn, eps_n, unit_n = norm_next if norm_next is not None else (None, 1.0, False)
+        if out is not None:
+            self._act(out, "pair output")
+            if out.dim() != 2 or out.shape[0] < n or out.shape[1] != h or not out.is_contiguous() or (resid is not None and wn is None) \
+                    or (wn is not None and (wn.numel() != h or not wn.is_contiguous())):
+                raise KernelLibraryError(f"pair_norm: output {tuple(out.shape)} does not fit [{n}, {h}]")
+        if n == 0:
+            return
+        item = ya.element_size()
+        self._note("mv_pair_norm_add_norm", n * h * (2 * item + (8 if resid is not None else 0) + (item if out is not None else 0)), 14 * n * h)
+
+        def side(y, w, r):
+            return (y.data_ptr(), y.stride(0) if n > 1 else h, w.data_ptr(), _ptr(None if r is None else r.sums),
+                    0 if r is None else r.sums.shape[1], 0 if r is None else r.inner)
+
+        inner_eps = sa.eps if sa is not None else (sb.eps if sb is not None else 0.0)
+        self.lib.call("mv_pair_norm_add_norm", *side(ya, wa, sa), *side(yb, wb, sb), _weight_code(wa, "pair weight"), pair.eps,
+                      float(inner_eps), _ptr(resid), _ptr(wn), DTYPE_F32 if wn is None else _weight_code(wn, "norm weight"),
+                      float(eps_n), int(unit_n), _ptr(out), h, n, h, self.code, self._stream())
+
+    def stream_entry(self, resid: torch.Tensor, delta: Optional[torch.Tensor], rows, step: Optional[torch.Tensor], norm_next,
+                     out: Optional[torch.Tensor]) -> None:
+        """resid += delta (when given) + table[ids] * scale (``rows`` = (ids, table, scale), when given) + step (a vector,
+        when given); with ``norm_next`` = (weight, eps, unit_offset), out = that norm of the new residual."""
+        _dev(resid, "residual")
+        n, h = resid.shape
+        if resid.dtype != torch.float32 or not resid.is_contiguous():
+            raise KernelLibraryError("stream_entry: the residual must be a contiguous float32 [n, h]")
+        if delta is not None:
+            self._act(delta, "delta")
+            if tuple(delta.shape) != (n, h) or delta.stride(1) != 1:
+                raise KernelLibraryError(f"stream_entry: delta {tuple(delta.shape)} is not [{n}, {h}]")
+        ids, table, scale = rows if rows is not None else (None, None, 1.0)
+        if ids is not None:
+            _dev(table, "embedding table")
+            self._ints(n, ids=(ids, n))
+            if table.dim() != 2 or table.shape[1] != h or not table.is_contiguous():
+                raise KernelLibraryError(f"stream_entry: table {tuple(table.shape)} does not fit rows of {h}")
+        if step is not None:
+            _dev(step, "step vector")
+            if step.numel() != h or not step.is_contiguous():
+                raise KernelLibraryError(f"stream_entry: a step vector of {step.numel()} elements for rows of {h}")
+        wn, eps_n, unit_n = norm_next if norm_next is not None else (None, 1.0, False)
+        if (out is None) != (wn is None):
+            raise KernelLibraryError("stream_entry: a norm and its output come together")
+        if out is not None:
+            self._act(out, "norm output")
+            if tuple(out.shape) != (n, h) or not out.is_contiguous() or wn.numel() != h or not wn.is_contiguous():
+                raise KernelLibraryError(f"stream_entry: output {tuple(out.shape)} does not fit [{n}, {h}]")
+        if n == 0:
+            return
+        self._note("mv_stream_entry", n * h * (8 + (0 if delta is None else delta.element_size())
+                                               + (0 if table is None else table.element_size()) + (0 if out is None else out.element_size())), 8 * n * h)
+        self.lib.call("mv_stream_entry", resid.data_ptr(), _ptr(delta), (delta.stride(0) if n > 1 else h) if delta is not None else 0,
+                      _ptr(ids), _ptr(table), DTYPE_F32 if table is None else _weight_code(table, "embedding table"),
+                      0 if table is None else table.shape[0], float(scale), _ptr(step),
+                      DTYPE_F32 if step is None else _weight_code(step, "step vector"), _ptr(wn),
+                      DTYPE_F32 if wn is None else _weight_code(wn, "norm weight"), float(eps_n), int(unit_n), _ptr(out), n, h, self.code,
+                      self._stream())
+
     def latent_prepare(self, packed: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, q_norm: torch.Tensor,
                        kv_norm: torch.Tensor, eps: float, table: Optional[torch.Tensor], positions: torch.Tensor,
                        token_seq: torch.Tensor, block_table: torch.Tensor, page_size: int, q_latent: torch.Tensor,
@@ -1441,14 +1791,16 @@ class Ops:
                       token_seq.data_ptr(), n, num_heads, num_kv_heads, head_dim, value_dim, float(scale), c, w,
                       _ptr(bias), _ptr(gate), gate_stride, self.code, self._stream())
 
-    def swiglu(self, gate_up: torch.Tensor, out: torch.Tensor) -> None:
-        """out[n, i] = silu(gate_up[n, i]) * gate_up[n, I + i]."""
+    def swiglu(self, gate_up: torch.Tensor, out: torch.Tensor, limit: float = 0.0, slope: float = 1.0) -> None:
+        """out[n, i] = silu(gate_up[n, i]) * gate_up[n, I + i]; with ``limit`` > 0 the clamped pair g = min(gate, limit),
+        u = clamp(up, -limit, limit), g * sigmoid(slope * g) * (u + 1)."""
         self._act(gate_up, "gate_up"); self._act(out, "swiglu output")
         n, two_i = gate_up.shape
         if two_i % 2 or out.shape != (n, two_i // 2) or not gate_up.is_contiguous() or not out.is_contiguous():
             raise KernelLibraryError(f"swiglu: {tuple(gate_up.shape)} -> {tuple(out.shape)} is not [n, 2I] -> [n, I]")
         self._note("mv_swiglu", self._size(gate_up, out), 6 * out.numel())
-        self.lib.call("mv_swiglu", gate_up.data_ptr(), out.data_ptr(), n, two_i // 2, self.code, self._stream())
+        self.lib.call("mv_swiglu", gate_up.data_ptr(), out.data_ptr(), n, two_i // 2, float(limit), float(slope), self.code,
+                      self._stream())
 
     # ------------------------------------------------------------------------------------
     def gemm(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
@@ -1610,7 +1962,7 @@ class Ops:
         return dict(kernel=counts[0], memset=counts[1], copy=counts[2], other=counts[3])
 
     def _gemm_mid(self, a: torch.Tensor, lda: int, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor,
-                  ldc: int, M: int, N: int, K: int, swiglu: bool, defer_sum: bool = False):
+                  ldc: int, M: int, N: int, K: int, swiglu: bool, defer_sum: bool = False, limit: float = 0.0, slope: float = 1.0):
         """The kernel for up to 64 rows against a large weight (activation rows shared through LDS,
         K split over workgroups); False when the shape is left to the weight-streaming kernel.
         With ``defer_sum`` the partial sums are not added up: a ``SplitSum`` is returned."""
@@ -1639,7 +1991,7 @@ class Ops:
         self._note("mv_gemm_mid", self._size(a, w, out) + 8 * M * N * int(self.lib.dll.mv_gemm_mid_splits(N, K)), 2 * M * N * K)
         self.lib.call("mv_gemm_mid", a.data_ptr(), lda, w.data_ptr(), _ptr(bias), out.data_ptr(), ldc,
                       _CODES[out.dtype], M, N, K, int(swiglu), self._mid_work.data_ptr(), self._mid_work.numel(),
-                      self._stream())
+                      float(limit), float(slope), self._stream())
         return True
 
     def wants_tile(self, M: int, N: int, K: int, gated: bool = False, fold_offered: bool = False) -> bool:
@@ -1696,7 +2048,7 @@ class Ops:
         return pending
 
     def gemm_tile(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
-                  gated: bool = False, force: int = 0) -> bool:
+                  gated: bool = False, force: int = 0, limit: float = 0.0, slope: float = 1.0) -> bool:
         """out[M, N] = a @ w^T (+ bias), or with ``gated`` out[M, N / 2] = silu(a Wg^T) * (a Wu^T), by the
         engine's tiled MFMA product for many rows. False, with nothing done, when the shape is not taken.
         ``force`` fixes the tile and the split of K (measurements)."""
@@ -1708,7 +2060,7 @@ class Ops:
         if (M == 0 or K % 64 or a.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or not w.is_contiguous()
                 or w.shape[1] != K or a.stride(1) != 1 or (M > 1 and a.stride(0) % 8) or a.data_ptr() % 16
                 or w.data_ptr() % 16 or out.shape != (M, n_out) or out.stride(1) != 1
-                or out.dtype not in (torch.bfloat16, torch.float32) or (gated and (N % 2 or bias is not None))
+                or out.dtype not in (torch.bfloat16, torch.float32) or (gated and N % 2)
                 or (bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != N))
                 or M * N >= 1 << 31):
             return False
@@ -1727,7 +2079,7 @@ class Ops:
         self._note("mv_gemm_tile", self._size(a, w, out) + 8 * need, 2 * M * N * K)
         self.lib.call("mv_gemm_tile", a.data_ptr(), a.stride(0) if M > 1 else K, w.data_ptr(), _ptr(bias), out.data_ptr(),
                       out.stride(0) if M > 1 else n_out, _CODES[out.dtype], M, N, K, int(gated), _ptr(work),
-                      0 if work is None else work.numel(), force, self._stream())
+                      0 if work is None else work.numel(), force, float(limit), float(slope), self._stream())
         return True
 
     @staticmethod
@@ -1769,7 +2121,7 @@ class Ops:
                 and fold.stream.weighted is None)
 
     def _gemm_scaled(self, rows: "WeightedRows", w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor],
-                     swiglu: bool) -> bool:
+                     swiglu: bool, limit: float = 0.0, slope: float = 1.0) -> bool:
         """The product (or gated pair) behind a folded norm: output rows divided by the input rows' root
         mean square; False if the shape is not taken (nothing has been done then)."""
         a = rows.weighted
@@ -1787,7 +2139,7 @@ class Ops:
             return False
         if self.prefers_library(M, w.shape[0], K, gated=swiglu) and self._library_allowed(M, w.shape[0], K, bias is not None):
             return False
-        if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != N):
+        if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != w.shape[0]):
             return False
         if (self.wants_tile(M, w.shape[0], K, gated=swiglu) and self.lib.has("mv_gemm_tile_scaled") and w.data_ptr() % 16 == 0
                 and int(self.lib.dll.mv_gemm_tile_splits(M, w.shape[0], K, int(swiglu), 0)) == 1):
@@ -1795,13 +2147,13 @@ class Ops:
             self._note("mv_gemm_tile", self._size(a, w, out) + M * rows.P * 4, 2 * M * w.shape[0] * K)
             self.lib.call("mv_gemm_tile_scaled", a.data_ptr(), a.stride(0) if M > 1 else K, w.data_ptr(), _ptr(bias),
                           out.data_ptr(), out.stride(0) if M > 1 else N, _CODES[out.dtype], M, w.shape[0], K, int(swiglu),
-                          rows.partial.data_ptr(), rows.P, rows.eps, self._stream())
+                          rows.partial.data_ptr(), rows.P, rows.eps, float(limit), float(slope), self._stream())
             return True
         rows.take()
         self._note("mv_gemm_skinny_scaled", self._size(a, w, out) + M * rows.P * 4, 2 * M * w.shape[0] * K)
         self.lib.call("mv_gemm_skinny_scaled", a.data_ptr(), a.stride(0) if M > 1 else K, w.data_ptr(), _ptr(bias),
                       out.data_ptr(), out.stride(0) if M > 1 else N, rows.partial.data_ptr(), rows.P, rows.eps, M, N, K,
-                      int(swiglu), self._stream())
+                      int(swiglu), float(limit), float(slope), self._stream())
         return True
 
     def scale_rows(self, weighted: torch.Tensor, partial: torch.Tensor, P: int, eps: float, out: torch.Tensor) -> None:
@@ -1822,7 +2174,7 @@ class Ops:
                 and rows * (width + 8) * 2 <= 44 * 1024)
 
     def _gemm_fused_norm(self, pending, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor],
-                         swiglu: bool) -> bool:
+                         swiglu: bool, limit: float = 0.0, slope: float = 1.0) -> bool:
         """add + RMSNorm + product (or gated pair) in one kernel; False if the shape is not taken
         (nothing has been done then)."""
         M, K = pending.shape
@@ -1842,36 +2194,41 @@ class Ops:
             return False    # the norm as a kernel of its own and the K-splitting product are faster here
         if self.prefers_library(M, w.shape[0], K, gated=swiglu):
             return False    # as are the norm and the library's product
-        if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != N):
+        if bias is not None and (bias.dtype != torch.bfloat16 or bias.numel() != w.shape[0]):
             return False
         resid_in, delta, resid_out = pending.fused()
-        if isinstance(delta, SplitSum):
+        if delta is not None and not isinstance(delta, torch.Tensor):
             delta = delta.materialize()
         self._note("mv_gemm_skinny_norm", M * K * (4 + (2 + 4 if delta is not None else 0)) + self._size(w, out),
                    2 * M * w.shape[0] * K + 4 * M * K)
         self.lib.call("mv_gemm_skinny_norm", resid_in.data_ptr(), _ptr(delta), _ptr(resid_out), weight.data_ptr(),
                       _weight_code(weight, "norm weight"), float(eps), int(unit_offset), w.data_ptr(),
                       _ptr(bias), out.data_ptr(), out.stride(0) if M > 1 else N, _CODES[out.dtype], M, N, K,
-                      int(swiglu), self._stream())
+                      int(swiglu), float(limit), float(slope), self._stream())
         return True
 
-    def gemm_swiglu(self, a: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor) -> bool:
+    def gemm_swiglu(self, a: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
+                    limit: float = 0.0, slope: float = 1.0) -> bool:
         """out[M, I] = silu(a Wg^T) * (a Wu^T) for the packed weight [2I, K] in one pass over the
         weight, when the weight-streaming kernel takes the shape. Returns False (and does nothing)
         otherwise; the caller then runs the product and the activation separately. ``a`` may be a
-        pending norm, as in ``gemm``."""
+        pending norm, as in ``gemm``. ``bias`` [2I] is added to the two products first; with ``limit`` > 0
+        the pair is the clamped one (see ``swiglu``)."""
+        if bias is not None and (bias.dtype != w_gate_up.dtype or bias.numel() != w_gate_up.shape[0]):
+            raise KernelLibraryError("gemm_swiglu: the bias must have the weight's dtype and an element for each of its rows")
         if not isinstance(a, torch.Tensor):
             if isinstance(a, WeightedRows):
-                if self._gemm_scaled(a, w_gate_up, out, None, swiglu=True):
+                if self._gemm_scaled(a, w_gate_up, out, bias, swiglu=True, limit=limit, slope=slope):
                     return True
-            elif self._gemm_fused_norm(a, w_gate_up, out, None, swiglu=True):
+            elif self._gemm_fused_norm(a, w_gate_up, out, bias, swiglu=True, limit=limit, slope=slope):
                 return True
             a = a.materialize()
         if not (self.use_fast_kernels and self.lib.has("mv_gemm_skinny_swiglu")):
             return False
         M, K = a.shape
         two_i = w_gate_up.shape[0]
-        if self.wants_tile(M, two_i, K, gated=True) and self.gemm_tile(a, w_gate_up, out, None, gated=True):
+        if self.wants_tile(M, two_i, K, gated=True) and self.gemm_tile(
+                a, w_gate_up, out, bias, gated=True, limit=limit, slope=slope):
             return True
         if self.prefers_library(M, two_i, K, gated=True) and self._library_allowed(M, two_i, K, False):
             return False
@@ -1885,12 +2242,13 @@ class Ops:
         self._act(a, "gemm input"); self._act(out, "swiglu output"); _dev(w_gate_up, "gate_up weight")
         if out.shape != (M, two_i // 2) or out.stride(1) != 1:
             raise KernelLibraryError(f"gemm_swiglu: output {tuple(out.shape)} is not [{M}, {two_i // 2}]")
-        if self._gemm_mid(a, a.stride(0) if M > 1 else K, w_gate_up, None, out, out.stride(0) if M > 1 else two_i // 2,
-                          M, two_i, K, swiglu=True):
+        if self._gemm_mid(a, a.stride(0) if M > 1 else K, w_gate_up, bias, out, out.stride(0) if M > 1 else two_i // 2,
+                          M, two_i, K, swiglu=True, limit=limit, slope=slope):
             return True
         self._note("mv_gemm_skinny_swiglu", self._size(a, w_gate_up, out), 2 * M * two_i * K)
-        self.lib.call("mv_gemm_skinny_swiglu", a.data_ptr(), a.stride(0) if M > 1 else K, w_gate_up.data_ptr(),
-                      out.data_ptr(), out.stride(0) if M > 1 else two_i // 2, M, two_i // 2, K, self._stream())
+        self.lib.call("mv_gemm_skinny_swiglu", a.data_ptr(), a.stride(0) if M > 1 else K, w_gate_up.data_ptr(), _ptr(bias),
+                      out.data_ptr(), out.stride(0) if M > 1 else two_i // 2, M, two_i // 2, K, float(limit), float(slope),
+                      self._stream())
         return True
 
     # ------------------------------------------------------------------------------------
@@ -1898,14 +2256,17 @@ class Ops:
                   block_table: torch.Tensor, page_size: int, positions: torch.Tensor, token_seq: torch.Tensor,
                   num_heads: int, num_kv_heads: int, head_dim: int, scale: float, window: Optional[int],
                   plan: Optional["AttentionPlan"] = None, keep_first: int = 0, gate: Optional[torch.Tensor] = None,
-                  value_dim: Optional[int] = None) -> None:
+                  value_dim: Optional[int] = None, softcap: Optional[float] = None, slopes: Optional[torch.Tensor] = None,
+                  sink: bool = False) -> None:
         """Causal attention of the step's queries over the paged cache.
 
         q: [n, >= H*D] rows (a view into the qkv rows), out: [n, H*Dv] (``value_dim`` Dv: the size of a value row
         where it differs from a key's; such sizes take the general kernel). The query at position p
         of sequence s sees keys max(0, p - window) .. p of s and, with ``keep_first``, the first
         ``keep_first`` positions of s however far back they lie. ``gate`` [n, >= H] (a view into the
-        packed rows): head h's output is multiplied by sigmoid(gate[:, h]). ``plan`` carries what the faster
+        packed rows): head h's output is multiplied by sigmoid(gate[:, h]). Scores may be capped, s <- softcap
+        tanh(s / softcap), and lose a distance bias, s <- s - slopes[h] (query position - key position) with
+        ``slopes`` float32 [H]; with ``sink`` the softmax's denominator is 1 + sum exp(s). ``plan`` carries what the faster
         kernels need to know about the step (see AttentionPlan); without it, or in float32, the
         general kernel runs."""
         self._act(q, "queries"); self._act(out, "attention output")
@@ -1942,14 +2303,23 @@ class Ops:
             if gate.dim() != 2 or gate.shape[0] != n or gate.shape[1] < num_heads or gate.stride(1) != 1:
                 raise KernelLibraryError(f"attention: gates {tuple(gate.shape)} do not hold {num_heads} numbers a row")
             gs = gate.stride(0) if n > 1 else gate.shape[1]
+        cap = 0.0 if softcap is None else float(softcap)
+        if softcap is not None and not cap > 0:
+            raise KernelLibraryError(f"attention: a soft cap must be positive, got {softcap}")
+        if slopes is not None:
+            _dev(slopes, "distance slopes")
+            if slopes.dtype != torch.float32 or slopes.numel() != num_heads or not slopes.is_contiguous():
+                raise KernelLibraryError(f"attention: the distance slopes must be float32 [{num_heads}]")
+        form = (cap, _ptr(slopes), int(bool(sink)))
         if vdim == head_dim and self._attention_fast(q, qs, out, os_, k_pages, v_pages, block_table, page_size, positions,
-                                                     token_seq, num_heads, num_kv_heads, head_dim, scale, w, plan, first, gate, gs):
+                                                     token_seq, num_heads, num_kv_heads, head_dim, scale, w, plan, first, gate, gs,
+                                                     form):
             return
         self._note_attention("mv_attention_ref", plan, n, num_heads, num_kv_heads, head_dim, q.element_size())
         self.lib.call("mv_attention_ref", q.data_ptr(), qs, out.data_ptr(), os_, k_pages.data_ptr(),
                       v_pages.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size,
                       positions.data_ptr(), token_seq.data_ptr(), n, num_heads, num_kv_heads, head_dim, vdim,
-                      float(scale), w, first, _ptr(gate), gs, self.code, self._stream())
+                      float(scale), w, first, _ptr(gate), gs, *form, self.code, self._stream())
 
     def _note_attention(self, entry: str, plan, n_tokens: int, H: int, Hkv: int, D: int, item: int, splits: int = 1) -> None:
         """Bytes: the keys and values of every sequence once (per key, so that the line can be priced
@@ -2110,7 +2480,7 @@ class Ops:
         return nt, kw, n_units, n_busy
 
     def _attention_fast(self, q, qs, out, os_, k_pages, v_pages, block_table, page_size, positions, token_seq,
-                        H, Hkv, D, scale, window, plan, first: int = 0, gate=None, gs: int = 0) -> bool:
+                        H, Hkv, D, scale, window, plan, first: int = 0, gate=None, gs: int = 0, form=(0.0, 0, 0)) -> bool:
         """The MFMA kernels, when the step and the sizes allow them."""
         if not self.use_fast_kernels or plan is None or not self.lib.has("mv_attention_decode"):
             return False
@@ -2129,7 +2499,7 @@ class Ops:
                           positions.data_ptr(), plan.cu_seqlens.data_ptr(), n_seqs, H, Hkv, D, float(scale), window,
                           _ptr(partials), self._split_counters(n_seqs * Hkv, partials), nsplit,
                           -(-max(1, plan.max_context_len) // page_size), DECODE_ATTENTION_WAVES, token_seq.data_ptr(),
-                          first, _ptr(gate), gs, self._stream())
+                          first, _ptr(gate), gs, *form, self._stream())
             return True
         if page_size & (page_size - 1):
             return False
@@ -2140,7 +2510,7 @@ class Ops:
         self.lib.call("mv_attention_prefill", q.data_ptr(), qs, out.data_ptr(), os_, k_pages.data_ptr(),
                       v_pages.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size,
                       positions.data_ptr(), plan.cu_seqlens.data_ptr(), n_seqs, n_units, n_busy, nt, kw, H, Hkv, D,
-                      float(scale), window, first, _ptr(gate), gs, self._stream())
+                      float(scale), window, first, _ptr(gate), gs, *form, self._stream())
         return True
 
     # ------------------------------------------------------------------------------------

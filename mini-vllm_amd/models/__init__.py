@@ -5,4 +5,5 @@ from . import bolapel  # registers "Bolapel"
 from . import dutilix  # registers "Dutilix"
 from . import zedudra  # registers "Zedudra"
 from . import furanex  # registers "Furanex"
+from . import sorulix  # registers "Sorulix"
 from .causal_lm import CausalLM, expected_tensors

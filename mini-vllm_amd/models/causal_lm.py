@@ -14,7 +14,7 @@ from typing import Dict, List, Optional, Tuple
 
 import torch
 
-from ..parts.base import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, POSITION_ENCODINGS, CacheNeed,
+from ..parts.base import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, POSITION_ENCODINGS, STREAM_ENTRIES, CacheNeed,
                           HiddenStream, Runtime, TensorDecl)
 from ..parts.plan import ModelPlan, TensorLocation
 from .registry import Architecture
@@ -28,6 +28,9 @@ def _model_level_decls(plan: ModelPlan) -> List[Tuple[TensorLocation, TensorDecl
         out.append((TensorLocation(None, "final_norm", name), decl))
     for name, decl in HEADS.get(plan.head.kind).tensors(plan.head).items():
         out.append((TensorLocation(None, "head", name), decl))
+    if plan.entry is not None:
+        for name, decl in STREAM_ENTRIES.get(plan.entry.kind).tensors(plan.entry).items():
+            out.append((TensorLocation(None, "entry", name), decl))
     return out
 
 
@@ -95,6 +98,11 @@ class CausalLM:
         head_cls = HEADS.get(plan.head.kind)
         self.head = head_cls(plan.head, fetch(None, "head", head_cls.tensors(plan.head)), rt)
 
+        self.entry = None
+        if plan.entry is not None:
+            entry_cls = STREAM_ENTRIES.get(plan.entry.kind)
+            self.entry = entry_cls(plan.entry, fetch(None, "entry", entry_cls.tensors(plan.entry)), rt, self.embedding)
+
         position_parts: Dict[object, object] = {}
         self.position_parts = position_parts
         self.graph_safe = True          # every part allows its forward to be captured in a graph
@@ -130,7 +138,8 @@ class CausalLM:
             parts = [mixer, ffn, kwargs.get("position")] + list(norms.values())
             self.graph_safe = self.graph_safe and all(getattr(p, "graph_safe", True) for p in parts if p is not None)
         self.graph_safe = self.graph_safe and all(getattr(p, "graph_safe", True)
-                                                  for p in (self.embedding, self.final_norm, self.head))
+                                                  for p in (self.embedding, self.final_norm, self.head, self.entry)
+                                                  if p is not None)
 
     # ------------------------------------------------------------------------------------
     def cache_needs(self) -> List[Optional[CacheNeed]]:
@@ -192,8 +201,11 @@ class CausalLM:
         stream = HiddenStream(resid, rt.workspace.get("resid.spare", (n, plan.hidden_size), torch.float32))
         for call_index, call in enumerate(plan.calls):
             block = self.blocks[call.layer]
+            if call.enters_pass is not None:
+                self.entry.forward(stream, ctx, call.enters_pass, block.entry_norm() if hasattr(block, "entry_norm") else None)
             after = None
-            if getattr(block, "accepts_next_norm", False) and call_index + 1 < len(plan.calls):
+            if getattr(block, "accepts_next_norm", False) and call_index + 1 < len(plan.calls) \
+                    and plan.calls[call_index + 1].enters_pass is None:
                 # the norm the next block starts with may be folded into this block's last product
                 after = self.blocks[plan.calls[call_index + 1].layer]
             if after is not None and hasattr(after, "entry_norm") and hasattr(after, "entry_part"):

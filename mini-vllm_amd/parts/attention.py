@@ -25,6 +25,14 @@ within a token: a layer with ``value_mix = "source"`` leaves the values it proje
 ``ctx.carry[value_mix_key]``; a layer with ``"blend"`` caches (1 - m) v + m v_source instead of its own v,
 with m its stored number ``value_mix`` (both must have the same kv heads and value size). Softmax weighting
 with either of these, or with values of another size than keys, runs ``_forward_rotated``.
+
+``row_norm``: q and k are divided by their root mean square over the whole projection, all heads together, and
+multiplied by weights as long as the projections (``q_norm``, ``k_norm``). With it, each off by default:
+``query_temperature`` = (coef, every): q at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1);
+``softcap``: a scaled score s becomes softcap tanh(s / softcap); ``distance_bias``: head h (counted from 0) of H then
+takes 2^(-8 (h + 1) / H) times the distance between query and key off its score; ``sink``: the softmax's denominator
+is 1 + sum exp(s). Softmax weighting with ``row_norm`` runs ``attend_scored``, which another part may call with a
+packed row of its own (``parts/parallel.py``).
 """
 from __future__ import annotations
 
@@ -65,6 +73,11 @@ class AttentionSpec(PartSpec):
     unit_norm_after_rotation: bool = False   # q, k <- x / rms(x) per head, behind the rotation, without a weight
     value_mix: Optional[str] = None          # "source" or "blend", see above
     value_mix_key: str = ""
+    row_norm: bool = False                   # q and k normed over the whole projection, see above
+    query_temperature: Optional[Tuple[float, int]] = None
+    softcap: Optional[float] = None
+    distance_bias: bool = False
+    sink: bool = False
 
     @property
     def q_dim(self) -> int:
@@ -89,14 +102,19 @@ class AttentionSpec(PartSpec):
     @property
     def plain(self) -> bool:
         """The reference's layer: softmax over all keys or a window, values as large as keys."""
-        return (self.weighting == "softmax" and self.chunk is None and self.value_dim in (None, self.head_dim)
+        return (self.weighting == "softmax" and not self.scored and self.chunk is None and self.value_dim in (None, self.head_dim)
                 and not self.head_gate and not self.score_bias and not self.keep_first and not self.value_from_key
-                and not self.unit_norm_after_rotation and self.value_mix is None)
+                and not self.unit_norm_after_rotation and self.value_mix is None and not self.scored)
+
+    @property
+    def scored(self) -> bool:
+        """Softmax over all keys or a window behind the whole-row norm; temperature, cap, distance bias and sink come with it."""
+        return self.row_norm
 
     @property
     def rotated(self) -> bool:
         """Softmax with the unit norm behind the rotation, values shared between layers, or values of a size of their own."""
-        return (self.weighting == "softmax" and self.chunk is None and not self.score_bias and not self.bias
+        return (self.weighting == "softmax" and not self.scored and self.chunk is None and not self.score_bias and not self.bias
                 and not self.qk_norm and not self.head_gate and not self.keep_first and not self.value_from_key
                 and not self.shares_kv
                 and (self.unit_norm_after_rotation or self.value_mix is not None or self.value_dim not in (None, self.head_dim)))
@@ -104,7 +122,7 @@ class AttentionSpec(PartSpec):
     @property
     def kept(self) -> bool:
         """Softmax over a window (or all keys) with kept first positions, head gates or values taken from the keys."""
-        return (self.weighting == "softmax" and self.chunk is None and self.value_dim in (None, self.head_dim)
+        return (self.weighting == "softmax" and not self.scored and self.chunk is None and self.value_dim in (None, self.head_dim)
                 and not self.score_bias and not self.bias and not self.qk_norm and not self.plain and not self.rotated
                 and not self.unit_norm_after_rotation and self.value_mix is None)
 
@@ -134,6 +152,9 @@ class Attention(Mixer):
             if not spec.shares_kv:
                 t["k_bias"] = TensorDecl((spec.kv_dim,), init="zeros_normal")
                 t["v_bias"] = TensorDecl((spec.kv_dim,), init="zeros_normal")
+        if spec.row_norm:
+            t["q_norm"] = TensorDecl((spec.q_dim,), init="ones_normal")
+            t["k_norm"] = TensorDecl((spec.kv_dim,), init="ones_normal")
         if spec.qk_norm:
             t["q_norm"] = TensorDecl((spec.head_dim,), init="ones_normal")
             if not spec.shares_kv:
@@ -168,7 +189,17 @@ class Attention(Mixer):
         if (spec.unit_norm_after_rotation or spec.value_mix) and not spec.rotated:
             raise NotImplementedError("the unit norm behind the rotation and values shared between layers are built for softmax "
                                       "weighting over all keys or a window, without biases, weighted q/k norms, gates or a shared cache")
-        if not spec.plain and not spec.kept and not spec.rotated and (spec.weighting != "sigmoid" or spec.bias):
+        if (spec.query_temperature or spec.softcap is not None or spec.distance_bias or spec.sink) and not spec.scored:
+            raise NotImplementedError("query temperature, capped scores, a distance bias and a sink are built behind the whole-row norm")
+        if spec.scored:
+            if (spec.weighting != "softmax" or spec.chunk is not None or spec.score_bias or spec.head_gate or spec.keep_first
+                    or spec.value_from_key or spec.unit_norm_after_rotation or spec.value_mix is not None or spec.bias or spec.qk_norm
+                    or spec.shares_kv or spec.position is not None):
+                raise NotImplementedError("the whole-row norm is built for softmax weighting over all keys or a window, without "
+                                          "rotation, biases, gates, per-head norms or a shared cache")
+            if (spec.softcap is not None and not spec.softcap > 0) or (spec.query_temperature and spec.query_temperature[1] < 1):
+                raise ValueError("a soft cap is positive and the query temperature changes every >= 1 positions")
+        elif not spec.plain and not spec.kept and not spec.rotated and (spec.weighting != "sigmoid" or spec.bias):
             raise NotImplementedError("chunks, a value size of its own and a score bias are built for sigmoid weighting "
                                       "without projection biases; kept first positions, head gates and values taken from "
                                       "the keys also for softmax weighting without biases and query/key norms")
@@ -195,6 +226,11 @@ class Attention(Mixer):
         self.q_norm = tensors.get("q_norm")
         self.k_norm = tensors.get("k_norm")
         self.value_mix = tensors.get("value_mix")
+        # distance slopes are a property of the head count alone
+        self.slopes = None
+        if spec.distance_bias:
+            self.slopes = torch.tensor([2.0 ** (-8.0 * (h + 1) / spec.num_heads) for h in range(spec.num_heads)], dtype=torch.float32,
+                                       device=rt.device)
         self.position = position
         self.rotary = position.rotary() if position is not None else None
         if position is not None and self.rotary is None and not hasattr(position, "apply"):
@@ -220,6 +256,14 @@ class Attention(Mixer):
 
     def forward(self, x: torch.Tensor, ctx, call: int, fold=None) -> torch.Tensor:
         spec, rt, ops = self.spec, self.rt, self.rt.ops
+        if spec.scored:
+            n = x.shape[0]
+            packed = rt.workspace.get("attn.qkv", (n, self.width), rt.dtype)
+            ops.gemm(x, self.w_qkv, packed)
+            self.norm_store(packed, self.offsets(0), ctx, call)
+            attn = self.attend_scored(packed, 0, ctx, call)
+            y = rt.workspace.get("mixer.out", (n, spec.hidden_size), rt.dtype)
+            return ops.gemm(attn, self.w_o, y, self.b_o, defer_sum=True, fold=fold) or y
         if spec.rotated:
             return self._forward_rotated(x, ctx, call)
         if spec.kept:
@@ -262,6 +306,30 @@ class Attention(Mixer):
         y = ws.get("mixer.out", (n, spec.hidden_size), rt.dtype)
         # (the sums of a product whose K was split may be left to the next norm)
         return ops.gemm(attn, self.w_o, y, self.b_o, defer_sum=True, fold=fold) or y
+
+    def offsets(self, base: int) -> Tuple[int, int, int]:
+        """Columns of q, k and v in rows that hold this mixer's projections from column ``base`` on."""
+        return base, base + self.spec.q_dim, base + self.spec.q_dim + self.spec.kv_dim
+
+    def norm_store_args(self, packed: torch.Tensor, offsets, ctx, call: int) -> dict:
+        """What ``ops.qkv_row_norm_store`` (or a kernel that runs it beside other work) takes for this mixer."""
+        spec, kv = self.spec, ctx.kv(call)
+        return dict(rows=packed, offsets=offsets, num_heads=spec.num_heads, num_kv_heads=spec.num_kv_heads, head_dim=spec.head_dim,
+                    value_dim=spec.v_head_dim, positions=ctx.positions, q_weight=self.q_norm, k_weight=self.k_norm,
+                    eps=spec.qk_norm_eps, temperature=spec.query_temperature, k_pages=kv.k_pages, v_pages=kv.v_pages,
+                    block_table=kv.block_table, page_size=kv.page_size)
+
+    def norm_store(self, packed: torch.Tensor, offsets, ctx, call: int) -> None:
+        self.rt.ops.qkv_row_norm_store(ctx.token_seq, **self.norm_store_args(packed, offsets, ctx, call))
+
+    def attend_scored(self, packed: torch.Tensor, q_offset: int, ctx, call: int) -> torch.Tensor:
+        """The heads' outputs [n, out_dim] for finished queries in ``packed`` and a finished cache."""
+        spec, rt, kv = self.spec, self.rt, ctx.kv(call)
+        attn = rt.workspace.get("attn.out", (packed.shape[0], spec.out_dim), rt.dtype)
+        rt.ops.attention(packed[:, q_offset:q_offset + spec.q_dim], attn, kv.k_pages, kv.v_pages, kv.block_table, kv.page_size,
+                         ctx.positions, ctx.token_seq, spec.num_heads, spec.num_kv_heads, spec.head_dim, spec.scale, spec.window,
+                         plan=ctx.attention_plan, value_dim=spec.v_head_dim, softcap=spec.softcap, slopes=self.slopes, sink=spec.sink)
+        return attn
 
     def _forward_sigmoid(self, x: torch.Tensor, ctx, call: int) -> torch.Tensor:
         """Sigmoid weighting (chunks, a window or all keys; values of any size; score bias; head gates)."""

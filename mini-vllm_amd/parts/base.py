@@ -16,8 +16,8 @@ Mixers additionally state what memory they need per request: ``cache_need(spec)`
 of keys and values, ``state_shape(spec)`` for a fixed-size state.
 
 New kinds are added with ``register_mixer`` / ``register_feed_forward`` / ``register_norm`` /
-``register_position_encoding`` / ``register_block`` / ``register_embedding`` / ``register_head``;
-nothing else in the engine changes.
+``register_position_encoding`` / ``register_block`` / ``register_embedding`` / ``register_head`` /
+``register_stream_entry``; nothing else in the engine changes.
 """
 from __future__ import annotations
 
@@ -268,6 +268,7 @@ POSITION_ENCODINGS = Registry("position encoding")
 BLOCKS = Registry("block arrangement")
 EMBEDDINGS = Registry("embedding")
 HEADS = Registry("output head")
+STREAM_ENTRIES = Registry("stream entry")
 
 register_mixer = MIXERS.register
 register_feed_forward = FEED_FORWARDS.register
@@ -276,6 +277,7 @@ register_position_encoding = POSITION_ENCODINGS.register
 register_block = BLOCKS.register
 register_embedding = EMBEDDINGS.register
 register_head = HEADS.register
+register_stream_entry = STREAM_ENTRIES.register
 
 
 # ---------------------------------------------------------------------------------------

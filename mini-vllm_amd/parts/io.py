@@ -36,6 +36,10 @@ class TokenEmbedding(Embedding):
     def forward(self, ctx, resid: torch.Tensor, gather=None) -> None:
         self.rt.ops.embedding(ctx.token_ids, self.table, resid, self.spec.scale, gather=gather)
 
+    def row_table(self):
+        """(table, factor): a token's output is its row of the table times the factor."""
+        return self.table, self.spec.scale
+
 
 @register_head(HeadSpec.kind)
 class LinearHead(Head):

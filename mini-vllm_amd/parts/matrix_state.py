@@ -22,19 +22,26 @@ so the read-out sees the token's own write.
   o <- o / (max(|n . q|, exp(-m')) + denom_eps). o is then divided by its root mean square per head,
   multiplied by a weight over all heads' channels and by sigmoid(W_g h).
 
-Both keep S as float32 [heads, columns, key_dim] per request (a head's matrix column by column),
+* ``channel_delta`` (the gated delta rule with a decay per key channel): as ``gated_delta``, but a is a vector over
+  the key channels, S <- diag(a) S, a = exp(-exp(A_log) * softplus(W_a2 (W_a1 h) + dt_bias)) per head and channel
+  (A_log per head), and o, after its norm, is multiplied by sigmoid(W_g2 (W_g1 h)).
+* ``constant_decay`` (lightning attention): [delta] is off, a is a constant per head and b = 1; q, k and v are SiLU of
+  their projections. All heads' o together are divided by their root mean square, multiplied by a weight over all
+  channels and by sigmoid(W_g h).
+
+All keep S as float32 [heads, columns, key_dim] per request (a head's matrix column by column),
 zero at a request's start; the convolution's last ``conv_taps - 1`` inputs (activation type) and the
 running maximum (float32 [heads]) are state too. Gates, unit vectors and the recurrence are float32
-whatever the activation type. All projections of the mixer's input are one packed product; the
-scan kernel is shared by the two mixers.
+whatever the activation type. All projections of the mixer's input are one packed product.
 """
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Dict, Optional
+from typing import Dict, Optional, Tuple
 
 import torch
 
+from ..kernels.ops import RowSums
 from .base import Mixer, PartSpec, Runtime, TensorDecl, register_mixer
 
 
@@ -198,4 +205,182 @@ class MLSTM(Mixer):
         ops.state_scan(qk, vals, gates, ctx.state(call), ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, H, H, dk, dv + 1, False, raw)
         ops.state_finish(raw, gates, packed, self.gate_offset, self.norm, H, dv, spec.out_norm_eps, ctx.token_seq, gated,
                          shared_weight=False, silu_gate=False, normaliser=True, denom_eps=spec.denom_eps)
+        return ops.gemm(gated, self.w_o, y, defer_sum=True) or y
+
+
+@dataclass(frozen=True)
+class ChannelDeltaSpec(PartSpec):
+    kind = "channel_delta"
+    hidden_size: int = 0
+    num_heads: int = 0
+    num_kv_heads: int = 0
+    key_dim: int = 0
+    value_dim: int = 0
+    conv_taps: int = 1                  # 1: no convolution (a single tap still scales each channel)
+    decay_rank: int = 0                 # rows of W_a1
+    gate_rank: int = 0                  # rows of W_g1
+    unit_eps: float = 1e-6              # inside the root of a query's or key's length
+    out_norm_eps: float = 1e-6          # of the per-head RMS of the output
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.num_kv_heads * self.key_dim + self.num_heads * self.value_dim
+
+
+@register_mixer(ChannelDeltaSpec.kind)
+class ChannelDelta(Mixer):
+    """Packed rows: [q | k | v | b, padded to a multiple of 8 | W_a1 h | W_g1 h, padded to a multiple of 32]. In steps with
+    prompt portions the two second matrices are one product against the low-rank columns (block-diagonal, in float32
+    rows [decays | gates]); in steps of single tokens the step's kernel makes them itself."""
+    spec_class = ChannelDeltaSpec
+    accepts_pending_norm = True         # the input is used by one packed product only
+    accepts_fold = True                 # the output comes from one product
+
+    @classmethod
+    def tensors(cls, spec: ChannelDeltaSpec) -> Dict[str, TensorDecl]:
+        hid, H = spec.hidden_size, spec.num_heads
+        qk, dk, vd = spec.num_kv_heads * spec.key_dim, H * spec.key_dim, H * spec.value_dim
+        return {"q": TensorDecl((qk, hid)), "k": TensorDecl((qk, hid)), "v": TensorDecl((vd, hid)), "b": TensorDecl((H, hid)),
+                "q_conv": TensorDecl((qk, spec.conv_taps)), "k_conv": TensorDecl((qk, spec.conv_taps)),
+                "v_conv": TensorDecl((vd, spec.conv_taps)),
+                "A_log": TensorDecl((H,), init="zeros_normal"), "dt_bias": TensorDecl((dk,), init="zeros_normal"),
+                "a1": TensorDecl((spec.decay_rank, hid)), "a2": TensorDecl((dk, spec.decay_rank)),
+                "g1": TensorDecl((spec.gate_rank, hid)), "g2": TensorDecl((vd, spec.gate_rank)),
+                "norm": TensorDecl((spec.value_dim,), init="ones_normal"), "o": TensorDecl((hid, vd))}
+
+    @classmethod
+    def state_shapes(cls, spec: ChannelDeltaSpec):
+        shapes = {"state": ((spec.num_heads, spec.value_dim, spec.key_dim), torch.float32)}
+        if spec.conv_taps > 1:
+            shapes["conv"] = ((spec.conv_taps - 1, spec.conv_channels), None)      # the activation type
+        return shapes
+
+    def __init__(self, spec: ChannelDeltaSpec, tensors: Dict[str, torch.Tensor], rt: Runtime, position: Optional[object] = None):
+        if min(spec.num_heads, spec.num_kv_heads, spec.key_dim, spec.value_dim, spec.conv_taps, spec.decay_rank, spec.gate_rank) < 1 \
+                or spec.num_heads % spec.num_kv_heads:
+            raise ValueError(f"channel-wise delta rule: bad sizes {spec}")
+        self.spec, self.rt = spec, rt
+        hid, H, dk, dv = spec.hidden_size, spec.num_heads, spec.key_dim, spec.value_dim
+        ra, rg = spec.decay_rank, spec.gate_rank
+        front = _pack(tensors, ("q", "k", "v", "b"), hid, "channel-wise delta rule")
+        low = torch.cat([tensors["a1"], tensors["g1"]], dim=0)
+        pad = (-low.shape[0]) % 32
+        if pad:
+            low = torch.cat([low, torch.zeros((pad, hid), dtype=low.dtype, device=low.device)], dim=0)
+        self.b_offset, self.low_offset, self.low_width = spec.conv_channels, front.shape[0], low.shape[0]
+        self.w_packed = torch.cat([front, low], dim=0).contiguous()
+        self.width = self.w_packed.shape[0]
+        second = torch.zeros((H * (dk + dv), self.low_width), dtype=low.dtype, device=low.device)
+        second[:H * dk, :ra] = tensors["a2"]
+        second[H * dk:, ra:ra + rg] = tensors["g2"]
+        self.w_second = second.contiguous()
+        self.conv_w = torch.cat([tensors["q_conv"], tensors["k_conv"], tensors["v_conv"]], dim=0).contiguous()
+        dt = self.conv_w.dtype
+        self.a_log, self.dt_bias = tensors["A_log"].to(dt).contiguous(), tensors["dt_bias"].to(dt).contiguous()
+        self.a2t, self.g2t = tensors["a2"].to(dt).t().contiguous(), tensors["g2"].to(dt).t().contiguous()
+        self.norm, self.w_o = tensors["norm"].to(dt).contiguous(), tensors["o"]
+
+    def first_product(self):
+        return self.w_packed.shape[0], self.w_packed.shape[1], False
+
+    def forward(self, x: torch.Tensor, ctx, call: int, fold=None) -> torch.Tensor:
+        spec, rt, ops, ws = self.spec, self.rt, self.rt.ops, self.rt.workspace
+        n, H, G, dk, dv = x.shape[0], spec.num_heads, spec.num_kv_heads, spec.key_dim, spec.value_dim
+        packed = ws.get("mstate.packed", (n, self.width), rt.dtype)
+        ops.gemm(x, self.w_packed, packed)
+        gated = ws.get("mstate.gated", (n, H * dv), rt.dtype)
+        y = ws.get("mixer.out", (n, spec.hidden_size), rt.dtype)
+        conv_state = ctx.state(call, "conv") if spec.conv_taps > 1 else None
+        plan = ctx.attention_plan
+        if plan is not None and plan.decode_only and ops.channel_step(
+                packed, H, G, dk, dv, spec.conv_taps, self.b_offset, self.low_offset, self.conv_w, self.a_log, self.dt_bias, self.a2t,
+                self.g2t, self.norm, conv_state, ctx.state(call), spec.unit_eps, spec.out_norm_eps, ctx.token_seq, ctx.cu_seqlens,
+                ctx.state_slots, ctx.n_seqs, gated):
+            return ops.gemm(gated, self.w_o, y, defer_sum=True, fold=fold) or y
+        z = ws.get("mstate.z", (n, H * (dk + dv)), torch.float32)
+        ops.gemm(packed[:, self.low_offset:self.low_offset + self.low_width], self.w_second, z)
+        qk = ws.get("mstate.qk", (n, G, 2, dk), torch.float32)
+        vals = ws.get("mstate.vals", (n, H, dv), torch.float32)
+        beta = ws.get("mstate.beta", (n, H), torch.float32)
+        ops.channel_prepare(packed, H, G, dk, dv, spec.conv_taps, self.b_offset, self.conv_w, self.a_log, self.dt_bias, conv_state,
+                            spec.unit_eps, ctx.token_seq, ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, qk, vals, beta, z)
+        raw = ws.get("mstate.raw", (n, H, dv), torch.float32)
+        ops.channel_scan(qk, vals, beta, z, ctx.state(call), ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, H, G, dk, dv, raw)
+        ops.state_finish(raw, None, z, H * dk, self.norm, H, dv, spec.out_norm_eps, ctx.token_seq, gated, shared_weight=True,
+                         silu_gate=False)
+        return ops.gemm(gated, self.w_o, y, defer_sum=True, fold=fold) or y
+
+
+@dataclass(frozen=True)
+class ConstantDecaySpec(PartSpec):
+    kind = "constant_decay"
+    hidden_size: int = 0
+    num_heads: int = 0
+    key_dim: int = 0
+    value_dim: int = 0
+    decay: Tuple[float, ...] = ()       # one per head
+    out_norm_eps: float = 1e-6          # of the RMS over all heads' outputs
+
+    @property
+    def inner(self) -> int:
+        return self.num_heads * self.value_dim
+
+
+@register_mixer(ConstantDecaySpec.kind)
+class ConstantDecay(Mixer):
+    spec_class = ConstantDecaySpec
+    PACKED = ("q", "k", "v", "g")
+
+    @classmethod
+    def tensors(cls, spec: ConstantDecaySpec) -> Dict[str, TensorDecl]:
+        hid, qk, vd = spec.hidden_size, spec.num_heads * spec.key_dim, spec.inner
+        return {"q": TensorDecl((qk, hid)), "k": TensorDecl((qk, hid)), "v": TensorDecl((vd, hid)), "g": TensorDecl((vd, hid)),
+                "norm": TensorDecl((vd,), init="ones_normal"), "o": TensorDecl((hid, vd))}
+
+    @classmethod
+    def state_shapes(cls, spec: ConstantDecaySpec):
+        return {"state": ((spec.num_heads, spec.value_dim, spec.key_dim), torch.float32)}
+
+    def __init__(self, spec: ConstantDecaySpec, tensors: Dict[str, torch.Tensor], rt: Runtime, position: Optional[object] = None):
+        if min(spec.num_heads, spec.key_dim, spec.value_dim) < 1 or len(spec.decay) != spec.num_heads:
+            raise ValueError(f"constant decay: bad sizes, or not one decay for each head: {spec}")
+        self.spec, self.rt = spec, rt
+        self.w_packed = _pack(tensors, self.PACKED, spec.hidden_size, "constant decay")
+        self.width = self.w_packed.shape[0]
+        self.decay = torch.tensor(spec.decay, dtype=torch.float32, device=rt.device)
+        self.norm, self.w_o = tensors["norm"].contiguous(), tensors["o"]
+
+    def recur(self, packed: torch.Tensor, base: int, ctx, call: int, beside: Optional[dict] = None):
+        """From rows that hold this mixer's projections from column ``base`` on: (the rows that go into the output
+        projection, a ``RowSums`` when they are still to be divided by their root mean square, whether ``beside`` ran).
+        ``beside``: a query/key norm and cache write on the same rows, to run in the same launch where there is one."""
+        spec, rt, ops, ws = self.spec, self.rt, self.rt.ops, self.rt.workspace
+        n, H, dk, dv = packed.shape[0], spec.num_heads, spec.key_dim, spec.value_dim
+        gated = ws.get("mstate.gated", (n, H * dv), rt.dtype)
+        plan = ctx.attention_plan
+        if plan is not None and plan.decode_only:
+            sums = ws.get("mstate.sums", (n, H), torch.float32)
+            if ops.constant_step(packed, base, H, dk, dv, self.decay, self.norm, ctx.state(call), ctx.token_seq, ctx.state_slots, gated,
+                                 sums, beside=beside):
+                return gated, RowSums(sums, H * dv, spec.out_norm_eps), beside is not None
+        qk = ws.get("mstate.qk", (n, H, 2, dk), torch.float32)
+        vals = ws.get("mstate.vals", (n, H, dv), torch.float32)
+        gates = ws.get("mstate.gates", (n, H, 4), torch.float32)
+        ops.constant_prepare(packed, base, H, dk, dv, self.decay, ctx.token_seq, qk, vals, gates)
+        raw = ws.get("mstate.raw", (n, H, dv), torch.float32)
+        ops.state_scan(qk, vals, gates, ctx.state(call), ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, H, H, dk, dv, False, raw)
+        ops.row_gate_finish(raw, packed, base + H * (2 * dk + dv), self.norm, spec.out_norm_eps, ctx.token_seq, gated)
+        return gated, None, False
+
+    def forward(self, x: torch.Tensor, ctx, call: int) -> torch.Tensor:
+        spec, rt, ops, ws = self.spec, self.rt, self.rt.ops, self.rt.workspace
+        n = x.shape[0]
+        packed = ws.get("mstate.packed", (n, self.width), rt.dtype)
+        ops.gemm(x, self.w_packed, packed)
+        gated, sums, _ = self.recur(packed, 0, ctx, call)
+        if sums is not None:
+            whole = ws.get("mstate.scaled", (n, spec.inner), rt.dtype)
+            ops.scale_rows(gated, sums.sums, sums.sums.shape[1], sums.eps, whole)
+            gated = whole
+        y = ws.get("mixer.out", (n, spec.hidden_size), rt.dtype)
         return ops.gemm(gated, self.w_o, y, defer_sum=True) or y

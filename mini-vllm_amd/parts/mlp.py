@@ -97,3 +97,60 @@ class XIELUFeedForward(FeedForward):
         ops.xielu(act, self.a_pos, self.a_neg, act)
         y = rt.workspace.get("ffn.out", (n, spec.hidden_size), rt.dtype)
         return ops.gemm(act, self.w_down, y, defer_sum=True) or y
+
+
+@dataclass(frozen=True)
+class ClampedGLUSpec(PartSpec):
+    """A gated pair with clamped halves: g = min(Wg x + bg, limit), u = clamp(Wu x + bu, -limit, limit),
+    y = Wd (g * sigmoid(slope * g) * (u + 1)) + bd; ``bias`` False leaves the three biases out."""
+    kind = "clamped_glu"
+    hidden_size: int = 0
+    intermediate_size: int = 0
+    limit: float = 0.0
+    slope: float = 1.702
+    bias: bool = True
+
+
+@register_feed_forward(ClampedGLUSpec.kind)
+class ClampedGLU(FeedForward):
+    spec_class = ClampedGLUSpec
+    accepts_pending_norm = True      # the input is used by one packed product only
+    accepts_fold = True              # the output comes from one product
+
+    @classmethod
+    def tensors(cls, spec: ClampedGLUSpec) -> Dict[str, TensorDecl]:
+        hid, ff = spec.hidden_size, spec.intermediate_size
+        t = {"gate": TensorDecl((ff, hid)), "up": TensorDecl((ff, hid)), "down": TensorDecl((hid, ff))}
+        if spec.bias:
+            t.update(gate_bias=TensorDecl((ff,), init="zeros_normal"), up_bias=TensorDecl((ff,), init="zeros_normal"),
+                     down_bias=TensorDecl((hid,), init="zeros_normal"))
+        return t
+
+    def __init__(self, spec: ClampedGLUSpec, tensors: Dict[str, torch.Tensor], rt: Runtime):
+        if not spec.limit > 0:
+            raise ValueError(f"a clamped pair needs a positive limit, got {spec.limit}")
+        self.spec, self.rt = spec, rt
+        if tensors["gate"].dtype != tensors["up"].dtype:
+            raise ValueError("gate and up projections are stored in different dtypes; cannot pack them")
+        self.w_gate_up = torch.cat([tensors["gate"], tensors["up"]], dim=0).contiguous()
+        self.w_down = tensors["down"]
+        self.b_gate_up = self.b_down = None
+        if spec.bias:
+            self.b_gate_up = torch.cat([tensors["gate_bias"], tensors["up_bias"]], dim=0).to(self.w_gate_up.dtype).contiguous()
+            self.b_down = tensors["down_bias"].to(self.w_down.dtype).contiguous()
+
+    def first_product(self):
+        return self.w_gate_up.shape[0], self.w_gate_up.shape[1], True
+
+    def forward(self, x: torch.Tensor, ctx, fold=None) -> torch.Tensor:
+        spec, rt, ops = self.spec, self.rt, self.rt.ops
+        n = x.shape[0]
+        act = rt.workspace.get("ffn.act", (n, spec.intermediate_size), rt.dtype)
+        if not ops.gemm_swiglu(x, self.w_gate_up, act, self.b_gate_up, limit=spec.limit, slope=spec.slope):
+            gu = rt.workspace.get("ffn.gate_up", (n, 2 * spec.intermediate_size), rt.dtype)
+            if not isinstance(x, torch.Tensor):
+                x = x.materialize()
+            ops.gemm(x, self.w_gate_up, gu, self.b_gate_up)
+            ops.swiglu(gu, act, limit=spec.limit, slope=spec.slope)
+        y = rt.workspace.get("ffn.out", (n, spec.hidden_size), rt.dtype)
+        return ops.gemm(act, self.w_down, y, self.b_down, defer_sum=True, fold=fold) or y

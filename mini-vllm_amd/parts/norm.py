@@ -87,6 +87,8 @@ class RMSNorm(Norm):
         taken = self._take_weighted(stream)
         if taken is not None:
             return taken
+        if getattr(stream.delta, "is_normed_pair", False):
+            return self.forward(stream, ctx)       # joining the pair is a kernel anyway: add and norm ride on it
         if stream.spare is not None and self.rt.ops.can_fuse_norm(stream.resid.shape[0], self.spec.size):
             return PendingNorm(self, stream, ctx)
         return self.forward(stream, ctx)

@@ -16,7 +16,7 @@ from .base import PartSpec
 @dataclass(frozen=True)
 class TensorLocation:
     """Where a tensor belongs: ``layer`` None for the model-level parts; ``role`` is
-    "embedding", "head", "final_norm", "mixer", "ffn" or "norm.<slot>"; ``name`` is the part's
+    "embedding", "head", "final_norm", "entry", "mixer", "ffn", "block" or "norm.<slot>"; ``name`` is the part's
     logical tensor name."""
     layer: Optional[int]
     role: str
@@ -40,6 +40,7 @@ class LayerPlan:
 class Call:
     layer: int
     cache_from: Optional[int] = None
+    enters_pass: Optional[int] = None      # number of the pass that starts with this call (see ``ModelPlan.entry``)
 
 
 @dataclass(frozen=True)
@@ -68,6 +69,8 @@ class ModelPlan:
     calls: Tuple[Call, ...]
     final_norm: PartSpec
     head: PartSpec                 # HeadSpec, or the spec of another registered head
+    # what happens to the residual stream in front of calls with ``enters_pass`` (a registered stream entry)
+    entry: Optional[PartSpec] = None
 
     def validate(self) -> None:
         if not self.layers:
@@ -75,6 +78,8 @@ class ModelPlan:
         for i, c in enumerate(self.calls):
             if not (0 <= c.layer < len(self.layers)):
                 raise ValueError(f"call {i} names layer {c.layer}, the plan has {len(self.layers)}")
+            if c.enters_pass is not None and self.entry is None:
+                raise ValueError(f"call {i} enters a pass, but the plan has no stream entry")
             if c.cache_from is not None:
                 if not (0 <= c.cache_from < i):
                     raise ValueError(f"call {i} reads the cache of call {c.cache_from}, which does not run before it")
