@@ -46,6 +46,11 @@ feed-forward dense and the others mixtures of ``--experts`` experts of which a t
 residual streams; grouped attention whose values are shared along the layers alternating with attention over a latent;
 every feed-forward a mixture of ``--experts`` experts named by a table, ``--top`` a token, beside a shared expert).
 
+``--design sorulix`` does the same for a Sorulix model of the named shape's sizes (``sorulix_shape``: layers of softmax
+attention beside linear attention with constant decays alternating with layers of the channel-wise gated delta rule, every
+feed-forward the clamped gated pair at the shape's dense width; with ``--loops`` above 1 the middle half of the layers
+runs that many times). Its dense sizes are those of Qwen3 of the same shape, so the two can be read side by side.
+
 Weights are seeded random tensors of the named shape and prompts are seeded uniform token ids
 (there is no network for checkpoints or datasets). The reference publishes no number for this
 metric, so ``vs_baseline`` is null.
@@ -101,6 +106,9 @@ def build_llm(args, shape, layers, max_seqs=None, token_budget=None, num_pages=N
         from minivllm_amd.config.shapes import furanex_shape
         raw = dict(furanex_shape(args.shape, layers, streams=args.streams, experts=args.experts, top=args.top,
                                  latent_every=args.latent_every), torch_dtype=args.dtype)
+    elif getattr(args, "design", "qwen3") == "sorulix":
+        from minivllm_amd.config.shapes import sorulix_shape
+        raw = dict(sorulix_shape(args.shape, layers, loops=args.loops), torch_dtype=args.dtype)
     else:
         raw = dict(shape, architectures=["Qwen3ForCausalLM"], num_hidden_layers=layers,
                    max_position_embeddings=40960, torch_dtype=args.dtype)
@@ -602,6 +610,73 @@ def bench_zedudra(args, llm, cfg, layers, layers_full, item) -> int:
     return 0
 
 
+def sorulix_numbers(llm, cfg):
+    """From the loaded model: elements of all tensors; of the matrices a token multiplies with, a layer that runs several
+    times counted each time; of the weights a decode step reads (again each time); bytes of state of one request; cache
+    elements a token takes and multiply-adds of a (query, key) pair, over all calls."""
+    from minivllm_amd.models.causal_lm import expected_tensors
+    ex = llm.executor
+    decls = expected_tensors(ex.arch, cfg, ex.plan)
+    runs = [0] * len(cfg.layers)
+    for call in ex.plan.calls:
+        runs[call.layer] += 1
+    sizes = {n: (_numel(d.shape), len(d.shape)) for n, d in decls.items()}
+    times = lambda n: runs[int(n[1:].split(".")[0])] if n[0] == "l" and n[1].isdigit() else 1
+    params = sum(k for k, _ in sizes.values())
+    matrices = sum(k * times(n) for n, (k, dims) in sizes.items() if dims == 2 and n not in ("embed", "loop.step")
+                   and not n.endswith(".conv"))
+    read = sum(k * times(n) for n, (k, _) in sizes.items() if n != "loop.step")
+    state = sum(t[0].numel() * t.element_size() for ts in ex.state_tensors.values() for t in ts.values())
+    attn = [cfg.layers[c.layer].left for c in ex.plan.calls if cfg.layers[c.layer].left is not None]
+    return dict(params=params, matrices=matrices, read=read, state=state, calls=len(ex.plan.calls),
+                cache=sum(a.kv_heads * (a.dim + a.vdim) for a in attn), pair=sum(a.heads * (a.dim + a.vdim) for a in attn))
+
+
+def bench_sorulix(args, llm, cfg, layers, layers_full, item) -> int:
+    """The default measurements for a Sorulix model of the named shape; the same fields in the line."""
+    nums = sorulix_numbers(llm, cfg)
+    prefill = None
+    if args.only in ("all", "prefill"):
+        prefill_s = measure_prefill(llm, cfg.vocab_size, args.prefill_tokens, repeats=3, seed=args.seed)
+        T = args.prefill_tokens
+        # the matrices, the softmax sides' causal pairs, the state updates (written and read once a token), the head
+        flops = 2 * T * nums["matrices"] + 2 * nums["pair"] * T * (T + 1) // 2 + T * nums["state"] + 2 * cfg.vocab_size * cfg.hidden_size
+        prefill = {"value": round(T / prefill_s, 1), "tokens": T, "ms": round(prefill_s * 1e3, 3),
+                   "frac": round(flops / prefill_s / PEAK_FLOPS[args.dtype], 4)}
+    tok_s = ms_step = roofline = None
+    ran = regions = 0
+    if args.only in ("all", "decode"):
+        tok_s, ms_step, mean_ctx, ran, regions = measure_decode(llm, cfg.vocab_size, args.batch, args.prompt_len,
+                                                                args.steps, args.warmup, args.seed)
+        # every weight once for each time its layer runs, each request's cache once, its states read and written
+        step_bytes = nums["read"] * item + args.batch * (nums["cache"] * item * mean_ctx + 2 * nums["state"])
+        achieved = step_bytes / (ms_step * 1e-3) / 1e9
+        roofline = {"bound": "hbm", "achieved": round(achieved, 1), "peak": PEAK_HBM_GBS, "unit": "GB/s",
+                    "frac": round(achieved / PEAK_HBM_GBS, 4)}
+    points = {}
+    if not args.no_points and args.only == "all":
+        for b, key in ((1, "decode_b1"), (64, "decode_b64")):
+            n = min(args.steps, 128)
+            points[key] = round(measure_decode(llm, cfg.vocab_size, b, args.prompt_len, n, min(args.warmup, 8),
+                                               args.seed + b)[0], 1)
+    kinds = [l.type for l in cfg.layers]
+    config = {"model": f"sorulix-{args.shape}-shape-random", "layers": layers, "layers_full": layers_full,
+              "layer_runs": nums["calls"], "hidden": cfg.hidden_size, "vocab": cfg.vocab_size,
+              "parallel_layers": kinds.count("parallel"), "channel_delta_layers": kinds.count("channel_delta"),
+              "weights": nums["params"], "global_batch": args.batch,
+              "seq_len": args.context, "prompt_len": args.prompt_len, "block_size": args.block_size, "graph": not args.no_graph,
+              "scheduler_steps": args.scheduler_steps, "launch_ahead": bool(llm.config.launch_ahead),
+              "parallelism": "single-gpu"}
+    print(json.dumps({"metric": "decode tok/s (batch %d, %d-token prompts)" % (args.batch, args.prompt_len),
+                      "value": round(tok_s, 1) if tok_s is not None else None, "unit": "tokens/s", "n_gpus": 1,
+                      "steps": ran if ran else args.steps, "warmup": args.warmup,
+                      "ms_per_step": round(ms_step, 4) if ms_step is not None else None, "higher_is_better": True,
+                      "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                      "data": "synthetic", "config": config, "timed_regions": regions, "prefill": prefill,
+                      "roofline": roofline, "points": points}))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser(description=__doc__, formatter_class=argparse.RawDescriptionHelpFormatter)
     ap.add_argument("--gpus", type=int, default=1)
@@ -619,7 +694,8 @@ def main() -> int:
     ap.add_argument("--latent-every", type=int, default=2,
                     help="--design furanex: every n-th layer attends over a latent, the others are grouped attention (a number "
                          "above the layer count: grouped attention everywhere)")
-    ap.add_argument("--design", choices=["qwen3", "bolapel", "dutilix", "zedudra", "furanex"], default="qwen3",
+    ap.add_argument("--loops", type=int, default=1, help="--design sorulix: times the middle half of the layers runs")
+    ap.add_argument("--design", choices=["qwen3", "bolapel", "dutilix", "zedudra", "furanex", "sorulix"], default="qwen3",
                     help="'bolapel': the same widths, head counts, vocabulary and number of layers as the named Qwen3 "
                          "shape, as a Bolapel model (three delta-rule layers to one attention layer in chunks of --chunk "
                          "tokens); decode and prefill are measured the same way and the line names the design")
@@ -726,6 +802,8 @@ def main() -> int:
         return bench_zedudra(args, llm, cfg, layers, layers_full, item)
     if args.design == "furanex":
         return bench_furanex(args, llm, cfg, layers, layers_full, item)
+    if args.design == "sorulix":
+        return bench_sorulix(args, llm, cfg, layers, layers_full, item)
     nums = model_numbers(shape, layers)
 
     prefill = None

@@ -172,7 +172,10 @@ def _align(trace: Sequence[Tuple[str, float]], start: int, patterns, limits) -> 
     (two products of the same kernel in a row are two launches, not one launch's pair)."""
     i, n = start, len(trace)
     times, names, other, other_count = [], [], 0.0, 0
-    for (pat, follow), limit in zip(patterns, limits):
+    for line, ((pat, follow), limit) in enumerate(zip(patterns, limits)):
+        # (several library products in a row: a kernel for each, what a split product adds goes to the last)
+        if follow is not None and follow.pattern == pat.pattern and line + 1 < len(patterns) and patterns[line + 1][0].pattern == pat.pattern:
+            limit = 1
         while i < n and not _OURS.search(trace[i][0]):
             other += trace[i][1]
             other_count += 1

@@ -1,0 +1,615 @@
+"""Each mechanism of Sorulix alone, the engine's kernels against the plain functions: the norm over whole query and key
+rows with temperature and cache write; softmax attention with capped scores, distance bias and sink (scattered pages, far
+keys, page borders, first tokens, prompts and single tokens, every split and variant); linear attention with constant
+decays and the channel-wise gated delta rule (any mix of requests, state carried, slots used again, padding, single-token
+steps); two parts' outputs joined with the residual add and the norm behind; entries into a run of layers; the clamped
+gated pair with biases in every product kernel."""
+import math
+
+import numpy as np
+import pytest
+import torch
+
+from plain import sorulix_plain as plain
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+DTYPES = [torch.float32, torch.bfloat16]
+
+
+def ops_for(dtype):
+    from minivllm_amd.kernels.ops import Ops
+    return Ops(dtype)
+
+
+def i32(values):
+    return torch.tensor(list(values), dtype=torch.int32, device=DEV)
+
+
+def step_ints(q_lens, slots, pad_rows=0, pad_seqs=0):
+    seq = [s for s, n in enumerate(q_lens) for _ in range(n)] + [-1] * pad_rows
+    cu = np.concatenate([[0], np.cumsum(q_lens)]).tolist()
+    cu += [cu[-1]] * pad_seqs
+    return i32(seq), i32(cu), i32(list(slots) + [0] * pad_seqs)
+
+
+def close(got, want, tol, what=""):
+    got, want = got.double().cpu(), want.double().cpu()
+    assert torch.isfinite(got).all(), what
+    err = float((got - want).abs().max() / want.abs().max().clamp_min(1e-30))
+    assert err <= tol, f"{what}: relative error {err:.3e} exceeds {tol:.1e}"
+
+
+def runtime(dtype, max_positions=4096):
+    from minivllm_amd.parts.base import Runtime, Workspace
+    return Runtime(device=torch.device(DEV), dtype=dtype, ops=ops_for(dtype), workspace=Workspace(torch.device(DEV)),
+                   max_positions=max_positions)
+
+
+# ---------------------------------------------------------------------------------------
+# norm over whole rows, temperature, cache write
+# ---------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H, G, D, Dv, n, every", [(4, 2, 16, 24, 9, 5), (3, 1, 10, 6, 7, 1), (16, 8, 128, 128, 3, 64), (6, 3, 64, 64, 80, 16),
+                                                   (1, 1, 12, 20, 70, 7), (2, 2, 64, 40, 65, 33)])
+@pytest.mark.parametrize("beside", [False, True])
+def test_row_norm_and_store(dtype, H, G, D, Dv, n, every, beside):
+    """Rows of a step with a padding row, positions on both sides of the temperature's edges, keys and values on scattered
+    pages; alone, and in the launch of the linear side's single-token step."""
+    ops = ops_for(dtype)
+    g = torch.Generator().manual_seed(H * 100 + D)
+    page, eps, coef = 16, 1e-5, 0.7
+    R, rd, rv = 3, 8, 8                                         # the linear side, for `beside`
+    q_dim, k_dim, v_dim = H * D, G * D, G * Dv
+    base = q_dim + k_dim + v_dim + (-(q_dim + k_dim + v_dim)) % 8
+    width = base + 2 * R * (rd + rv)
+    rows = (2.0 * torch.randn(n, width, generator=g)).to(dtype)
+    qw, kw = [(1 + 0.2 * torch.randn(s, generator=g)).to(torch.bfloat16) for s in (q_dim, k_dim)]
+    start = every - 2 if every > 2 else 0
+    n_seq = 1 if not beside else n
+    positions = list(range(start, start + n))
+    table = torch.randperm(-(-(start + n) // page) + 3, generator=g).tolist()
+    bt = i32(table).view(1, -1).repeat(n_seq, 1).contiguous()
+    k_pages = torch.full((len(table), G, page, D), float("nan"), dtype=dtype, device=DEV)
+    v_pages = torch.full((len(table), G, Dv, page), float("nan"), dtype=dtype, device=DEV)
+    seq = [0] * n if not beside else list(range(n))
+    seq[n // 2] = -1                                            # a padding row
+    dev = rows.to(DEV)
+    args = dict(rows=dev, offsets=(0, q_dim, q_dim + k_dim), num_heads=H, num_kv_heads=G, head_dim=D, value_dim=Dv, positions=i32(positions),
+                q_weight=qw.to(DEV), k_weight=kw.to(DEV), eps=eps, temperature=(coef, every), k_pages=k_pages, v_pages=v_pages,
+                block_table=bt, page_size=page)
+    if beside:
+        state = torch.zeros(n, R, rv, rd, device=DEV)
+        out, sums = torch.empty(n, R * rv, dtype=dtype, device=DEV), torch.empty(n, R, device=DEV)
+        assert ops.constant_step(dev, base, R, rd, rv, torch.tensor([0.5, 0.9, 1.0], device=DEV), torch.ones(R * rv, device=DEV).to(torch.bfloat16),
+                                 state, i32(seq), i32(range(n)), out, sums, beside=args)
+    else:
+        ops.qkv_row_norm_store(i32(seq), **args)
+    torch.cuda.synchronize()
+    x = rows.double()
+    temp = torch.tensor([plain.query_temperature(p, coef, every) for p in positions], dtype=torch.float64)[:, None]
+    want_q = plain.rms_norm(x[:, :q_dim], qw.double(), eps) * temp
+    want_k = plain.rms_norm(x[:, q_dim:q_dim + k_dim], kw.double(), eps)
+    live = [t for t in range(n) if seq[t] >= 0]
+    tol = 3e-6 if dtype == torch.float32 else 8e-3
+    close(dev[live, :q_dim], want_q[live], tol, "queries")
+    assert torch.equal(dev[n // 2].cpu(), rows[n // 2]), "a padding row was touched"
+    assert torch.equal(dev[:, q_dim + k_dim:].cpu(), rows[:, q_dim + k_dim:]), "columns behind the keys were touched"
+    got_k = torch.stack([k_pages[table[positions[t] // page], :, positions[t] % page] for t in live]).reshape(len(live), k_dim)
+    got_v = torch.stack([v_pages[table[positions[t] // page], :, :, positions[t] % page] for t in live]).reshape(len(live), v_dim)
+    close(got_k, want_k[live], tol, "keys")
+    assert torch.equal(got_v.cpu(), rows[live, q_dim + k_dim:q_dim + k_dim + v_dim])
+    assert int(torch.isfinite(k_pages.float()).sum()) == len(live) * k_dim, "a slot of nobody was written"
+
+
+# ---------------------------------------------------------------------------------------
+# scored attention
+# ---------------------------------------------------------------------------------------
+class Scored:
+    """One request's keys and values on scattered pages (everything else NaN) and the plain answer."""
+
+    def __init__(self, H, G, D, Dv, n, page, dtype, seed, cap=20.0, biased=True, sink=True, far=None):
+        self.H, self.G, self.D, self.Dv, self.n, self.page, self.dtype = H, G, D, Dv, n, page, dtype
+        g = torch.Generator().manual_seed(seed)
+        self.q = torch.randn(n, H, D, generator=g)
+        self.k = torch.randn(n, G, D, generator=g)
+        self.v = torch.randn(n, G, Dv, generator=g)
+        if far is not None:                              # queries from position `far[1]` on single out the key at far[0]
+            mark = torch.randn(D, generator=g)
+            mark = mark / mark.norm() * D ** 0.5
+            self.k[far[0]] = 2.2 * mark
+            self.q[far[1]:] = 0.3 * self.q[far[1]:] + 2.2 * mark
+        self.q, self.k, self.v = self.q.to(dtype), self.k.to(dtype), self.v.to(dtype)
+        self.scale, self.cap, self.biased, self.sink = 1.3 / D ** 0.5, cap, biased, sink
+        self.slopes = torch.tensor([plain.distance_slope(h, H) for h in range(H)], dtype=torch.float32, device=DEV) if biased else None
+        count = -(-n // page)
+        self.table = torch.randperm(count + 4, generator=g)[:count].tolist()
+        self.k_pages = torch.full((count + 4, G, page, D), float("nan"), dtype=dtype)
+        self.v_pages = torch.full((count + 4, G, Dv, page), float("nan"), dtype=dtype)
+        for p in range(n):
+            self.k_pages[self.table[p // page], :, p % page] = self.k[p]
+            self.v_pages[self.table[p // page], :, :, p % page] = self.v[p]
+        self.k_pages, self.v_pages = self.k_pages.to(DEV), self.v_pages.to(DEV)
+
+    def want(self, first, count):
+        out = torch.empty(count, self.H, self.Dv, dtype=torch.float64)
+        m = {"scale": self.scale, "softcap": self.cap}
+        for h in range(self.H):
+            kv = h // (self.H // self.G)
+            q, k = self.q[first:first + count, h].double(), self.k[:first + count, kv].double()
+            s = plain.attention_scores(q, k, first, h, self.H, m)
+            if not self.biased:
+                i, j = torch.arange(first, first + count)[:, None], torch.arange(first + count)[None]
+                s = torch.where(j <= i, plain.capped((q @ k.T) * self.scale, self.cap), torch.full_like(s, -math.inf))
+            p = plain.sink_softmax(s) if self.sink else torch.softmax(s, -1)
+            out[:, h] = p @ self.v[:first + count, kv].double()
+        return out.reshape(count, self.H * self.Dv)
+
+    def run(self, ops, first, count, splits=None, variant=None, fast=True, hide_later=True):
+        from minivllm_amd.engine.step import AttentionPlan
+        from minivllm_amd.parts.base import Workspace
+        plan = AttentionPlan(decode_only=(count == 1), max_q_len=count, max_context_len=first + count, n_seqs=1, q_lens=[count],
+                             cu_seqlens=i32([0, count]), workspace=Workspace(torch.device(DEV)), decode_splits=splits,
+                             prefill_variant=variant, kv_tokens=first + count)
+        k_pages, v_pages = self.k_pages, self.v_pages
+        if hide_later and first + count < self.n:        # slots that nobody has written yet hold anything
+            k_pages, v_pages = k_pages.clone(), v_pages.clone()
+            for p in range(first + count, self.n):
+                k_pages[self.table[p // self.page], :, p % self.page] = float("nan")
+                v_pages[self.table[p // self.page], :, :, p % self.page] = float("nan")
+        q = self.q[first:first + count].reshape(count, -1).contiguous().to(DEV)
+        out = torch.empty(count, self.H * self.Dv, dtype=self.dtype, device=DEV)
+        ops.ledger = []
+        ops.attention(q, out, k_pages, v_pages, i32(self.table).view(1, -1), self.page, i32(range(first, first + count)), i32([0] * count),
+                      self.H, self.G, self.D, self.scale, None, plan=plan if fast else None, value_dim=self.Dv, softcap=self.cap,
+                      slopes=self.slopes, sink=self.sink)
+        torch.cuda.synchronize()
+        entry, ops.ledger = ops.ledger[0][0], None
+        return out, entry
+
+
+FORMS = [dict(), dict(cap=None), dict(biased=False), dict(sink=False), dict(cap=3.0, biased=False, sink=False)]
+
+
+@pytest.mark.parametrize("form", FORMS, ids=["all", "nocap", "nobias", "nosink", "cap"])
+@pytest.mark.parametrize("H, G, D, Dv, page", [(4, 2, 16, 24, 8), (3, 1, 10, 6, 4), (6, 2, 64, 64, 16), (2, 1, 128, 128, 32), (5, 5, 64, 32, 16)])
+def test_scored_attention_float32(H, G, D, Dv, page, form):
+    ops = ops_for(torch.float32)
+    c = Scored(H, G, D, Dv, 150, page, torch.float32, seed=D, far=(17, 120), **form)
+    for first, count in ((0, 150), (0, 1), (1, 2), (127, 5), (128, 1), (149, 1)):
+        out, entry = c.run(ops, first, count)
+        assert entry == "mv_attention_ref"
+        close(out, c.want(first, count), 2e-5, f"{count} queries from {first}")
+
+
+@pytest.mark.parametrize("form", FORMS, ids=["all", "nocap", "nobias", "nosink", "cap"])
+@pytest.mark.parametrize("variant", [(1, 1), (2, 1), (1, 2), (2, 2)])
+@pytest.mark.parametrize("H, G, D, page", [(6, 2, 64, 16), (2, 1, 128, 32), (16, 1, 64, 64), (4, 4, 128, 16)])
+def test_scored_attention_prompts(H, G, D, page, variant, form):
+    """Every variant of the MFMA prompt kernel: whole prompts, portions of odd lengths at odd places, a key far back that
+    the later queries single out at the border of a page."""
+    ops = ops_for(torch.bfloat16)
+    c = Scored(H, G, D, D, 300, page, torch.bfloat16, seed=H + D, far=(page - 1, 200), **form)
+    for first, count in ((0, 300), (0, 2), (3, 40), (95, 66), (250, 33)):
+        out, entry = c.run(ops, first, count, variant=variant)
+        assert entry == "mv_attention_prefill"
+        close(out, c.want(first, count), 1.2e-2, f"{count} queries from {first}")
+
+
+@pytest.mark.parametrize("form", FORMS, ids=["all", "nocap", "nobias", "nosink", "cap"])
+@pytest.mark.parametrize("splits", [None, 1, 3, 16])
+@pytest.mark.parametrize("H, G, D, page", [(6, 2, 64, 16), (2, 1, 128, 32), (16, 1, 64, 64), (4, 4, 128, 16)])
+def test_scored_attention_single_tokens(H, G, D, page, splits, form):
+    ops = ops_for(torch.bfloat16)
+    c = Scored(H, G, D, D, 700, page, torch.bfloat16, seed=H + D + 1, far=(page, 300), **form)
+    for first in (0, 1, 15, 16, 31, 32, 127, 128, 301, 511, 699):
+        out, entry = c.run(ops, first, 1, splits=splits)
+        assert entry == "mv_attention_decode"
+        close(out, c.want(first, 1), 1.2e-2, f"position {first}")
+
+
+def test_scored_attention_many_single_tokens():
+    """More (sequence, kv head) pairs than compute units: two workgroups share a unit and the keys are not split."""
+    from minivllm_amd.engine.step import AttentionPlan
+    from minivllm_amd.parts.base import Workspace
+    for D, H, G in ((64, 8, 4), (128, 4, 4)):
+        ops = ops_for(torch.bfloat16)
+        c = Scored(H, G, D, D, 90, 16, torch.bfloat16, seed=5, far=(3, 60))
+        B = 80
+        pos = [(7 * i + 3) % 90 for i in range(B)]
+        plan = AttentionPlan(decode_only=True, max_q_len=1, max_context_len=90, n_seqs=B, q_lens=[1] * B, cu_seqlens=i32(range(B + 1)),
+                             workspace=Workspace(torch.device(DEV)))
+        q = c.q[pos].reshape(B, -1).contiguous().to(DEV)
+        out = torch.empty(B, H * D, dtype=torch.bfloat16, device=DEV)
+        ops.attention(q, out, c.k_pages, c.v_pages, i32(c.table).view(1, -1).repeat(B, 1).contiguous(), 16, i32(pos), i32(range(B)), H, G, D,
+                      c.scale, None, plan=plan, softcap=c.cap, slopes=c.slopes, sink=True)
+        torch.cuda.synchronize()
+        want = torch.cat([c.want(p, 1) for p in pos])
+        close(out, want, 1.2e-2, "many single tokens")
+
+
+# ---------------------------------------------------------------------------------------
+# linear attention with constant decays
+# ---------------------------------------------------------------------------------------
+def constant_plain(rows, off, H, dk, dv, decay, norm, eps, S):
+    p = rows.double()[:, off:]
+    n = p.shape[0]
+    q, k = (plain.silu(p[:, i * H * dk:(i + 1) * H * dk]).view(n, H, dk) for i in (0, 1))
+    v = plain.silu(p[:, 2 * H * dk:2 * H * dk + H * dv]).view(n, H, dv)
+    gate = torch.sigmoid(p[:, 2 * H * dk + H * dv:2 * H * (dk + dv)])
+    raw, new = torch.empty(n, H, dv, dtype=torch.float64), []
+    for h in range(H):
+        raw[:, h], s = plain.constant_decay_scan(q[:, h], k[:, h], v[:, h], decay[h], S[h])
+        new.append(s)
+    return plain.rms_norm(raw.reshape(n, H * dv), norm.double(), eps) * gate, torch.stack(new)
+
+
+CONSTANT_SIZES = [(3, 12, 8, 8), (5, 6, 10, 0), (2, 64, 64, 16), (1, 8, 16, 3), (4, 32, 100, 8), (2, 128, 64, 24), (1, 200, 7, 5), (2, 16, 128, 0),
+                  (3, 70, 40, 8), (16, 64, 64, 0), (2, 128, 128, 8)]
+
+
+def build_constant(rt, H, dk, dv, decay, norm, eps, width):
+    from minivllm_amd.parts.matrix_state import ConstantDecay, ConstantDecaySpec
+    spec = ConstantDecaySpec(hidden_size=width, num_heads=H, key_dim=dk, value_dim=dv, decay=tuple(decay), out_norm_eps=eps)
+    t = {"q": torch.zeros(H * dk, width), "k": torch.zeros(H * dk, width), "v": torch.zeros(H * dv, width), "g": torch.zeros(H * dv, width),
+         "norm": norm, "o": torch.zeros(width, H * dv)}
+    return ConstantDecay(spec, {k: v.to(torch.bfloat16).to(DEV) for k, v in t.items()}, rt)
+
+
+def state_ctx(q_lens, slots, state, pad_rows=0, pad_seqs=0, conv=None):
+    from minivllm_amd.engine.step import AttentionPlan, StepContext
+    ctx = StepContext()
+    ctx.token_seq, ctx.cu_seqlens, ctx.state_slots = step_ints(q_lens, slots, pad_rows, pad_seqs)
+    ctx.n_tokens, ctx.n_seqs = sum(q_lens) + pad_rows, len(q_lens) + pad_seqs
+    ctx._state = {0: {"state": state} if conv is None else {"state": state, "conv": conv}}
+    ctx.attention_plan = AttentionPlan(decode_only=all(n == 1 for n in q_lens) and not pad_rows, max_q_len=max(q_lens), max_context_len=64,
+                                       n_seqs=ctx.n_seqs, q_lens=q_lens, cu_seqlens=ctx.cu_seqlens)
+    return ctx
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H, dk, dv, off", CONSTANT_SIZES)
+@pytest.mark.parametrize("q_lens", [[9, 1, 4, 2], [150, 3, 67, 64], [1, 130]])
+def test_constant_decay_mixed_step(dtype, H, dk, dv, off, q_lens):
+    """Requests on slots out of order, padding rows and a padding sequence, states that are not zero."""
+    rt = runtime(dtype)
+    g = torch.Generator().manual_seed(H * 1000 + dk + dv)
+    slots, n, eps = [2, 0, 3, 1][:len(q_lens)], sum(q_lens), 1e-5
+    rows = (1.5 * torch.randn(n + 2, off + 2 * H * (dk + dv) + (-(off + 2 * H * (dk + dv))) % 8, generator=g)).to(dtype)
+    decay = [1.0 if h == 0 and H > 1 else float(x) for h, x in enumerate(torch.rand(H, generator=g) * 0.9 + 0.1)]
+    norm = (1 + 0.2 * torch.randn(H * dv, generator=g)).to(torch.bfloat16)
+    part = build_constant(rt, H, dk, dv, decay, norm, eps, 32)
+    S0 = torch.randn(5, H, dk, dv, generator=g)
+    state = S0.transpose(2, 3).contiguous().to(DEV)
+    ctx = state_ctx(q_lens, slots, state, pad_rows=2, pad_seqs=1)
+    gated, sums, _ = part.recur(rows.to(DEV), off, ctx, 0)
+    torch.cuda.synchronize()
+    assert sums is None
+    tol = 2e-5 if dtype == torch.float32 else 1.5e-2
+    base = 0
+    decay32 = torch.tensor(decay, dtype=torch.float32).double().tolist()
+    for qn, slot in zip(q_lens, slots):
+        want, S = constant_plain(rows[base:base + qn], off, H, dk, dv, decay32, norm, eps, S0[slot].double())
+        close(gated[base:base + qn], want, tol, f"request of {qn}")
+        close(state[slot].transpose(1, 2), S, 2e-5, "state")
+        base += qn
+    assert float(gated[n:].float().abs().max()) == 0.0
+    untouched = sorted(set(range(5)) - set(slots))
+    assert torch.equal(state[untouched].cpu(), S0[untouched].transpose(2, 3)), "a slot of nobody was touched"
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H, dk, dv, off", CONSTANT_SIZES)
+def test_constant_decay_single_tokens(dtype, H, dk, dv, off):
+    """Twelve tokens one by one for three requests side by side (one row of padding in some steps) against the plain scan;
+    the rows the step leaves undivided come out right once divided by their root mean square."""
+    rt = runtime(dtype)
+    g = torch.Generator().manual_seed(H * 77 + dk)
+    eps, T = 1e-5, 12
+    width = off + 2 * H * (dk + dv) + (-(off + 2 * H * (dk + dv))) % 8
+    rows = (1.5 * torch.randn(T, 3, width, generator=g)).to(dtype)
+    decay = [float(x) for x in torch.rand(H, generator=g) * 0.9 + 0.1]
+    norm = (1 + 0.2 * torch.randn(H * dv, generator=g)).to(torch.bfloat16)
+    part = build_constant(rt, H, dk, dv, decay, norm, eps, 32)
+    slots = [3, 0, 2]
+    state = torch.zeros(4, H, dv, dk, device=DEV)
+    want = [constant_plain(rows[:, i], off, H, dk, dv, torch.tensor(decay, dtype=torch.float32).double().tolist(), norm, eps,
+                           torch.zeros(H, dk, dv, dtype=torch.float64)) for i in range(3)]
+    for t in range(T):
+        ctx = state_ctx([1, 1, 1], slots, state)
+        gated, sums, _ = part.recur(rows[t].to(DEV), off, ctx, 0)
+        assert sums is not None and sums.inner == H * dv
+        whole = torch.empty_like(gated)
+        rt.ops.scale_rows(gated, sums.sums, H, sums.eps, whole)
+        torch.cuda.synchronize()
+        for i in range(3):
+            close(whole[i:i + 1], want[i][0][t:t + 1], 2e-5 if dtype == torch.float32 else 2e-2, f"token {t} of request {i}")
+    for i, s in enumerate(slots):
+        close(state[s].transpose(1, 2), want[i][1], 2e-5, "state after the last token")
+    assert float(state[1].abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_constant_decay_portions_and_long_runs(dtype):
+    """700 tokens whole against portions of many sizes, down to one token, with a decay of almost one and one that forgets
+    within a token or two."""
+    H, dk, dv, eps = 3, 64, 64, 1e-6
+    rt = runtime(dtype)
+    g = torch.Generator().manual_seed(9)
+    rows = torch.randn(700, 2 * H * (dk + dv), generator=g).to(dtype)
+    norm = torch.ones(H * dv).to(torch.bfloat16)
+    part = build_constant(rt, H, dk, dv, [0.9999, 0.9, 0.05], norm, eps, 32)
+    decay32 = torch.tensor([0.9999, 0.9, 0.05], dtype=torch.float32).double().tolist()
+    want, S = constant_plain(rows, 0, H, dk, dv, decay32, norm, eps, torch.zeros(H, dk, dv, dtype=torch.float64))
+    tol = 3e-5 if dtype == torch.float32 else 1.5e-2
+    for sizes in ([700], [64, 63, 65, 128, 127, 1, 2, 250], [1, 2, 3, 31, 32, 33, 598]):
+        state, p, out = torch.zeros(1, H, dv, dk, device=DEV), 0, []
+        for n in sizes:
+            ctx = state_ctx([n], [0], state)
+            gated, sums, _ = part.recur(rows[p:p + n].to(DEV), 0, ctx, 0)
+            if sums is not None:
+                whole = torch.empty_like(gated)
+                rt.ops.scale_rows(gated, sums.sums, H, sums.eps, whole)
+                gated = whole
+            out.append(gated.clone())
+            p += n
+        torch.cuda.synchronize()
+        got = torch.cat(out)
+        if dtype == torch.bfloat16:                      # (rows left undivided are rounded once more)
+            close(got, want[:p], 2e-2, str(sizes))
+        else:
+            close(got, want[:p], tol, str(sizes))
+        close(state[0].transpose(1, 2), S if p == 700 else constant_plain(rows[:p], 0, H, dk, dv, decay32, norm, eps,
+                                                                           torch.zeros(H, dk, dv, dtype=torch.float64))[1], 3e-5, "state")
+
+
+# ---------------------------------------------------------------------------------------
+# channel-wise gated delta rule
+# ---------------------------------------------------------------------------------------
+def channel_case(H, G, dk, dv, taps, ra, rg, hid, seed):
+    g = torch.Generator().manual_seed(seed)
+    shapes = {"q": (G * dk, hid), "k": (G * dk, hid), "v": (H * dv, hid), "b": (H, hid), "q.conv": (G * dk, taps), "k.conv": (G * dk, taps),
+              "v.conv": (H * dv, taps), "A_log": (H,), "dt_bias": (H * dk,), "a1": (ra, hid), "a2": (H * dk, ra), "g1": (rg, hid),
+              "g2": (H * dv, rg), "norm": (dv,), "o": (hid, H * dv)}
+    w = {}
+    for name, shape in shapes.items():
+        t = torch.randn(shape, generator=g)
+        if len(shape) == 2 and not name.endswith("conv"):
+            t = t / shape[1] ** 0.5
+        if name == "A_log":
+            t = t - 1.0
+        if name == "norm":
+            t = 1 + 0.2 * t
+        w[name] = t.to(torch.bfloat16)
+    return w
+
+
+def build_channel(rt, w, H, G, dk, dv, taps, ra, rg, hid, eps):
+    from minivllm_amd.parts.matrix_state import ChannelDelta, ChannelDeltaSpec
+    spec = ChannelDeltaSpec(hidden_size=hid, num_heads=H, num_kv_heads=G, key_dim=dk, value_dim=dv, conv_taps=taps, decay_rank=ra,
+                            gate_rank=rg, unit_eps=plain.UNIT_EPS, out_norm_eps=eps)
+    return ChannelDelta(spec, {k.replace(".", "_"): v.to(DEV) for k, v in w.items()}, rt)
+
+
+def plain_channel(x, w, m, eps, state, dtype):
+    rnd = None if dtype == torch.float32 else plain.round_to_bfloat16
+    return plain.channel_delta_mixer(x.double(), {k: v.double() for k, v in w.items()}, "", m, eps, state, rnd)
+
+
+def split_state(conv, S, G, H, dk, dv):
+    """The plain state of a slot from the engine's layout."""
+    d = {"S": S.transpose(1, 2).double().cpu()}
+    if conv is not None:
+        c = conv.double().cpu()
+        d.update({"conv.q": c[:, :G * dk], "conv.k": c[:, G * dk:2 * G * dk], "conv.v": c[:, 2 * G * dk:]})
+    return d
+
+
+CHANNEL_SIZES = [(4, 2, 16, 24, 3, 12, 20), (3, 3, 6, 10, 2, 3, 7), (2, 1, 64, 128, 4, 32, 48), (1, 1, 12, 8, 1, 4, 4), (6, 2, 40, 20, 5, 17, 2),
+                 (2, 2, 128, 64, 4, 64, 64), (1, 1, 200, 7, 2, 9, 5), (8, 8, 64, 64, 4, 64, 32), (2, 2, 32, 256, 3, 130, 8), (2, 1, 10, 300, 6, 8, 8)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H, G, dk, dv, taps, ra, rg", CHANNEL_SIZES)
+@pytest.mark.parametrize("q_lens", [[9, 1, 4, 2], [1, 1, 1, 1], [70, 2, 1, 33]])
+def test_channel_delta_step(dtype, H, G, dk, dv, taps, ra, rg, q_lens):
+    """Four requests on slots out of order from states and kept inputs that are not zero: prompt portions with padding rows
+    and a padding sequence, and single tokens (one kernel)."""
+    rt = runtime(dtype)
+    hid, eps = 96, 1e-5
+    w = channel_case(H, G, dk, dv, taps, ra, rg, hid, seed=H * 100 + dk)
+    part = build_channel(rt, w, H, G, dk, dv, taps, ra, rg, hid, eps)
+    m = {"heads": H, "kv_heads": G, "dim": dk, "vdim": dv}
+    g = torch.Generator().manual_seed(3)
+    slots, n = [2, 0, 3, 1], sum(q_lens)
+    single = all(k == 1 for k in q_lens)
+    pad = 0 if single else 2
+    x = torch.randn(n + pad, hid, generator=g).to(dtype)
+    C = 2 * G * dk + H * dv
+    S0 = 0.3 * torch.randn(5, H, dv, dk, generator=g)
+    c0 = torch.randn(5, taps - 1, C, generator=g).to(dtype) if taps > 1 else None
+    state, conv = S0.clone().to(DEV), None if c0 is None else c0.clone().to(DEV)
+    ctx = state_ctx(q_lens, slots, state, pad_rows=pad, pad_seqs=1 if pad else 0, conv=conv)
+    rt.ops.ledger = []
+    y = part.forward(x.to(DEV), ctx, 0)
+    y = y if isinstance(y, torch.Tensor) else y.materialize()
+    torch.cuda.synchronize()
+    ran, rt.ops.ledger = [e[0] for e in rt.ops.ledger], None
+    assert ("mv_channel_step" in ran) == (single and dv <= 256) and ("mv_channel_scan" in ran) == (not (single and dv <= 256))
+    tol = 3e-5 if dtype == torch.float32 else 2e-2
+    base = 0
+    for qn, slot in zip(q_lens, slots):
+        before = split_state(None if c0 is None else c0[slot], S0[slot], G, H, dk, dv)
+        want, after = plain_channel(x[base:base + qn], w, m, eps, before, dtype)
+        close(y[base:base + qn], want, tol, f"request of {qn}")
+        got = split_state(None if conv is None else conv[slot], state[slot], G, H, dk, dv)
+        close(got["S"], after["S"], 3e-5 if dtype == torch.float32 else 5e-3, "state")
+        if taps > 1:
+            for name in ("q", "k", "v"):
+                close(got["conv." + name], after["conv." + name], 1e-6 if dtype == torch.float32 else 8e-3, "kept inputs")
+        base += qn
+    assert torch.equal(state[4].cpu(), S0[4]) and (conv is None or torch.equal(conv[4].cpu(), c0[4]))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("G", [4, 2])
+def test_channel_delta_portions(dtype, G):
+    """260 tokens whole, in portions down to two tokens, and token by token: the same rows, within rounding."""
+    H, dk, dv, taps, ra, rg, hid, eps = 4, 32, 24, 4, 16, 8, 64, 1e-6
+    rt = runtime(dtype)
+    w = channel_case(H, G, dk, dv, taps, ra, rg, hid, seed=4)
+    part = build_channel(rt, w, H, G, dk, dv, taps, ra, rg, hid, eps)
+    x = torch.randn(260, hid, generator=torch.Generator().manual_seed(1)).to(dtype)
+    want, _ = plain_channel(x, w, {"heads": H, "kv_heads": G, "dim": dk, "vdim": dv}, eps, None, dtype)
+    for sizes in ([260], [2, 3, 64, 15, 16, 17, 2, 2, 139], [100] + [1] * 160):
+        state = torch.zeros(1, H, dv, dk, device=DEV)
+        conv = torch.zeros(1, taps - 1, 2 * G * dk + H * dv, dtype=dtype, device=DEV)
+        out, p = [], 0
+        for n in sizes:
+            y = part.forward(x[p:p + n].to(DEV), state_ctx([n], [0], state, conv=conv), 0)
+            out.append((y if isinstance(y, torch.Tensor) else y.materialize()).clone())
+            p += n
+        torch.cuda.synchronize()
+        close(torch.cat(out), want, 3e-5 if dtype == torch.float32 else 2e-2, str(sizes[:6]))
+
+
+# ---------------------------------------------------------------------------------------
+# two parts joined, entries into a run of layers
+# ---------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W", [64, 50, 1024, 2056, 4096, 8192, 8200])
+@pytest.mark.parametrize("undivided", [False, True])
+def test_pair_norm(dtype, W, undivided):
+    """Joined alone, added to the residual, and with the next norm; with one side's rows still to be divided by the root
+    mean square that was left out in front of its linear map."""
+    from minivllm_amd.kernels.ops import NormedPair, RowSums
+    ops = ops_for(dtype)
+    g = torch.Generator().manual_seed(W)
+    n, eps, inner_eps, inner, parts = 5, 1e-5, 1e-5, 36, 3
+    a, b = (3 * torch.randn(n, W, generator=g)), (0.2 * torch.randn(n, W, generator=g))
+    sums = 4.0 * torch.rand(n, parts, generator=g) + 0.1
+    c = torch.sqrt(sums.double().sum(1, keepdim=True) / inner + inner_eps) if undivided else torch.ones(n, 1, dtype=torch.float64)
+    a, b = a.to(dtype), b.to(dtype)
+    wa, wb, wn = [(s + 0.2 * torch.randn(W, generator=g)).to(torch.bfloat16) for s in (1.0, 1.0, 0.0)]
+    x0 = torch.randn(n, W, generator=g)
+    delta = 0.5 * (plain.rms_norm(a.double(), wa.double(), eps) + plain.rms_norm(b.double() / c, wb.double(), eps))
+    total = x0.double() + delta
+    rows = RowSums(sums.to(DEV), inner, inner_eps) if undivided else None
+
+    def pair():
+        return NormedPair(ops, (a.to(DEV), b.to(DEV)), (wa.to(DEV), wb.to(DEV)), eps, (None, rows), torch.empty(n, W, dtype=dtype, device=DEV))
+    tol = 3e-6 if dtype == torch.float32 else 6e-3
+    close(pair().materialize(), delta, tol, "joined")
+    resid = x0.to(DEV)
+    ops.add_rmsnorm(resid, pair(), None, eps, None)
+    close(resid, total, 1e-6, "residual")
+    resid, out = x0.to(DEV), torch.empty(n, W, dtype=dtype, device=DEV)
+    ops.add_rmsnorm(resid, pair(), wn.to(DEV), 1e-6, out, unit_offset=True)
+    close(resid, total, 1e-6, "residual")
+    close(out, plain.rms_norm(total, wn.double(), 1e-6, around_zero=True), tol, "next norm")
+    pick = i32([3, 0])
+    out = torch.empty(2, W, dtype=dtype, device=DEV)
+    ops.add_rmsnorm(x0.to(DEV), pair(), wn.to(DEV), 1e-6, out, rows=pick, unit_offset=True)
+    close(out, plain.rms_norm(total[[3, 0]], wn.double(), 1e-6, around_zero=True), tol if dtype == torch.float32 else 1.2e-2, "chosen rows")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W", [64, 50, 1024])
+@pytest.mark.parametrize("with_delta, with_rows, with_norm", [(True, True, True), (False, False, True), (True, False, False), (False, True, False)])
+def test_stream_entry(dtype, W, with_delta, with_rows, with_norm):
+    ops = ops_for(dtype)
+    g = torch.Generator().manual_seed(W)
+    n, V = 6, 30
+    x0, d = torch.randn(n, W, generator=g), torch.randn(n, W, generator=g).to(dtype)
+    table, step, wn = torch.randn(V, W, generator=g).to(torch.bfloat16), torch.randn(W, generator=g).to(torch.bfloat16), \
+        (0.2 * torch.randn(W, generator=g)).to(torch.bfloat16)
+    ids = [3, 29, 0, 7, 7, 12]
+    want = x0.double() + step.double()
+    if with_delta:
+        want = want + d.double()
+    if with_rows:
+        want = want + table.double()[ids] * 1.5
+    resid, out = x0.to(DEV), torch.empty(n, W, dtype=dtype, device=DEV) if with_norm else None
+    ops.stream_entry(resid, d.to(DEV) if with_delta else None, (i32(ids), table.to(DEV), 1.5) if with_rows else None, step.to(DEV),
+                     (wn.to(DEV), 1e-5, True) if with_norm else None, out)
+    torch.cuda.synchronize()
+    close(resid, want, 1e-6, "residual")
+    if with_norm:
+        close(out, plain.rms_norm(want, wn.double(), 1e-5, around_zero=True), 3e-6 if dtype == torch.float32 else 6e-3, "norm")
+
+
+# ---------------------------------------------------------------------------------------
+# the clamped gated pair with biases, in whatever kernel takes the shape
+# ---------------------------------------------------------------------------------------
+def feed_forward_case(hid, ff, seed, limit):
+    g = torch.Generator().manual_seed(seed)
+    w = {"gate": torch.randn(ff, hid, generator=g) / hid ** 0.5, "up": torch.randn(ff, hid, generator=g) / hid ** 0.5,
+         "down": torch.randn(hid, ff, generator=g) / ff ** 0.5, "gate.b": 0.8 * torch.randn(ff, generator=g),
+         "up.b": 0.8 * torch.randn(ff, generator=g), "down.b": 0.8 * torch.randn(hid, generator=g)}
+    return {k: v.to(torch.bfloat16) for k, v in w.items()}
+
+
+def build_feed_forward(rt, w, hid, ff, limit):
+    from minivllm_amd.parts.mlp import ClampedGLU, ClampedGLUSpec
+    return ClampedGLU(ClampedGLUSpec(hidden_size=hid, intermediate_size=ff, limit=limit, slope=plain.GATE_SLOPE),
+                      {k.replace(".b", "_bias"): v.to(DEV) for k, v in w.items()}, rt)
+
+
+@pytest.mark.parametrize("dtype, hid, ff, rows", [
+    (torch.float32, 50, 30, 7), (torch.float32, 64, 96, 65), (torch.bfloat16, 50, 30, 9), (torch.bfloat16, 64, 96, 1),
+    (torch.bfloat16, 192, 256, 40), (torch.bfloat16, 1024, 3072, 8), (torch.bfloat16, 1024, 3072, 64), (torch.bfloat16, 1024, 3072, 200),
+    (torch.bfloat16, 2048, 3072, 20), (torch.bfloat16, 1024, 3072, 2000)])
+@pytest.mark.parametrize("limit", [0.6, 7.0])
+def test_clamped_pair(dtype, hid, ff, rows, limit):
+    rt = runtime(dtype)
+    w = feed_forward_case(hid, ff, hid + ff, limit)
+    x = torch.randn(rows, hid, generator=torch.Generator().manual_seed(rows)).to(dtype)
+    y = build_feed_forward(rt, w, hid, ff, limit).forward(x.to(DEV), None)
+    y = y if isinstance(y, torch.Tensor) else y.materialize()
+    torch.cuda.synchronize()
+    want = plain.clamped_feed_forward(x.double(), {k: v.double() for k, v in w.items()}, "", limit)
+    close(y, want, 1e-5 if dtype == torch.float32 else 1.2e-2, f"{rows} rows")
+
+
+@pytest.mark.parametrize("rows, hid, ff", [(1, 256, 320), (8, 1024, 3072), (16, 1024, 1024), (40, 1024, 3072), (64, 256, 512), (96, 512, 768)])
+def test_clamped_pair_behind_folded_and_pending_norms(rows, hid, ff):
+    """The gated pair with biases as the product behind a norm: the norm pending (few rows), and folded into a product with
+    a bias in front (its rows arrive weighted but not divided)."""
+    from minivllm_amd.parts.base import HiddenStream
+    from minivllm_amd.parts.norm import RMSNorm, RMSNormSpec
+    rt = runtime(torch.bfloat16)
+    ops, g = rt.ops, torch.Generator().manual_seed(rows)
+    w = feed_forward_case(hid, ff, 5, 0.9)
+    part = build_feed_forward(rt, w, hid, ff, 0.9)
+    nw = (0.2 * torch.randn(hid, generator=g)).to(torch.bfloat16)
+    norm = RMSNorm(RMSNormSpec(size=hid, eps=1e-5, unit_offset=True), {"weight": nw.to(DEV)}, rt)
+    x0 = torch.randn(rows, hid, generator=g)
+    dense = {k: v.double() for k, v in w.items()}
+
+    def want(x):
+        return plain.clamped_feed_forward(plain.rms_norm(x, nw.double(), 1e-5, around_zero=True), dense, "", 0.9)
+
+    def finished(y):
+        y = y if isinstance(y, torch.Tensor) else y.materialize()
+        torch.cuda.synchronize()
+        return y
+    d = torch.randn(rows, hid, generator=g).to(torch.bfloat16)
+    stream = HiddenStream(x0.to(DEV), torch.empty(rows, hid, device=DEV))
+    stream.delta = d.to(DEV)
+    y = finished(part.forward(norm.pending(stream, None), None))
+    close(y, want(x0.double() + d.double()), 1.5e-2, "pending norm")
+    # a product with a bias in front of the norm
+    pw, pb, a = torch.randn(hid, 192, generator=g) / 192 ** 0.5, 0.5 * torch.randn(hid, generator=g), torch.randn(rows, 192, generator=g)
+    pw, pb, a = pw.to(torch.bfloat16), pb.to(torch.bfloat16), a.to(torch.bfloat16)
+    stream = HiddenStream(x0.to(DEV), torch.empty(rows, hid, device=DEV))
+    fold = norm.fold(stream, None, part.first_product())
+    out = torch.empty(rows, hid, dtype=torch.bfloat16, device=DEV)
+    got = ops.gemm(a.to(DEV), pw.to(DEV), out, pb.to(DEV), fold=fold)
+    if getattr(got, "is_weighted_rows", False):
+        stream.weighted = got
+    else:
+        stream.delta = out if got is None else got
+    y = finished(part.forward(norm.pending(stream, None), None))
+    total = x0.double() + plain.round_to_bfloat16(a.double() @ pw.double().T + pb.double())
+    close(stream.resid, total, 4e-3, "residual behind the folded product")      # (the product is rounded once: an ulp of it)
+    close(y, want(total), 1.5e-2, "folded norm")

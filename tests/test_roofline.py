@@ -92,3 +92,16 @@ def test_two_products_of_one_kernel_in_a_row_are_two_launches(tmp_path):
     assert [len(t) for t in found[0].times] == [1, 1, 1, 1, 2, 1]
     text = roofline.kernel_table(path, roofline.launches(step), "bfloat16", title="t")
     assert "3 occurrences" in text
+
+
+def test_library_products_in_a_row(tmp_path):
+    """Two library products behind each other are two launches; a single one may bring a second kernel along."""
+    step = [("mv_embedding", 100, 0), ("mv_gemm_lt", 4000, 8000), ("mv_gemm_lt", 2000, 4000), ("mv_swiglu", 500, 0),
+            ("mv_gemm_lt", 3000, 6000), ("mv_sample", 300, 600)]
+    kernels = [("void embedding_kernel(int const*)", 1.0), ("Cijk_Alik_Bljk_BBS_BH_MT64x128x128_MI16", 18.0),
+               ("Cijk_Alik_Bljk_BBS_BH_MT64x128x64_MI16", 13.0), ("void swiglu_vec_kernel<bf16>(int)", 10.0),
+               ("Cijk_Alik_Bljk_BBS_BH_MT128x64x128_MI16", 25.0), ("Cijk_Alik_Bljk_BBS_BH_PostGSU", 2.0), ("void sample_kernel(float const*)", 2.0)]
+    path = str(tmp_path / "lt_kernel_trace.csv")
+    write_trace(path, kernels * 2)
+    found = roofline.find_windows(roofline.read_trace(path), roofline.launches(step))
+    assert len(found) == 2 and [len(t) for t in found[0].times] == [1, 1, 1, 1, 2, 1]
