@@ -82,6 +82,7 @@ KERNELS_OF: Dict[str, Tuple[str, Optional[str], int]] = {
     "mv_add_rows": (r"\badd_rows_kernel", None, 1),
     "mv_qkv_row_norm_store": (r"\bqkv_row_norm_store_kernel", r"\bstore_v_pages_kernel", 2),
     "mv_constant_prepare": (r"\bconstant_prepare_kernel", None, 1),
+    "mv_constant_chunks": (r"\bchunk_sums_kernel", r"\bchunk_(walk|out)_kernel", 3),
     "mv_row_gate_finish": (r"\brow_gate_finish_kernel", None, 1),
     "mv_constant_step": (r"\bconstant_step_kernel", None, 1),
     "mv_pair_norm_add_norm": (r"\bpair_norm_add_norm_kernel", None, 1),

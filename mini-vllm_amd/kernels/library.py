@@ -62,6 +62,10 @@ _SIGNATURES = {
     # packed, ld, off, n, H, DK, DV, decay, token_seq, qk, vals, gates, dtype, stream
     "mv_constant_prepare": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                     c_void_p, c_int, c_void_p]),
+    "mv_constant_chunk_tokens": (c_int, []),
+    # packed, ld, off, n, H, DK, DV, decay, state, cu_seqlens, state_slots, n_seqs, chunks, sums, out, dtype, stream
+    "mv_constant_chunks": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                                   c_int, c_int, c_void_p, c_void_p, c_int, c_void_p]),
     # raw, packed, ld, g_off, weight, weight_dtype, n, W, eps, token_seq, out, ldo, dtype, stream
     "mv_row_gate_finish": (c_int, [c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p,
                                    c_long, c_int, c_void_p]),

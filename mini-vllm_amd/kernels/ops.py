@@ -1043,6 +1043,32 @@ class Ops:
                       dk, dv, decay.data_ptr(), token_seq.data_ptr(), qk.data_ptr(), vals.data_ptr(), gates.data_ptr(), self.code,
                       self._stream())
 
+    def constant_chunk_tokens(self) -> int:
+        """Tokens in a chunk of ``constant_chunks``."""
+        return int(self.lib.dll.mv_constant_chunk_tokens())
+
+    def constant_chunks(self, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, decay: torch.Tensor, state: torch.Tensor,
+                        token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int, chunks: int,
+                        sums: torch.Tensor, out: torch.Tensor) -> None:
+        """Per request and head over the step's tokens: S <- decay S + k v^T; out = S^T q, with q, k, v the SiLU of the rows'
+        columns [q | k (heads*dk each) | v (heads*dv)] from ``offset`` on, as products over chunks of tokens. Decays in
+        (0, 1]. ``chunks``: how many chunks of ``constant_chunk_tokens`` the requests' rows form (or more); sums float32
+        [chunks, heads, dv, dk] is scratch. state float32 [slots, heads, dv, dk] is read and left advanced; out float32
+        [n, heads, dv]."""
+        n = self._constant_rows("constant_chunks", packed, offset, heads, dk, dv, decay, token_seq)
+        self._matrix_state("constant_chunks", state, heads, dv, dk)
+        _dev(sums, "chunk sums"); _dev(out, "chunk outputs")
+        for t, shape, name in ((sums, (chunks, heads, dv, dk), "chunk sums"), (out, (n, heads, dv), "outputs")):
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"constant_chunks: the {name} must be contiguous float32 {shape}")
+        self._ints(n, cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        C = self.constant_chunk_tokens()
+        self._note("mv_constant_chunks", n * heads * (2 * dk + dv) * packed.element_size() + self._size(out)
+                   + 2 * min(n_seqs, max(n, 1)) * heads * dv * dk * 4, n * heads * (4 * dk * dv + C * (dk + dv)))
+        self.lib.call("mv_constant_chunks", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(offset), n, heads, dk,
+                      dv, decay.data_ptr(), state.data_ptr(), cu_seqlens.data_ptr(), state_slots.data_ptr(), n_seqs, int(chunks),
+                      sums.data_ptr(), out.data_ptr(), self.code, self._stream())
+
     def row_gate_finish(self, raw: torch.Tensor, packed: torch.Tensor, gate_offset: int, weight: torch.Tensor, eps: float,
                         token_seq: torch.Tensor, out: torch.Tensor) -> None:
         """out[t] = o / rms(o) * weight * sigmoid(g), the root mean square over the whole row of o = raw[t] (all heads

@@ -348,6 +348,8 @@ class ConstantDecay(Mixer):
         self.w_packed = _pack(tensors, self.PACKED, spec.hidden_size, "constant decay")
         self.width = self.w_packed.shape[0]
         self.decay = torch.tensor(spec.decay, dtype=torch.float32, device=rt.device)
+        # prompts go chunk by chunk through matrix products where the decays' powers are powers of two's logarithm
+        self.chunked = all(0.0 < d <= 1.0 for d in spec.decay)
         self.norm, self.w_o = tensors["norm"].contiguous(), tensors["o"]
 
     def recur(self, packed: torch.Tensor, base: int, ctx, call: int, beside: Optional[dict] = None):
@@ -363,12 +365,18 @@ class ConstantDecay(Mixer):
             if ops.constant_step(packed, base, H, dk, dv, self.decay, self.norm, ctx.state(call), ctx.token_seq, ctx.state_slots, gated,
                                  sums, beside=beside):
                 return gated, RowSums(sums, H * dv, spec.out_norm_eps), beside is not None
-        qk = ws.get("mstate.qk", (n, H, 2, dk), torch.float32)
-        vals = ws.get("mstate.vals", (n, H, dv), torch.float32)
-        gates = ws.get("mstate.gates", (n, H, 4), torch.float32)
-        ops.constant_prepare(packed, base, H, dk, dv, self.decay, ctx.token_seq, qk, vals, gates)
         raw = ws.get("mstate.raw", (n, H, dv), torch.float32)
-        ops.state_scan(qk, vals, gates, ctx.state(call), ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, H, H, dk, dv, False, raw)
+        if self.chunked and plan is not None:
+            chunks = plan.units(ops.constant_chunk_tokens())
+            sums = ws.get("mstate.chunks", (chunks, H, dv, dk), torch.float32)
+            ops.constant_chunks(packed, base, H, dk, dv, self.decay, ctx.state(call), ctx.token_seq, ctx.cu_seqlens, ctx.state_slots,
+                                ctx.n_seqs, chunks, sums, raw)
+        else:
+            qk = ws.get("mstate.qk", (n, H, 2, dk), torch.float32)
+            vals = ws.get("mstate.vals", (n, H, dv), torch.float32)
+            gates = ws.get("mstate.gates", (n, H, 4), torch.float32)
+            ops.constant_prepare(packed, base, H, dk, dv, self.decay, ctx.token_seq, qk, vals, gates)
+            ops.state_scan(qk, vals, gates, ctx.state(call), ctx.cu_seqlens, ctx.state_slots, ctx.n_seqs, H, H, dk, dv, False, raw)
         ops.row_gate_finish(raw, packed, base + H * (2 * dk + dv), self.norm, spec.out_norm_eps, ctx.token_seq, gated)
         return gated, None, False
 

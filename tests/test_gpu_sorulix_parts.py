@@ -269,9 +269,11 @@ def state_ctx(q_lens, slots, state, pad_rows=0, pad_seqs=0, conv=None):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H, dk, dv, off", CONSTANT_SIZES)
-@pytest.mark.parametrize("q_lens", [[9, 1, 4, 2], [150, 3, 67, 64], [1, 130]])
-def test_constant_decay_mixed_step(dtype, H, dk, dv, off, q_lens):
-    """Requests on slots out of order, padding rows and a padding sequence, states that are not zero."""
+@pytest.mark.parametrize("q_lens", [[9, 1, 4, 2], [150, 3, 67, 64], [1, 130], [2] * 4])
+@pytest.mark.parametrize("chunked", [True, False])
+def test_constant_decay_mixed_step(dtype, H, dk, dv, off, q_lens, chunked):
+    """Requests on slots out of order, padding rows and a padding sequence, states that are not zero; in chunks (products
+    of small matrices) and token by token (what decays outside (0, 1] take)."""
     rt = runtime(dtype)
     g = torch.Generator().manual_seed(H * 1000 + dk + dv)
     slots, n, eps = [2, 0, 3, 1][:len(q_lens)], sum(q_lens), 1e-5
@@ -279,6 +281,8 @@ def test_constant_decay_mixed_step(dtype, H, dk, dv, off, q_lens):
     decay = [1.0 if h == 0 and H > 1 else float(x) for h, x in enumerate(torch.rand(H, generator=g) * 0.9 + 0.1)]
     norm = (1 + 0.2 * torch.randn(H * dv, generator=g)).to(torch.bfloat16)
     part = build_constant(rt, H, dk, dv, decay, norm, eps, 32)
+    assert part.chunked and not build_constant(rt, H, dk, dv, [-0.5] + decay[1:], norm, eps, 32).chunked
+    part.chunked = chunked
     S0 = torch.randn(5, H, dk, dv, generator=g)
     state = S0.transpose(2, 3).contiguous().to(DEV)
     ctx = state_ctx(q_lens, slots, state, pad_rows=2, pad_seqs=1)
@@ -327,6 +331,29 @@ def test_constant_decay_single_tokens(dtype, H, dk, dv, off):
     for i, s in enumerate(slots):
         close(state[s].transpose(1, 2), want[i][1], 2e-5, "state after the last token")
     assert float(state[1].abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_constant_decay_many_requests(dtype):
+    """More requests than a workgroup has threads, of one to three tokens and a few chunks, in one step."""
+    H, dk, dv, eps = 2, 8, 12, 1e-5
+    rt = runtime(dtype)
+    g = torch.Generator().manual_seed(2)
+    q_lens = [int(x) for x in torch.randint(1, 4, (290,), generator=g)]
+    q_lens[5], q_lens[256], q_lens[289] = 130, 70, 65
+    rows = torch.randn(sum(q_lens), 2 * H * (dk + dv), generator=g).to(dtype)
+    norm = torch.ones(H * dv).to(torch.bfloat16)
+    part = build_constant(rt, H, dk, dv, [0.9, 0.99], norm, eps, 32)
+    state = torch.zeros(290, H, dv, dk, device=DEV)
+    gated, sums, _ = part.recur(rows.to(DEV), 0, state_ctx(q_lens, list(range(289, -1, -1)), state), 0)
+    torch.cuda.synchronize()
+    decay32 = torch.tensor([0.9, 0.99], dtype=torch.float32).double().tolist()
+    base = 0
+    for s, n in enumerate(q_lens):
+        want, S = constant_plain(rows[base:base + n], 0, H, dk, dv, decay32, norm, eps, torch.zeros(H, dk, dv, dtype=torch.float64))
+        close(gated[base:base + n], want, 2e-5 if dtype == torch.float32 else 1.5e-2, f"request {s}")
+        close(state[289 - s].transpose(1, 2), S, 2e-5, f"state of request {s}")
+        base += n
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
