@@ -52,14 +52,15 @@ static inline int skinny_blocks(int N, int rows) { return (N + rows - 1) / rows;
 // a full one (320 tiles on 256 units: two rounds for the work of 1.25). So a workgroup takes 8 to
 // `most` columns, not a whole number of tiles, such that the rounds are as few and as full as
 // possible: rounds * columns is what a unit streams. (The rows of a tile beyond the workgroup's
-// own are loaded again from its last row.) Of equal choices the largest: fewer workgroups read
-// the tokens.
+// own are loaded again from its last row.) A round costs its columns and what a workgroup costs whatever
+// its size (it reads the tokens, joins its waves' sums), about four columns more: without that, widths of
+// just over a full round fall to 4 columns a workgroup ([12480, 4096] at 8 rows: 51 us).
 static inline int pick_rows(int N, int most) {
     int rows = most;
     long best = -1;
     for (int p = most; p >= SK_MIN_ROWS; p -= 4) {
         const long wgs = (N + p - 1) / p;
-        const long cost = ((wgs + SK_COMPUTE_UNITS - 1) / SK_COMPUTE_UNITS) * p;
+        const long cost = ((wgs + SK_COMPUTE_UNITS - 1) / SK_COMPUTE_UNITS) * (p + 4);
         if (best < 0 || cost < best) {
             best = cost;
             rows = p;

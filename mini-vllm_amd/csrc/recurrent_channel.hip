@@ -83,6 +83,120 @@ channel_prepare_kernel(ChannelRows A, const T* __restrict__ conv_state, const in
     if (tid == 0) beta[(size_t)t * H + head] = sigmoid_f(to_f(packed[(size_t)t * A.ld + A.b_off + head]));
 }
 
+// The same for CP_ROWS neighbouring rows a workgroup and 2 to 4 taps: a thread's filter stays in registers, and a row's
+// input is read once for all the taps it falls under. The sums are those of the kernel above, term by term.
+#define CP_ROWS 8
+
+// silu(convolution) of channel c in rows t0 .. t0 + CP_ROWS - 1 (first[r]: row r's request's first row, -1 for a row
+// that does not count; hist[r]: the request's kept inputs)
+template <typename T, int TAPS>
+__device__ __forceinline__ void conv_rows(float (&x)[CP_ROWS], const ChannelRows& A, const T* __restrict__ conv_state,
+                                          const int (&first)[CP_ROWS], const int (&slot)[CP_ROWS], int t0, int n, int C, int c) {
+    const T* packed = (const T*)A.packed;
+    float w[TAPS], in[CP_ROWS + TAPS - 1];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = A.conv_w.at((size_t)c * TAPS + j);
+#pragma unroll
+    for (int i = 0; i < CP_ROWS + TAPS - 1; ++i) {
+        const int r = min(max(t0 - (TAPS - 1) + i, 0), n - 1);
+        in[i] = to_f(packed[(size_t)r * A.ld + c]);
+    }
+#pragma unroll
+    for (int r = 0; r < CP_ROWS; ++r) {
+        float acc = 0.f;
+        if (t0 + r - (TAPS - 1) >= first[r]) {
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) acc = fmaf(w[j], in[r + j], acc);
+        } else {
+            const T* hist = conv_state + (size_t)slot[r] * (TAPS - 1) * C;
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j)
+                acc = fmaf(w[j], conv_input(packed, A.ld, hist, C, TAPS, first[r], t0 + r - (TAPS - 1) + j, c), acc);
+        }
+        x[r] = silu_f(acc);
+    }
+}
+
+template <typename T, int TAPS>
+__global__ void __launch_bounds__(128)
+channel_prepare_rows_kernel(ChannelRows A, const T* __restrict__ conv_state, const int* __restrict__ token_seq,
+                            const int* __restrict__ cu_seqlens, const int* __restrict__ state_slots, int n, float* __restrict__ qk,
+                            float* __restrict__ vals, float* __restrict__ beta, float* __restrict__ z, long ldz) {
+    __shared__ float scratch[CP_ROWS][4];
+    const int t0 = blockIdx.x * CP_ROWS, unit = blockIdx.y, tid = threadIdx.x;
+    const int G = A.G, H = A.H, DK = A.DK, DV = A.DV;
+    const int C = 2 * G * DK + H * DV;
+    int first[CP_ROWS], slot[CP_ROWS];
+    bool live[CP_ROWS];
+#pragma unroll
+    for (int r = 0; r < CP_ROWS; ++r) {
+        // (a row that does not count is computed as if it were row 0's request's first row and not stored)
+        const int seq = t0 + r < n ? token_seq[t0 + r] : -1;
+        live[r] = seq >= 0;
+        first[r] = live[r] ? cu_seqlens[seq] : -TAPS;
+        slot[r] = live[r] ? state_slots[seq] : 0;
+    }
+    if (unit < G) {
+        float x[2][2][CP_ROWS];
+#pragma unroll
+        for (int which = 0; which < 2; ++which)
+#pragma unroll
+            for (int u = 0; u < 2; ++u) {
+                const int d = u * 128 + tid;
+                if (d < DK) conv_rows<T, TAPS>(x[which][u], A, conv_state, first, slot, t0, n, C, which * G * DK + unit * DK + d);
+                else
+#pragma unroll
+                    for (int r = 0; r < CP_ROWS; ++r) x[which][u][r] = 0.f;
+            }
+#pragma unroll
+        for (int r = 0; r < CP_ROWS; ++r) {
+            const float sq = wave_sum(fmaf(x[0][1][r], x[0][1][r], x[0][0][r] * x[0][0][r]));
+            const float sk = wave_sum(fmaf(x[1][1][r], x[1][1][r], x[1][0][r] * x[1][0][r]));
+            if (tid % MV_WAVE == 0) {
+                scratch[r][tid / MV_WAVE] = sq;
+                scratch[r][2 + tid / MV_WAVE] = sk;
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int r = 0; r < CP_ROWS; ++r) {
+            if (!live[r]) continue;
+            const float inv[2] = {(1.f / sqrtf((float)DK)) / sqrtf(scratch[r][0] + scratch[r][1] + A.unit_eps),
+                                  1.f / sqrtf(scratch[r][2] + scratch[r][3] + A.unit_eps)};
+            float* o = qk + ((size_t)(t0 + r) * G + unit) * 2 * DK;
+#pragma unroll
+            for (int which = 0; which < 2; ++which)
+#pragma unroll
+                for (int u = 0; u < 2; ++u) {
+                    const int d = u * 128 + tid;
+                    if (d < DK) o[which * DK + d] = x[which][u][r] * inv[which];
+                }
+        }
+        return;
+    }
+    const int head = unit - G;
+    for (int d = tid; d < DV; d += 128) {
+        float x[CP_ROWS];
+        conv_rows<T, TAPS>(x, A, conv_state, first, slot, t0, n, C, 2 * G * DK + head * DV + d);
+#pragma unroll
+        for (int r = 0; r < CP_ROWS; ++r)
+            if (live[r]) vals[((size_t)(t0 + r) * H + head) * DV + d] = x[r];
+    }
+    const float rate = -expf(A.a_log.at(head));
+    for (int d = tid; d < DK; d += 128) {
+        const float bias = A.dt_bias.at((size_t)head * DK + d);
+        float x[CP_ROWS];
+#pragma unroll
+        for (int r = 0; r < CP_ROWS; ++r) x[r] = live[r] ? z[(size_t)(t0 + r) * ldz + (size_t)head * DK + d] : 0.f;
+#pragma unroll
+        for (int r = 0; r < CP_ROWS; ++r)
+            if (live[r]) z[(size_t)(t0 + r) * ldz + (size_t)head * DK + d] = expf(rate * softplus_f(x[r] + bias));
+    }
+    const int row = t0 + tid;
+    if (tid < CP_ROWS && row < n && token_seq[row] >= 0)
+        beta[(size_t)row * H + head] = sigmoid_f(to_f(((const T*)A.packed)[(size_t)row * A.ld + A.b_off + head]));
+}
+
 static int channel_check(const char* what, const ChannelRows& A, int n, int n_seqs, const void* conv_state) {
     MV_REQUIRE(n >= 0 && n_seqs >= 0 && A.H > 0 && A.G > 0 && A.H % A.G == 0 && A.DK > 0 && A.DV > 0,
                "%s: bad sizes n=%d H=%d G=%d DK=%d DV=%d", what, n, A.H, A.G, A.DK, A.DV);
@@ -105,9 +219,24 @@ extern "C" int mv_channel_prepare(const void* packed, long ld, int n, int n_seqs
     if (int rc = channel_check("channel_prepare", A, n, n_seqs, conv_state)) return rc;
     MV_REQUIRE(token_seq && cu_seqlens && state_slots && qk && vals && beta && z && ldz >= (long)H * DK, "channel_prepare: missing operand");
     if (n == 0) return 0;
-    MV_DISPATCH_T(dtype, "channel_prepare",
-                  hipLaunchKernelGGL(channel_prepare_kernel<T>, dim3(n, G + H), dim3(128), 0, stream, A, (const T*)conv_state,
-                                     token_seq, cu_seqlens, state_slots, qk, vals, beta, z, ldz));
+#define CHANNEL_ROWS(TAPS)                                                                                                 \
+    MV_DISPATCH_T(dtype, "channel_prepare",                                                                               \
+                  hipLaunchKernelGGL((channel_prepare_rows_kernel<T, TAPS>), dim3((n + CP_ROWS - 1) / CP_ROWS, G + H), dim3(128), \
+                                     0, stream, A, (const T*)conv_state, token_seq, cu_seqlens, state_slots, n, qk, vals, beta, \
+                                     z, ldz))
+    // (few rows fill the chip only one a workgroup)
+    if (taps < 2 || taps > 4 || (long)n * (G + H) < 2L * CP_ROWS * mv_compute_units()) {
+        MV_DISPATCH_T(dtype, "channel_prepare",
+                      hipLaunchKernelGGL(channel_prepare_kernel<T>, dim3(n, G + H), dim3(128), 0, stream, A, (const T*)conv_state,
+                                         token_seq, cu_seqlens, state_slots, qk, vals, beta, z, ldz));
+    } else if (taps == 2) {
+        CHANNEL_ROWS(2);
+    } else if (taps == 3) {
+        CHANNEL_ROWS(3);
+    } else {
+        CHANNEL_ROWS(4);
+    }
+#undef CHANNEL_ROWS
     if (mv_check_launch("channel_prepare")) return 1;
     if (taps > 1 && n_seqs > 0) {
         const int C = 2 * G * DK + H * DV;

@@ -87,7 +87,7 @@ KERNELS_OF: Dict[str, Tuple[str, Optional[str], int]] = {
     "mv_constant_step": (r"\bconstant_step_kernel", None, 1),
     "mv_pair_norm_add_norm": (r"\bpair_norm_add_norm_kernel", None, 1),
     "mv_stream_entry": (r"\bstream_entry_kernel", None, 1),
-    "mv_channel_prepare": (r"\bchannel_prepare_kernel", r"\bconv_state_kernel", 2),
+    "mv_channel_prepare": (r"\bchannel_prepare(_rows)?_kernel", r"\bconv_state_kernel", 2),
     "mv_channel_scan": (r"\bchannel_scan_kernel", None, 1),
     "mv_channel_step": (r"\bchannel_step_kernel", r"\bconv_state_kernel", 2),
 }

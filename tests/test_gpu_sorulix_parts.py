@@ -479,6 +479,16 @@ def test_channel_delta_step(dtype, H, G, dk, dv, taps, ra, rg, q_lens):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H, G, dk, dv, taps, q_lens", [(4, 4, 8, 12, 4, [513, 2, 1, 37]), (6, 2, 20, 10, 3, [3, 1, 5, 520]),
+                                                       (5, 5, 10, 160, 2, [2, 450, 6, 1]), (2, 2, 140, 6, 4, [700, 1, 2, 341])])
+def test_channel_delta_steps_of_many_rows(dtype, H, G, dk, dv, taps, q_lens):
+    """Steps large enough for the kernel that prepares several rows a workgroup: requests that begin anywhere in such a run
+    of rows, portions shorter than the filter, padding rows behind the last."""
+    assert (sum(q_lens) + 2) * (G + H) >= 2 * 8 * 256
+    test_channel_delta_step(dtype, H, G, dk, dv, taps, 7, 9, q_lens)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("G", [4, 2])
 def test_channel_delta_portions(dtype, G):
     """260 tokens whole, in portions down to two tokens, and token by token: the same rows, within rounding."""
