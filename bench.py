@@ -51,6 +51,10 @@ attention beside linear attention with constant decays alternating with layers o
 feed-forward the clamped gated pair at the shape's dense width; with ``--loops`` above 1 the middle half of the layers
 runs that many times). Its dense sizes are those of Qwen3 of the same shape, so the two can be read side by side.
 
+``--design setirax`` does the same for a Setirax model of the named shape's sizes (``setirax_shape``: attention over a
+latent, softmax attention on convolved projections beside gated linear attention, and the real-gated linear recurrent unit
+take turns, the softmax mixers see ``--window`` positions, every feed-forward has as many weights as the shape's).
+
 Weights are seeded random tensors of the named shape and prompts are seeded uniform token ids
 (there is no network for checkpoints or datasets). The reference publishes no number for this
 metric, so ``vs_baseline`` is null.
@@ -109,6 +113,9 @@ def build_llm(args, shape, layers, max_seqs=None, token_budget=None, num_pages=N
     elif getattr(args, "design", "qwen3") == "sorulix":
         from minivllm_amd.config.shapes import sorulix_shape
         raw = dict(sorulix_shape(args.shape, layers, loops=args.loops), torch_dtype=args.dtype)
+    elif getattr(args, "design", "qwen3") == "setirax":
+        from minivllm_amd.config.shapes import setirax_shape
+        raw = dict(setirax_shape(args.shape, layers, window=args.window), torch_dtype=args.dtype)
     else:
         raw = dict(shape, architectures=["Qwen3ForCausalLM"], num_hidden_layers=layers,
                    max_position_embeddings=40960, torch_dtype=args.dtype)
@@ -677,6 +684,80 @@ def bench_sorulix(args, llm, cfg, layers, layers_full, item) -> int:
     return 0
 
 
+def setirax_numbers(llm, cfg):
+    """From the loaded model: elements of all tensors; of the matrices a token multiplies with and of the weights a decode step
+    reads, a layer that runs several times counted each time; bytes of state of one request; per call with a cache: its window
+    (None: all keys), cache elements a token takes, multiply-adds of a (query, key) pair."""
+    from minivllm_amd.models.causal_lm import expected_tensors
+    ex = llm.executor
+    decls = expected_tensors(ex.arch, cfg, ex.plan)
+    runs = {}
+    for i in range(len(cfg.layers)):
+        runs[cfg.owner_of(i)] = runs.get(cfg.owner_of(i), 0) + 1
+    sizes = {n: (_numel(d.shape), len(d.shape)) for n, d in decls.items()}
+    times = lambda n: runs[int(n[1:].split(".")[0])] if n[0] == "l" and n[1].isdigit() else 1
+    params = sum(k for k, _ in sizes.values())
+    matrices = sum(k * times(n) for n, (k, dims) in sizes.items() if dims >= 2 and n != "embed" and not n.endswith((".conv", ".b")))
+    read = sum(k * times(n) for n, (k, _) in sizes.items())
+    state = sum(t[0].numel() * t.element_size() for ts in ex.state_tensors.values() for t in ts.values())
+    attn = []
+    for l in cfg.layers:
+        if l.left is not None:
+            attn.append((l.left.window, l.left.kv_heads * (l.left.dim + l.left.vdim), l.left.heads * (l.left.dim + l.left.vdim)))
+        elif l.latent is not None:
+            # (attention runs in the latent's space: a score and a weighted sum of kv_rank numbers each)
+            attn.append((l.latent.window, l.latent.kv_rank, 2 * l.latent.heads * l.latent.kv_rank))
+    return dict(params=params, matrices=matrices, read=read, state=state, attn=attn)
+
+
+def bench_setirax(args, llm, cfg, layers, layers_full, item) -> int:
+    """The default measurements for a Setirax model of the named shape; the same fields in the line."""
+    nums = setirax_numbers(llm, cfg)
+    prefill = None
+    if args.only in ("all", "prefill"):
+        prefill_s = measure_prefill(llm, cfg.vocab_size, args.prefill_tokens, repeats=3, seed=args.seed)
+        T = args.prefill_tokens
+        # the matrices, the softmax mixers' visible pairs, the state updates (written and read once a token), the head
+        flops = 2 * T * nums["matrices"] + T * nums["state"] + 2 * cfg.vocab_size * cfg.hidden_size
+        for window, _, pair in nums["attn"]:
+            flops += 2 * pair * _visible_pairs(T, T if window is None else window, 0)
+        prefill = {"value": round(T / prefill_s, 1), "tokens": T, "ms": round(prefill_s * 1e3, 3),
+                   "frac": round(flops / prefill_s / PEAK_FLOPS[args.dtype], 4)}
+    tok_s = ms_step = roofline = None
+    ran = regions = 0
+    if args.only in ("all", "decode"):
+        tok_s, ms_step, mean_ctx, ran, regions = measure_decode(llm, cfg.vocab_size, args.batch, args.prompt_len,
+                                                                args.steps, args.warmup, args.seed)
+        # every weight once for each time its layer runs, the keys each request's query sees, its states read and written
+        seen = sum(cache * (mean_ctx if window is None else min(mean_ctx, window)) for window, cache, _ in nums["attn"])
+        step_bytes = nums["read"] * item + args.batch * (seen * item + 2 * nums["state"])
+        achieved = step_bytes / (ms_step * 1e-3) / 1e9
+        roofline = {"bound": "hbm", "achieved": round(achieved, 1), "peak": PEAK_HBM_GBS, "unit": "GB/s",
+                    "frac": round(achieved / PEAK_HBM_GBS, 4)}
+    points = {}
+    if not args.no_points and args.only == "all":
+        for b, key in ((1, "decode_b1"), (64, "decode_b64")):
+            n = min(args.steps, 128)
+            points[key] = round(measure_decode(llm, cfg.vocab_size, b, args.prompt_len, n, min(args.warmup, 8),
+                                               args.seed + b)[0], 1)
+    kinds = [l.type for l in cfg.layers]
+    config = {"model": f"setirax-{args.shape}-shape-random", "layers": layers, "layers_full": layers_full,
+              "hidden": cfg.hidden_size, "vocab": cfg.vocab_size, "window": args.window,
+              **{f"{kind}_layers": kinds.count(kind) for kind in ("latent_attention", "parallel", "rglru")},
+              "weights": nums["params"], "global_batch": args.batch,
+              "seq_len": args.context, "prompt_len": args.prompt_len, "block_size": args.block_size, "graph": not args.no_graph,
+              "scheduler_steps": args.scheduler_steps, "launch_ahead": bool(llm.config.launch_ahead),
+              "parallelism": "single-gpu"}
+    print(json.dumps({"metric": "decode tok/s (batch %d, %d-token prompts)" % (args.batch, args.prompt_len),
+                      "value": round(tok_s, 1) if tok_s is not None else None, "unit": "tokens/s", "n_gpus": 1,
+                      "steps": ran if ran else args.steps, "warmup": args.warmup,
+                      "ms_per_step": round(ms_step, 4) if ms_step is not None else None, "higher_is_better": True,
+                      "scaling": "weak", "vs_baseline": None, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+                      "data": "synthetic", "config": config, "timed_regions": regions, "prefill": prefill,
+                      "roofline": roofline, "points": points}))
+    return 0
+
+
 def main() -> int:
     ap = argparse.ArgumentParser(description=__doc__, formatter_class=argparse.RawDescriptionHelpFormatter)
     ap.add_argument("--gpus", type=int, default=1)
@@ -685,7 +766,7 @@ def main() -> int:
     ap.add_argument("--shape", choices=sorted(SHAPES), default="0.6b")
     ap.add_argument("--experts", type=int, default=32, help="--design dutilix: experts of each mixture layer")
     ap.add_argument("--top", type=int, default=4, help="--design dutilix: experts a token uses (each 1/top of the dense width)")
-    ap.add_argument("--window", type=int, default=1024, help="--design zedudra: positions a query sees behind it (itself among them)")
+    ap.add_argument("--window", type=int, default=1024, help="--design zedudra, setirax: positions a query sees behind it (itself among them)")
     ap.add_argument("--keep-first", type=int, default=64, help="--design zedudra: first positions every query keeps seeing")
     ap.add_argument("--dense-every", type=int, default=2,
                     help="--design zedudra: every n-th feed-forward is dense, the others are routed (1: all dense; a number "
@@ -695,7 +776,7 @@ def main() -> int:
                     help="--design furanex: every n-th layer attends over a latent, the others are grouped attention (a number "
                          "above the layer count: grouped attention everywhere)")
     ap.add_argument("--loops", type=int, default=1, help="--design sorulix: times the middle half of the layers runs")
-    ap.add_argument("--design", choices=["qwen3", "bolapel", "dutilix", "zedudra", "furanex", "sorulix"], default="qwen3",
+    ap.add_argument("--design", choices=["qwen3", "bolapel", "dutilix", "zedudra", "furanex", "sorulix", "setirax"], default="qwen3",
                     help="'bolapel': the same widths, head counts, vocabulary and number of layers as the named Qwen3 "
                          "shape, as a Bolapel model (three delta-rule layers to one attention layer in chunks of --chunk "
                          "tokens); decode and prefill are measured the same way and the line names the design")
@@ -804,6 +885,8 @@ def main() -> int:
         return bench_furanex(args, llm, cfg, layers, layers_full, item)
     if args.design == "sorulix":
         return bench_sorulix(args, llm, cfg, layers, layers_full, item)
+    if args.design == "setirax":
+        return bench_setirax(args, llm, cfg, layers, layers_full, item)
     nums = model_numbers(shape, layers)
 
     prefill = None

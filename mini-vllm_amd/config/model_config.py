@@ -1513,3 +1513,310 @@ class SorulixConfig(ModelConfig):
         if self.max_position_embeddings != (1 << 24):
             d["max_position_embeddings"] = self.max_position_embeddings
         return d
+
+
+# ---------------------------------------------------------------------------------------
+# Setirax
+# ---------------------------------------------------------------------------------------
+@dataclass(frozen=True)
+class SetiraxAttention:
+    """The softmax side of a "parallel" layer. ``conv``: taps of the convolution behind q, k and v; ``window`` counts the
+    query's own position (None: all keys); ``rot_dims`` 0: no rotation; ``rot_scaling`` = (factor, low, high, original)."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    conv: int = UNSTATED
+    softcap: Optional[float] = None
+    window: Optional[int] = None
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    rot_scaling: Optional[Tuple[float, float, float, float]] = None
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+                             "conv": self.conv, "softcap": self.softcap,
+                             "mask": None if self.window is None else {"size": self.window}}
+        if self.rot_dims:
+            d["rot"] = {"dims": self.rot_dims, "base": self.rot_base}
+            if self.rot_scaling is not None:
+                d["rot"]["scaling"] = dict(zip(("factor", "low", "high", "original"), self.rot_scaling))
+        return {k: v for k, v in d.items() if v is not None and v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SetiraxLinear:
+    """The linear-attention side of a "parallel" layer. ``rank``: width between the decay's two matrices (the stored tensors
+    state it; config.json may leave it out)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    rank: int = UNSTATED
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "tau": self.tau, "rank": self.rank}
+        return {k: v for k, v in d.items() if v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SetiraxUnit:
+    """An "rglru" mixer: ``width`` channels in ``blocks`` parts, ``conv`` taps."""
+    width: int
+    blocks: int
+    conv: int
+
+    def to_dict(self) -> Dict[str, Any]:
+        return {k: v for k, v in (("width", self.width), ("blocks", self.blocks), ("conv", self.conv)) if v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SetiraxLatent:
+    """A "latent_attention" mixer; ``window`` counts the query's own position (None: all keys)."""
+    heads: int
+    dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: Optional[int] = None
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {"heads": self.heads, "dim": self.dim, "vdim": self.vdim, "kv_rank": self.kv_rank, "scale": self.scale,
+                             "mask": None if self.window is None else {"size": self.window}}
+        return {k: v for k, v in d.items() if v is not None and v != UNSTATED}
+
+
+@dataclass(frozen=True)
+class SetiraxLayer:
+    """``left``, ``right`` and their scales for a "parallel" layer, ``unit`` for an "rglru" layer, ``latent`` for a
+    "latent_attention" layer. ``ff`` is the width of the feed-forward, None for a layer without one. ``weights_of``: the layer
+    whose tensors this one uses."""
+    type: str
+    left: Optional[SetiraxAttention] = None
+    right: Optional[SetiraxLinear] = None
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+    unit: Optional[SetiraxUnit] = None
+    latent: Optional[SetiraxLatent] = None
+    ff: Optional[int] = None
+    weights_of: Optional[int] = None
+
+    def to_dict(self) -> Dict[str, Any]:
+        if self.type == "parallel":
+            mixer: Dict[str, Any] = {"left": self.left.to_dict(), "right": self.right.to_dict(), "left_scale": self.left_scale,
+                                     "right_scale": self.right_scale}
+        else:
+            mixer = (self.unit if self.type == "rglru" else self.latent).to_dict()
+        d = {"type": self.type, "mixer": mixer,
+             "mlp": None if self.ff is None else {k: v for k, v in (("kind", "dense"), ("ff", self.ff)) if v != UNSTATED}}
+        if self.weights_of is not None:
+            d["weights_of"] = self.weights_of
+        return d
+
+
+@dataclass(frozen=True)
+class SetiraxConfig(ModelConfig):
+    """Setirax: a decoder with norms behind its sublayers only, whose ``layers`` are listed one by one; each has a mixer
+    (``type``: "parallel", softmax attention beside gated linear attention; "rglru", the real-gated linear recurrent unit;
+    "latent_attention") and a feed-forward with squared ReLU or none, and may use another layer's tensors (``weights_of``).
+    The output head is the embedding's table, its logits are capped. Keys: ``vocab``, ``width``, ``layers``, ``norm.eps``,
+    ``logit_softcap``. Sizes that config.json leaves out are UNSTATED until ``completed`` fills them in from the stored
+    tensors' shapes."""
+
+    architecture: ClassVar[str] = "Setirax"
+
+    vocab_size: int = UNSTATED
+    hidden_size: int = UNSTATED
+    layers: Tuple[SetiraxLayer, ...] = ()
+    norm_eps: float = 1e-6
+    logit_softcap: Optional[float] = None
+    max_position_embeddings: int = 1 << 24
+    dtype: str = "bfloat16"
+    eos_token_ids: Tuple[int, ...] = ()
+
+    @staticmethod
+    def _window(m: Dict[str, Any], mw: str) -> Optional[int]:
+        mask = _section(m, "mask", mw, optional=True)
+        return None if mask is None else _require(mask, "size", int, mw + ".mask")
+
+    @classmethod
+    def _left(cls, m: Dict[str, Any], mw: str) -> SetiraxAttention:
+        cap = m.get("softcap")
+        rot = _section(m, "rot", mw, optional=True)
+        dims, base, scaling = 0, 10000.0, None
+        if rot is not None:
+            rw = mw + ".rot"
+            dims, base = _require(rot, "dims", int, rw), _require(rot, "base", float, rw)
+            sc = _section(rot, "scaling", rw, optional=True)
+            if sc is not None:
+                scaling = tuple(_require(sc, key, float, rw + ".scaling") for key in ("factor", "low", "high", "original"))
+        return SetiraxAttention(heads=_require(m, "heads", int, mw), kv_heads=_size(m, "kv_heads", mw), dim=_size(m, "dim", mw),
+                                vdim=_size(m, "vdim", mw), scale=_require(m, "scale", float, mw), conv=_size(m, "conv", mw),
+                                softcap=None if cap is None else _typed(cap, "softcap", float, mw), window=cls._window(m, mw),
+                                rot_dims=dims, rot_base=base, rot_scaling=scaling)
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any], where: str = "config.json") -> "SetiraxConfig":
+        raw_layers = d.get("layers")
+        if not isinstance(raw_layers, (list, tuple)) or not raw_layers:
+            raise ConfigError(f"{where}: 'layers' must be a non-empty list")
+        layers = []
+        for i, entry in enumerate(raw_layers):
+            lw = f"{where}: layers[{i}]"
+            if not isinstance(entry, dict):
+                raise ConfigError(f"{lw} must be an object")
+            kind = entry.get("type")
+            m, mw = _section(entry, "mixer", lw), lw + ".mixer"
+            parts: Dict[str, Any] = {}
+            if kind == "parallel":
+                parts["left"] = cls._left(_section(m, "left", mw), mw + ".left")
+                r, rw = _section(m, "right", mw), mw + ".right"
+                parts["right"] = SetiraxLinear(heads=_require(r, "heads", int, rw), dim=_size(r, "dim", rw), vdim=_size(r, "vdim", rw),
+                                               tau=_require(r, "tau", float, rw), rank=_size(r, "rank", rw))
+                for key in ("left_scale", "right_scale"):
+                    parts[key] = _require(m, key, float, mw)
+            elif kind == "rglru":
+                parts["unit"] = SetiraxUnit(width=_size(m, "width", mw), blocks=_size(m, "blocks", mw), conv=_size(m, "conv", mw))
+            elif kind == "latent_attention":
+                parts["latent"] = SetiraxLatent(heads=_require(m, "heads", int, mw), dim=_size(m, "dim", mw), vdim=_size(m, "vdim", mw),
+                                                kv_rank=_size(m, "kv_rank", mw), scale=_require(m, "scale", float, mw),
+                                                window=cls._window(m, mw))
+            else:
+                raise ConfigError(f"{lw}: layer type {kind!r} is not supported (parallel, rglru, latent_attention)")
+            mlp = _section(entry, "mlp", lw, optional=True)
+            if mlp is not None:
+                if mlp.get("kind", "dense") != "dense":
+                    raise ConfigError(f"{lw}.mlp: kind {mlp.get('kind')!r} is not supported (dense)")
+                parts["ff"] = _size(mlp, "ff", lw + ".mlp")
+            shared = entry.get("weights_of")
+            layers.append(SetiraxLayer(type=kind, weights_of=None if shared is None else _typed(shared, "weights_of", int, lw), **parts))
+        dtype = d.get("dtype", d.get("torch_dtype", "bfloat16")) or "bfloat16"
+        if str(dtype) not in _DTYPE_NAMES:
+            raise ConfigError(f"{where}: unknown dtype {dtype!r}")
+        eos = d.get("eos_token_id")
+        eos_ids: Tuple[int, ...] = ()
+        if isinstance(eos, int) and not isinstance(eos, bool):
+            eos_ids = (eos,)
+        elif isinstance(eos, (list, tuple)) and all(isinstance(e, int) for e in eos):
+            eos_ids = tuple(eos)
+        elif eos is not None:
+            raise ConfigError(f"{where}: eos_token_id must be an integer or a list of integers, got {eos!r}")
+        max_pos, cap = d.get("max_position_embeddings"), d.get("logit_softcap")
+        cfg = cls(
+            vocab_size=_size(d, "vocab", where), hidden_size=_size(d, "width", where), layers=tuple(layers),
+            norm_eps=_require(_section(d, "norm", where), "eps", float, where + ".norm"),
+            logit_softcap=None if cap is None else _typed(cap, "logit_softcap", float, where),
+            max_position_embeddings=(1 << 24) if max_pos is None else _typed(max_pos, "max_position_embeddings", int, where),
+            dtype=_DTYPE_NAMES[str(dtype)],
+            eos_token_ids=eos_ids,
+        )
+        cfg.validate(where)
+        return cfg
+
+    def owner_of(self, i: int, where: str = "layers") -> int:
+        """The layer whose tensors layer ``i`` uses: itself, or the end of its chain of ``weights_of``."""
+        seen = {i}
+        while self.layers[i].weights_of is not None:
+            j = self.layers[i].weights_of
+            if not (0 <= j < len(self.layers)) or j in seen:
+                raise ConfigError(f"{where}: weights_of {j} must name another layer of the model, and the chain must end "
+                                  f"at a layer with tensors of its own")
+            seen.add(j)
+            i = j
+        return i
+
+    def completed(self, sizes=None, where: str = "config") -> "SetiraxConfig":
+        """The configuration with nothing UNSTATED. ``sizes(name) -> shape or None`` looks a stored tensor's shape up."""
+        import dataclasses
+        sizes = sizes or (lambda name: None)
+
+        def need(value: int, name: str, axis: int, what: str, per: int = 1) -> int:
+            if value != UNSTATED:
+                return value
+            shape = sizes(name)
+            if shape is not None and len(shape) > axis and shape[axis] % per == 0:
+                return int(shape[axis]) // per
+            raise ConfigError(f"{where}: {what} is stated neither in config.json nor by a stored tensor's shape")
+
+        layers = []
+        for i, l in enumerate(self.layers):
+            owner = self.owner_of(i)
+            p, lw = f"l{owner}.mix.", f"layers[{i}]"
+            if l.type == "parallel":
+                a, b = l.left, l.right
+                dim = need(a.dim, p + "left.q", 0, lw + ".left.dim", a.heads)
+                kv = need(a.kv_heads, p + "left.k", 0, lw + ".left.kv_heads", dim)
+                a = dataclasses.replace(a, dim=dim, kv_heads=kv, vdim=need(a.vdim, p + "left.v", 0, lw + ".left.vdim", kv),
+                                        conv=need(a.conv, p + "left.q.conv", 1, lw + ".left.conv"))
+                b = dataclasses.replace(b, dim=need(b.dim, p + "right.q", 0, lw + ".right.dim", b.heads),
+                                        vdim=need(b.vdim, p + "right.v", 0, lw + ".right.vdim", b.heads),
+                                        rank=need(b.rank, p + "right.a1", 0, lw + ".right.rank"))
+                l = dataclasses.replace(l, left=a, right=b)
+            elif l.type == "rglru":
+                l = dataclasses.replace(l, unit=SetiraxUnit(
+                    width=need(l.unit.width, p + "lam", 0, lw + ".width"), blocks=need(l.unit.blocks, p + "ra", 0, lw + ".blocks"),
+                    conv=need(l.unit.conv, p + "conv", 1, lw + ".conv")))
+            else:
+                c = l.latent
+                l = dataclasses.replace(l, latent=dataclasses.replace(
+                    c, dim=need(c.dim, p + "q", 0, lw + ".dim", c.heads), vdim=need(c.vdim, p + "uv", 0, lw + ".vdim", c.heads),
+                    kv_rank=need(c.kv_rank, p + "dkv", 0, lw + ".kv_rank")))
+            if l.ff is not None:
+                l = dataclasses.replace(l, ff=need(l.ff, f"l{owner}.mlp.up", 0, lw + ".mlp.ff"))
+            layers.append(l)
+        done = dataclasses.replace(self, vocab_size=need(self.vocab_size, "embed", 0, "vocab"),
+                                   hidden_size=need(self.hidden_size, "embed", 1, "width"), layers=tuple(layers))
+        done.validate(where)
+        return done
+
+    def validate(self, where: str = "config") -> None:
+        import dataclasses
+        positive = lambda *values: all(v == UNSTATED or v > 0 for v in values)
+        if not positive(self.vocab_size, self.hidden_size):
+            raise ConfigError(f"{where}: vocab and width must be positive")
+        if self.norm_eps <= 0 or (self.logit_softcap is not None and not self.logit_softcap > 0):
+            raise ConfigError(f"{where}: norm.eps and logit_softcap must be positive")
+        for i, l in enumerate(self.layers):
+            lw = f"{where}: layers[{i}]"
+            a, b, u, c = l.left, l.right, l.unit, l.latent
+            if a is not None:
+                if not positive(a.heads, a.kv_heads, a.dim, a.vdim, a.conv) or (a.kv_heads != UNSTATED and a.heads % a.kv_heads):
+                    raise ConfigError(f"{lw}: sizes must be positive, and {a.heads} heads a multiple of {a.kv_heads} kv_heads")
+                if not a.scale > 0 or (a.softcap is not None and not a.softcap > 0):
+                    raise ConfigError(f"{lw}: scale and softcap must be positive")
+                if a.rot_dims < 0 or a.rot_dims % 2 or (a.dim != UNSTATED and a.rot_dims > a.dim) or not a.rot_base > 0:
+                    raise ConfigError(f"{lw}: rot.dims {a.rot_dims} must be even and at most dim {a.dim}, rot.base positive")
+                if a.rot_scaling is not None:
+                    factor, low, high, original = a.rot_scaling
+                    if not (factor > 0 and original > 0 and 0 < low <= high):
+                        raise ConfigError(f"{lw}: rot.scaling needs a positive factor and original, and 0 < low <= high")
+            if b is not None and (not positive(b.heads, b.dim, b.vdim, b.rank) or not b.tau > 0):
+                raise ConfigError(f"{lw}: the linear side needs positive sizes and a positive tau")
+            if u is not None and (not positive(u.width, u.blocks, u.conv) or (UNSTATED not in (u.width, u.blocks) and u.width % u.blocks)):
+                raise ConfigError(f"{lw}: width {u.width} must form {u.blocks} equal blocks, with at least one tap")
+            if c is not None and (not positive(c.heads, c.dim, c.vdim, c.kv_rank) or not c.scale > 0):
+                raise ConfigError(f"{lw}: sizes and scale must be positive")
+            for window in (None if a is None else a.window, None if c is None else c.window):
+                if window is not None and window < 1:
+                    raise ConfigError(f"{lw}: mask.size counts the query's own position, so it is >= 1, got {window}")
+            if l.ff is not None and not positive(l.ff):
+                raise ConfigError(f"{lw}: the feed-forward's width must be positive")
+            if l.weights_of is not None:
+                j = self.owner_of(i, lw)
+                if dataclasses.replace(self.layers[j], weights_of=None) != dataclasses.replace(l, weights_of=None):
+                    raise ConfigError(f"{lw}: weights_of {j} names a layer with other sizes or constants than this one")
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {"architecture": self.architecture, "layers": [l.to_dict() for l in self.layers],
+                             "norm": {"eps": self.norm_eps}, "torch_dtype": self.dtype}
+        for key, value in (("vocab", self.vocab_size), ("width", self.hidden_size)):
+            if value != UNSTATED:
+                d[key] = value
+        if self.logit_softcap is not None:
+            d["logit_softcap"] = self.logit_softcap
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids) if len(self.eos_token_ids) > 1 else self.eos_token_ids[0]
+        if self.max_position_embeddings != (1 << 24):
+            d["max_position_embeddings"] = self.max_position_embeddings
+        return d

@@ -31,6 +31,7 @@ def named_shapes() -> Dict[str, Dict[str, Any]]:
     shapes["zedudra-tiny"] = zedudra_tiny_shape()
     shapes["furanex-tiny"] = furanex_tiny_shape()
     shapes["sorulix-tiny"] = sorulix_tiny_shape()
+    shapes["setirax-tiny"] = setirax_tiny_shape()
     for name in QWEN3_SHAPES:
         if name != "tiny":
             shapes[f"bolapel-{name}"] = bolapel_shape(name)
@@ -38,6 +39,7 @@ def named_shapes() -> Dict[str, Dict[str, Any]]:
             shapes[f"zedudra-{name}"] = zedudra_shape(name)
             shapes[f"furanex-{name}"] = furanex_shape(name)
             shapes[f"sorulix-{name}"] = sorulix_shape(name)
+            shapes[f"setirax-{name}"] = setirax_shape(name)
     return shapes
 
 
@@ -258,3 +260,47 @@ def sorulix_tiny_shape() -> Dict[str, Any]:
             "layers": [{"type": "channel_delta", "mixer": dict(delta), "mlp": None},
                        {"type": "parallel", "mixer": parallel, "mlp": dict(mlp)},
                        {"type": "channel_delta", "mixer": dict(delta, kv_heads=4), "mlp": dict(mlp)}]}
+
+
+def setirax_shape(name: str, layers: int = None, window: int = 1024, kv_rank: int = 256, state_head_dim: int = 64, conv: int = 4,
+                  tau: float = 16.0, softcap: float = 50.0) -> Dict[str, Any]:
+    """A Setirax configuration with the width, vocabulary, head counts, head size and number of layers of the named Qwen3
+    shape: attention over a latent of ``kv_rank`` numbers, softmax attention beside gated linear attention with heads of
+    ``state_head_dim``, and the real-gated linear recurrent unit (as wide as the model, a block for each attention head) take
+    turns; the softmax mixers see ``window`` positions; every feed-forward is half as wide again as the shape's gated one, so
+    that it has as many weights. For random-weights models at sizes that resemble a real model's layers."""
+    q = QWEN3_SHAPES[name]
+    n = layers or q["num_hidden_layers"]
+    hid, hd, heads = q["hidden_size"], q["head_dim"], q["num_attention_heads"]
+    state_heads = hid // state_head_dim
+    mask = {"size": window}
+    scaling = {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}
+    mixers = {
+        "latent_attention": {"heads": heads, "dim": hd, "vdim": hd, "kv_rank": kv_rank, "scale": hd ** -0.5, "mask": dict(mask)},
+        "parallel": {"left": {"heads": heads, "kv_heads": q["num_key_value_heads"], "dim": hd, "vdim": hd, "scale": hd ** -0.5,
+                              "conv": conv, "softcap": softcap, "mask": dict(mask),
+                              "rot": {"dims": hd, "base": q["rope_theta"], "scaling": scaling}},
+                     "right": {"heads": state_heads, "dim": state_head_dim, "vdim": state_head_dim, "tau": tau, "rank": 16},
+                     "left_scale": 0.7, "right_scale": 0.7},
+        "rglru": {"width": hid, "blocks": heads, "conv": conv},
+    }
+    kinds = list(mixers)
+    out = [{"type": kinds[i % 3], "mixer": mixers[kinds[i % 3]], "mlp": {"kind": "dense", "ff": q["intermediate_size"] * 3 // 2}}
+           for i in range(n)]
+    return {"architecture": "Setirax", "vocab": q["vocab_size"], "width": hid, "layers": out, "norm": {"eps": q["rms_norm_eps"]},
+            "logit_softcap": 30.0}
+
+
+def setirax_tiny_shape() -> Dict[str, Any]:
+    """A Setirax model of a few thousand weights: every kind of layer, one without a feed-forward, one that runs another's
+    tensors again."""
+    mlp = {"kind": "dense", "ff": 88}
+    parallel = {"left": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "scale": 0.3, "conv": 3, "softcap": 12.0, "mask": {"size": 20},
+                         "rot": {"dims": 8, "base": 5000.0, "scaling": {"factor": 4.0, "low": 1.0, "high": 3.0, "original": 64}}},
+                "right": {"heads": 3, "dim": 12, "vdim": 8, "tau": 8.0, "rank": 6}, "left_scale": 0.8, "right_scale": 0.5}
+    latent = {"heads": 3, "dim": 12, "vdim": 20, "kv_rank": 24, "scale": 0.25, "mask": {"size": 13}}
+    return {"architecture": "Setirax", "vocab": 256, "width": 64, "norm": {"eps": 1e-5}, "logit_softcap": 15.0,
+            "layers": [{"type": "rglru", "mixer": {"width": 48, "blocks": 3, "conv": 4}, "mlp": None},
+                       {"type": "parallel", "mixer": parallel, "mlp": dict(mlp)},
+                       {"type": "latent_attention", "mixer": latent, "mlp": dict(mlp)},
+                       {"type": "parallel", "mixer": parallel, "mlp": dict(mlp), "weights_of": 1}]}

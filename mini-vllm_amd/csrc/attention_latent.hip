@@ -9,12 +9,14 @@
 //                        the way; weighted latents into values, times the output gate)
 //     attention_latent   softmax attention with one shared key row of R + DR numbers whose first R
 //                        are also the value
+// A query may see only a window (the keys from `window` positions behind it on; < 0: all), and the softmax's denominator may
+// have one more term e^sink[h] (a float per head, not scaled; null: none).
 // Page layout: rows[page][slot][R + DR] in the activation type, and the latents once more with a page's slots side
 // by side, [page][R][slot], which is how the MFMA kernel's second product wants them. Scores, weights and sums are float.
 #include "dispatch.h"
 
 // ---------------------------------------------------------------------------------------
-// Prepare. Packed rows: [dq (QR) | dkv (R + DR) | ...]. One workgroup per row:
+// Prepare. Packed rows: [dq (QR, may be 0: no query latent) | dkv (R + DR) | ...]. One workgroup per row:
 //   cq[t]           = dq / rms(dq) * wq                      (the query's latent, activation type)
 //   page row of t   = [dkv[:R] / rms(dkv[:R]) * wkv | rot(dkv[R:], position)]
 // rot pairs channel i with i + DR/2; table[p] = [cos (DR/2) | sin (DR/2)] of position p.
@@ -34,14 +36,16 @@ latent_prepare_kernel(const T* __restrict__ packed, long ld, int QR, int R, int 
         return;
     }
     const T* p = packed + (size_t)t * ld;
-    float ss = 0.f;
-    for (int c = tid; c < QR; c += 256) {
-        const float x = to_f(p[c]);
-        ss = fmaf(x, x, ss);
+    float ss = 0.f, inv;
+    if (QR > 0) {
+        for (int c = tid; c < QR; c += 256) {
+            const float x = to_f(p[c]);
+            ss = fmaf(x, x, ss);
+        }
+        ss = block_sum(ss, scratch);
+        inv = 1.f / sqrtf(ss / (float)QR + eps);
+        for (int c = tid; c < QR; c += 256) qo[c] = from_f<T>(to_f(p[c]) * inv * wq.at(c));
     }
-    ss = block_sum(ss, scratch);
-    float inv = 1.f / sqrtf(ss / (float)QR + eps);
-    for (int c = tid; c < QR; c += 256) qo[c] = from_f<T>(to_f(p[c]) * inv * wq.at(c));
     const T* kv = p + QR;
     ss = 0.f;
     for (int c = tid; c < R; c += 256) {
@@ -74,10 +78,10 @@ extern "C" int mv_latent_prepare(const void* packed, long ld, int n, int QR, int
                                  int weight_dtype, float eps, const float* table, int table_rows, const int* positions,
                                  const int* token_seq, const int* block_table, int bt_width, int page_size, void* cq,
                                  long ldq, void* pages, void* pages_t, int dtype, hipStream_t stream) {
-    MV_REQUIRE(n >= 0 && QR > 0 && R > 0 && DR >= 0 && DR % 2 == 0, "latent_prepare: bad sizes n=%d QR=%d R=%d DR=%d", n, QR, R, DR);
+    MV_REQUIRE(n >= 0 && QR >= 0 && R > 0 && DR >= 0 && DR % 2 == 0, "latent_prepare: bad sizes n=%d QR=%d R=%d DR=%d", n, QR, R, DR);
     MV_REQUIRE(ld >= (long)QR + R + DR && ldq >= QR && page_size > 0 && bt_width > 0, "latent_prepare: row pitches too small");
-    MV_REQUIRE(mv_valid_dtype(weight_dtype) && packed && wq && wkv && (table || DR == 0) && table_rows >= 0 && positions && token_seq
-               && block_table && cq && pages && eps > 0.f, "latent_prepare: missing operand");
+    MV_REQUIRE(mv_valid_dtype(weight_dtype) && packed && (QR == 0 || (wq && cq)) && wkv && (table || DR == 0) && table_rows >= 0 && positions && token_seq
+               && block_table && pages && eps > 0.f, "latent_prepare: missing operand");
     if (n == 0) return 0;
     WeightPtr a{wq, weight_dtype}, b{wkv, weight_dtype};
     MV_DISPATCH_T(dtype, "latent_prepare",
@@ -214,7 +218,7 @@ extern "C" int mv_head_linear(const void* x, long ldx, int ldx_head, const void*
 // ---------------------------------------------------------------------------------------
 // Attention. One workgroup per (row, group of AL_HEADS heads): the query heads of a row read the same
 // key rows, so a key row that a thread has fetched serves all heads of the group. Keys are visited in
-// tiles of AL_THREADS from position 0 (causal: a query at position p sees 0..p), so the order of
+// tiles of AL_THREADS from the first visible position (a query at position p sees max(0, p - window)..p), so the order of
 // additions depends on the position alone. q float [n][H][R + DR]; out float [n][H][R]: the
 // weighted sum of the visible latents.
 // ---------------------------------------------------------------------------------------
@@ -227,7 +231,8 @@ template <typename T>
 __global__ void __launch_bounds__(AL_THREADS)
 attention_latent_kernel(const float* __restrict__ q, long ldq, float* __restrict__ out, long ldo, const T* __restrict__ pages,
                         const int* __restrict__ block_table, int bt_width, int page_size, const int* __restrict__ positions,
-                        const int* __restrict__ token_seq, int H, int R, int DR, float scale) {
+                        const int* __restrict__ token_seq, int H, int R, int DR, float scale, int window,
+                        const float* __restrict__ sink) {
     __shared__ float qs[AL_HEADS][AL_MAX_KEY];
     __shared__ float ps[AL_HEADS][AL_THREADS];
     __shared__ long roff[AL_THREADS];
@@ -251,12 +256,13 @@ attention_latent_kernel(const float* __restrict__ q, long ldq, float* __restrict
     float acc[AL_HEADS][AL_MAX_R / AL_THREADS];
 #pragma unroll
     for (int hh = 0; hh < AL_HEADS; ++hh) {
-        m[hh] = -INFINITY;
-        l[hh] = 0.f;
+        // (the sink is a key whose weight counts and whose value is zero)
+        m[hh] = sink != nullptr && hh < nh ? sink[h0 + hh] : -INFINITY;
+        l[hh] = sink != nullptr && hh < nh ? 1.f : 0.f;
 #pragma unroll
         for (int i = 0; i < AL_MAX_R / AL_THREADS; ++i) acc[hh][i] = 0.f;
     }
-    for (int base = 0; base <= hi; base += AL_THREADS) {
+    for (int base = window >= 0 ? max(0, hi - window) : 0; base <= hi; base += AL_THREADS) {
         const int j = base + tid;
         const bool valid = j <= hi;
         float s[AL_HEADS];
@@ -324,7 +330,7 @@ attention_latent_kernel(const float* __restrict__ q, long ldq, float* __restrict
 
 extern "C" int mv_attention_latent(const float* q, long ldq, float* out, long ldo, const void* pages, const int* block_table,
                                    int bt_width, int page_size, const int* positions, const int* token_seq, int n, int H,
-                                   int R, int DR, float scale, int dtype, hipStream_t stream) {
+                                   int R, int DR, float scale, int window, const float* sink, int dtype, hipStream_t stream) {
     MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0, "attention_latent: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
     MV_REQUIRE(R <= AL_MAX_R && R + DR <= AL_MAX_KEY, "attention_latent: a latent of %d and a rotated part of %d exceed %d / %d",
                R, DR, AL_MAX_R, AL_MAX_KEY);
@@ -335,14 +341,14 @@ extern "C" int mv_attention_latent(const float* q, long ldq, float* out, long ld
     MV_DISPATCH_T(dtype, "attention_latent",
                   hipLaunchKernelGGL(attention_latent_kernel<T>, dim3(n, (H + AL_HEADS - 1) / AL_HEADS), dim3(AL_THREADS), 0,
                                      stream, q, ldq, out, ldo, (const T*)pages, block_table, bt_width, page_size, positions,
-                                     token_seq, H, R, DR, scale));
+                                     token_seq, H, R, DR, scale, window, sink));
     return mv_check_launch("attention_latent");
 }
 
 // ---------------------------------------------------------------------------------------
 // Attention for steps of few rows (single decoded tokens): a row's keys are dealt out to workgroups in
-// runs of `run` positions (run s holds positions s * run ..., so the cutting depends on the position and
-// the launch's run length alone), a workgroup serves up to ALS_HEADS heads of the row at once and brings each tile of
+// runs of `run` positions (a run begins at a multiple of `run`, so the cutting depends on the position and
+// the launch's run length alone; under a window the first run is the one that the window begins in), a workgroup serves up to ALS_HEADS heads of the row at once and brings each tile of
 // ALS_TILE key rows into LDS with 16-byte loads, where all its heads read them. It leaves per run the
 // running maximum, the sum of weights and the weighted sum of latents; a second kernel joins the runs
 // in their order. Requires (R + DR) * sizeof(T) to be a multiple of 16.
@@ -370,7 +376,7 @@ template <typename T>
 __global__ void __launch_bounds__(ALS_THREADS)
 attention_latent_split_kernel(const float* __restrict__ q, long ldq, const T* __restrict__ pages, const int* __restrict__ block_table,
                               int bt_width, int page_size, const int* __restrict__ positions, const int* __restrict__ token_seq,
-                              int H, int R, int DR, float scale, int row_words, int run, int max_splits,
+                              int H, int R, int DR, float scale, int window, int row_words, int run, int max_splits,
                               float* __restrict__ part_o, float* __restrict__ part_ml) {
     extern __shared__ __attribute__((aligned(16))) unsigned char als_lds[];
     constexpr int PER = AlsWord<T>::per;
@@ -384,9 +390,10 @@ attention_latent_split_kernel(const float* __restrict__ q, long ldq, const T* __
     const int seq = token_seq[tok];
     if (seq < 0) return;
     const int pos = positions[tok];
-    const int lo = split * run;
-    if (lo > pos) return;
-    const int hi = min(pos, lo + run - 1);
+    const int seen = window >= 0 ? max(0, pos - window) : 0;
+    const int begin = (seen / run + split) * run;
+    if (begin > pos) return;
+    const int lo = max(begin, seen), hi = min(pos, begin + run - 1);
     const int nh = min(ALS_HEADS, H - h0);
     const int* bt = block_table + (size_t)seq * bt_width;
     for (int e = tid; e < ALS_HEADS * DK; e += ALS_THREADS) {
@@ -519,19 +526,20 @@ attention_latent_split_kernel(const float* __restrict__ q, long ldq, const T* __
 
 __global__ void __launch_bounds__(256)
 attention_latent_join_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ positions,
-                             const int* __restrict__ token_seq, int H, int R, int run, int max_splits, float* __restrict__ out,
-                             long ldo) {
+                             const int* __restrict__ token_seq, int H, int R, int window, const float* __restrict__ sink, int run,
+                             int max_splits, float* __restrict__ out, long ldo) {
     const int tok = blockIdx.x, head = blockIdx.y;
     float* o = out + (size_t)tok * ldo + (size_t)head * R;
     if (token_seq[tok] < 0) {
         for (int d = threadIdx.x; d < R; d += 256) o[d] = 0.f;
         return;
     }
-    const int runs = positions[tok] / run + 1;
+    const int pos = positions[tok];
+    const int runs = pos / run + 1 - (window >= 0 ? max(0, pos - window) / run : 0);
     const float* ml = part_ml + ((size_t)tok * H + head) * max_splits * 2;
-    float m = -INFINITY;
+    float m = sink != nullptr ? sink[head] : -INFINITY;
     for (int s = 0; s < runs; ++s) m = fmaxf(m, ml[2 * s]);
-    float l = 0.f;
+    float l = sink != nullptr ? expf(sink[head] - m) : 0.f;
     for (int s = 0; s < runs; ++s) l += expf(ml[2 * s] - m) * ml[2 * s + 1];
     const float inv = 1.f / l;
     const float* po = part_o + ((size_t)tok * H + head) * max_splits * R;
@@ -553,17 +561,22 @@ static void als_layout(int R, int DR, int elem, int& row_words, size_t& lds) {
 // so few tiles a workgroup and many workgroups is what a step of few rows wants)
 static int als_run(int max_context) { return max_context <= 8192 ? 64 : (max_context <= 32768 ? 256 : 1024); }
 
-// floats of scratch for n rows whose contexts reach max_context positions: (weighted sums, maxima and sums)
-extern "C" long mv_attention_latent_split_workspace(int n, int H, int R, int max_context) {
+// most runs a query reads whose context reaches max_context positions
+static long als_runs(int max_context, int window) {
     const int run = als_run(max_context);
-    const long runs = (max_context + run - 1) / run;
-    return (long)n * H * runs * (R + 2);
+    const long all = (max_context + run - 1) / run;
+    return window < 0 ? all : min(all, (long)window / run + 2);
+}
+
+// floats of scratch for n rows whose contexts reach max_context positions: (weighted sums, maxima and sums)
+extern "C" long mv_attention_latent_split_workspace(int n, int H, int R, int max_context, int window) {
+    return (long)n * H * als_runs(max_context, window) * (R + 2);
 }
 
 // returns 2 (nothing done) when the sizes are not served: the caller takes the general kernel
 extern "C" int mv_attention_latent_split(const float* q, long ldq, float* out, long ldo, const void* pages, const int* block_table,
                                          int bt_width, int page_size, const int* positions, const int* token_seq, int n, int H,
-                                         int R, int DR, float scale, int max_context, float* work, long work_floats, int dtype,
+                                         int R, int DR, float scale, int window, const float* sink, int max_context, float* work, long work_floats, int dtype,
                                          hipStream_t stream) {
     MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0 && max_context > 0, "attention_latent_split: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
     const int elem = (int)mv_dtype_size(dtype);
@@ -575,8 +588,8 @@ extern "C" int mv_attention_latent_split(const float* q, long ldq, float* out, l
     MV_REQUIRE(page_size > 0 && bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_split: pitches too small");
     MV_REQUIRE(q && out && pages && block_table && positions && token_seq && work, "attention_latent_split: missing operand");
     const int run = als_run(max_context);
-    const int runs = (max_context + run - 1) / run;
-    MV_REQUIRE(work_floats >= mv_attention_latent_split_workspace(n, H, R, max_context) && runs <= 65535,
+    const int runs = (int)als_runs(max_context, window);
+    MV_REQUIRE(work_floats >= mv_attention_latent_split_workspace(n, H, R, max_context, window) && runs <= 65535,
                "attention_latent_split: scratch of %ld floats is too small", work_floats);
     if (n == 0) return 0;
     float* part_o = work;
@@ -584,11 +597,11 @@ extern "C" int mv_attention_latent_split(const float* q, long ldq, float* out, l
     dim3 grid(n, (H + ALS_HEADS - 1) / ALS_HEADS, runs);
     MV_DISPATCH_T(dtype, "attention_latent_split",
                   hipLaunchKernelGGL(attention_latent_split_kernel<T>, grid, dim3(ALS_THREADS), lds, stream, q, ldq, (const T*)pages,
-                                     block_table, bt_width, page_size, positions, token_seq, H, R, DR, scale, row_words, run, runs,
+                                     block_table, bt_width, page_size, positions, token_seq, H, R, DR, scale, window, row_words, run, runs,
                                      part_o, part_ml));
     if (mv_check_launch("attention_latent_split")) return 1;
     hipLaunchKernelGGL(attention_latent_join_kernel, dim3(n, H), dim3(256), 0, stream, part_o, part_ml, positions, token_seq, H, R,
-                       run, runs, out, ldo);
+                       window, sink, run, runs, out, ldo);
     return mv_check_launch("attention_latent_join");
 }
 
@@ -596,12 +609,12 @@ extern "C" int mv_attention_latent_split(const float* q, long ldq, float* out, l
 #ifdef MV_WITH_BF16
 // ---------------------------------------------------------------------------------------
 // Attention for steps with prompt portions (bfloat16, MFMA). One wave per (row, group of 16 heads): the heads of a row
-// are the 16 rows of the first operand, since they all read the same key rows. Keys are walked 32 at a time from
-// position 0:   S = Q K^T (NQ products of 16 x 16 x 32 for each half of the block, key rows straight from the pages),
+// are the 16 rows of the first operand, since they all read the same key rows. Keys are walked 32 at a time from the
+// multiple of eight at or in front of the first visible position:   S = Q K^T (NQ products of 16 x 16 x 32 for each half of the block, key rows straight from the pages),
 // a running maximum and sum per head in float, P rounded to bfloat16 and turned from "a lane holds a key's column" to
 // "a lane holds a head's row" through the wave's own 1 KB of LDS,   O += P V with V from the pages that hold the
 // latents slot-contiguous (a lane's eight keys are eight neighbouring slots of one page: page_size % 8 == 0).
-// Keys behind the row's position are masked in S and zeroed in V (their slots may hold anything).
+// Keys that the row does not see are masked in S and zeroed in V (their slots may hold anything).
 // v_mfma_f32_16x16x32_bf16: lane l holds row l % 16 of the first operand (k = 8 (l / 16) .. + 7), column l % 16 of the
 // second, and column l % 16 of rows 4 (l / 16) .. + 3 of the result.
 // ---------------------------------------------------------------------------------------
@@ -628,7 +641,8 @@ template <int NQ, int NR>
 __global__ void __launch_bounds__(256)
 attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __restrict__ out, long ldo, const bf16* __restrict__ pages,
                              const bf16* __restrict__ pages_t, const int* __restrict__ block_table, int bt_width, int page_size,
-                             const int* __restrict__ positions, const int* __restrict__ token_seq, int n, int H, float scale) {
+                             const int* __restrict__ positions, const int* __restrict__ token_seq, int n, int H, float scale, int window,
+                             const float* __restrict__ sink) {
     constexpr int DK = NQ * 32, R = NR * 16;
     __shared__ __attribute__((aligned(16))) uint16_t pl[4][16][40];          // a wave's P: [head][key], rows 80 bytes apart
     const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
@@ -658,18 +672,21 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     alm_f4 acc[NR];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        m[i] = -INFINITY;
-        l[i] = 0.f;
+        // (the sink is a key whose weight counts and whose value is zero)
+        const bool has = sink != nullptr && 4 * kq + i < nh;
+        m[i] = has ? sink[h0 + 4 * kq + i] : -INFINITY;
+        l[i] = has ? 1.f : 0.f;
     }
+    const int lo = window >= 0 ? max(0, pos - window) : 0;
 #pragma unroll
     for (int t = 0; t < NR; ++t) acc[t] = alm_f4{0.f, 0.f, 0.f, 0.f};
-    for (int kb = 0; kb <= pos; kb += 32) {
+    for (int kb = lo & ~7; kb <= pos; kb += 32) {
         alm_f4 s[2];
 #pragma unroll
         for (int sub = 0; sub < 2; ++sub) {
             s[sub] = alm_f4{0.f, 0.f, 0.f, 0.f};
             const int key = kb + 16 * sub + r;
-            const int kc = key <= pos ? key : pos;           // keys behind the row: some valid row, masked below
+            const int kc = key <= pos ? max(key, lo) : pos;  // keys the row does not see: some valid row, masked below
             const bf16* krow = pages + ((size_t)bt[kc / page_size] * page_size + kc % page_size) * DK + 8 * kq;
 #pragma unroll
             for (int c = 0; c < NQ; ++c) {
@@ -678,7 +695,7 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
                 s[sub] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qf[c].v, kf.v, s[sub], 0, 0, 0);
             }
         }
-        const bool ok0 = kb + r <= pos, ok1 = kb + 16 + r <= pos;
+        const bool ok0 = kb + r <= pos && kb + r >= lo, ok1 = kb + 16 + r <= pos;     // (kb + 16 > lo)
         float corr[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -712,7 +729,7 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
             vf.u = *reinterpret_cast<const uint4*>(vbase + (size_t)16 * t * page_size);
 #pragma unroll
             for (int e = 0; e < 8; ++e)
-                if (e >= live) vf.h[e] = 0;
+                if (e >= live || key0 + e < lo) vf.h[e] = 0;
             acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf.v, vf.v, acc[t], 0, 0, 0);
         }
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -729,13 +746,15 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     }
 }
 
-// returns 2 (nothing done) for sizes it does not serve: (R, DR) in (64, 32), (128, 32), (128, 64), (256, 64), pages
-// whose size is a multiple of 8
+// returns 2 (nothing done) for sizes it does not serve: (R, DR) in (64, 32), (128, 32), (128, 64), (256, 64), without a rotated
+// part R in 32, 64, 96, 128, 160, 192, 256, 384, 512; pages whose size is a multiple of 8
 extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, long ldo, const void* pages, const void* pages_t,
                                         const int* block_table, int bt_width, int page_size, const int* positions,
-                                        const int* token_seq, int n, int H, int R, int DR, float scale, hipStream_t stream) {
+                                        const int* token_seq, int n, int H, int R, int DR, float scale, int window, const float* sink,
+                                        hipStream_t stream) {
     MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0, "attention_latent_mfma: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
-    const bool served = (R == 64 && DR == 32) || (R == 128 && DR == 32) || (R == 128 && DR == 64) || (R == 256 && DR == 64);
+    const bool plain = DR == 0 && R % 32 == 0 && (R <= 192 || R == 256 || R == 384 || R == 512);
+    const bool served = plain || (R == 64 && DR == 32) || (R == 128 && DR == 32) || (R == 128 && DR == 64) || (R == 256 && DR == 64);
     if (!served || page_size % 8 != 0 || !pages_t || ((uintptr_t)pages % 16) || ((uintptr_t)pages_t % 16)) return 2;
     MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_mfma: pitches too small");
     MV_REQUIRE(q && out && pages && block_table && positions && token_seq, "attention_latent_mfma: missing operand");
@@ -743,8 +762,20 @@ extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, lo
     dim3 grid((n + 3) / 4, (H + 15) / 16);
 #define ALM_LAUNCH(NQ, NR)                                                                                                 \
     hipLaunchKernelGGL((attention_latent_mfma_kernel<NQ, NR>), grid, dim3(256), 0, stream, q, ldq, out, ldo, (const bf16*)pages, \
-                       (const bf16*)pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, scale)
-    if (R == 64) ALM_LAUNCH(3, 4);
+                       (const bf16*)pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, scale, window, sink)
+    if (plain) {
+        switch (R) {
+            case 32: ALM_LAUNCH(1, 2); break;
+            case 64: ALM_LAUNCH(2, 4); break;
+            case 96: ALM_LAUNCH(3, 6); break;
+            case 128: ALM_LAUNCH(4, 8); break;
+            case 160: ALM_LAUNCH(5, 10); break;
+            case 192: ALM_LAUNCH(6, 12); break;
+            case 256: ALM_LAUNCH(8, 16); break;
+            case 384: ALM_LAUNCH(12, 24); break;
+            default: ALM_LAUNCH(16, 32); break;
+        }
+    } else if (R == 64) ALM_LAUNCH(3, 4);
     else if (R == 128 && DR == 32) ALM_LAUNCH(5, 8);
     else if (R == 128) ALM_LAUNCH(6, 8);
     else ALM_LAUNCH(10, 16);

@@ -29,7 +29,7 @@ ARCH = "gfx950"
 COMMON_SOURCES = ["runtime.hip", "elementwise.hip", "gemm_ref.hip", "attention_ref.hip", "sampling.hip", "recurrent.hip",
                   "attention_sigmoid.hip", "attention_latent.hip", "moe.hip", "group_norm.hip", "hyper.hip", "qkv_rotate.hip",
                   "qkv_row_norm.hip", "recurrent_channel.hip", "recurrent_constant.hip", "recurrent_chunks.hip",
-                  "pair_norm.hip"]
+                  "pair_norm.hip", "qkv_conv.hip", "recurrent_gated.hip", "recurrent_unit.hip"]
 VARIANT_SOURCES: Dict[str, List[str]] = {
     "f32": COMMON_SOURCES,
     "bf16": COMMON_SOURCES + ["gemm_skinny.hip", "gemm_mid.hip", "gemm_tile.hip", "gemm_lt.hip", "attention_fast.hip",

@@ -930,9 +930,64 @@ extern "C" int mv_xielu(const void* x, long ldx, void* out, long ldo, int n, int
 }
 
 // ---------------------------------------------------------------------------------------
+// The square of ReLU in place, and float rows rounded to the activation type: contiguous, eight elements a thread (the
+// last thread takes what is left one by one)
+// ---------------------------------------------------------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256)
+squared_relu_kernel(T* __restrict__ x, long total) {
+    const long i = ((long)blockIdx.x * 256 + threadIdx.x) * 8;
+    if (i + 8 <= total) {
+        float v[8];
+        Vec8<T>::load(x + i, v);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const float p = fmaxf(v[e], 0.f);
+            v[e] = p * p;
+        }
+        Vec8<T>::store(x + i, v);
+        return;
+    }
+    for (long k = i; k < total; ++k) {
+        const float p = fmaxf(to_f(x[k]), 0.f);
+        x[k] = from_f<T>(p * p);
+    }
+}
+
+extern "C" int mv_squared_relu(void* x, long total, int dtype, hipStream_t stream) {
+    MV_REQUIRE(total >= 0 && x && ((uintptr_t)x % 16) == 0, "squared_relu: contiguous rows of a 16-byte aligned tensor are needed");
+    if (total == 0) return 0;
+    const dim3 grid((unsigned)((total + 2047) / 2048));
+    MV_DISPATCH_T(dtype, "squared_relu", hipLaunchKernelGGL(squared_relu_kernel<T>, grid, dim3(256), 0, stream, (T*)x, total));
+    return mv_check_launch("squared_relu");
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+round_rows_kernel(const float* __restrict__ x, T* __restrict__ out, long total) {
+    const long i = ((long)blockIdx.x * 256 + threadIdx.x) * 8;
+    if (i + 8 <= total) {
+        float v[8];
+        Vec8<float>::load(x + i, v);
+        Vec8<T>::store(out + i, v);
+        return;
+    }
+    for (long k = i; k < total; ++k) out[k] = from_f<T>(x[k]);
+}
+
+extern "C" int mv_round_rows(const float* x, void* out, long total, int dtype, hipStream_t stream) {
+    MV_REQUIRE(total >= 0 && x && out && ((uintptr_t)x % 16) == 0 && ((uintptr_t)out % 16) == 0,
+               "round_rows: contiguous rows of 16-byte aligned tensors are needed");
+    if (total == 0) return 0;
+    const dim3 grid((unsigned)((total + 2047) / 2048));
+    MV_DISPATCH_T(dtype, "round_rows", hipLaunchKernelGGL(round_rows_kernel<T>, grid, dim3(256), 0, stream, x, (T*)out, total));
+    return mv_check_launch("round_rows");
+}
+
+// ---------------------------------------------------------------------------------------
 // A norm behind a sublayer, the residual add, and the norm in front of the next sublayer:
 //   v = resid[r] + y[r] / sqrt(mean(y[r]^2) + eps_a) * wa ;  resid[r] = v ;
-//   out[r] = v / sqrt(mean(v^2) + eps_b) * wb                          (out == null: the add alone)
+//   out[r] = v / sqrt(mean(v^2) + eps_b) * wb                          (out == null: the add alone; wb == null: out[r] = v)
 // One workgroup per row; the sum stays float from the first norm to the second.
 // ---------------------------------------------------------------------------------------
 // NE > 0: a thread keeps its NE columns (c = thread + 256 e) in registers from the first sum to the last
@@ -985,7 +1040,7 @@ norm_add_norm_kernel(const T* __restrict__ y, long ldy, WeightPtr wa, float eps_
         // the value dropped): a load under a condition would be a branch with a wait of its own, and the
         // kernel would wait for memory once per column instead of once
         const T* stl = st != nullptr ? st : yr;
-        const WeightPtr wbl = o != nullptr ? wb : wa;
+        const WeightPtr wbl = o != nullptr && wb.p != nullptr ? wb : wa;
 #pragma unroll
         for (int e = 0; e < NE; ++e) {
             const int c = threadIdx.x + 256 * e;
@@ -1016,6 +1071,12 @@ norm_add_norm_kernel(const T* __restrict__ y, long ldy, WeightPtr wa, float eps_
             }
         }
         if (o == nullptr) return;
+        if (wb.p == nullptr) {               // the sum itself, rounded
+#pragma unroll
+            for (int e = 0; e < NE; ++e)
+                if ((int)threadIdx.x + 256 * e < h) o[threadIdx.x + 256 * e] = from_f<T>(v[e]);
+            return;
+        }
         ss2 = wave_sum(ss2);
         if (lane == 0) part_b[wave] = ss2;
         __syncthreads();
@@ -1052,6 +1113,10 @@ norm_add_norm_kernel(const T* __restrict__ y, long ldy, WeightPtr wa, float eps_
             ss2 = fmaf(v, v, ss2);
         }
         if (o == nullptr) return;
+        if (wb.p == nullptr) {               // the sum itself, rounded
+            for (int c = threadIdx.x; c < h; c += 256) o[c] = from_f<T>(x[c]);
+            return;
+        }
         ss2 = wave_sum(ss2);
         if (lane == 0) part_b[wave] = ss2;
         __syncthreads();
@@ -1082,7 +1147,7 @@ norm_add_norm_vec_kernel(const T* __restrict__ y, long ldy, WeightPtr wa, float 
     T* st = (shifted && seq >= 0) ? (T*)shift.state + (size_t)shift.state_slots[seq] * h : nullptr;
     const WeightPtr mix{shift.mix != nullptr ? shift.mix : wa.p, shift.mix != nullptr ? shift.mix_dtype : wa.dtype};
     const T* stl = st != nullptr ? st : yr;
-    const WeightPtr wbl = o != nullptr ? wb : wa;
+    const WeightPtr wbl = o != nullptr && wb.p != nullptr ? wb : wa;
     float v[NC][8], xr[NC][8], fa[NC][8], fb[NC][8], prev[NC][8], fm[NC][8];
     float ss = 0.f;
 #pragma unroll
@@ -1120,6 +1185,14 @@ norm_add_norm_vec_kernel(const T* __restrict__ y, long ldy, WeightPtr wa, float 
         }
     }
     if (o == nullptr) return;
+    if (wb.p == nullptr) {                   // the sum itself, rounded
+#pragma unroll
+        for (int c = 0; c < NC; ++c) {
+            const int d = (threadIdx.x + 256 * c) * 8;
+            if (d < h) Vec8<T>::store(o + d, v[c]);
+        }
+        return;
+    }
     ss2 = wave_sum(ss2);
     if (lane == 0) part_b[wave] = ss2;
     __syncthreads();
@@ -1155,7 +1228,8 @@ extern "C" int mv_norm_add_norm(const void* y, long ldy, const void* wa, int wa_
     const ShiftArgs shift{shift_mix, shift_mix_dtype, shift_state, token_seq, state_slots};
     MV_REQUIRE(n >= 0 && h > 0 && ldy >= h, "norm_add_norm: bad sizes n=%d h=%d", n, h);
     MV_REQUIRE(y && wa && resid && mv_valid_dtype(wa_dtype) && eps_a > 0.f, "norm_add_norm: missing operand");
-    MV_REQUIRE(out == nullptr || (wb && mv_valid_dtype(wb_dtype) && eps_b > 0.f), "norm_add_norm: the second norm lacks its weight");
+    MV_REQUIRE(wb == nullptr || (mv_valid_dtype(wb_dtype) && eps_b > 0.f), "norm_add_norm: bad constants of the second norm");
+    MV_REQUIRE(wb != nullptr || shift_mix == nullptr, "norm_add_norm: a token shift needs the second norm");
     if (n == 0) return 0;
     WeightPtr pa{wa, wa_dtype}, pb{wb, out ? wb_dtype : MV_F32};
 #define NAN_LAUNCH(NE)                                                                                               \

@@ -9,54 +9,7 @@
 // q, k and v are SiLU of the packed rows' columns [q (H*DK) | k (H*DK) | v (H*DV)] from column `off` on. States and
 // the chunks' sums are floats [..][H][DV][DK], a head's matrix column by column. Powers of the decay are 2^(n log2 a),
 // so 0 < a <= 1.
-#include "recurrent.h"
-
-typedef float floatx4_t __attribute__((ext_vector_type(4)));
-
-#define CL_TOKENS 64
-#define CL_TILE 64                 // channels of a tile
-// LDS rows of 68 floats: a lane takes four neighbours of a row for four steps of a product (16 bytes; the four
-// steps then sum over k in another order, the same for both operands), and the 16 rows that 16 lanes touch lie in
-// different banks
-#define CL_PITCH 68
-typedef float Tile[CL_TILE][CL_PITCH];
-
-// The chunk `unit` of the step: which request it belongs to, its first row and its number of rows (0: no such chunk).
-// All 256 threads call it; sh holds 8 ints.
-__device__ __forceinline__ void find_chunk(const int* __restrict__ cu, int n_seqs, int unit, int* sh, int& seq, int& row0, int& count) {
-    const int tid = threadIdx.x, lane = tid % MV_WAVE, wave = tid / MV_WAVE;
-    if (tid == 0) sh[4] = -1;
-    int base = 0;
-    for (int s0 = 0; s0 < n_seqs; s0 += 256) {
-        const int s = s0 + tid;
-        const int first = s < n_seqs ? cu[s] : 0, len = s < n_seqs ? cu[s + 1] - first : 0;
-        const int mine = (len + CL_TOKENS - 1) / CL_TOKENS;
-        int incl = mine;
-#pragma unroll
-        for (int o = 1; o < MV_WAVE; o <<= 1) {
-            const int t = __shfl_up(incl, o, MV_WAVE);
-            if (lane >= o) incl += t;
-        }
-        __syncthreads();
-        if (lane == MV_WAVE - 1) sh[wave] = incl;
-        __syncthreads();
-        int before = base;
-        for (int w = 0; w < wave; ++w) before += sh[w];
-        incl += before;
-        if (unit < incl && unit >= incl - mine) {
-            const int c = unit - (incl - mine);
-            sh[4] = s;
-            sh[5] = first + c * CL_TOKENS;
-            sh[6] = len - c * CL_TOKENS < CL_TOKENS ? len - c * CL_TOKENS : CL_TOKENS;
-        }
-        base += sh[0] + sh[1] + sh[2] + sh[3];
-        if (base > unit) break;                        // (the same for every thread)
-    }
-    __syncthreads();
-    seq = sh[4];
-    row0 = sh[5];
-    count = seq >= 0 ? sh[6] : 0;
-}
+#include "recurrent_chunk.h"
 
 // silu of up to CL_TOKENS rows x CL_TILE channels into LDS, zero beyond the rows and channels there are: dst[row][channel],
 // or TRANSPOSED dst[channel][row], there multiplied by 2^((count - 1 - row) * l2) when WEIGHTED
@@ -88,16 +41,6 @@ __device__ __forceinline__ void load_tile(Tile& dst, const T* __restrict__ src, 
     }
 }
 
-// acc += A B^T over four k of each lane group: a and b hold a lane's four neighbours of the operands' rows
-__device__ __forceinline__ void mfma4(floatx4_t& acc, const float4& a, const float4& b) {
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
-}
-
-__device__ __forceinline__ float4 four(const Tile& t, int row, int k) { return *reinterpret_cast<const float4*>(&t[row][k]); }
-
 struct ChunkArgs {
     const void* packed; long ld; int off;
     int H, DK, DV;
@@ -114,7 +57,7 @@ chunk_sums_kernel(ChunkArgs A) {
     __shared__ __attribute__((aligned(16))) Tile sK, sV;                       // transposed: [channel][token]
     __shared__ int sh[8];
     int seq, row0, count;
-    find_chunk(A.cu_seqlens, A.n_seqs, blockIdx.x, sh, seq, row0, count);
+    find_chunk<CL_TOKENS>(A.cu_seqlens, A.n_seqs, blockIdx.x, sh, seq, row0, count);
     if (count <= 0) return;
     const int head = blockIdx.y, tk = (A.DK + CL_TILE - 1) / CL_TILE;
     const int k0 = (blockIdx.z % tk) * CL_TILE, v0 = (blockIdx.z / tk) * CL_TILE;
@@ -148,15 +91,9 @@ __global__ void __launch_bounds__(256)
 chunk_walk_kernel(ChunkArgs A, float* __restrict__ state, const int* __restrict__ state_slots) {
     __shared__ int part[4];
     const int seq = blockIdx.x, head = blockIdx.y;
-    const int first = A.cu_seqlens[seq], len = A.cu_seqlens[seq + 1] - first;
+    const int len = A.cu_seqlens[seq + 1] - A.cu_seqlens[seq];
     if (len <= 0) return;
-    int before = 0;
-    for (int s = threadIdx.x; s < seq; s += 256) before += (A.cu_seqlens[s + 1] - A.cu_seqlens[s] + CL_TOKENS - 1) / CL_TOKENS;
-#pragma unroll
-    for (int o = MV_WAVE / 2; o > 0; o >>= 1) before += __shfl_xor(before, o, MV_WAVE);
-    if (threadIdx.x % MV_WAVE == 0) part[threadIdx.x / MV_WAVE] = before;
-    __syncthreads();
-    const int c0 = part[0] + part[1] + part[2] + part[3];
+    const int c0 = chunks_before<CL_TOKENS>(A.cu_seqlens, seq, part);
     const int chunks = (len + CL_TOKENS - 1) / CL_TOKENS;
     const int size = A.DV * A.DK, e = blockIdx.z * 256 + threadIdx.x;
     if (e >= size) return;
@@ -190,7 +127,7 @@ chunk_out_kernel(ChunkArgs A, float* __restrict__ out) {
     __shared__ __attribute__((aligned(16))) Tile s0, s1, s2;
     __shared__ int sh[8];
     int seq, row0, count;
-    find_chunk(A.cu_seqlens, A.n_seqs, blockIdx.x, sh, seq, row0, count);
+    find_chunk<CL_TOKENS>(A.cu_seqlens, A.n_seqs, blockIdx.x, sh, seq, row0, count);
     if (count <= 0) return;
     const int head = blockIdx.y, v0 = blockIdx.z * CL_TILE, DK = A.DK, DV = A.DV;
     const T* rows = (const T*)A.packed + (size_t)row0 * A.ld + A.off;

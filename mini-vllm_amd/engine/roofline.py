@@ -90,6 +90,14 @@ KERNELS_OF: Dict[str, Tuple[str, Optional[str], int]] = {
     "mv_channel_prepare": (r"\bchannel_prepare(_rows)?_kernel", r"\bconv_state_kernel", 2),
     "mv_channel_scan": (r"\bchannel_scan_kernel", None, 1),
     "mv_channel_step": (r"\bchannel_step_kernel", r"\bconv_state_kernel", 2),
+    "mv_squared_relu": (r"\bsquared_relu_kernel", None, 1),
+    "mv_round_rows": (r"\bround_rows_kernel", None, 1),
+    "mv_qkv_conv_store": (r"\bqkv_conv_store(_vec)?_kernel", r"\b(store_v_pages|conv_state)_kernel", 3),
+    "mv_gated_linear_chunks": (r"\bgated_sums_kernel", r"\bgated_(walk|out)_kernel", 3),
+    "mv_gated_linear_step": (r"\bgated_step_kernel", None, 1),
+    "mv_short_conv": (r"\bshort_conv_kernel", r"\bconv_state_kernel", 2),
+    "mv_unit_scan": (r"\bunit_chunk_kernel", r"\bunit_(walk|chunk)_kernel", 3),
+    "mv_unit_step": (r"\bunit_step_kernel", None, 1),
 }
 _OURS = re.compile("|".join(f"(?:{p})" for spec in KERNELS_OF.values() for p in spec[:2] if p))
 

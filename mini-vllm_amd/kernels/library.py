@@ -142,6 +142,40 @@ _SIGNATURES = {
     "mv_norm_add_norm": (c_int, [c_void_p, c_long, c_void_p, c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_float,
                                  c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                  c_void_p]),
+    # x, total, dtype, stream
+    "mv_squared_relu": (c_int, [c_void_p, c_long, c_int, c_void_p]),
+    # x, out, total, dtype, stream
+    "mv_round_rows": (c_int, [c_void_p, c_void_p, c_long, c_int, c_void_p]),
+    # rows, ld, base, n, n_seqs, H, Hkv, D, Dv, taps, w, conv_state, single, positions, token_seq, cu_seqlens, state_slots,
+    # block_table, bt_width, page_size, k_pages, v_pages, table, rot, unit_norm, eps, out, ldo, dtype, stream
+    "mv_qkv_conv_store": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int,
+                                  c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int,
+                                  c_int, c_float, c_void_p, c_long, c_int, c_void_p]),
+    "mv_gated_linear_chunk_tokens": (c_int, []),
+    # packed, ld, off, n, H, DK, DV, z, ldz, bias, tau, state, cu_seqlens, state_slots, n_seqs, chunks, sums, decays, out, dtype,
+    # stream
+    "mv_gated_linear_chunks": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p, c_float, c_void_p,
+                                       c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
+    # packed, ld, off, low_off, n, H, DK, DV, ra, a2t, a2_dtype, bias, tau, norm_w, eps, state, token_seq, state_slots, out, ldo,
+    # then the softmax mixer beside it: rows, rows_ld, base, H, Hkv, D, Dv, taps, w, conv_state, positions, cu_seqlens,
+    # block_table, bt_width, page_size, k_pages, v_pages, table, rot, unit_norm, eps, out, ldo, dtype, stream
+    "mv_gated_linear_step": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_float,
+                                     c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_long,
+                                     c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                                     c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_long,
+                                     c_int, c_void_p]),
+    # rows, ld, n, n_seqs, C, taps, w, bias, conv_state, token_seq, cu_seqlens, state_slots, out, ldo, dtype, stream
+    "mv_short_conv": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                              c_void_p, c_long, c_int, c_void_p]),
+    "mv_unit_chunk_tokens": (c_int, []),
+    # z, u, ldu, packed, ld, y_off, n, W, B, gate_bias, rate, state, cu_seqlens, state_slots, n_seqs, chunks, sums, out, ldo, dtype,
+    # stream
+    "mv_unit_scan": (c_int, [c_void_p, c_void_p, c_long, c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p,
+                             c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_long, c_int, c_void_p]),
+    # packed, ld, y_off, n, W, B, taps, w, conv_bias, conv_state, gates, gates_dtype, gate_bias, rate, state, token_seq,
+    # state_slots, out, ldo, dtype, stream
+    "mv_unit_step": (c_int, [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
+                             c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p]),
     # x, ld, rows, cols, cap, stream
     "mv_soft_cap": (c_int, [c_void_p, c_long, c_int, c_int, c_float, c_void_p]),
     "mv_sample": (c_int, [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -156,9 +190,10 @@ _OPTIONAL_SIGNATURES = {
     # x, ldx, ldx_head, w, n, H, IN, OUT, y, ldy, ldy_head, tail, table, positions, gate, ldg, gate_per_head, token_seq, mode, stream
     "mv_head_linear_mfma": (c_int, [c_void_p, c_long, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_long, c_int, c_int,
                                     c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_void_p]),
-    # q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, R, DR, scale, stream
+    # q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, R, DR, scale, window, sink,
+    # stream
     "mv_attention_latent_mfma": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
-                                         c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p]),
+                                         c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p]),
     "mv_moe_grouped_ints": (c_long, [c_int, c_int, c_int]),
     # x, ldx, n, hidden, w_gate_up, w_down, n_real, identity, F, ids, weights, top, dense, ld_dense, ints, act, out, y, ldy,
     # limit, slope, stream
@@ -265,14 +300,15 @@ _OPTIONAL_SIGNATURES = {
     # dtype, stream
     "mv_head_linear": (c_int, [c_void_p, c_long, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_int,
                                c_int, c_void_p, c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_int, c_void_p]),
-    # q, ldq, out, ldo, pages, block_table, bt_width, page_size, positions, token_seq, n, H, R, DR, scale, dtype, stream
+    # q, ldq, out, ldo, pages, block_table, bt_width, page_size, positions, token_seq, n, H, R, DR, scale, window, sink, dtype,
+    # stream
     "mv_attention_latent": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p,
-                                    c_int, c_int, c_int, c_int, c_float, c_int, c_void_p]),
-    "mv_attention_latent_split_workspace": (c_long, [c_int, c_int, c_int, c_int]),
-    # as mv_attention_latent up to scale, then max_context, work, work_floats, dtype, stream
+                                    c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_int, c_void_p]),
+    "mv_attention_latent_split_workspace": (c_long, [c_int, c_int, c_int, c_int, c_int]),
+    # as mv_attention_latent up to sink, then max_context, work, work_floats, dtype, stream
     "mv_attention_latent_split": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_void_p,
-                                          c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_long, c_int,
-                                          c_void_p]),
+                                          c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_int, c_void_p, c_long,
+                                          c_int, c_void_p]),
     # logits, ld, n, E, correction, weight_dtype, groups, keep, top, sum_eps, flags, dense, ids, weights, stream
     "mv_moe_route": (c_int, [c_void_p, c_long, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p,
                              c_void_p, c_void_p, c_void_p]),

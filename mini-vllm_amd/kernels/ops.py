@@ -1247,23 +1247,28 @@ class Ops:
 
     def latent_prepare(self, packed: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, q_norm: torch.Tensor,
                        kv_norm: torch.Tensor, eps: float, table: Optional[torch.Tensor], positions: torch.Tensor,
-                       token_seq: torch.Tensor, block_table: torch.Tensor, page_size: int, q_latent: torch.Tensor,
+                       token_seq: torch.Tensor, block_table: torch.Tensor, page_size: int, q_latent: Optional[torch.Tensor],
                        pages: torch.Tensor, pages_t: Optional[torch.Tensor] = None) -> None:
-        """From rows [dq (q_rank) | dkv (kv_rank + rot_dim) | ...]: q_latent = rmsnorm(dq) * q_norm; the row's cache
+        """From rows [dq (q_rank) | dkv (kv_rank + rot_dim) | ...]: q_latent = rmsnorm(dq) * q_norm (``q_rank`` 0: no query
+        latent, q_norm and q_latent None); the row's cache
         entry [rmsnorm(dkv[:kv_rank]) * kv_norm | rot(dkv[kv_rank:])] goes to pages [pages, page_size, kv_rank + rot_dim]
         at the row's position (``table``: float32 [positions, rot_dim] = cat(cos, sin), pairs i, i + rot_dim/2).
         ``pages_t`` [pages, kv_rank, page_size], when given, gets the latent once more, a page's slots side by side."""
-        self._act(packed, "latent rows"); self._act(q_latent, "query latent"); self._act(pages, "latent pages")
+        self._act(packed, "latent rows"); self._act(pages, "latent pages")
+        if q_rank:
+            self._act(q_latent, "query latent")
         n = packed.shape[0]
         if packed.dim() != 2 or packed.stride(1) != 1 or packed.shape[1] < q_rank + kv_rank + rot_dim:
             raise KernelLibraryError(f"latent_prepare: rows {tuple(packed.shape)} are too short")
-        if tuple(q_latent.shape) != (n, q_rank) or q_latent.stride(1) != 1:
+        if q_rank and (tuple(q_latent.shape) != (n, q_rank) or q_latent.stride(1) != 1):
             raise KernelLibraryError(f"latent_prepare: the query latent must be [{n}, {q_rank}]")
         if pages.dim() != 3 or tuple(pages.shape[1:]) != (page_size, kv_rank + rot_dim) or not pages.is_contiguous():
             raise KernelLibraryError(f"latent_prepare: pages must be [pages, {page_size}, {kv_rank + rot_dim}]")
         for t, size, name in ((q_norm, q_rank, "query latent norm"), (kv_norm, kv_rank, "latent norm")):
+            if size == 0:
+                continue
             _dev(t, name)
-            if t.numel() != size or not t.is_contiguous() or t.dtype != q_norm.dtype:
+            if t.numel() != size or not t.is_contiguous() or t.dtype != kv_norm.dtype:
                 raise KernelLibraryError(f"latent_prepare: the {name} weight must hold {size} numbers")
         if pages_t is not None:
             self._act(pages_t, "slot-contiguous latent pages")
@@ -1281,9 +1286,9 @@ class Ops:
         self._ints(n, positions=(positions, n), token_seq=(token_seq, n))
         self._note("mv_latent_prepare", n * (q_rank + kv_rank + rot_dim) * 2 * packed.element_size(), 8 * n * (q_rank + kv_rank + rot_dim))
         self.lib.call("mv_latent_prepare", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], n, q_rank, kv_rank,
-                      rot_dim, q_norm.data_ptr(), kv_norm.data_ptr(), _weight_code(q_norm, "latent norm"), float(eps),
+                      rot_dim, _ptr(q_norm), kv_norm.data_ptr(), _weight_code(kv_norm, "latent norm"), float(eps),
                       _ptr(table), rows, positions.data_ptr(), token_seq.data_ptr(), block_table.data_ptr(),
-                      block_table.shape[1], page_size, q_latent.data_ptr(), q_latent.stride(0) if n > 1 else q_rank,
+                      block_table.shape[1], page_size, _ptr(q_latent), q_latent.stride(0) if q_rank and n > 1 else q_rank,
                       pages.data_ptr(), _ptr(pages_t), self.code, self._stream())
 
     def head_linear(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, token_seq: torch.Tensor, tail: int = 0,
@@ -1344,10 +1349,12 @@ class Ops:
 
     def attention_latent(self, q: torch.Tensor, out: torch.Tensor, pages: torch.Tensor, block_table: torch.Tensor,
                          page_size: int, positions: torch.Tensor, token_seq: torch.Tensor, heads: int, kv_rank: int,
-                         rot_dim: int, scale: float, plan=None, pages_t: Optional[torch.Tensor] = None) -> None:
+                         rot_dim: int, scale: float, plan=None, pages_t: Optional[torch.Tensor] = None,
+                         window: Optional[int] = None, sink: Optional[torch.Tensor] = None) -> None:
         """Causal softmax attention of q float32 [n, heads, kv_rank + rot_dim] over the cached rows [latent | rotated
         key part] of each row's request (pages [pages, page_size, kv_rank + rot_dim]); out float32 [n, heads, kv_rank] is
-        the weighted sum of the latents. Steps of single tokens take the kernel that deals a row's keys out over workgroups;
+        the weighted sum of the latents. With ``window`` the query at position p sees the keys from p - window on; ``sink`` float32
+        [heads]: the softmax's denominator has one more term exp(sink[h]). Steps of single tokens take the kernel that deals a row's keys out over workgroups;
         in bfloat16 other steps take the MFMA kernel where it serves the sizes (it reads the values from ``pages_t``
         [pages, kv_rank, page_size], the latents with a page's slots side by side); everything else the general kernel."""
         _dev(q, "latent queries"); _dev(out, "latent attention output"); self._act(pages, "latent pages")
@@ -1362,10 +1369,16 @@ class Ops:
         if block_table.dtype != torch.int32 or block_table.dim() != 2 or not block_table.is_contiguous():
             raise KernelLibraryError("attention_latent: the block table must be contiguous int32 [sequences, width]")
         self._ints(n, positions=(positions, n), token_seq=(token_seq, n))
-        kv_tokens = plan.kv_tokens if plan is not None else 0
-        pairs = plan.attention_pairs if plan is not None else 0
+        if sink is not None:
+            _dev(sink, "sinks")
+            if sink.dtype != torch.float32 or sink.numel() != heads or not sink.is_contiguous():
+                raise KernelLibraryError(f"attention_latent: the sinks must be float32 [{heads}]")
+        w = -1 if window is None else int(window)
+        priced = self._window_priced(plan, w, 0) if self.ledger is not None else plan
+        kv_tokens = priced.kv_tokens if plan is not None else 0
+        pairs = priced.attention_pairs if plan is not None else 0
         if plan is not None and plan.decode_only and plan.max_context_len > 0 and self._attention_latent_split(
-                q, out, pages, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim, scale,
+                q, out, pages, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim, scale, w, sink,
                 plan.max_context_len, kv_tokens):
             return
         if pages_t is not None and self.use_fast_kernels and self.lib.has("mv_attention_latent_mfma") \
@@ -1375,7 +1388,7 @@ class Ops:
                 raise KernelLibraryError(f"attention_latent: the slot-contiguous pages must be [{pages.shape[0]}, {kv_rank}, {page_size}]")
             if self.lib.offer("mv_attention_latent_mfma", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank, pages.data_ptr(),
                               pages_t.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(),
-                              token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), self._stream()):
+                              token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), w, _ptr(sink), self._stream()):
                 self._note("mv_attention_latent_mfma", self._size(q, out) + kv_tokens * (dk + kv_rank) * pages.element_size(),
                            2 * pairs * heads * (dk + kv_rank))
                 return
@@ -1383,13 +1396,13 @@ class Ops:
                    2 * pairs * heads * (dk + kv_rank))
         self.lib.call("mv_attention_latent", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank, pages.data_ptr(),
                       block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(), token_seq.data_ptr(),
-                      n, heads, kv_rank, rot_dim, float(scale), self.code, self._stream())
+                      n, heads, kv_rank, rot_dim, float(scale), w, _ptr(sink), self.code, self._stream())
 
     def _attention_latent_split(self, q, out, pages, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim,
-                                scale, max_context, kv_tokens) -> bool:
+                                scale, window, sink, max_context, kv_tokens) -> bool:
         """Steps of single tokens: each row's keys dealt out to workgroups in runs of 256 positions, every workgroup
         serving 16 heads from key rows staged in LDS; False when the sizes are not served (the general kernel runs)."""
-        need = int(self.lib.dll.mv_attention_latent_split_workspace(n, heads, kv_rank, max_context))
+        need = int(self.lib.dll.mv_attention_latent_split_workspace(n, heads, kv_rank, max_context, window))
         if self._latent_work is None or self._latent_work.numel() < need:
             if torch.cuda.is_current_stream_capturing():
                 return False                                   # no allocation inside a capture
@@ -1399,7 +1412,7 @@ class Ops:
         dk = kv_rank + rot_dim
         if not self.lib.offer("mv_attention_latent_split", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank,
                               pages.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(),
-                              token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), int(max_context),
+                              token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), window, _ptr(sink), int(max_context),
                               self._latent_work.data_ptr(), self._latent_work.numel(), self.code, self._stream()):
             return False
         self._note("mv_attention_latent_split", self._size(q, out) + kv_tokens * dk * pages.element_size(), 0)
@@ -1668,7 +1681,7 @@ class Ops:
     def norm_add_norm(self, y: torch.Tensor, norm_y, resid: torch.Tensor, norm_next, out: Optional[torch.Tensor],
                       shift: Optional[tuple] = None) -> None:
         """resid += rmsnorm(y) * w (``norm_y`` = (weight, eps, unit_offset)); with ``norm_next`` of the same
-        form, out = rmsnorm(resid) * w'. The sum stays float32 in between.
+        form, out = rmsnorm(resid) * w'; without it, out = resid rounded. The sum stays float32 in between.
 
         ``shift`` = (mix, state [slots, h], token_seq, state_slots), for steps in which every request brings
         one token: ``out`` gets the rows after the token shift that ``token_shift`` would apply to them (row r
@@ -1683,19 +1696,18 @@ class Ops:
             raise KernelLibraryError(f"norm_add_norm: weight of {wa.numel()} elements for rows of {h}")
         wb, eps_b, unit_b, wb_code = None, 1.0, False, DTYPE_F32
         if out is not None:
-            if norm_next is None:
-                raise KernelLibraryError("norm_add_norm: an output needs the second norm")
             self._act(out, "norm output")
-            wb, eps_b, unit_b = norm_next
-            _dev(wb, "norm weight")
-            wb_code = _weight_code(wb, "norm weight")
-            if wb.numel() != h or not wb.is_contiguous() or tuple(out.shape) != (n, h) or not out.is_contiguous():
+            if norm_next is not None:
+                wb, eps_b, unit_b = norm_next
+                _dev(wb, "norm weight")
+                wb_code = _weight_code(wb, "norm weight")
+            if (wb is not None and (wb.numel() != h or not wb.is_contiguous())) or tuple(out.shape) != (n, h) or not out.is_contiguous():
                 raise KernelLibraryError("norm_add_norm: the second norm's weight or output does not fit")
         mix = state = tsq = slots = None
         mix_code = DTYPE_F32
         if shift is not None:
             mix, state, tsq, slots = shift
-            if out is None:
+            if out is None or wb is None:
                 raise KernelLibraryError("norm_add_norm: a token shift needs the second norm and its output")
             self._act(state, "shift state"); _dev(mix, "shift weight")
             mix_code = _weight_code(mix, "shift weight")
@@ -1707,6 +1719,263 @@ class Ops:
                       _weight_code(wa, "norm weight"), float(eps_a), int(unit_a), resid.data_ptr(), _ptr(wb), wb_code,
                       float(eps_b), int(unit_b), _ptr(out), n, h, _ptr(mix), mix_code, _ptr(state), _ptr(tsq), _ptr(slots),
                       self.code, self._stream())
+
+    def squared_relu(self, x: torch.Tensor) -> None:
+        """In place: x <- max(x, 0)^2 (contiguous rows of the activation type)."""
+        self._act(x, "rows")
+        if not x.is_contiguous():
+            raise KernelLibraryError("squared_relu: contiguous rows are needed")
+        if x.numel() == 0:
+            return
+        self._note("mv_squared_relu", 2 * self._size(x), 2 * x.numel())
+        self.lib.call("mv_squared_relu", x.data_ptr(), x.numel(), self.code, self._stream())
+
+    def round_rows(self, x: torch.Tensor, out: torch.Tensor) -> None:
+        """out = x float32, rounded to the activation type (contiguous)."""
+        _dev(x, "rows"); self._act(out, "rounded rows")
+        if x.dtype != torch.float32 or not x.is_contiguous() or not out.is_contiguous() or out.shape != x.shape:
+            raise KernelLibraryError("round_rows: contiguous float32 rows and rows of the same shape are needed")
+        if x.numel() == 0:
+            return
+        self._note("mv_round_rows", self._size(x, out), 0)
+        self.lib.call("mv_round_rows", x.data_ptr(), out.data_ptr(), x.numel(), self.code, self._stream())
+
+    # ------------------------------------------------------------------------------------
+    # projections behind a short convolution; gated linear attention; the real-gated linear recurrent unit
+    # ------------------------------------------------------------------------------------
+    def _conv_operands(self, token_seq: torch.Tensor, rows: torch.Tensor, base: int, num_heads: int, num_kv_heads: int, head_dim: int,
+                       value_dim: int, taps_t: torch.Tensor, conv_state: Optional[torch.Tensor], positions: torch.Tensor,
+                       cu_seqlens: torch.Tensor, state_slots: torch.Tensor, n_seqs: int, rope_table: Optional[torch.Tensor],
+                       unit_norm: bool, eps: float, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
+                       page_size: int, out: torch.Tensor) -> dict:
+        self._act(rows, "qkv rows"); self._act(k_pages, "key pages"); self._act(v_pages, "value pages"); self._act(out, "convolved rows")
+        n = rows.shape[0]
+        q_dim, k_dim, v_dim = num_heads * head_dim, num_kv_heads * head_dim, num_kv_heads * value_dim
+        C, taps = q_dim + k_dim + v_dim, taps_t.shape[0]
+        if rows.dim() != 2 or rows.stride(1) != 1 or rows.shape[1] < base + C or out.dim() != 2 or out.shape[0] != n or out.stride(1) != 1 \
+                or out.shape[1] < q_dim + v_dim:
+            raise KernelLibraryError(f"qkv_conv_store: rows {tuple(rows.shape)} / {tuple(out.shape)} are too short")
+        if tuple(k_pages.shape[1:]) != (num_kv_heads, page_size, head_dim) or tuple(v_pages.shape[1:]) != (num_kv_heads, value_dim, page_size) \
+                or not k_pages.is_contiguous() or not v_pages.is_contiguous():
+            raise KernelLibraryError(f"qkv_conv_store: pages {tuple(k_pages.shape)} / {tuple(v_pages.shape)} do not match "
+                                     f"[pages, {num_kv_heads}, {page_size}, {head_dim}] / [pages, {num_kv_heads}, {value_dim}, {page_size}]")
+        _dev(taps_t, "convolution taps"); _dev(block_table, "block table")
+        if taps_t.dtype != torch.float32 or tuple(taps_t.shape) != (taps, C) or not taps_t.is_contiguous():
+            raise KernelLibraryError(f"qkv_conv_store: the taps must be contiguous float32 [taps, {C}]")
+        self._conv_state("qkv_conv_store", conv_state, taps, C)
+        if block_table.dtype != torch.int32 or block_table.dim() != 2 or not block_table.is_contiguous():
+            raise KernelLibraryError("qkv_conv_store: the block table must be a contiguous int32 matrix")
+        rot = 0
+        if rope_table is not None:
+            _dev(rope_table, "rope table")
+            rot = rope_table.shape[1]
+            if rope_table.dtype != torch.float32 or rope_table.dim() != 2 or not rope_table.is_contiguous() or rot > head_dim or rot % 2:
+                raise KernelLibraryError("qkv_conv_store: the rope table must be contiguous float32 [positions, rot <= head_dim]")
+        self._ints(n, positions=(positions, n), token_seq=(token_seq, n), cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        return {"rows": rows.data_ptr(), "ld": rows.stride(0) if n > 1 else rows.shape[1], "base": int(base), "n": n, "n_seqs": n_seqs,
+                "sizes": (num_heads, num_kv_heads, head_dim, value_dim, taps), "w": taps_t.data_ptr(), "conv_state": _ptr(conv_state),
+                "positions": positions.data_ptr(), "cu_seqlens": cu_seqlens.data_ptr(), "state_slots": state_slots.data_ptr(),
+                "block_table": block_table.data_ptr(), "bt_width": block_table.shape[1], "page_size": page_size,
+                "k_pages": k_pages.data_ptr(), "v_pages": v_pages.data_ptr(), "table": _ptr(rope_table), "rot": rot,
+                "unit_norm": int(bool(unit_norm)), "eps": float(eps), "out": out.data_ptr(), "ldo": out.stride(0) if n > 1 else out.shape[1],
+                "bytes": n * (2 * C * rows.element_size() + 4 * rot), "flops": n * C * (2 * taps + 6)}
+
+    def _conv_state(self, what: str, conv_state: Optional[torch.Tensor], taps: int, channels: int) -> None:
+        if taps > 1:
+            if conv_state is None:
+                raise KernelLibraryError(f"{what}: {taps} taps need the kept inputs")
+            self._act(conv_state, "convolution state")
+            if conv_state.dim() != 3 or tuple(conv_state.shape[1:]) != (taps - 1, channels) or not conv_state.is_contiguous():
+                raise KernelLibraryError(f"{what}: the convolution's state must be [slots, {taps - 1}, {channels}]")
+
+    def qkv_conv_store(self, token_seq: torch.Tensor, single: bool, **args) -> None:
+        """On ``rows`` with q, k and v side by side from column ``base`` on: a causal convolution over time per channel
+        (``taps_t`` float32 [taps, channels], the last tap the current token's; ``conv_state`` [slots, taps - 1, channels] the
+        request's inputs in front of the step, advanced); then q and k heads are rotated over their first channels
+        (``rope_table``) and, with ``unit_norm``, divided by their root mean square. q goes to the first columns of ``out``, k and
+        v (``value_dim`` a head) to the cache pages; the rows stay as they are (columns of ``out`` behind the queries are room
+        for the values). ``single``: the step has one row of each request."""
+        a = self._conv_operands(token_seq, **args)
+        if a["n"] == 0:
+            return
+        self._note("mv_qkv_conv_store", a["bytes"], a["flops"])
+        self.lib.call("mv_qkv_conv_store", a["rows"], a["ld"], a["base"], a["n"], a["n_seqs"], *a["sizes"], a["w"], a["conv_state"],
+                      int(bool(single)), a["positions"], token_seq.data_ptr(), a["cu_seqlens"], a["state_slots"], a["block_table"],
+                      a["bt_width"], a["page_size"], a["k_pages"], a["v_pages"], a["table"], a["rot"], a["unit_norm"], a["eps"], a["out"],
+                      a["ldo"], self.code, self._stream())
+
+    def _gated_linear_rows(self, what: str, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, bias: torch.Tensor,
+                           token_seq: torch.Tensor) -> int:
+        self._act(packed, "mixer rows"); _dev(bias, "decay bias")
+        n = packed.shape[0]
+        if packed.dim() != 2 or packed.stride(1) != 1 or packed.shape[1] < offset + 2 * heads * (dk + dv):
+            raise KernelLibraryError(f"{what}: rows {tuple(packed.shape)} are too short")
+        if bias.dtype != torch.float32 or bias.numel() != heads * dk or not bias.is_contiguous():
+            raise KernelLibraryError(f"{what}: the decay's bias must be float32 [{heads * dk}]")
+        self._ints(n, token_seq=(token_seq, n))
+        return n
+
+    def gated_linear_chunk_tokens(self) -> int:
+        """Tokens in a chunk of ``gated_linear_chunks``."""
+        return int(self.lib.dll.mv_gated_linear_chunk_tokens())
+
+    def gated_linear_chunks(self, packed: torch.Tensor, offset: int, heads: int, dk: int, dv: int, z: torch.Tensor, bias: torch.Tensor,
+                            tau: float, state: torch.Tensor, token_seq: torch.Tensor, cu_seqlens: torch.Tensor,
+                            state_slots: torch.Tensor, n_seqs: int, chunks: int, sums: torch.Tensor, decays: torch.Tensor,
+                            out: torch.Tensor) -> None:
+        """Per request and head over the step's tokens: S <- diag(a) S + k v^T; out = S^T q, with [q | k (heads*dk each) |
+        v (heads*dv)] the rows' columns from ``offset`` on, q times dk^-1/2, and a = sigmoid(z + bias)^(1 / tau) (z float32
+        [n, heads*dk]), as products over chunks of tokens. ``chunks``: how many chunks of ``gated_linear_chunk_tokens`` the
+        requests' rows form (or more); sums float32 [chunks, heads, dv, dk] and decays [chunks, heads, dk] are scratch. state
+        float32 [slots, heads, dv, dk] is read and left advanced; out float32 [n, heads, dv]."""
+        n = self._gated_linear_rows("gated_linear_chunks", packed, offset, heads, dk, dv, bias, token_seq)
+        self._matrix_state("gated_linear_chunks", state, heads, dv, dk)
+        for t, shape, name in ((sums, (chunks, heads, dv, dk), "chunk sums"), (decays, (chunks, heads, dk), "chunk decays"),
+                               (out, (n, heads, dv), "outputs"), (z, (n, heads * dk), "decay rows")):
+            _dev(t, name)
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"gated_linear_chunks: the {name} must be contiguous float32 {shape}")
+        self._ints(n, cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        if n == 0:
+            return
+        C = self.gated_linear_chunk_tokens()
+        self._note("mv_gated_linear_chunks", n * heads * (2 * dk + dv) * packed.element_size() + self._size(out, z)
+                   + 2 * min(n_seqs, max(n, 1)) * heads * dv * dk * 4, n * heads * (4 * dk * dv + C * (dk + dv)))
+        self.lib.call("mv_gated_linear_chunks", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(offset), n, heads,
+                      dk, dv, z.data_ptr(), z.stride(0) if n > 1 else z.shape[1], bias.data_ptr(), float(tau), state.data_ptr(),
+                      cu_seqlens.data_ptr(), state_slots.data_ptr(), n_seqs, int(chunks), sums.data_ptr(), decays.data_ptr(),
+                      out.data_ptr(), self.code, self._stream())
+
+    def gated_linear_step(self, packed: torch.Tensor, offset: int, low_offset: int, heads: int, dk: int, dv: int, a2t: torch.Tensor,
+                          bias: torch.Tensor, tau: float, weight: torch.Tensor, eps: float, state: torch.Tensor,
+                          token_seq: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor, beside: Optional[dict] = None) -> int:
+        """For a step in which every request brings one token: the decays (W_a1 h from column ``low_offset`` on, a2t [rank,
+        heads*dk] the transposed second matrix), the recurrence, the head's norm (``weight`` float32 [dv]) and the gate silu(g)
+        (g behind v) of one (row, head) in one workgroup, into ``out`` [n, heads*dv]. ``beside``: the arguments of a
+        ``qkv_conv_store`` on the same rows that runs in the same launch where it can. 0: the sizes are not served and nothing
+        was done; 1: it ran; 2: it ran together with ``beside``."""
+        n = self._gated_linear_rows("gated_linear_step", packed, offset, heads, dk, dv, bias, token_seq)
+        rank = a2t.shape[0]
+        self._act(out, "mixer output"); _dev(weight, "output norm weight"); _dev(a2t, "second decay matrix")
+        if tuple(out.shape) != (n, heads * dv) or out.stride(1) != 1 or weight.dtype != torch.float32 or weight.numel() != dv \
+                or not weight.is_contiguous() or tuple(a2t.shape) != (rank, heads * dk) or not a2t.is_contiguous() \
+                or packed.shape[1] < low_offset + rank:
+            raise KernelLibraryError("gated_linear_step: operands do not fit")
+        self._matrix_state("gated_linear_step", state, heads, dv, dk)
+        self._ints(n, state_slots=(state_slots, 1))
+        if n == 0:
+            return 1
+        mine = (packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(offset), int(low_offset), n, heads, dk, dv, rank,
+                a2t.data_ptr(), _weight_code(a2t, "second decay matrix"), bias.data_ptr(), float(tau), weight.data_ptr(), float(eps),
+                state.data_ptr(), token_seq.data_ptr(), state_slots.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else heads * dv)
+        nothing = (0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0, 0.0, 0, 0)
+        ran = 0
+        extra = 0
+        if beside is not None:
+            a = self._conv_operands(token_seq, **beside)
+            if self.lib.offer("mv_gated_linear_step", *mine, a["rows"], a["ld"], a["base"], *a["sizes"], a["w"], a["conv_state"],
+                              a["positions"], a["cu_seqlens"], a["block_table"], a["bt_width"], a["page_size"], a["k_pages"], a["v_pages"],
+                              a["table"], a["rot"], a["unit_norm"], a["eps"], a["out"], a["ldo"], self.code, self._stream()):
+                ran, extra = 2, a["bytes"]
+        if not ran and self.lib.offer("mv_gated_linear_step", *mine, *nothing, self.code, self._stream()):
+            ran = 1
+        if ran:
+            self._note("mv_gated_linear_step", n * (heads * (2 * dk + 3 * dv) + rank) * packed.element_size() + self._size(a2t)
+                       + 2 * n * heads * dv * dk * 4 + extra, n * heads * (4 * dv * dk + 2 * rank * dk))
+        return ran
+
+    def short_conv(self, rows: torch.Tensor, channels: int, taps_t: torch.Tensor, bias: Optional[torch.Tensor],
+                   conv_state: Optional[torch.Tensor], token_seq: torch.Tensor, cu_seqlens: torch.Tensor, state_slots: torch.Tensor,
+                   n_seqs: int, out: torch.Tensor) -> None:
+        """out [n, channels] = a causal convolution over time of the rows' first ``channels`` columns (``taps_t`` float32
+        [taps, channels], the last tap the current token's) plus ``bias`` (float32 [channels] or None). conv_state [slots,
+        taps - 1, channels]: the request's inputs in front of the step, advanced."""
+        self._act(rows, "rows"); self._act(out, "convolved rows"); _dev(taps_t, "convolution taps")
+        n, taps = rows.shape[0], taps_t.shape[0]
+        if rows.dim() != 2 or rows.stride(1) != 1 or rows.shape[1] < channels or tuple(out.shape) != (n, channels) or out.stride(1) != 1:
+            raise KernelLibraryError(f"short_conv: rows {tuple(rows.shape)} / {tuple(out.shape)} do not fit {channels} channels")
+        if taps_t.dtype != torch.float32 or tuple(taps_t.shape) != (taps, channels) or not taps_t.is_contiguous():
+            raise KernelLibraryError(f"short_conv: the taps must be contiguous float32 [taps, {channels}]")
+        if bias is not None:
+            _dev(bias, "convolution bias")
+            if bias.dtype != torch.float32 or bias.numel() != channels or not bias.is_contiguous():
+                raise KernelLibraryError(f"short_conv: the bias must be float32 [{channels}]")
+        self._conv_state("short_conv", conv_state, taps, channels)
+        self._ints(n, token_seq=(token_seq, n), cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        if n == 0:
+            return
+        self._note("mv_short_conv", 2 * n * channels * rows.element_size(), 2 * n * channels * taps)
+        self.lib.call("mv_short_conv", rows.data_ptr(), rows.stride(0) if n > 1 else rows.shape[1], n, n_seqs, channels, taps,
+                      taps_t.data_ptr(), _ptr(bias), _ptr(conv_state), token_seq.data_ptr(), cu_seqlens.data_ptr(),
+                      state_slots.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else channels, self.code, self._stream())
+
+    def unit_chunk_tokens(self) -> int:
+        """Tokens in a chunk of ``unit_scan``."""
+        return int(self.lib.dll.mv_unit_chunk_tokens())
+
+    def _unit_operands(self, what: str, packed: torch.Tensor, y_offset: int, blocks: int, gate_bias: torch.Tensor, rate: torch.Tensor,
+                       state: torch.Tensor, token_seq: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor):
+        self._act(packed, "mixer rows"); self._act(out, "mixer output"); _dev(state, "unit state")
+        n, W = out.shape
+        if packed.dim() != 2 or packed.shape[0] != n or packed.stride(1) != 1 or packed.shape[1] < y_offset + W or y_offset < W \
+                or out.stride(1) != 1 or W % blocks:
+            raise KernelLibraryError(f"{what}: rows {tuple(packed.shape)} / {tuple(out.shape)} do not fit")
+        for t, shape, name in ((gate_bias, (2, W), "gate biases"), (rate, (W,), "decay rates")):
+            _dev(t, name)
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"{what}: the {name} must be contiguous float32 {shape}")
+        if state.dtype != torch.float32 or state.dim() != 2 or state.shape[1] != W or not state.is_contiguous():
+            raise KernelLibraryError(f"{what}: the state must be float32 [slots, {W}]")
+        self._ints(n, token_seq=(token_seq, n), state_slots=(state_slots, 1))
+        return n, W
+
+    def unit_scan(self, z: torch.Tensor, u: torch.Tensor, packed: torch.Tensor, y_offset: int, blocks: int, gate_bias: torch.Tensor,
+                  rate: torch.Tensor, state: torch.Tensor, token_seq: torch.Tensor, cu_seqlens: torch.Tensor,
+                  state_slots: torch.Tensor, n_seqs: int, chunks: int, sums: torch.Tensor, out: torch.Tensor) -> None:
+        """Per request and channel over the step's tokens: log a = rate sigmoid(zr + br), S <- a S + sqrt(1 - a^2)
+        sigmoid(zi + bi) u, out = S gelu_tanh(y), with z float32 [n, blocks, 2 * width / blocks] (a block's zr in front of its zi),
+        gate_bias float32 [2, width], u [n, width], y the rows' columns from ``y_offset`` on. ``chunks``: how many chunks of
+        ``unit_chunk_tokens`` the requests' rows form (or more); sums float32 [chunks, 2, width] is scratch. state float32
+        [slots, width] is read and left advanced."""
+        n, W = self._unit_operands("unit_scan", packed, y_offset, blocks, gate_bias, rate, state, token_seq, state_slots, out)
+        self._act(u, "convolved rows")
+        if tuple(u.shape) != (n, W) or u.stride(1) != 1:
+            raise KernelLibraryError(f"unit_scan: convolved rows {tuple(u.shape)} are not [{n}, {W}]")
+        for t, shape, name in ((z, (n, blocks, 2 * W // blocks), "gate products"), (sums, (chunks, 2, W), "chunk sums")):
+            _dev(t, name)
+            if t.dtype != torch.float32 or tuple(t.shape) != shape or not t.is_contiguous():
+                raise KernelLibraryError(f"unit_scan: the {name} must be contiguous float32 {shape}")
+        self._ints(n, cu_seqlens=(cu_seqlens, n_seqs + 1), state_slots=(state_slots, n_seqs))
+        if n == 0:
+            return
+        self._note("mv_unit_scan", self._size(z, u, out) + n * W * packed.element_size() + 2 * min(n_seqs, n) * W * 4, 40 * n * W)
+        self.lib.call("mv_unit_scan", z.data_ptr(), u.data_ptr(), u.stride(0) if n > 1 else W, packed.data_ptr(),
+                      packed.stride(0) if n > 1 else packed.shape[1], int(y_offset), n, W, blocks, gate_bias.data_ptr(), rate.data_ptr(),
+                      state.data_ptr(), cu_seqlens.data_ptr(), state_slots.data_ptr(), n_seqs, int(chunks), sums.data_ptr(),
+                      out.data_ptr(), out.stride(0) if n > 1 else W, self.code, self._stream())
+
+    def unit_step(self, packed: torch.Tensor, y_offset: int, blocks: int, taps_t: torch.Tensor, conv_bias: torch.Tensor,
+                  conv_state: Optional[torch.Tensor], gate_rows: torch.Tensor, gate_cols: torch.Tensor, gate_bias: torch.Tensor,
+                  rate: torch.Tensor, state: torch.Tensor, token_seq: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor) -> bool:
+        """For a step in which every request brings one token: ``short_conv``, both gates' products (gate_cols [blocks, inputs,
+        2 * outputs], gate_rows the same with outputs and inputs changed over) and ``unit_scan`` as one kernel. False when the
+        sizes are not served (nothing was done)."""
+        n, W = self._unit_operands("unit_step", packed, y_offset, blocks, gate_bias, rate, state, token_seq, state_slots, out)
+        P, taps = W // blocks, taps_t.shape[0]
+        _dev(taps_t, "convolution taps"); _dev(conv_bias, "convolution bias"); _dev(gate_cols, "gate matrices")
+        if taps_t.dtype != torch.float32 or tuple(taps_t.shape) != (taps, W) or not taps_t.is_contiguous() \
+                or conv_bias.dtype != torch.float32 or conv_bias.numel() != W or not conv_bias.is_contiguous() \
+                or tuple(gate_cols.shape) != (blocks, P, 2 * P) or not gate_cols.is_contiguous():
+            raise KernelLibraryError("unit_step: operands do not fit")
+        self._conv_state("unit_step", conv_state, taps, W)
+        if not self.lib.offer("mv_unit_step", packed.data_ptr(), packed.stride(0) if n > 1 else packed.shape[1], int(y_offset), n, W, blocks,
+                              taps, taps_t.data_ptr(), conv_bias.data_ptr(), _ptr(conv_state), gate_cols.data_ptr(),
+                              _weight_code(gate_cols, "gate matrices"), gate_bias.data_ptr(), rate.data_ptr(), state.data_ptr(),
+                              token_seq.data_ptr(), state_slots.data_ptr(), out.data_ptr(), out.stride(0) if n > 1 else W, self.code,
+                              self._stream()):
+            return False
+        self._note("mv_unit_step", n * W * (3 + 2 * taps) * packed.element_size() + self._size(gate_cols) + 8 * n * W, 4 * n * W * P)
+        return True
 
     def soft_cap(self, logits: torch.Tensor, cap: float) -> None:
         """In place on float32 [rows, cols]: x <- cap * tanh(x / cap)."""

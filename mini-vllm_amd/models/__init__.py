@@ -6,4 +6,5 @@ from . import dutilix  # registers "Dutilix"
 from . import zedudra  # registers "Zedudra"
 from . import furanex  # registers "Furanex"
 from . import sorulix  # registers "Sorulix"
+from . import setirax  # registers "Setirax"
 from .causal_lm import CausalLM, expected_tensors

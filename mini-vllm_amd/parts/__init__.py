@@ -7,12 +7,13 @@ from .plan import Call, EmbeddingSpec, HeadSpec, LayerPlan, ModelPlan, TensorLoc
 from .norm import RMSNorm, RMSNormSpec
 from .rope import RotaryEmbedding, RotarySpec, inverse_frequencies
 from .attention import Attention, AttentionSpec
-from .mlp import ClampedGLU, ClampedGLUSpec, SwiGLU, SwiGLUSpec
-from .block import PreNormBlock, PreNormBlockSpec, SandwichBlock, SandwichBlockSpec
+from .mlp import ClampedGLU, ClampedGLUSpec, SquaredReLU, SquaredReLUSpec, SwiGLU, SwiGLUSpec
+from .block import (PostNormBlock, PostNormBlockSpec, PreNormBlock, PreNormBlockSpec, SandwichBlock, SandwichBlockSpec)
 from .delta_rule import DeltaRule, DeltaRuleSpec
 from .matrix_state import (MLSTM, ChannelDelta, ChannelDeltaSpec, ConstantDecay, ConstantDecaySpec, GatedDelta, GatedDeltaSpec,
-                           MLSTMSpec)
+                           GatedLinear, GatedLinearSpec, MLSTMSpec)
 from .parallel import ParallelMixer, ParallelMixerSpec
+from .recurrent_unit import RecurrentUnit, RecurrentUnitSpec
 from .entry import PassEntry, PassEntrySpec
 from .latent_attention import LatentAttention, LatentAttentionSpec, LatentNeed
 from .moe import RoutedExperts, RoutedExpertsSpec

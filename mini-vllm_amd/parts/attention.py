@@ -33,6 +33,12 @@ multiplied by weights as long as the projections (``q_norm``, ``k_norm``). With 
 takes 2^(-8 (h + 1) / H) times the distance between query and key off its score; ``sink``: the softmax's denominator
 is 1 + sum exp(s). Softmax weighting with ``row_norm`` runs ``attend_scored``, which another part may call with a
 packed row of its own (``parts/parallel.py``).
+
+``conv_taps`` >= 1: a short causal convolution over time on each channel of q, k and v (no activation) comes directly behind
+the projection; the last ``conv_taps - 1`` projected rows of a request are its state. With it rotation over the first channels
+of a head (any number), ``unit_norm_after_rotation``, ``softcap``, a window, values of any size, and ``out_scale``, a constant
+on the heads' outputs (they are linear in the values, so it goes into the values' taps). Softmax weighting with ``conv_taps``
+runs ``conv_store`` and ``attend_scored``, which another part may call like those of ``row_norm``.
 """
 from __future__ import annotations
 
@@ -78,6 +84,17 @@ class AttentionSpec(PartSpec):
     softcap: Optional[float] = None
     distance_bias: bool = False
     sink: bool = False
+    conv_taps: int = 0                       # 0: no convolution; 1 scales each channel
+    out_scale: float = 1.0                   # with a convolution: on the heads' outputs
+
+    @property
+    def convolved(self) -> bool:
+        """Softmax over all keys or a window on projections that pass a short convolution."""
+        return self.conv_taps > 0
+
+    @property
+    def conv_channels(self) -> int:
+        return self.q_dim + self.kv_dim + self.v_dim
 
     @property
     def q_dim(self) -> int:
@@ -104,7 +121,7 @@ class AttentionSpec(PartSpec):
         """The reference's layer: softmax over all keys or a window, values as large as keys."""
         return (self.weighting == "softmax" and not self.scored and self.chunk is None and self.value_dim in (None, self.head_dim)
                 and not self.head_gate and not self.score_bias and not self.keep_first and not self.value_from_key
-                and not self.unit_norm_after_rotation and self.value_mix is None and not self.scored)
+                and not self.unit_norm_after_rotation and self.value_mix is None and not self.scored and not self.convolved)
 
     @property
     def scored(self) -> bool:
@@ -116,7 +133,7 @@ class AttentionSpec(PartSpec):
         """Softmax with the unit norm behind the rotation, values shared between layers, or values of a size of their own."""
         return (self.weighting == "softmax" and not self.scored and self.chunk is None and not self.score_bias and not self.bias
                 and not self.qk_norm and not self.head_gate and not self.keep_first and not self.value_from_key
-                and not self.shares_kv
+                and not self.shares_kv and not self.convolved
                 and (self.unit_norm_after_rotation or self.value_mix is not None or self.value_dim not in (None, self.head_dim)))
 
     @property
@@ -124,7 +141,7 @@ class AttentionSpec(PartSpec):
         """Softmax over a window (or all keys) with kept first positions, head gates or values taken from the keys."""
         return (self.weighting == "softmax" and not self.scored and self.chunk is None and self.value_dim in (None, self.head_dim)
                 and not self.score_bias and not self.bias and not self.qk_norm and not self.plain and not self.rotated
-                and not self.unit_norm_after_rotation and self.value_mix is None)
+                and not self.unit_norm_after_rotation and self.value_mix is None and not self.convolved)
 
 
 @register_mixer(AttentionSpec.kind)
@@ -152,6 +169,9 @@ class Attention(Mixer):
             if not spec.shares_kv:
                 t["k_bias"] = TensorDecl((spec.kv_dim,), init="zeros_normal")
                 t["v_bias"] = TensorDecl((spec.kv_dim,), init="zeros_normal")
+        if spec.convolved:
+            for name, rows in (("q", spec.q_dim), ("k", spec.kv_dim), ("v", spec.v_dim)):
+                t[name + "_conv"] = TensorDecl((rows, spec.conv_taps))
         if spec.row_norm:
             t["q_norm"] = TensorDecl((spec.q_dim,), init="ones_normal")
             t["k_norm"] = TensorDecl((spec.kv_dim,), init="ones_normal")
@@ -178,6 +198,11 @@ class Attention(Mixer):
         return KeyValueNeed(retention=retention, num_kv_heads=spec.num_kv_heads, head_dim=spec.head_dim,
                             value_dim=spec.value_dim)
 
+    @classmethod
+    def state_shapes(cls, spec: AttentionSpec):
+        # the projections' rows of the request's last taps - 1 tokens, in the activation type (None: the runtime's)
+        return {"conv": ((spec.conv_taps - 1, spec.conv_channels), None)} if spec.conv_taps > 1 else {}
+
     def __init__(self, spec: AttentionSpec, tensors: Dict[str, torch.Tensor], rt: Runtime,
                  position: Optional[object] = None):
         if spec.num_heads % spec.num_kv_heads:
@@ -186,11 +211,21 @@ class Attention(Mixer):
             raise ValueError(f"attention weighting must be 'softmax' or 'sigmoid', got {spec.weighting!r}")
         if spec.value_mix not in (None, "source", "blend") or (spec.value_mix and not spec.value_mix_key):
             raise ValueError(f"value_mix must be None, 'source' or 'blend' with a key, got {spec.value_mix!r}, {spec.value_mix_key!r}")
-        if (spec.unit_norm_after_rotation or spec.value_mix) and not spec.rotated:
+        if (spec.unit_norm_after_rotation or spec.value_mix) and not spec.rotated and not spec.convolved:
             raise NotImplementedError("the unit norm behind the rotation and values shared between layers are built for softmax "
                                       "weighting over all keys or a window, without biases, weighted q/k norms, gates or a shared cache")
-        if (spec.query_temperature or spec.softcap is not None or spec.distance_bias or spec.sink) and not spec.scored:
+        if (spec.query_temperature or spec.distance_bias or spec.sink or (spec.softcap is not None and not spec.convolved)) \
+                and not spec.scored:
             raise NotImplementedError("query temperature, capped scores, a distance bias and a sink are built behind the whole-row norm")
+        if spec.convolved:
+            if (spec.weighting != "softmax" or spec.scored or spec.chunk is not None or spec.score_bias or spec.head_gate
+                    or spec.keep_first or spec.value_from_key or spec.value_mix is not None or spec.bias or spec.qk_norm
+                    or spec.shares_kv or (spec.softcap is not None and not spec.softcap > 0)):
+                raise NotImplementedError("a convolution behind the projections is built for softmax weighting over all keys or a "
+                                          "window, without biases, gates, weighted norms, shared values or a shared cache, with a "
+                                          "positive soft cap or none")
+        elif spec.out_scale != 1.0:
+            raise NotImplementedError("out_scale is built into the taps of a convolution")
         if spec.scored:
             if (spec.weighting != "softmax" or spec.chunk is not None or spec.score_bias or spec.head_gate or spec.keep_first
                     or spec.value_from_key or spec.unit_norm_after_rotation or spec.value_mix is not None or spec.bias or spec.qk_norm
@@ -199,7 +234,7 @@ class Attention(Mixer):
                                           "rotation, biases, gates, per-head norms or a shared cache")
             if (spec.softcap is not None and not spec.softcap > 0) or (spec.query_temperature and spec.query_temperature[1] < 1):
                 raise ValueError("a soft cap is positive and the query temperature changes every >= 1 positions")
-        elif not spec.plain and not spec.kept and not spec.rotated and (spec.weighting != "sigmoid" or spec.bias):
+        elif not spec.convolved and not spec.plain and not spec.kept and not spec.rotated and (spec.weighting != "sigmoid" or spec.bias):
             raise NotImplementedError("chunks, a value size of its own and a score bias are built for sigmoid weighting "
                                       "without projection biases; kept first positions, head gates and values taken from "
                                       "the keys also for softmax weighting without biases and query/key norms")
@@ -226,6 +261,13 @@ class Attention(Mixer):
         self.q_norm = tensors.get("q_norm")
         self.k_norm = tensors.get("k_norm")
         self.value_mix = tensors.get("value_mix")
+        self.conv_t = None
+        if spec.convolved:
+            # tap by tap, [taps, channels], float32: eight channels' weights of a tap are one load, and the constant on the
+            # outputs costs the values no rounding of their own
+            taps = [tensors[name + "_conv"].to(torch.float32) for name in ("q", "k", "v")]
+            taps[2] = taps[2] * spec.out_scale
+            self.conv_t = torch.cat(taps, dim=0).t().contiguous()
         # distance slopes are a property of the head count alone
         self.slopes = None
         if spec.distance_bias:
@@ -264,6 +306,14 @@ class Attention(Mixer):
             attn = self.attend_scored(packed, 0, ctx, call)
             y = rt.workspace.get("mixer.out", (n, spec.hidden_size), rt.dtype)
             return ops.gemm(attn, self.w_o, y, self.b_o, defer_sum=True, fold=fold) or y
+        if spec.convolved:
+            n = x.shape[0]
+            packed = rt.workspace.get("attn.qkv", (n, self.width), rt.dtype)
+            ops.gemm(x, self.w_qkv, packed)
+            rows = self.conv_store(packed, 0, ctx, call)
+            attn = self.attend_scored(rows, 0, ctx, call)
+            y = rt.workspace.get("mixer.out", (n, spec.hidden_size), rt.dtype)
+            return ops.gemm(attn, self.w_o, y, defer_sum=True, fold=fold) or y
         if spec.rotated:
             return self._forward_rotated(x, ctx, call)
         if spec.kept:
@@ -322,10 +372,31 @@ class Attention(Mixer):
     def norm_store(self, packed: torch.Tensor, offsets, ctx, call: int) -> None:
         self.rt.ops.qkv_row_norm_store(ctx.token_seq, **self.norm_store_args(packed, offsets, ctx, call))
 
-    def attend_scored(self, packed: torch.Tensor, q_offset: int, ctx, call: int) -> torch.Tensor:
-        """The heads' outputs [n, out_dim] for finished queries in ``packed`` and a finished cache."""
+    def conv_store_args(self, packed: torch.Tensor, base: int, ctx, call: int) -> dict:
+        """What ``ops.qkv_conv_store`` (or a kernel that runs it beside other work) takes for this mixer's projections from
+        column ``base`` on; the finished queries (and room for the values) are ``args["out"]``."""
+        spec, kv = self.spec, ctx.kv(call)
+        table, interleaved = self.rotary if self.rotary is not None else (None, False)
+        if interleaved or (self.position is not None and self.rotary is None):
+            raise NotImplementedError("a convolution behind the projections is followed by a rotary table with half-split pairs")
+        out = self.rt.workspace.get("attn.convolved", (packed.shape[0], spec.q_dim + spec.v_dim), self.rt.dtype)
+        return dict(rows=packed, base=base, num_heads=spec.num_heads, num_kv_heads=spec.num_kv_heads, head_dim=spec.head_dim,
+                    value_dim=spec.v_head_dim, taps_t=self.conv_t, conv_state=ctx.state(call, "conv") if spec.conv_taps > 1 else None,
+                    positions=ctx.positions, cu_seqlens=ctx.cu_seqlens, state_slots=ctx.state_slots, n_seqs=ctx.n_seqs,
+                    rope_table=table, unit_norm=spec.unit_norm_after_rotation, eps=spec.qk_norm_eps, k_pages=kv.k_pages,
+                    v_pages=kv.v_pages, block_table=kv.block_table, page_size=kv.page_size, out=out)
+
+    def conv_store(self, packed: torch.Tensor, base: int, ctx, call: int) -> torch.Tensor:
+        """Convolution, rotation, unit norm and cache write; returns rows whose first columns are the finished queries."""
+        args = self.conv_store_args(packed, base, ctx, call)
+        plan = ctx.attention_plan
+        self.rt.ops.qkv_conv_store(ctx.token_seq, single=plan is not None and plan.decode_only, **args)
+        return args["out"]
+
+    def attend_scored(self, packed: torch.Tensor, q_offset: int, ctx, call: int, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """The heads' outputs [n, out_dim] (in ``out`` when given) for finished queries in ``packed`` and a finished cache."""
         spec, rt, kv = self.spec, self.rt, ctx.kv(call)
-        attn = rt.workspace.get("attn.out", (packed.shape[0], spec.out_dim), rt.dtype)
+        attn = rt.workspace.get("attn.out", (packed.shape[0], spec.out_dim), rt.dtype) if out is None else out
         rt.ops.attention(packed[:, q_offset:q_offset + spec.q_dim], attn, kv.k_pages, kv.v_pages, kv.block_table, kv.page_size,
                          ctx.positions, ctx.token_seq, spec.num_heads, spec.num_kv_heads, spec.head_dim, spec.scale, spec.window,
                          plan=ctx.attention_plan, value_dim=spec.v_head_dim, softcap=spec.softcap, slopes=self.slopes, sink=spec.sink)

@@ -346,7 +346,7 @@ class HiddenStream:
     defer_sum=True)`` returned in its place (an output whose partial sums the norm's kernel adds
     up itself; it has ``shape``, ``materialize()`` and ``discard()``)."""
 
-    __slots__ = ("resid", "delta", "spare", "weighted", "normed", "lanes", "lanes_write")
+    __slots__ = ("resid", "delta", "spare", "weighted", "normed", "lanes", "lanes_write", "copy")
 
     def __init__(self, resid: torch.Tensor, spare: Optional[torch.Tensor] = None):
         self.resid = resid
@@ -355,6 +355,8 @@ class HiddenStream:
         # that made ``resid`` (a block that closes a sublayer and opens the next in one launch);
         # that norm takes them from here instead of running
         self.normed = None
+        # the rows of ``resid`` in the activation type, left by a block whose successor reads the residual itself
+        self.copy = None
         # rows that the last product already added to ``resid`` and left half normalised for the
         # norm that comes next (see NormFold); that norm takes them from here
         self.weighted = None

@@ -252,6 +252,82 @@ class TokenShiftEntry:
 
 
 @dataclass(frozen=True)
+class PostNormBlockSpec(PartSpec):
+    """Norms behind the sublayers only."""
+    kind = "post_norm"
+
+
+class PostNormEntry:
+    """What a post-norm block offers the block in front of it: it reads the residual itself, so that block's last kernel may
+    leave the residual's rows in the activation type as well."""
+
+
+@register_block(PostNormBlockSpec.kind)
+class PostNormBlock(Block):
+    """x = x + norm1(mixer(x)); x = x + norm2(ffn(x)); a layer without a feed-forward has only the first half. The sublayers
+    read the residual itself, rounded to the activation type: the kernel that adds a sublayer's normed output to the float32
+    residual leaves that copy too (``HiddenStream.copy``), so that between two sublayers there is one launch. In float32 the
+    residual is its own copy."""
+    norm_slots: Tuple[str, ...] = ("norm1", "norm2")
+    accepts_next_norm = True
+    wants_runtime = True
+
+    @classmethod
+    def slots_for(cls, has_ffn: bool) -> Tuple[str, ...]:
+        return cls.norm_slots if has_ffn else cls.norm_slots[:1]
+
+    def __init__(self, spec: PostNormBlockSpec, norms: Dict[str, Norm], mixer: Mixer, ffn: FeedForward, tensors=None, rt=None):
+        if rt is None:
+            raise ValueError("a post-norm block needs the runtime")
+        self.spec, self.rt, self.mixer, self.ffn = spec, rt, mixer, ffn
+        self.norm_mixer = norms["norm1"]
+        self.norm_ffn = norms["norm2"] if ffn is not None else None
+        for norm in (self.norm_mixer, self.norm_ffn):
+            if norm is not None and norm.as_scaled_rms() is None:
+                raise ValueError("the norms of a post-norm block must be plain scaled RMS norms")
+
+    def entry_part(self):
+        return PostNormEntry()
+
+    def _read(self, stream: HiddenStream, ctx) -> torch.Tensor:
+        """The residual's rows in the activation type."""
+        rows, stream.copy = stream.copy, None
+        stream.normed = None
+        if stream.delta is not None:               # a block of another kind in front left its last sum to us
+            delta = stream.delta
+            if not isinstance(delta, torch.Tensor):
+                delta = delta.materialize()
+            self.rt.ops.stream_entry(stream.resid, delta, None, None, None, None)
+            stream.delta, rows = None, None
+        if self.rt.dtype == torch.float32:
+            return stream.resid
+        if rows is None:
+            rows = self.rt.workspace.get("stream.copy", tuple(stream.resid.shape), self.rt.dtype)
+            self.rt.ops.round_rows(stream.resid, rows)
+        return rows
+
+    def forward(self, stream: HiddenStream, ctx, call: int, next_norm: Optional[Norm] = None, next_part=None) -> None:
+        if stream.lanes is not None or stream.weighted is not None:
+            raise RuntimeError("a post-norm block takes a plain residual stream")
+        last = self.ffn is None
+        y = self.mixer.forward(self._read(stream, ctx), ctx, call)
+        self._close(stream, y, self.norm_mixer, isinstance(next_part, PostNormEntry) if last else True)
+        if not last:
+            y = self.ffn.forward(self._read(stream, ctx), ctx)
+            self._close(stream, y, self.norm_ffn, isinstance(next_part, PostNormEntry))
+
+    def _close(self, stream: HiddenStream, y, norm: Norm, wants_copy: bool) -> None:
+        """resid += norm(y); the residual's rows in the activation type with it when the next sublayer reads them."""
+        if not isinstance(y, torch.Tensor):
+            y = y.materialize()
+        rows = None
+        if wants_copy and self.rt.dtype != torch.float32:
+            rows = self.rt.workspace.get("stream.copy", tuple(y.shape), self.rt.dtype)
+        self.rt.ops.norm_add_norm(y, norm.as_scaled_rms(), stream.resid, None, rows)
+        stream.delta, stream.normed, stream.copy = None, None, rows
+
+
+@dataclass(frozen=True)
 class HyperConnectionBlockSpec(PartSpec):
     """Pre-norm sublayers on ``streams`` residual streams of width ``hidden_size`` instead of one."""
     kind = "hyper_connections"

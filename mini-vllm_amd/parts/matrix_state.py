@@ -29,6 +29,11 @@ so the read-out sees the token's own write.
   their projections. All heads' o together are divided by their root mean square, multiplied by a weight over all
   channels and by sigmoid(W_g h).
 
+* ``gated_linear`` (gated linear attention): [delta] is off, b = 1, a is a vector over the key channels, S <- diag(a) S with
+  a = sigmoid(z)^(1 / tau), z = W_a2 (W_a1 h) + bias per head and channel; q = W_q h * key_dim^-1/2, k and v are plain
+  projections. o is divided by its root mean square per head, multiplied by a weight of ``value_dim`` numbers that the
+  heads share and by silu(W_g h); ``out_scale`` is a constant on the result.
+
 All keep S as float32 [heads, columns, key_dim] per request (a head's matrix column by column),
 zero at a request's start; the convolution's last ``conv_taps - 1`` inputs (activation type) and the
 running maximum (float32 [heads]) are state too. Gates, unit vectors and the recurrence are float32
@@ -392,3 +397,101 @@ class ConstantDecay(Mixer):
             gated = whole
         y = ws.get("mixer.out", (n, spec.hidden_size), rt.dtype)
         return ops.gemm(gated, self.w_o, y, defer_sum=True) or y
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec(PartSpec):
+    kind = "gated_linear"
+    hidden_size: int = 0
+    num_heads: int = 0
+    key_dim: int = 0
+    value_dim: int = 0
+    decay_rank: int = 0                 # rows of W_a1
+    tau: float = 1.0                    # a channel's decay is sigmoid(z)^(1 / tau)
+    out_norm_eps: float = 1e-6          # of the per-head RMS of the output
+    out_scale: float = 1.0              # on the gated rows (it goes into the norm's weight)
+
+    @property
+    def inner(self) -> int:
+        return self.num_heads * self.value_dim
+
+
+@register_mixer(GatedLinearSpec.kind)
+class GatedLinear(Mixer):
+    """Packed rows: [q | k | v | g, padded to a multiple of 8 | W_a1 h, padded to a multiple of 32]. In steps with prompt
+    portions W_a2 is one product with float32 rows; in steps of single tokens the step's kernel makes them itself."""
+    spec_class = GatedLinearSpec
+    accepts_pending_norm = True         # the input is used by one packed product only
+    accepts_fold = True                 # the output comes from one product
+    PACKED = ("q", "k", "v", "g")
+
+    @classmethod
+    def tensors(cls, spec: GatedLinearSpec) -> Dict[str, TensorDecl]:
+        hid, qk, vd = spec.hidden_size, spec.num_heads * spec.key_dim, spec.inner
+        return {"q": TensorDecl((qk, hid)), "k": TensorDecl((qk, hid)), "v": TensorDecl((vd, hid)), "g": TensorDecl((vd, hid)),
+                "a1": TensorDecl((spec.decay_rank, hid)), "a2": TensorDecl((qk, spec.decay_rank)),
+                "a2_bias": TensorDecl((qk,), init="zeros_normal"), "norm": TensorDecl((spec.value_dim,), init="ones_normal"),
+                "o": TensorDecl((hid, vd))}
+
+    @classmethod
+    def state_shapes(cls, spec: GatedLinearSpec):
+        return {"state": ((spec.num_heads, spec.value_dim, spec.key_dim), torch.float32)}
+
+    def __init__(self, spec: GatedLinearSpec, tensors: Dict[str, torch.Tensor], rt: Runtime, position: Optional[object] = None):
+        if min(spec.num_heads, spec.key_dim, spec.value_dim, spec.decay_rank) < 1 or not spec.tau > 0:
+            raise ValueError(f"gated linear attention: bad sizes {spec}")
+        self.spec, self.rt = spec, rt
+        hid, qk = spec.hidden_size, spec.num_heads * spec.key_dim
+        front = _pack(tensors, self.PACKED, hid, "gated linear attention")
+        pad = (-spec.decay_rank) % 32
+        low, a2 = tensors["a1"], tensors["a2"]
+        self.a2t = a2.t().contiguous()
+        if pad:
+            low = torch.cat([low, torch.zeros((pad, hid), dtype=low.dtype, device=low.device)], dim=0)
+            a2 = torch.cat([a2, torch.zeros((qk, pad), dtype=a2.dtype, device=a2.device)], dim=1)
+        self.low_offset, self.low_width = front.shape[0], low.shape[0]
+        self.w_packed = torch.cat([front, low], dim=0).contiguous()
+        self.width = self.w_packed.shape[0]
+        self.w_second = a2.contiguous()
+        self.a2_bias = tensors["a2_bias"].to(torch.float32).contiguous()
+        # float32: the constant on the output costs no rounding of its own
+        self.norm = (tensors["norm"].to(torch.float32) * spec.out_scale).contiguous()
+        self.w_o = tensors["o"]
+
+    def first_product(self):
+        return self.w_packed.shape[0], self.w_packed.shape[1], False
+
+    def recur(self, packed: torch.Tensor, base: int, ctx, call: int, out: torch.Tensor, beside: Optional[dict] = None) -> bool:
+        """From rows that hold this mixer's projections from column ``base`` on: the gated rows that go into the output
+        projection, in ``out`` [n, heads * value_dim]. ``beside``: a convolution and cache write of a softmax mixer on the same
+        rows (``Attention.conv_store_args``), to run in the same launch where there is one; returns whether it ran."""
+        spec, rt, ops, ws = self.spec, self.rt, self.rt.ops, self.rt.workspace
+        n, H, dk, dv = packed.shape[0], spec.num_heads, spec.key_dim, spec.value_dim
+        plan = ctx.attention_plan
+        if plan is not None and plan.decode_only:
+            ran = ops.gated_linear_step(packed, base, base + self.low_offset, H, dk, dv, self.a2t, self.a2_bias, spec.tau, self.norm,
+                                        spec.out_norm_eps, ctx.state(call), ctx.token_seq, ctx.state_slots, out, beside=beside)
+            if ran:
+                return ran == 2
+        z = ws.get("mstate.z", (n, H * dk), torch.float32)
+        low = base + self.low_offset
+        ops.gemm(packed[:, low:low + self.low_width], self.w_second, z)
+        raw = ws.get("mstate.raw", (n, H, dv), torch.float32)
+        chunks = plan.units(ops.gated_linear_chunk_tokens()) if plan is not None else n
+        sums = ws.get("mstate.chunks", (chunks, H, dv, dk), torch.float32)
+        decays = ws.get("mstate.decays", (chunks, H, dk), torch.float32)
+        ops.gated_linear_chunks(packed, base, H, dk, dv, z, self.a2_bias, spec.tau, ctx.state(call), ctx.token_seq, ctx.cu_seqlens,
+                                ctx.state_slots, ctx.n_seqs, chunks, sums, decays, raw)
+        ops.state_finish(raw, None, packed, base + H * (2 * dk + dv), self.norm, H, dv, spec.out_norm_eps, ctx.token_seq, out,
+                         shared_weight=True, silu_gate=True)
+        return False
+
+    def forward(self, x: torch.Tensor, ctx, call: int, fold=None) -> torch.Tensor:
+        spec, rt, ops, ws = self.spec, self.rt, self.rt.ops, self.rt.workspace
+        n = x.shape[0]
+        packed = ws.get("mstate.packed", (n, self.width), rt.dtype)
+        ops.gemm(x, self.w_packed, packed)
+        gated = ws.get("mstate.gated", (n, spec.inner), rt.dtype)
+        self.recur(packed, 0, ctx, call, gated)
+        y = ws.get("mixer.out", (n, spec.hidden_size), rt.dtype)
+        return ops.gemm(gated, self.w_o, y, defer_sum=True, fold=fold) or y

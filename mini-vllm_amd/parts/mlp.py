@@ -100,6 +100,49 @@ class XIELUFeedForward(FeedForward):
 
 
 @dataclass(frozen=True)
+class SquaredReLUSpec(PartSpec):
+    """Two projections with the square of ReLU between them: y = Wd max(Wu x + bu, 0)^2 + bd; ``bias`` False leaves both
+    biases out."""
+    kind = "squared_relu_mlp"
+    hidden_size: int = 0
+    intermediate_size: int = 0
+    bias: bool = True
+
+
+@register_feed_forward(SquaredReLUSpec.kind)
+class SquaredReLU(FeedForward):
+    spec_class = SquaredReLUSpec
+
+    @classmethod
+    def tensors(cls, spec: SquaredReLUSpec) -> Dict[str, TensorDecl]:
+        t = {"up": TensorDecl((spec.intermediate_size, spec.hidden_size)),
+             "down": TensorDecl((spec.hidden_size, spec.intermediate_size))}
+        if spec.bias:
+            t.update(up_bias=TensorDecl((spec.intermediate_size,), init="zeros_normal"),
+                     down_bias=TensorDecl((spec.hidden_size,), init="zeros_normal"))
+        return t
+
+    def __init__(self, spec: SquaredReLUSpec, tensors: Dict[str, torch.Tensor], rt: Runtime):
+        self.spec, self.rt = spec, rt
+        self.w_up, self.w_down = tensors["up"], tensors["down"]
+        self.b_up = self.b_down = None
+        if spec.bias:
+            self.b_up = tensors["up_bias"].to(self.w_up.dtype).contiguous()
+            self.b_down = tensors["down_bias"].to(self.w_down.dtype).contiguous()
+
+    def forward(self, x: torch.Tensor, ctx) -> torch.Tensor:
+        spec, rt, ops = self.spec, self.rt, self.rt.ops
+        if not isinstance(x, torch.Tensor):
+            x = x.materialize()
+        n = x.shape[0]
+        act = rt.workspace.get("ffn.act", (n, spec.intermediate_size), rt.dtype)
+        ops.gemm(x, self.w_up, act, self.b_up)
+        ops.squared_relu(act)
+        y = rt.workspace.get("ffn.out", (n, spec.hidden_size), rt.dtype)
+        return ops.gemm(act, self.w_down, y, self.b_down, defer_sum=True) or y
+
+
+@dataclass(frozen=True)
 class ClampedGLUSpec(PartSpec):
     """A gated pair with clamped halves: g = min(Wg x + bg, limit), u = clamp(Wu x + bu, -limit, limit),
     y = Wd (g * sigmoid(slope * g) * (u + 1)) + bd; ``bias`` False leaves the three biases out."""

@@ -27,6 +27,8 @@ class RotarySpec(PartSpec):
     # stretched low frequencies for contexts longer than the model was made for: (factor, original length, fast, slow),
     # see ``stretched_frequencies``; None: the plain geometric frequencies
     stretch: Optional[Tuple[float, float, float, float]] = None
+    # the low frequencies slowed down by their wavelength: (factor, low, high, original), see ``wavelength_frequencies``
+    by_wavelength: Optional[Tuple[float, float, float, float]] = None
 
 
 def inverse_frequencies(rotary_dim: int, theta: float) -> torch.Tensor:
@@ -64,6 +66,28 @@ def stretched_frequencies(rotary_dim: int, theta: float, stretch: Tuple[float, f
     return torch.tensor(freqs, dtype=torch.float32), MAGNITUDE_SLOPE * math.log(factor) + 1.0
 
 
+def wavelength_frequencies(rotary_dim: int, theta: float, scaling: Tuple[float, float, float, float]) -> torch.Tensor:
+    """float32 [rotary_dim / 2] for ``scaling`` = (factor, low, high, original). A pair of frequency f turns
+    t = original f / (2 pi) times over ``original`` positions: above ``high`` turns it keeps f, below ``low`` it turns at
+    f / factor, and between them the two are blended, s f + (1 - s) f / factor with s = (t - low) / (high - low).
+    Evaluated in double precision, rounded once."""
+    factor, low, high, original = (float(v) for v in scaling)
+    if not (factor > 0 and original > 0 and 0 < low <= high and theta > 0):
+        raise ValueError(f"rotary frequencies by wavelength need positive constants and low <= high, got {scaling}, theta {theta}")
+    freqs = []
+    for i in range(rotary_dim // 2):
+        f = theta ** (-2.0 * i / rotary_dim)
+        turns = original * f / (2.0 * math.pi)
+        if turns > high:
+            kept = 1.0
+        elif turns < low:
+            kept = 0.0
+        else:
+            kept = (turns - low) / (high - low) if high > low else 1.0
+        freqs.append(f / factor * (1.0 - kept) + f * kept)
+    return torch.tensor(freqs, dtype=torch.float32)
+
+
 @register_position_encoding(RotarySpec.kind)
 class RotaryEmbedding(PositionEncoding):
     spec_class = RotarySpec
@@ -73,7 +97,11 @@ class RotaryEmbedding(PositionEncoding):
             raise ValueError(f"rotary_dim must be positive and even, got {spec.rotary_dim}")
         self.spec = spec
         self.rt = rt
-        if spec.stretch is None:
+        if spec.stretch is not None and spec.by_wavelength is not None:
+            raise ValueError("rotary frequencies are stretched in one way at a time")
+        if spec.by_wavelength is not None:
+            inv_freq, magnitude = wavelength_frequencies(spec.rotary_dim, spec.theta, spec.by_wavelength), 1.0
+        elif spec.stretch is None:
             inv_freq, magnitude = inverse_frequencies(spec.rotary_dim, spec.theta), 1.0
         else:
             inv_freq, magnitude = stretched_frequencies(spec.rotary_dim, spec.theta, spec.stretch)
@@ -91,7 +119,7 @@ class RotaryEmbedding(PositionEncoding):
         plan = ctx.attention_plan
         if plan is None or not plan.decode_only or self.spec.interleaved or not self.rt.ops.use_fast_kernels:
             return None
-        rows = self.rt.workspace.get(f"rotary.rows.{self.spec.rotary_dim}.{self.spec.theta}.{self.spec.stretch}",
+        rows = self.rt.workspace.get(f"rotary.rows.{self.spec.rotary_dim}.{self.spec.theta}.{self.spec.stretch}.{self.spec.by_wavelength}",
                                      (ctx.n_tokens, self.spec.rotary_dim), torch.float32)
         ctx.position_rows[self] = rows
         return ctx.positions, self.table, rows
