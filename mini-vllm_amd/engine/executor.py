@@ -870,6 +870,9 @@ class Executor:
                 plan.decode_only, plan.max_q_len, plan.q_lens = False, mixed_key[0], ()
                 plan.bound = (mixed_key[0], mixed_key[1])
                 ctx.q_lens = ctx.starts = ctx.host_state_slots = None
+            else:
+                # ... and any number of sequences up to the bucket, of which this step may fill only some
+                plan.q_lens = [1] * plan.n_seqs
             self.model.forward(ctx)                # loads every kernel before the capture
             torch.cuda.synchronize()
             self._graph_workspace.frozen = True    # the eager run above sized everything: nothing is allocated now

@@ -257,7 +257,7 @@ def forward(cfg: dict, w: Tensors, tokens: List[int], state: Optional[list] = No
         if layer.get("mlp") is not None:
             x = x + rms_norm(feed_forward(rnd(x), w, p + "mlp.", rnd), w[p + "norm2"], eps)
         kept.append(x)
-    logits = capped(rnd(rms_norm(x, w["final.norm"], eps)) @ w["embed"].T, cfg["logit_softcap"])
+    logits = capped(rnd(rms_norm(x, w["final.norm"], eps)) @ w["embed"].T, cfg.get("logit_softcap"))
     return (logits, new, kept) if keep_layers else (logits, new)
 
 
