@@ -637,25 +637,41 @@ __device__ __forceinline__ float alm_row16_sum(float v) {
     return v;
 }
 
-template <int NQ, int NR>
+// SPLIT (steps of single tokens): a wave takes one run of one row (runs as in the split kernel above) and leaves its sums for
+// attention_latent_join_kernel, which also brings the sink in.
+struct AlmSplit {
+    int run, max_splits;
+    float *part_o, *part_ml;
+};
+
+template <int NQ, int NR, bool SPLIT>
 __global__ void __launch_bounds__(256)
 attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __restrict__ out, long ldo, const bf16* __restrict__ pages,
                              const bf16* __restrict__ pages_t, const int* __restrict__ block_table, int bt_width, int page_size,
                              const int* __restrict__ positions, const int* __restrict__ token_seq, int n, int H, float scale, int window,
-                             const float* __restrict__ sink) {
+                             const float* __restrict__ sink, AlmSplit split) {
     constexpr int DK = NQ * 32, R = NR * 16;
     __shared__ __attribute__((aligned(16))) uint16_t pl[4][16][40];          // a wave's P: [head][key], rows 80 bytes apart
     const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
-    const int tok = blockIdx.x * 4 + wave, h0 = blockIdx.y * 16;
+    const int tok = SPLIT ? (int)blockIdx.x : (int)blockIdx.x * 4 + wave, h0 = blockIdx.y * 16;
     if (tok >= n) return;
     const int r = lane % 16, kq = lane / 16;
     const int nh = min(16, H - h0);
     const int seq = token_seq[tok];
     if (seq < 0) {
+        if (SPLIT) return;
         for (int e = lane; e < nh * R; e += 64) out[(size_t)tok * ldo + (size_t)(h0 + e / R) * R + e % R] = 0.f;
         return;
     }
-    const int pos = positions[tok];
+    int pos = positions[tok];                                // the last key to visit ...
+    int lo = window >= 0 ? max(0, pos - window) : 0;         // ... and the first
+    const int part = SPLIT ? (int)blockIdx.z * 4 + wave : 0;
+    if (SPLIT) {
+        const int begin = (lo / split.run + part) * split.run;
+        if (begin > pos) return;
+        lo = max(lo, begin);
+        pos = min(pos, begin + split.run - 1);
+    }
     const int* bt = block_table + (size_t)seq * bt_width;
     AlmFrag qf[NQ];
 #pragma unroll
@@ -673,14 +689,24 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         // (the sink is a key whose weight counts and whose value is zero)
-        const bool has = sink != nullptr && 4 * kq + i < nh;
+        const bool has = !SPLIT && sink != nullptr && 4 * kq + i < nh;
         m[i] = has ? sink[h0 + 4 * kq + i] : -INFINITY;
         l[i] = has ? 1.f : 0.f;
     }
-    const int lo = window >= 0 ? max(0, pos - window) : 0;
 #pragma unroll
     for (int t = 0; t < NR; ++t) acc[t] = alm_f4{0.f, 0.f, 0.f, 0.f};
     for (int kb = lo & ~7; kb <= pos; kb += 32) {
+        const int key0 = kb + 8 * kq;                        // this lane's eight keys: one page's neighbouring slots
+        const int live = min(8, pos - key0 + 1);             // how many of them the row sees (<= 0: none)
+        // (every lane loads and multiplies, whatever it sees: a matrix instruction is the whole wave's. A lane that
+        // sees none of its keys reads the row's own page instead and zeroes all eight.)
+        const int keyc = live > 0 ? key0 : (pos / 8) * 8;
+        const bf16* vbase = pages_t + ((size_t)bt[keyc / page_size] * R + r) * page_size + keyc % page_size;
+        AlmFrag held[SPLIT ? NR : 1];
+        if (SPLIT) {                                         // few waves: the second product's operand comes while the scores are made
+#pragma unroll
+            for (int t = 0; t < NR; ++t) held[t].u = *reinterpret_cast<const uint4*>(vbase + (size_t)16 * t * page_size);
+        }
         alm_f4 s[2];
 #pragma unroll
         for (int sub = 0; sub < 2; ++sub) {
@@ -717,16 +743,11 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
         __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
         AlmFrag pf;
         pf.u = *reinterpret_cast<const uint4*>(&pl[wave][r][8 * kq]);
-        const int key0 = kb + 8 * kq;                        // this lane's eight keys: one page's neighbouring slots
-        const int live = min(8, pos - key0 + 1);             // how many of them the row sees (<= 0: none)
-        // (every lane loads and multiplies, whatever it sees: a matrix instruction is the whole wave's. A lane that
-        // sees none of its keys reads the row's own page instead and zeroes all eight.)
-        const int keyc = live > 0 ? key0 : (pos / 8) * 8;
-        const bf16* vbase = pages_t + ((size_t)bt[keyc / page_size] * R + r) * page_size + keyc % page_size;
 #pragma unroll
         for (int t = 0; t < NR; ++t) {
             AlmFrag vf;
-            vf.u = *reinterpret_cast<const uint4*>(vbase + (size_t)16 * t * page_size);
+            if constexpr (SPLIT) vf = held[t];
+            else vf.u = *reinterpret_cast<const uint4*>(vbase + (size_t)16 * t * page_size);
 #pragma unroll
             for (int e = 0; e < 8; ++e)
                 if (e >= live || key0 + e < lo) vf.h[e] = 0;
@@ -738,7 +759,16 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
         const int head = 4 * kq + i;
-        if (head < nh) {
+        if (head >= nh) continue;
+        if (SPLIT) {
+            const size_t at = ((size_t)tok * H + h0 + head) * split.max_splits + part;
+#pragma unroll
+            for (int t = 0; t < NR; ++t) split.part_o[at * R + 16 * t + r] = acc[t][i];
+            if (r == 0) {
+                split.part_ml[2 * at] = m[i];
+                split.part_ml[2 * at + 1] = l[i];
+            }
+        } else {
             const float inv = 1.f / l[i];
 #pragma unroll
             for (int t = 0; t < NR; ++t) out[(size_t)tok * ldo + (size_t)(h0 + head) * R + 16 * t + r] = acc[t][i] * inv;
@@ -746,24 +776,22 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     }
 }
 
-// returns 2 (nothing done) for sizes it does not serve: (R, DR) in (64, 32), (128, 32), (128, 64), (256, 64), without a rotated
-// part R in 32, 64, 96, 128, 160, 192, 256, 384, 512; pages whose size is a multiple of 8
-extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, long ldo, const void* pages, const void* pages_t,
-                                        const int* block_table, int bt_width, int page_size, const int* positions,
-                                        const int* token_seq, int n, int H, int R, int DR, float scale, int window, const float* sink,
-                                        hipStream_t stream) {
-    MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0, "attention_latent_mfma: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
-    const bool plain = DR == 0 && R % 32 == 0 && (R <= 192 || R == 256 || R == 384 || R == 512);
+// sizes served: (R, DR) in (64, 32), (128, 32), (128, 64), (256, 64), without a rotated part R in 32, 64, 96, 128, 160, 192,
+// 256, 384, 512; pages whose size is a multiple of 8
+static bool alm_served(const void* pages, const void* pages_t, int page_size, int R, int DR) {
+    const bool plain = DR == 0 && R % 32 == 0 && R > 0 && (R <= 192 || R == 256 || R == 384 || R == 512);
     const bool served = plain || (R == 64 && DR == 32) || (R == 128 && DR == 32) || (R == 128 && DR == 64) || (R == 256 && DR == 64);
-    if (!served || page_size % 8 != 0 || !pages_t || ((uintptr_t)pages % 16) || ((uintptr_t)pages_t % 16)) return 2;
-    MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_mfma: pitches too small");
-    MV_REQUIRE(q && out && pages && block_table && positions && token_seq, "attention_latent_mfma: missing operand");
-    if (n == 0) return 0;
-    dim3 grid((n + 3) / 4, (H + 15) / 16);
+    return served && page_size % 8 == 0 && pages_t && ((uintptr_t)pages % 16) == 0 && ((uintptr_t)pages_t % 16) == 0;
+}
+
+template <bool SPLIT>
+static void alm_launch(dim3 grid, const float* q, long ldq, float* out, long ldo, const void* pages, const void* pages_t,
+                       const int* block_table, int bt_width, int page_size, const int* positions, const int* token_seq, int n, int H,
+                       int R, int DR, float scale, int window, const float* sink, const AlmSplit& split, hipStream_t stream) {
 #define ALM_LAUNCH(NQ, NR)                                                                                                 \
-    hipLaunchKernelGGL((attention_latent_mfma_kernel<NQ, NR>), grid, dim3(256), 0, stream, q, ldq, out, ldo, (const bf16*)pages, \
-                       (const bf16*)pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, scale, window, sink)
-    if (plain) {
+    hipLaunchKernelGGL((attention_latent_mfma_kernel<NQ, NR, SPLIT>), grid, dim3(256), 0, stream, q, ldq, out, ldo, (const bf16*)pages, \
+                       (const bf16*)pages_t, block_table, bt_width, page_size, positions, token_seq, n, H, scale, window, sink, split)
+    if (DR == 0) {
         switch (R) {
             case 32: ALM_LAUNCH(1, 2); break;
             case 64: ALM_LAUNCH(2, 4); break;
@@ -780,7 +808,45 @@ extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, lo
     else if (R == 128) ALM_LAUNCH(6, 8);
     else ALM_LAUNCH(10, 16);
 #undef ALM_LAUNCH
+}
+
+// returns 2 (nothing done) for sizes it does not serve
+extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, long ldo, const void* pages, const void* pages_t,
+                                        const int* block_table, int bt_width, int page_size, const int* positions,
+                                        const int* token_seq, int n, int H, int R, int DR, float scale, int window, const float* sink,
+                                        hipStream_t stream) {
+    MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0, "attention_latent_mfma: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
+    if (!alm_served(pages, pages_t, page_size, R, DR)) return 2;
+    MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_mfma: pitches too small");
+    MV_REQUIRE(q && out && pages && block_table && positions && token_seq, "attention_latent_mfma: missing operand");
+    if (n == 0) return 0;
+    alm_launch<false>(dim3((n + 3) / 4, (H + 15) / 16), q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions,
+                      token_seq, n, H, R, DR, scale, window, sink, AlmSplit{}, stream);
     return mv_check_launch("attention_latent_mfma");
+}
+
+// The same for steps of single tokens, a row's keys dealt out in runs and joined (scratch as for mv_attention_latent_split).
+// Returns 2 (nothing done) for sizes it does not serve.
+extern "C" int mv_attention_latent_split_mfma(const float* q, long ldq, float* out, long ldo, const void* pages, const void* pages_t,
+                                              const int* block_table, int bt_width, int page_size, const int* positions,
+                                              const int* token_seq, int n, int H, int R, int DR, float scale, int window,
+                                              const float* sink, int max_context, float* work, long work_floats, hipStream_t stream) {
+    MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0 && max_context > 0, "attention_latent_split_mfma: bad sizes n=%d H=%d R=%d DR=%d", n, H,
+               R, DR);
+    if (!alm_served(pages, pages_t, page_size, R, DR)) return 2;
+    MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R && H <= 65535, "attention_latent_split_mfma: pitches too small");
+    MV_REQUIRE(q && out && pages && block_table && positions && token_seq && work, "attention_latent_split_mfma: missing operand");
+    const int run = als_run(max_context), runs = (int)als_runs(max_context, window);
+    MV_REQUIRE(work_floats >= mv_attention_latent_split_workspace(n, H, R, max_context, window) && (runs + 3) / 4 <= 65535,
+               "attention_latent_split_mfma: scratch of %ld floats is too small", work_floats);
+    if (n == 0) return 0;
+    const AlmSplit split{run, runs, work, work + (size_t)n * H * runs * R};
+    alm_launch<true>(dim3(n, (H + 15) / 16, (runs + 3) / 4), q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions,
+                     token_seq, n, H, R, DR, scale, window, nullptr, split, stream);
+    if (mv_check_launch("attention_latent_split_mfma")) return 1;
+    hipLaunchKernelGGL(attention_latent_join_kernel, dim3(n, H), dim3(256), 0, stream, split.part_o, split.part_ml, positions, token_seq, H,
+                       R, window, sink, run, runs, out, ldo);
+    return mv_check_launch("attention_latent_join");
 }
 #endif
 

@@ -572,6 +572,7 @@ gemm_skinny_kernel(const bf16* __restrict__ A, long lda, const bf16* __restrict_
                     if (col >= n_end) continue;
                     float v = acc[r][t][e];
                     if (bias) v += to_f(bias[col]);
+                    if (EPI == EPI_NONE && !NORM && fold.square_relu) v = v > 0.f ? v * v : 0.f;
                     store_c<TC>(C + (size_t)tok * ldc + col, v);
                 }
             }
@@ -666,24 +667,26 @@ static int dispatch_tm(const void* A, long lda, const void* W, const void* bias,
     return 0;
 }
 
-// c_dtype: MV_BF16 or MV_F32.
+// c_dtype: MV_BF16 or MV_F32. square_relu: C = max(., 0)^2.
 extern "C" int mv_gemm_skinny(const void* A, long lda, const void* W, long ldw, const void* bias, void* C, long ldc,
-                              int c_dtype, int M, int N, int K, hipStream_t stream) {
+                              int c_dtype, int M, int N, int K, int square_relu, hipStream_t stream) {
     if (int rc = check_skinny("gemm_skinny", A, lda, W, ldc, M, N, K)) return rc;
     MV_REQUIRE(ldw == K, "gemm_skinny: the weight must be contiguous (ldw=%ld, K=%d)", ldw, K);
     MV_REQUIRE(c_dtype == MV_F32 || c_dtype == MV_BF16, "gemm_skinny: bad output dtype %d", c_dtype);
     if (M == 0) return 0;
     int S, R, rows;
     skinny_shape(M, N, K, S, R, rows);
+    RowsInput after{};
+    after.square_relu = square_relu;
     int rc = 0;
     if (c_dtype == MV_F32) {
-        if (R == 4) rc = dispatch_tm<4, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
-        else if (R == 2) rc = dispatch_tm<2, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
-        else rc = dispatch_tm<1, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
+        if (R == 4) rc = dispatch_tm<4, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
+        else if (R == 2) rc = dispatch_tm<2, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
+        else rc = dispatch_tm<1, false, float>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
     } else {
-        if (R == 4) rc = dispatch_tm<4, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
-        else if (R == 2) rc = dispatch_tm<2, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
-        else rc = dispatch_tm<1, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream);
+        if (R == 4) rc = dispatch_tm<4, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
+        else if (R == 2) rc = dispatch_tm<2, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
+        else rc = dispatch_tm<1, false, bf16>(A, lda, W, bias, C, ldc, M, N, K, S, rows, stream, after);
     }
     if (rc) return rc;
     return mv_check_launch("gemm_skinny");

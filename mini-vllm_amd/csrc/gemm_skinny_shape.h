@@ -27,7 +27,7 @@ union Frag {
 #define SK_WAVE_K 128      // fewest K elements of a wave
 #endif
 
-// What the FOLD and SCALED variants need beside the product (EPI below).
+// What the variants need beside the product (EPI below).
 struct RowsInput {
     float* resid;            // FOLD: [M, N] float, updated in place: resid += bf16(product)
     long ldr;
@@ -41,6 +41,7 @@ struct RowsInput {
     int P;
     float eps;               // SCALED
     int width;               // SCALED: elements of an input row (the norm's size)
+    int square_relu;         // without FOLD and the gated pair: c <- max(c, 0)^2
 };
 
 enum { EPI_NONE = 0, EPI_FOLD = 1, EPI_SCALED = 2 };

@@ -194,13 +194,17 @@ _OPTIONAL_SIGNATURES = {
     # stream
     "mv_attention_latent_mfma": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
                                          c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p]),
+    # the same up to sink, then max_context, work, work_floats, stream
+    "mv_attention_latent_split_mfma": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p,
+                                               c_void_p, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_int, c_void_p, c_long,
+                                               c_void_p]),
     "mv_moe_grouped_ints": (c_long, [c_int, c_int, c_int]),
     # x, ldx, n, hidden, w_gate_up, w_down, n_real, identity, F, ids, weights, top, dense, ld_dense, ints, act, out, y, ldy,
     # limit, slope, stream
     "mv_moe_grouped": (c_int, [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int,
                                c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_float, c_float, c_void_p]),
     "mv_gemm_skinny": (c_int, [c_void_p, c_long, c_void_p, c_long, c_void_p, c_void_p, c_long, c_int,
-                               c_int, c_int, c_int, c_void_p]),
+                               c_int, c_int, c_int, c_int, c_void_p]),
     # A, lda, W, bias, out, ldo, M, I, K, limit, slope, stream
     "mv_gemm_skinny_swiglu": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_float, c_float,
                                       c_void_p]),

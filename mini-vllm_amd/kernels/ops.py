@@ -132,6 +132,9 @@ def _weight_code(w: torch.Tensor, what: str) -> int:
     return code
 
 
+_SQUARED = object()      # what ``Ops.gemm`` returns when the product's kernel applied the squared ReLU too
+
+
 class SplitSum:
     """The output of a matrix product that exists only as the float partial sums of its splits of K
     so far: ``out[m, n] = round(sum_f work[f, m, n] + bias[n])``. The next residual add + norm can
@@ -1373,19 +1376,20 @@ class Ops:
             _dev(sink, "sinks")
             if sink.dtype != torch.float32 or sink.numel() != heads or not sink.is_contiguous():
                 raise KernelLibraryError(f"attention_latent: the sinks must be float32 [{heads}]")
+        if pages_t is not None:
+            self._act(pages_t, "slot-contiguous latent pages")
+            if tuple(pages_t.shape) != (pages.shape[0], kv_rank, page_size) or not pages_t.is_contiguous():
+                raise KernelLibraryError(f"attention_latent: the slot-contiguous pages must be [{pages.shape[0]}, {kv_rank}, {page_size}]")
         w = -1 if window is None else int(window)
         priced = self._window_priced(plan, w, 0) if self.ledger is not None else plan
         kv_tokens = priced.kv_tokens if plan is not None else 0
         pairs = priced.attention_pairs if plan is not None else 0
         if plan is not None and plan.decode_only and plan.max_context_len > 0 and self._attention_latent_split(
-                q, out, pages, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim, scale, w, sink,
+                q, out, pages, pages_t, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim, scale, w, sink,
                 plan.max_context_len, kv_tokens):
             return
         if pages_t is not None and self.use_fast_kernels and self.lib.has("mv_attention_latent_mfma") \
                 and not (plan is not None and plan.decode_only):
-            self._act(pages_t, "slot-contiguous latent pages")
-            if tuple(pages_t.shape) != (pages.shape[0], kv_rank, page_size) or not pages_t.is_contiguous():
-                raise KernelLibraryError(f"attention_latent: the slot-contiguous pages must be [{pages.shape[0]}, {kv_rank}, {page_size}]")
             if self.lib.offer("mv_attention_latent_mfma", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank, pages.data_ptr(),
                               pages_t.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(),
                               token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), w, _ptr(sink), self._stream()):
@@ -1398,10 +1402,11 @@ class Ops:
                       block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(), token_seq.data_ptr(),
                       n, heads, kv_rank, rot_dim, float(scale), w, _ptr(sink), self.code, self._stream())
 
-    def _attention_latent_split(self, q, out, pages, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim,
+    def _attention_latent_split(self, q, out, pages, pages_t, block_table, page_size, positions, token_seq, n, heads, kv_rank, rot_dim,
                                 scale, window, sink, max_context, kv_tokens) -> bool:
-        """Steps of single tokens: each row's keys dealt out to workgroups in runs of 256 positions, every workgroup
-        serving 16 heads from key rows staged in LDS; False when the sizes are not served (the general kernel runs)."""
+        """Steps of single tokens: each row's keys dealt out in runs whose sums a second kernel joins. In bfloat16 a run is a
+        wave of the MFMA kernel where it serves the sizes; else a workgroup that serves 16 heads from key rows staged in
+        LDS. False when the sizes are not served by either (the general kernel runs)."""
         need = int(self.lib.dll.mv_attention_latent_split_workspace(n, heads, kv_rank, max_context, window))
         if self._latent_work is None or self._latent_work.numel() < need:
             if torch.cuda.is_current_stream_capturing():
@@ -1410,6 +1415,14 @@ class Ops:
                 self._mid_retired.append(self._latent_work)    # captured graphs may hold its address
             self._latent_work = torch.empty(max(need, 1 << 20), dtype=torch.float32, device=q.device)
         dk = kv_rank + rot_dim
+        if pages_t is not None and self.use_fast_kernels and self.lib.has("mv_attention_latent_split_mfma") and self.lib.offer(
+                "mv_attention_latent_split_mfma", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank, pages.data_ptr(),
+                pages_t.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(), token_seq.data_ptr(),
+                n, heads, kv_rank, rot_dim, float(scale), window, _ptr(sink), int(max_context), self._latent_work.data_ptr(),
+                self._latent_work.numel(), self._stream()):
+            self._note("mv_attention_latent_split_mfma", self._size(q, out) + kv_tokens * (dk + kv_rank) * pages.element_size(),
+                       2 * kv_tokens * heads * (dk + kv_rank))
+            return True
         if not self.lib.offer("mv_attention_latent_split", q.data_ptr(), heads * dk, out.data_ptr(), heads * kv_rank,
                               pages.data_ptr(), block_table.data_ptr(), block_table.shape[1], page_size, positions.data_ptr(),
                               token_seq.data_ptr(), n, heads, kv_rank, rot_dim, float(scale), window, _ptr(sink), int(max_context),
@@ -2098,9 +2111,16 @@ class Ops:
                       self._stream())
 
     # ------------------------------------------------------------------------------------
+    def gemm_squared_relu(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
+        """out = max(a @ w^T (+ bias), 0)^2, contiguous rows of the activation type; the weight-streaming kernel applies it to
+        its float sums, behind every other product it is a pass of its own."""
+        if self.gemm(a, w, out, bias, square_relu=True) is not _SQUARED:
+            self.squared_relu(out)
+
     def gemm(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
-             exact: bool = False, defer_sum: bool = False, fold=None):
-        """out[M, N] = a[M, K] @ w[N, K]^T (+ bias). ``out`` is the activation type or float32.
+             exact: bool = False, defer_sum: bool = False, fold=None, square_relu: bool = False):
+        """out[M, N] = a[M, K] @ w[N, K]^T (+ bias). ``out`` is the activation type or float32. (``square_relu`` is
+        ``gemm_squared_relu``'s: ``_SQUARED`` is returned where the kernel has applied it.)
 
         With ``defer_sum`` the caller can take a ``SplitSum`` instead of the finished ``out``: when
         the product runs on the kernel that splits K, its partial sums are left to whoever uses the
@@ -2184,9 +2204,9 @@ class Ops:
                 m = min(SKINNY_LAUNCH_ROWS, M - m0)
                 self._note("mv_gemm_skinny", m * K * 2 + (N * K * 2 if m0 == 0 else 0) + m * N * out.element_size(), 2 * m * N * K)
                 self.lib.call("mv_gemm_skinny", a.data_ptr() + m0 * lda * 2, lda, w.data_ptr(), K, _ptr(bias),
-                              out.data_ptr() + m0 * ldc * out.element_size(), ldc, _CODES[out.dtype], m, N, K,
+                              out.data_ptr() + m0 * ldc * out.element_size(), ldc, _CODES[out.dtype], m, N, K, int(square_relu),
                               self._stream())
-            return
+            return _SQUARED if square_relu else None
         if fast and M > SKINNY_MAX_M and self._library_serves(out) and \
                 self._library_allowed(M, N, K, bias is not None, out.dtype) and self._library_product(a, w, bias, out):
             return

@@ -136,8 +136,7 @@ class SquaredReLU(FeedForward):
             x = x.materialize()
         n = x.shape[0]
         act = rt.workspace.get("ffn.act", (n, spec.intermediate_size), rt.dtype)
-        ops.gemm(x, self.w_up, act, self.b_up)
-        ops.squared_relu(act)
+        ops.gemm_squared_relu(x, self.w_up, act, self.b_up)
         y = rt.workspace.get("ffn.out", (n, spec.hidden_size), rt.dtype)
         return ops.gemm(act, self.w_down, y, self.b_down, defer_sum=True) or y
 

@@ -558,17 +558,19 @@ def test_latent_attention_single_token_kernel(dtype, H, R, dr):
 
 @pytest.mark.parametrize("H, R, dr", [(16, 256, 64), (5, 64, 32), (20, 128, 32), (8, 128, 64)])
 @pytest.mark.parametrize("page_size", [16, 8])
-def test_latent_attention_mfma_kernel(H, R, dr, page_size):
+@pytest.mark.parametrize("single", [None, 1024, 20000])
+def test_latent_attention_mfma_kernel(H, R, dr, page_size, single):
     """bfloat16 steps with prompt portions take an MFMA kernel (a row's 16 heads are the rows of its first operand, the
     values come from the slot-contiguous pages): a prompt of 100 tokens, a portion that starts in the middle of a block of
     32 keys, single rows at positions 0, 31, 32, 33 and 700, a padding row; NaN in every slot nobody wrote. Against the
-    softmax written out on the stored rows."""
+    softmax written out on the stored rows. ``single``: the requests' last rows alone, a step of single tokens that deals
+    their keys out in runs (whose length follows the longest context the step must serve)."""
     from minivllm_amd.engine.step import AttentionPlan
     dtype = torch.bfloat16
     ops = ops_for(dtype)
     g = torch.Generator().manual_seed(H + R)
     ctx = [100, 77, 1, 32, 33, 34, 701]                    # contexts of the seven requests after the step
-    qlens = [100, 20, 1, 1, 1, 1, 1]
+    qlens = [100, 20, 1, 1, 1, 1, 1] if single is None else [1] * 7
     n_pages = sum(-(-c // page_size) for c in ctx) + 3
     pages = torch.full((n_pages, page_size, R + dr), float("nan"), dtype=dtype, device=DEV)
     pages_t = torch.full((n_pages, R, page_size), float("nan"), dtype=dtype, device=DEV)
@@ -591,12 +593,12 @@ def test_latent_attention_mfma_kernel(H, R, dr, page_size):
     pos.append(0); tsq.append(-1)
     n = len(pos)
     qa = (1.2 * torch.randn(n, H, R + dr, generator=g)).to(DEV)
-    plan = AttentionPlan(decode_only=False, max_q_len=100, max_context_len=1024, n_seqs=len(ctx))
+    plan = AttentionPlan(decode_only=single is not None, max_q_len=max(qlens), max_context_len=single or 1024, n_seqs=len(ctx))
     got = torch.full((n, H, R), float("nan"), device=DEV)
     ops.ledger = []
     ops.attention_latent(qa, got, pages, bt.to(DEV), page_size, i32(pos), i32(tsq), H, R, dr, 0.15, plan=plan, pages_t=pages_t)
     torch.cuda.synchronize()
-    assert [e[0] for e in ops.ledger] == ["mv_attention_latent_mfma"]
+    assert [e[0] for e in ops.ledger] == ["mv_attention_latent_mfma" if single is None else "mv_attention_latent_split_mfma"]
     ops.ledger = None
     bad = (~torch.isfinite(got)).nonzero()
     assert bad.numel() == 0, f"non-finite outputs at (row, head, channel) {bad[:8].tolist()} ... of rows at positions {sorted({pos[i] for i in bad[:, 0].tolist()})[:12]}"

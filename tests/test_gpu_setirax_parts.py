@@ -285,7 +285,7 @@ def test_latent_attention_under_a_window(dtype, H, d, dv, R, page, size):
 
 
 @pytest.mark.parametrize("R", [32, 64, 96, 128, 160, 192, 256, 384, 512])
-@pytest.mark.parametrize("kernel", ["general", "split", "mfma"])
+@pytest.mark.parametrize("kernel", ["general", "split", "mfma", "split_mfma"])
 @pytest.mark.parametrize("size", [1, 8, 50, 300])
 def test_latent_kernels_find_the_first_key_of_a_window(R, kernel, size):
     """A key that the query singles out just inside the window, then just outside; with and without a sink that stands out."""
@@ -312,18 +312,18 @@ def test_latent_kernels_find_the_first_key_of_a_window(R, kernel, size):
                 pages[perm[p // page], p % page] = keys[p]
             bt = torch.where(torch.arange(len(perm)) >= low, perm, torch.full_like(perm, -1)).to(torch.int32).view(1, -1).to(DEV)
             for sink in (None, torch.linspace(-1.0, 14.0, H)):
-                plan = AttentionPlan(decode_only=kernel == "split", max_q_len=1, max_context_len=pos + 1, n_seqs=1, q_lens=[1],
+                plan = AttentionPlan(decode_only=kernel.startswith("split"), max_q_len=1, max_context_len=pos + 1, n_seqs=1, q_lens=[1],
                                      cu_seqlens=i32([0, 1]), workspace=Workspace(torch.device(DEV)))
                 out = torch.empty(1, H, R, device=DEV)
                 ops.ledger = []
                 pages_dev = pages.to(DEV)
                 ops.attention_latent(q.to(DEV), out, pages_dev, bt, page, i32([pos]), i32([0]), H, R, 0, scale,
                                      plan=None if kernel == "general" else plan, window=size - 1, sink=None if sink is None else sink.to(DEV),
-                                     pages_t=pages_dev.transpose(1, 2).contiguous() if kernel == "mfma" else None)
+                                     pages_t=pages_dev.transpose(1, 2).contiguous() if kernel.endswith("mfma") else None)
                 torch.cuda.synchronize()
                 ran, ops.ledger = ops.ledger[0][0], None
                 # (key rows of 1,024 bytes do not fit the split kernel's LDS beside the queries)
-                assert ran == {"general": "mv_attention_latent", "split": "mv_attention_latent_split" if R < 512 else "mv_attention_latent", "mfma": "mv_attention_latent_mfma"}[kernel]
+                assert ran == {"general": "mv_attention_latent", "split": "mv_attention_latent_split" if R < 512 else "mv_attention_latent", "mfma": "mv_attention_latent_mfma", "split_mfma": "mv_attention_latent_split_mfma"}[kernel]
                 s = [plain.windowed(q[0, h:h + 1].double() @ keys[:pos + 1].double().T * scale, pos, size) for h in range(H)]
                 want = torch.cat([plain.sink_softmax(s[h], None if sink is None else sink[h].double()) for h in range(H)]) @ keys[:pos + 1].double()
                 close(out[0], want, 1.2e-2, f"position {pos}, marked key {edge}")
