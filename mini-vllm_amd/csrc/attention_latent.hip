@@ -107,6 +107,23 @@ extern "C" int mv_latent_prepare(const void* packed, long ld, int n, int QR, int
 // order through LDS. (64 columns x 4 slices for steps of many rows; 16 x 16 for steps of few rows, whose few
 // workgroups a head would otherwise walk long runs of inputs one load after the other.) The order of additions
 // depends on IN and the variant.
+// acc[row] += the slice's share of one output column; w points at the column's first weight, eight weights are asked for at a time
+template <typename TW, int HL_SLICES>
+__device__ __forceinline__ void head_dots(const TW* __restrict__ w, int IN, int OUT, int slice, const float (&xs)[HL_TOKENS][HL_MAX_IN],
+                                          float (&acc)[HL_TOKENS]) {
+    constexpr int AHEAD = 8;
+    for (int i0 = slice; i0 < IN; i0 += AHEAD * HL_SLICES) {
+        float wv[AHEAD];
+#pragma unroll
+        for (int u = 0; u < AHEAD; ++u) wv[u] = to_f(w[(size_t)min(i0 + u * HL_SLICES, IN - 1) * OUT]);
+#pragma unroll
+        for (int u = 0; u < AHEAD; ++u)
+            if (i0 + u * HL_SLICES < IN)
+#pragma unroll
+                for (int tt = 0; tt < HL_TOKENS; ++tt) acc[tt] = fmaf(xs[tt][i0 + u * HL_SLICES], wv[u], acc[tt]);
+    }
+}
+
 template <typename TIN, typename TOUT, typename TG, int HL_COLS, int HL_SLICES>
 __global__ void __launch_bounds__(256)
 head_linear_kernel(const TIN* __restrict__ x, long ldx, int ldx_head, WeightPtr w, int IN, int OUT, TOUT* __restrict__ y, long ldy,
@@ -116,9 +133,18 @@ head_linear_kernel(const TIN* __restrict__ x, long ldx, int ldx_head, WeightPtr 
     __shared__ float part[HL_SLICES][HL_TOKENS][HL_COLS];
     const int t0 = blockIdx.x * HL_TOKENS, head = blockIdx.y, tid = threadIdx.x;
     const int nt = min(HL_TOKENS, n - t0);
-    for (int e = tid; e < HL_TOKENS * IN; e += 256) {
-        const int tt = e / IN, i = e % IN;
-        xs[tt][i] = tt < nt ? to_f(x[(size_t)(t0 + tt) * ldx + (size_t)head * ldx_head + i]) : 0.f;
+    for (int e0 = tid; e0 < HL_TOKENS * IN; e0 += 8 * 256) {               // eight loads in flight (addresses that exist, values dropped)
+        float v[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int e = min(e0 + 256 * u, HL_TOKENS * IN - 1);
+            v[u] = to_f(x[(size_t)(t0 + min(e / IN, nt - 1)) * ldx + (size_t)head * ldx_head + e % IN]);
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int e = e0 + 256 * u;
+            if (e < HL_TOKENS * IN) xs[e / IN][e % IN] = e / IN < nt ? v[u] : 0.f;
+        }
     }
     __syncthreads();
     const int col = tid % HL_COLS, slice = tid / HL_COLS;
@@ -128,21 +154,8 @@ head_linear_kernel(const TIN* __restrict__ x, long ldx, int ldx_head, WeightPtr 
     for (int tt = 0; tt < HL_TOKENS; ++tt) acc[tt] = 0.f;
     if (j < OUT) {
         const size_t w0 = (size_t)head * IN * OUT + j;
-        int i = slice;
-        for (; i + 3 * HL_SLICES < IN; i += 4 * HL_SLICES) {          // four loads in flight
-            float wv[4];
-#pragma unroll
-            for (int u = 0; u < 4; ++u) wv[u] = w.at(w0 + (size_t)(i + u * HL_SLICES) * OUT);
-#pragma unroll
-            for (int u = 0; u < 4; ++u)
-#pragma unroll
-                for (int tt = 0; tt < HL_TOKENS; ++tt) acc[tt] = fmaf(xs[tt][i + u * HL_SLICES], wv[u], acc[tt]);
-        }
-        for (; i < IN; i += HL_SLICES) {
-            const float wv = w.at(w0 + (size_t)i * OUT);
-#pragma unroll
-            for (int tt = 0; tt < HL_TOKENS; ++tt) acc[tt] = fmaf(xs[tt][i], wv, acc[tt]);
-        }
+        if (w.dtype == MV_F32) head_dots<float, HL_SLICES>((const float*)w.p + w0, IN, OUT, slice, xs, acc);
+        else head_dots<bf16, HL_SLICES>((const bf16*)w.p + w0, IN, OUT, slice, xs, acc);
     }
 #pragma unroll
     for (int tt = 0; tt < HL_TOKENS; ++tt) part[slice][tt][col] = acc[tt];
@@ -524,30 +537,56 @@ attention_latent_split_kernel(const float* __restrict__ q, long ldq, const T* __
     }
 }
 
+// joins the runs of a (row, head) in their order
 __global__ void __launch_bounds__(256)
 attention_latent_join_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ positions,
                              const int* __restrict__ token_seq, int H, int R, int window, const float* __restrict__ sink, int run,
                              int max_splits, float* __restrict__ out, long ldo) {
-    const int tok = blockIdx.x, head = blockIdx.y;
+    __shared__ float weights[256];
+    const int tok = blockIdx.x, head = blockIdx.y, tid = threadIdx.x, lane = tid % MV_WAVE;
     float* o = out + (size_t)tok * ldo + (size_t)head * R;
     if (token_seq[tok] < 0) {
-        for (int d = threadIdx.x; d < R; d += 256) o[d] = 0.f;
+        for (int d = tid; d < R; d += 256) o[d] = 0.f;
         return;
     }
     const int pos = positions[tok];
     const int runs = pos / run + 1 - (window >= 0 ? max(0, pos - window) / run : 0);
     const float* ml = part_ml + ((size_t)tok * H + head) * max_splits * 2;
     float m = sink != nullptr ? sink[head] : -INFINITY;
-    for (int s = 0; s < runs; ++s) m = fmaxf(m, ml[2 * s]);
-    float l = sink != nullptr ? expf(sink[head] - m) : 0.f;
-    for (int s = 0; s < runs; ++s) l += expf(ml[2 * s] - m) * ml[2 * s + 1];
+    for (int s = lane; s < runs; s += MV_WAVE) m = fmaxf(m, ml[2 * s]);
+    m = wave_max(m);
+    float l = 0.f;
+    for (int s = lane; s < runs; s += MV_WAVE) l += expf(ml[2 * s] - m) * ml[2 * s + 1];
+    l = wave_sum(l);
+    if (sink != nullptr) l += expf(sink[head] - m);
     const float inv = 1.f / l;
     const float* po = part_o + ((size_t)tok * H + head) * max_splits * R;
-    for (int d = threadIdx.x; d < R; d += 256) {
-        float a = 0.f;
-        for (int s = 0; s < runs; ++s) a = fmaf(expf(ml[2 * s] - m), po[(size_t)s * R + d], a);
-        o[d] = a * inv;
+    float acc[AL_MAX_R / 256];
+#pragma unroll
+    for (int c = 0; c < AL_MAX_R / 256; ++c) acc[c] = 0.f;
+    for (int s0 = 0; s0 < runs; s0 += 256) {
+        if (s0 > 0) __syncthreads();
+        weights[tid] = s0 + tid < runs ? expf(ml[2 * (s0 + tid)] - m) : 0.f;
+        __syncthreads();
+        const int count = min(256, runs - s0);
+#pragma unroll
+        for (int c = 0; c < AL_MAX_R / 256; ++c) {
+            const int d = tid + 256 * c;
+            if (d >= R) continue;
+            constexpr int AHEAD = 8;
+            for (int b = 0; b < count; b += AHEAD) {
+                float v[AHEAD];
+#pragma unroll
+                for (int e = 0; e < AHEAD; ++e) v[e] = po[(size_t)(s0 + min(b + e, count - 1)) * R + d];
+#pragma unroll
+                for (int e = 0; e < AHEAD; ++e)
+                    if (b + e < count) acc[c] = fmaf(weights[b + e], v[e], acc[c]);
+            }
+        }
     }
+#pragma unroll
+    for (int c = 0; c < AL_MAX_R / 256; ++c)
+        if (tid + 256 * c < R) o[tid + 256 * c] = acc[c] * inv;
 }
 
 // bytes of LDS the split kernel needs for these sizes, and the pitch of a key row in it (32-bit words, odd)
@@ -562,15 +601,14 @@ static void als_layout(int R, int DR, int elem, int& row_words, size_t& lds) {
 static int als_run(int max_context) { return max_context <= 8192 ? 64 : (max_context <= 32768 ? 256 : 1024); }
 
 // most runs a query reads whose context reaches max_context positions
-static long als_runs(int max_context, int window) {
-    const int run = als_run(max_context);
+static long als_runs(int max_context, int window, int run) {
     const long all = (max_context + run - 1) / run;
     return window < 0 ? all : min(all, (long)window / run + 2);
 }
 
 // floats of scratch for n rows whose contexts reach max_context positions: (weighted sums, maxima and sums)
 extern "C" long mv_attention_latent_split_workspace(int n, int H, int R, int max_context, int window) {
-    return (long)n * H * als_runs(max_context, window) * (R + 2);
+    return (long)n * H * als_runs(max_context, window, als_run(max_context)) * (R + 2);
 }
 
 // returns 2 (nothing done) when the sizes are not served: the caller takes the general kernel
@@ -588,7 +626,7 @@ extern "C" int mv_attention_latent_split(const float* q, long ldq, float* out, l
     MV_REQUIRE(page_size > 0 && bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_split: pitches too small");
     MV_REQUIRE(q && out && pages && block_table && positions && token_seq && work, "attention_latent_split: missing operand");
     const int run = als_run(max_context);
-    const int runs = (int)als_runs(max_context, window);
+    const int runs = (int)als_runs(max_context, window, run);
     MV_REQUIRE(work_floats >= mv_attention_latent_split_workspace(n, H, R, max_context, window) && runs <= 65535,
                "attention_latent_split: scratch of %ld floats is too small", work_floats);
     if (n == 0) return 0;
@@ -637,7 +675,8 @@ __device__ __forceinline__ float alm_row16_sum(float v) {
     return v;
 }
 
-// SPLIT (steps of single tokens): a wave takes one run of one row (runs as in the split kernel above) and leaves its sums for
+// SPLIT (steps of single tokens): a workgroup takes one run of one row (runs as in the split kernel above, 128 positions and
+// more), its waves take the run's blocks of 32 keys in turn and are joined through LDS, and the run's sums are left for
 // attention_latent_join_kernel, which also brings the sink in.
 struct AlmSplit {
     int run, max_splits;
@@ -652,7 +691,8 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
                              const float* __restrict__ sink, AlmSplit split) {
     constexpr int DK = NQ * 32, R = NR * 16;
     __shared__ __attribute__((aligned(16))) uint16_t pl[4][16][40];          // a wave's P: [head][key], rows 80 bytes apart
-    const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
+    __shared__ float sh_o[SPLIT ? 4 : 1][SPLIT ? 16 : 1][SPLIT ? R + 4 : 1], sh_ml[SPLIT ? 4 : 1][16][2];
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lane = threadIdx.x % 64;
     const int tok = SPLIT ? (int)blockIdx.x : (int)blockIdx.x * 4 + wave, h0 = blockIdx.y * 16;
     if (tok >= n) return;
     const int r = lane % 16, kq = lane / 16;
@@ -665,7 +705,7 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     }
     int pos = positions[tok];                                // the last key to visit ...
     int lo = window >= 0 ? max(0, pos - window) : 0;         // ... and the first
-    const int part = SPLIT ? (int)blockIdx.z * 4 + wave : 0;
+    const int part = blockIdx.z;
     if (SPLIT) {
         const int begin = (lo / split.run + part) * split.run;
         if (begin > pos) return;
@@ -674,14 +714,19 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     }
     const int* bt = block_table + (size_t)seq * bt_width;
     AlmFrag qf[NQ];
+    {
+        // (rows of heads that do not exist read the last one's, and count as zeros: a load under a condition would wait alone)
+        const float* src = q + (size_t)tok * ldq + (size_t)(h0 + min(r, nh - 1)) * DK + 8 * kq;
+        const float on = r < nh ? scale : 0.f;
+        float x[NQ][8];
 #pragma unroll
-    for (int c = 0; c < NQ; ++c) {
-        if (r < nh) {
-            const float* src = q + (size_t)tok * ldq + (size_t)(h0 + r) * DK + 32 * c + 8 * kq;
+        for (int c = 0; c < NQ; ++c) Vec8<float>::load(src + 32 * c, x[c]);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) qf[c].h[e] = f32_to_bf16_bits(src[e] * scale);
-        } else {
-            qf[c].u = uint4{0u, 0u, 0u, 0u};
+        for (int c = 0; c < NQ; ++c) {
+            qf[c].u.x = f32x2_to_bf16x2_bits(x[c][0] * on, x[c][1] * on);
+            qf[c].u.y = f32x2_to_bf16x2_bits(x[c][2] * on, x[c][3] * on);
+            qf[c].u.z = f32x2_to_bf16x2_bits(x[c][4] * on, x[c][5] * on);
+            qf[c].u.w = f32x2_to_bf16x2_bits(x[c][6] * on, x[c][7] * on);
         }
     }
     float m[4], l[4];
@@ -695,13 +740,16 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
     }
 #pragma unroll
     for (int t = 0; t < NR; ++t) acc[t] = alm_f4{0.f, 0.f, 0.f, 0.f};
-    for (int kb = lo & ~7; kb <= pos; kb += 32) {
+    for (int kb = (lo & ~7) + (SPLIT ? 32 * wave : 0); kb <= pos; kb += SPLIT ? 128 : 32) {
         const int key0 = kb + 8 * kq;                        // this lane's eight keys: one page's neighbouring slots
         const int live = min(8, pos - key0 + 1);             // how many of them the row sees (<= 0: none)
         // (every lane loads and multiplies, whatever it sees: a matrix instruction is the whole wave's. A lane that
         // sees none of its keys reads the row's own page instead and zeroes all eight.)
         const int keyc = live > 0 ? key0 : (pos / 8) * 8;
         const bf16* vbase = pages_t + ((size_t)bt[keyc / page_size] * R + r) * page_size + keyc % page_size;
+        AlmFrag seen;                                        // ones where the row sees the lane's key
+#pragma unroll
+        for (int e = 0; e < 8; ++e) seen.h[e] = e < live && key0 + e >= lo ? 0xffff : 0;
         AlmFrag held[SPLIT ? NR : 1];
         if (SPLIT) {                                         // few waves: the second product's operand comes while the scores are made
 #pragma unroll
@@ -734,10 +782,12 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
             pl[wave][4 * kq + i][r] = f32_to_bf16_bits(p0);
             pl[wave][4 * kq + i][16 + r] = f32_to_bf16_bits(p1);
         }
+        if (!SPLIT || kb > (lo & ~7) + 32 * wave) {          // (nothing to scale in front of a wave's first block)
 #pragma unroll
-        for (int t = 0; t < NR; ++t)
+            for (int t = 0; t < NR; ++t)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) acc[t][i] *= corr[i];
+                for (int i = 0; i < 4; ++i) acc[t][i] *= corr[i];
+        }
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
         __builtin_amdgcn_wave_barrier();
         __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
@@ -748,30 +798,61 @@ attention_latent_mfma_kernel(const float* __restrict__ q, long ldq, float* __res
             AlmFrag vf;
             if constexpr (SPLIT) vf = held[t];
             else vf.u = *reinterpret_cast<const uint4*>(vbase + (size_t)16 * t * page_size);
-#pragma unroll
-            for (int e = 0; e < 8; ++e)
-                if (e >= live || key0 + e < lo) vf.h[e] = 0;
+            vf.u.x &= seen.u.x;
+            vf.u.y &= seen.u.y;
+            vf.u.z &= seen.u.z;
+            vf.u.w &= seen.u.w;
             acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf.v, vf.v, acc[t], 0, 0, 0);
         }
         __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
         __builtin_amdgcn_wave_barrier();
     }
+    if constexpr (SPLIT) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int head = 4 * kq + i;
-        if (head >= nh) continue;
-        if (SPLIT) {
-            const size_t at = ((size_t)tok * H + h0 + head) * split.max_splits + part;
+        for (int i = 0; i < 4; ++i) {
 #pragma unroll
-            for (int t = 0; t < NR; ++t) split.part_o[at * R + 16 * t + r] = acc[t][i];
+            for (int t = 0; t < NR; ++t) sh_o[wave][4 * kq + i][16 * t + r] = acc[t][i];
             if (r == 0) {
-                split.part_ml[2 * at] = m[i];
-                split.part_ml[2 * at + 1] = l[i];
+                sh_ml[wave][4 * kq + i][0] = m[i];
+                sh_ml[wave][4 * kq + i][1] = l[i];
             }
-        } else {
-            const float inv = 1.f / l[i];
+        }
+        __syncthreads();
+        // the waves' shares (wave 0 has seen a key, so the maximum is finite; a wave without keys counts nothing)
+        if (threadIdx.x < 16) {
+            const int head = threadIdx.x;
+            float top = -INFINITY, den = 0.f;
 #pragma unroll
-            for (int t = 0; t < NR; ++t) out[(size_t)tok * ldo + (size_t)(h0 + head) * R + 16 * t + r] = acc[t][i] * inv;
+            for (int w = 0; w < 4; ++w) top = fmaxf(top, sh_ml[w][head][0]);
+#pragma unroll
+            for (int w = 0; w < 4; ++w) {
+                const float c = expf(sh_ml[w][head][0] - top);
+                den = fmaf(c, sh_ml[w][head][1], den);
+                sh_ml[w][head][0] = c;
+            }
+            if (head < nh) {
+                float* ml = split.part_ml + 2 * (((size_t)tok * H + h0 + head) * split.max_splits + part);
+                ml[0] = top;
+                ml[1] = den;
+            }
+        }
+        __syncthreads();
+        for (int e = threadIdx.x; e < nh * R; e += 256) {
+            const int head = e / R, d = e % R;
+            float o = 0.f;
+#pragma unroll
+            for (int w = 0; w < 4; ++w) o = fmaf(sh_ml[w][head][0], sh_o[w][head][d], o);
+            split.part_o[(((size_t)tok * H + h0 + head) * split.max_splits + part) * R + d] = o;
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int head = 4 * kq + i;
+            if (head < nh) {
+                const float inv = 1.f / l[i];
+#pragma unroll
+                for (int t = 0; t < NR; ++t) out[(size_t)tok * ldo + (size_t)(h0 + head) * R + 16 * t + r] = acc[t][i] * inv;
+            }
         }
     }
 }
@@ -818,7 +899,8 @@ extern "C" int mv_attention_latent_mfma(const float* q, long ldq, float* out, lo
     MV_REQUIRE(n >= 0 && H > 0 && R > 0 && DR >= 0, "attention_latent_mfma: bad sizes n=%d H=%d R=%d DR=%d", n, H, R, DR);
     if (!alm_served(pages, pages_t, page_size, R, DR)) return 2;
     MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R, "attention_latent_mfma: pitches too small");
-    MV_REQUIRE(q && out && pages && block_table && positions && token_seq, "attention_latent_mfma: missing operand");
+    MV_REQUIRE(q && out && pages && block_table && positions && token_seq && ((uintptr_t)q % 16) == 0 && ldq % 4 == 0,
+               "attention_latent_mfma: missing operand or queries not aligned");
     if (n == 0) return 0;
     alm_launch<false>(dim3((n + 3) / 4, (H + 15) / 16), q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions,
                       token_seq, n, H, R, DR, scale, window, sink, AlmSplit{}, stream);
@@ -835,13 +917,15 @@ extern "C" int mv_attention_latent_split_mfma(const float* q, long ldq, float* o
                R, DR);
     if (!alm_served(pages, pages_t, page_size, R, DR)) return 2;
     MV_REQUIRE(bt_width > 0 && ldq >= (long)H * (R + DR) && ldo >= (long)H * R && H <= 65535, "attention_latent_split_mfma: pitches too small");
-    MV_REQUIRE(q && out && pages && block_table && positions && token_seq && work, "attention_latent_split_mfma: missing operand");
-    const int run = als_run(max_context), runs = (int)als_runs(max_context, window);
-    MV_REQUIRE(work_floats >= mv_attention_latent_split_workspace(n, H, R, max_context, window) && (runs + 3) / 4 <= 65535,
+    MV_REQUIRE(q && out && pages && block_table && positions && token_seq && work && ((uintptr_t)q % 16) == 0 && ldq % 4 == 0,
+               "attention_latent_split_mfma: missing operand or queries not aligned");
+    // (never shorter than the runs the scratch is sized for)
+    const int run = max(128, als_run(max_context)), runs = (int)als_runs(max_context, window, run);
+    MV_REQUIRE(work_floats >= (long)n * H * runs * (R + 2) && runs <= 65535,
                "attention_latent_split_mfma: scratch of %ld floats is too small", work_floats);
     if (n == 0) return 0;
     const AlmSplit split{run, runs, work, work + (size_t)n * H * runs * R};
-    alm_launch<true>(dim3(n, (H + 15) / 16, (runs + 3) / 4), q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions,
+    alm_launch<true>(dim3(n, (H + 15) / 16, runs), q, ldq, out, ldo, pages, pages_t, block_table, bt_width, page_size, positions,
                      token_seq, n, H, R, DR, scale, window, nullptr, split, stream);
     if (mv_check_launch("attention_latent_split_mfma")) return 1;
     hipLaunchKernelGGL(attention_latent_join_kernel, dim3(n, H), dim3(256), 0, stream, split.part_o, split.part_ml, positions, token_seq, H,
