@@ -236,11 +236,31 @@ struct UnitStepArgs {
 #define RU_MAX_PART 512
 #define RU_THREADS 1024
 
+// acc[row][e] += the slice's inputs times the weights of eight neighbouring outputs (w points at the first); four rows of weights
+// are asked for at a time
+template <typename TW, int ROWS>
+__device__ __forceinline__ void unit_dots(const TW* __restrict__ w, int P, int slice, int slices, const float (&su)[ROWS][RU_MAX_PART],
+                                          float (&acc)[ROWS][8]) {
+    for (int k0 = slice; k0 < P; k0 += 4 * slices) {
+        float v[4][8];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) Vec8<TW>::load(w + (size_t)min(k0 + q * slices, P - 1) * 2 * P, v[q]);
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+            if (k0 + q * slices < P)
+#pragma unroll
+                for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) acc[r][e] = fmaf(su[r][k0 + q * slices], v[q][e], acc[r][e]);
+    }
+}
+
 template <typename T, int ROWS>
 __global__ void __launch_bounds__(RU_THREADS)
 unit_step_kernel(UnitStepArgs A) {
     __shared__ float su[ROWS][RU_MAX_PART];
     __shared__ float partial[ROWS][RU_THREADS * 8];        // [slice][2 P]
+    __shared__ float sums[ROWS][2 * RU_MAX_PART];
     const int t0 = blockIdx.x * ROWS, part = blockIdx.y, tid = threadIdx.x;
     const int W = A.W, P = A.P, taps = A.taps;
     for (int e = tid; e < ROWS * P; e += RU_THREADS) {
@@ -249,13 +269,21 @@ unit_step_kernel(UnitStepArgs A) {
         float acc = 0.f;
         if (seq >= 0) {
             T* hist = (T*)A.conv_state + (taps > 1 ? (size_t)A.state_slots[seq] * (taps - 1) * W : 0) + c;
-            acc = A.conv_bias[c];
-            for (int j = 0; j < taps - 1; ++j) {
-                const T x = hist[(size_t)j * W];
-                acc = fmaf(A.w[(size_t)j * W + c], to_f(x), acc);
-                if (j > 0) hist[(size_t)(j - 1) * W] = x;
-            }
             const T now = ((const T*)A.packed)[(size_t)t * A.ld + c];
+            acc = A.conv_bias[c];
+            if (taps == 4) {                                // everything is asked for before anything is used or stored
+                const T x0 = hist[0], x1 = hist[(size_t)W], x2 = hist[2 * (size_t)W];
+                const float w0 = A.w[c], w1 = A.w[(size_t)W + c], w2 = A.w[2 * (size_t)W + c];
+                acc = fmaf(w2, to_f(x2), fmaf(w1, to_f(x1), fmaf(w0, to_f(x0), acc)));
+                hist[0] = x1;
+                hist[(size_t)W] = x2;
+            } else {
+                for (int j = 0; j < taps - 1; ++j) {
+                    const T x = hist[(size_t)j * W];
+                    acc = fmaf(A.w[(size_t)j * W + c], to_f(x), acc);
+                    if (j > 0) hist[(size_t)(j - 1) * W] = x;
+                }
+            }
             acc = fmaf(A.w[(size_t)(taps - 1) * W + c], to_f(now), acc);
             if (taps > 1) hist[(size_t)(taps - 2) * W] = now;
         }
@@ -271,28 +299,21 @@ unit_step_kernel(UnitStepArgs A) {
 #pragma unroll
             for (int e = 0; e < 8; ++e) acc[r][e] = 0.f;
         const size_t w0 = (size_t)part * P * 2 * P + o;
-        int k = slice;
-        for (; k + 3 * slices < P; k += 4 * slices) {       // four loads in flight
-            float w[4][8];
-#pragma unroll
-            for (int q = 0; q < 4; ++q) A.gates.at8(w0 + (size_t)(k + q * slices) * 2 * P, w[q]);
-#pragma unroll
-            for (int q = 0; q < 4; ++q)
-#pragma unroll
-                for (int r = 0; r < ROWS; ++r)
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) acc[r][e] = fmaf(su[r][k + q * slices], w[q][e], acc[r][e]);
-        }
-        for (; k < P; k += slices) {
-            float w[8];
-            A.gates.at8(w0 + (size_t)k * 2 * P, w);
-#pragma unroll
-            for (int r = 0; r < ROWS; ++r)
-#pragma unroll
-                for (int e = 0; e < 8; ++e) acc[r][e] = fmaf(su[r][k], w[e], acc[r][e]);
-        }
+        if (A.gates.dtype == MV_F32) unit_dots<float, ROWS>((const float*)A.gates.p + w0, P, slice, slices, su, acc);
+        else unit_dots<bf16, ROWS>((const bf16*)A.gates.p + w0, P, slice, slices, su, acc);
 #pragma unroll
         for (int r = 0; r < ROWS; ++r) Vec8<float>::store(&partial[r][slice * 2 * P + o], acc[r]);
+    }
+    __syncthreads();
+    // the slices of an output are added by eight neighbouring lanes (all lanes of a wave take part: 16 P is a multiple of 64)
+    for (int e = tid; e < ROWS * 2 * P * 8; e += RU_THREADS) {
+        const int r = e / (16 * P), j = e / 8 % (2 * P);
+        float v = 0.f;
+        for (int s = e % 8; s < slices; s += 8) v += partial[r][s * 2 * P + j];
+        v += __shfl_xor(v, 1, MV_WAVE);
+        v += __shfl_xor(v, 2, MV_WAVE);
+        v += __shfl_xor(v, 4, MV_WAVE);
+        if (e % 8 == 0) sums[r][j] = v;
     }
     __syncthreads();
     for (int e = tid; e < ROWS * P; e += RU_THREADS) {
@@ -304,11 +325,7 @@ unit_step_kernel(UnitStepArgs A) {
             *out = from_f<T>(0.f);
             continue;
         }
-        float zr = A.gate_bias[c], zi = A.gate_bias[W + c];
-        for (int s = 0; s < slices; ++s) {
-            zr += partial[r][s * 2 * P + k];
-            zi += partial[r][s * 2 * P + P + k];
-        }
+        const float zr = A.gate_bias[c] + sums[r][k], zi = A.gate_bias[W + c] + sums[r][P + k];
         float a, x;
         unit_coefficients(zr, zi, su[r][k], A.rate[c], a, x);
         float* st = A.state + (size_t)A.state_slots[seq] * W + c;
