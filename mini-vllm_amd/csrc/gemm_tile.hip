@@ -70,6 +70,7 @@ struct TileArgs {
     int P;
     float eps;
     GatedPair pair;       // GATED: what becomes of the two products (with biases [2 I] added where given)
+    int square_relu;      // without GATED, K not split: c <- max(c, 0)^2
 };
 
 template <int WM, int WN, bool GATED, int STAGES, int OCC>
@@ -281,6 +282,7 @@ gemm_tile_kernel(TileArgs a) {
                     v[e] = a.pair.of(fmaf(acc[t][u][e], rinv, bv[e]), fmaf(acc[t + WN / 2][u][e], rinv, bu[e]));
                 } else {
                     v[e] = acc[t][u][e] * rinv + bv[e];
+                    if (a.square_relu) v[e] = v[e] > 0.f ? v[e] * v[e] : 0.f;
                 }
             }
             const bool whole = col + 3 < n_out;
@@ -414,7 +416,8 @@ extern "C" int mv_gemm_mid_reduce(const float* work, const void* bias, void* C, 
 // asks for none).
 static int tile_launch(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int c_dtype, int M,
                        int N, int K, int gated, float* work, long work_floats, int force, bool reduce,
-                       const float* partial, int P, float eps, hipStream_t stream, GatedPair pair = GatedPair{0.f, 1.f}) {
+                       const float* partial, int P, float eps, hipStream_t stream, GatedPair pair = GatedPair{0.f, 1.f},
+                       int square_relu = 0) {
     MV_REQUIRE(M > 0 && N > 0 && K > 0 && K % GT_KC == 0, "gemm_tile: K=%d must be a positive multiple of %d (M=%d, N=%d)",
                K, GT_KC, M, N);
     MV_REQUIRE(lda >= K && lda % 8 == 0, "gemm_tile: lda=%ld must be a multiple of 8 and at least K=%d", lda, K);
@@ -430,8 +433,10 @@ static int tile_launch(const void* A, long lda, const void* W, const void* bias,
                "gemm_tile: the work area holds %ld floats, %ld are needed", work_floats, (long)p.F * M * N);
     MV_REQUIRE(partial == nullptr || (p.F == 1 && P > 0 && eps > 0.f),
                "gemm_tile: rows without their norm's division need an unsplit K (F=%d), their sums (P=%d) and eps", p.F, P);
+    MV_REQUIRE(!square_relu || (p.F == 1 && !gated), "gemm_tile: the squared ReLU needs an unsplit K (F=%d) and no gated pair", p.F);
     TileArgs a{(const bf16*)A, lda, (const bf16*)W, (const bf16*)bias, C, ldc, c_dtype == MV_F32, p.F > 1 ? work : nullptr,
-               M, N, K, p.F, p.chunks_per_split, p.tiles_m, p.tiles_n, gated ? N / 2 : 0, partial, P, eps, pair};
+               M, N, K, p.F, p.chunks_per_split, p.tiles_m, p.tiles_n, gated ? N / 2 : 0, partial, P, eps, pair,
+               square_relu};
     const dim3 grid((unsigned)((long)p.tiles_m * p.tiles_n * p.F));
     // rings: 128 x 128 tiles 2 stages of 32 KB with two workgroups a compute unit, or 4 with one;
     // 64 x 128 and 128 x 64 3 stages of 24 KB, 64 x 64 4 stages of 16 KB, two workgroups a unit
@@ -455,11 +460,12 @@ static int tile_launch(const void* A, long lda, const void* W, const void* bias,
     return 0;
 }
 
+// square_relu (K not split: mv_gemm_tile_splits == 1): C = max(., 0)^2
 extern "C" int mv_gemm_tile(const void* A, long lda, const void* W, const void* bias, void* C, long ldc, int c_dtype,
                             int M, int N, int K, int gated, float* work, long work_floats, int force, float limit,
-                            float slope, hipStream_t stream) {
+                            float slope, int square_relu, hipStream_t stream) {
     return tile_launch(A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, true, nullptr, 0, 0.f,
-                       stream, GatedPair{limit, slope});
+                       stream, GatedPair{limit, slope}, square_relu);
 }
 
 // The same for rows that a product in front left weighted but not yet divided by their root mean

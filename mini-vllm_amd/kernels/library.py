@@ -239,9 +239,9 @@ _OPTIONAL_SIGNATURES = {
     "mv_device_compute_units": (c_int, []),
     "mv_gemm_tile_workspace": (c_long, [c_int, c_int, c_int, c_int, c_int]),
     "mv_gemm_tile_splits": (c_int, [c_int, c_int, c_int, c_int, c_int]),
-    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, limit, slope, stream
+    # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, work, work_floats, force, limit, slope, square_relu, stream
     "mv_gemm_tile": (c_int, [c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_long, c_int, c_int, c_int, c_int, c_int,
-                             c_void_p, c_long, c_int, c_float, c_float, c_void_p]),
+                             c_void_p, c_long, c_int, c_float, c_float, c_int, c_void_p]),
     # A, lda, W, M, N, K, work, work_floats, force, stream
     "mv_gemm_tile_sums": (c_int, [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_int, c_void_p]),
     # A, lda, W, bias, C, ldc, c_dtype, M, N, K, gated, partial, P, eps, limit, slope, stream

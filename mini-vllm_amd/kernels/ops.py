@@ -2112,8 +2112,8 @@ class Ops:
 
     # ------------------------------------------------------------------------------------
     def gemm_squared_relu(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
-        """out = max(a @ w^T (+ bias), 0)^2, contiguous rows of the activation type; the weight-streaming kernel applies it to
-        its float sums, behind every other product it is a pass of its own."""
+        """out = max(a @ w^T (+ bias), 0)^2, contiguous rows of the activation type; the weight-streaming and the tiled
+        kernel apply it to their float sums (the tiled one where K is not split), behind every other product it is a pass of its own."""
         if self.gemm(a, w, out, bias, square_relu=True) is not _SQUARED:
             self.squared_relu(out)
 
@@ -2179,8 +2179,9 @@ class Ops:
                 pending = self._gemm_tile_sums(a, lda, w, bias, out, M, N, K)
                 if pending is not None:
                     return pending
-            if self.gemm_tile(a, w, out, bias):
-                return None
+            squares = square_relu and int(self.lib.dll.mv_gemm_tile_splits(M, N, K, 0, 0)) == 1
+            if self.gemm_tile(a, w, out, bias, square_relu=squares):
+                return _SQUARED if squares else None
         if fast and K % 32 == 0 and lda % 8 == 0 and a.data_ptr() % 16 == 0 and self.lib.has("mv_gemm_skinny"):
             done = self._gemm_mid(a, lda, w, bias, out, ldc, M, N, K, swiglu=False,
                                   defer_sum=defer_sum and out.dtype == self.dtype and out.is_contiguous())
@@ -2363,9 +2364,9 @@ class Ops:
         return pending
 
     def gemm_tile(self, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Optional[torch.Tensor] = None,
-                  gated: bool = False, force: int = 0, limit: float = 0.0, slope: float = 1.0) -> bool:
+                  gated: bool = False, force: int = 0, limit: float = 0.0, slope: float = 1.0, square_relu: bool = False) -> bool:
         """out[M, N] = a @ w^T (+ bias), or with ``gated`` out[M, N / 2] = silu(a Wg^T) * (a Wu^T), by the
-        engine's tiled MFMA product for many rows. False, with nothing done, when the shape is not taken.
+        engine's tiled MFMA product for many rows (``square_relu``: max(., 0)^2 of it, where K is not split). False, with nothing done, when the shape is not taken.
         ``force`` fixes the tile and the split of K (measurements)."""
         if not (self.use_fast_kernels and self.lib.has("mv_gemm_tile")):
             return False
@@ -2394,7 +2395,7 @@ class Ops:
         self._note("mv_gemm_tile", self._size(a, w, out) + 8 * need, 2 * M * N * K)
         self.lib.call("mv_gemm_tile", a.data_ptr(), a.stride(0) if M > 1 else K, w.data_ptr(), _ptr(bias), out.data_ptr(),
                       out.stride(0) if M > 1 else n_out, _CODES[out.dtype], M, N, K, int(gated), _ptr(work),
-                      0 if work is None else work.numel(), force, float(limit), float(slope), self._stream())
+                      0 if work is None else work.numel(), force, float(limit), float(slope), int(square_relu), self._stream())
         return True
 
     @staticmethod

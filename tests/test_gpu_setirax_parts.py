@@ -580,19 +580,26 @@ def test_recurrent_unit_constants_by_hand():
     (torch.float32, 50, 30, 7), (torch.float32, 64, 96, 65), (torch.bfloat16, 50, 30, 9), (torch.bfloat16, 64, 96, 1), (torch.bfloat16, 64, 96, 300),
     (torch.bfloat16, 192, 256, 40), (torch.bfloat16, 1024, 4608, 1), (torch.bfloat16, 1024, 4608, 8), (torch.bfloat16, 1024, 4608, 16),
     (torch.bfloat16, 1024, 4608, 64), (torch.bfloat16, 1024, 4608, 200), (torch.bfloat16, 2048, 3072, 20), (torch.bfloat16, 1024, 4608, 2000),
-    (torch.bfloat16, 4096, 4608, 8), (torch.bfloat16, 4096, 4608, 64)])
+    (torch.bfloat16, 4096, 4608, 8), (torch.bfloat16, 4096, 4608, 64), (torch.bfloat16, 4096, 18432, 8)])
 @pytest.mark.parametrize("bias", [True, False])
 def test_squared_relu(dtype, hid, ff, rows, bias):
+    """... which the weight-streaming and the tiled product apply themselves, the latter where it does not split K."""
     from minivllm_amd.parts.mlp import SquaredReLU, SquaredReLUSpec
     rt = runtime(dtype)
     g = torch.Generator().manual_seed(hid + ff)
-    w = {"up": torch.randn(ff, hid, generator=g) / hid ** 0.5, "down": torch.randn(hid, ff, generator=g) / ff ** 0.5,
-         "up.b": 0.8 * torch.randn(ff, generator=g), "down.b": 0.8 * torch.randn(hid, generator=g)}
+    some = torch.randn(min(ff, 2048), hid, generator=g).repeat(-(-ff // 2048), 1)[:ff]          # (many rows: the same ones again)
+    w = {"up": some / hid ** 0.5, "down": torch.randn(hid, ff, generator=g) / ff ** 0.5, "up.b": 0.8 * torch.randn(ff, generator=g), "down.b": 0.8 * torch.randn(hid, generator=g)}
     w = {k: (v if bias or not k.endswith(".b") else 0 * v).to(torch.bfloat16) for k, v in w.items()}
     part = SquaredReLU(SquaredReLUSpec(hidden_size=hid, intermediate_size=ff, bias=bias),
                        {k.replace(".b", "_bias"): v.to(DEV) for k, v in w.items() if bias or not k.endswith(".b")}, rt)
     x = torch.randn(rows, hid, generator=torch.Generator().manual_seed(rows)).to(dtype)
+    rt.ops.ledger = []
     y = finished(part.forward(x.to(DEV), None))
+    ran, rt.ops.ledger = [e[0] for e in rt.ops.ledger], None
+    fused = ran[0] == "mv_gemm_skinny" or (ran[0] == "mv_gemm_tile" and rt.ops.lib.dll.mv_gemm_tile_splits(rows, ff, hid, 0, 0) == 1)
+    assert ("mv_squared_relu" in ran) != fused, ran
+    if ff == 18432:
+        assert ran[0] == "mv_gemm_tile" and fused, ran
     want = plain.feed_forward(x.double(), {k: v.double() for k, v in w.items()}, "")
     close(y, want, 1e-5 if dtype == torch.float32 else 1.2e-2, f"{rows} rows")
 
