@@ -272,8 +272,8 @@ def test_long_prompt(tmp_path, dtype):
     """A prompt of 1,100 tokens through sizes that the MFMA kernels serve, one softmax layer without a window: whole, and the
     last 40 tokens one by one behind a prompt fed in two portions. A token of the first page is repeated at the end."""
     cfg = model(400, 128, 1e-6, 20.0, [
-        latent(6, 64, 64, 96, 0.3, None, dense(256)),
-        parallel((6, 3, 64, 64, 0.3, 25.0, 200, 4, (64, 1e5, (8.0, 1.0, 4.0, 512.0))), (3, 64, 64, 16.0, 24), dense(128)),
+        latent(6, 32, 64, 160, 0.3, None, dense(256)),
+        parallel((8, 2, 64, 64, 0.3, 25.0, 200, 3, (32, 1e5, (8.0, 1.0, 4.0, 512.0))), (3, 64, 64, 16.0, 24), dense(128)),
         unit(96, 3, 4, None)])
     cfg["layers"].append(dict(cfg["layers"][1], weights_of=1))
     weights = make_weights(cfg, seed=8)
